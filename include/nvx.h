@@ -46,8 +46,12 @@ typedef void* nvx_stream_t;
  *   9: nvx_boundary_norm can apply the convolution of a decode step in the same launch.
  *  17: several residual streams (`nvx_hyper_mix`), the real-gated recurrence (`nvx_rglru_scan`), a latent with a rotated key part
  *      (`nvx_latent_rope_prep`), the softmax router with groups (`nvx_moe_route_softmax`), `nvx_short_conv`; nvx_softcap_attn gained a
- *      sink and a gate per head. */
-#define NVX_ABI_VERSION 17
+ *      sink and a gate per head.
+ *  18: keys and values tied in one cached row (`nvx_tied_prep_store`), chunks of positions, a linear distance penalty and keys normed as
+ *      they are scored in nvx_softcap_attn; gated linear attention (`nvx_gla_scan`); nvx_mlstm_scan takes long portions in chunks; the
+ *      sigmoid router with groups (`nvx_moe_route_sigmoid`), `nvx_gelu_glu`, `nvx_residual_norm`, `nvx_embed_sum`; nvx_skinny_proj has a bias
+ *      and an output activation. */
+#define NVX_ABI_VERSION 18
 
 /* Library identification and diagnostics. */
 int nvx_abi_version(void);
@@ -517,6 +521,13 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     N (slots, heads, dim), M (slots, heads) are continued and written back; all start from zero.  dim <= 512.  They are read
  *     through N_in / M_in: the same pointers where a head is one column block (nvx_scan_column_blocks(dim, vdim) == 1), copies
  *     taken before the launch otherwise (a column block that starts late must not read what the first one has written).
+ *     chunk > 0: the portions are cut into chunks of that many tokens (n_chunk_max: chunks of the longest portion) that run side by side
+ *     in two walks with a carry between them; ws takes n_seq * n_chunk_max * heads * (dim * (vdim + 1) + 3) floats, and N_in, M_in are
+ *     not read.
+ * nvx_gla_scan:  x[t] holds q at q_off, k at k_off (heads * dim) and v at v_off (heads * vdim); alpha (n_tok, heads * dim) float32, the
+ *     decay of every key channel at every token.  S <- diag(alpha[t]) S + k v^T;  out[t] = q_mul S^T q  (float32, heads * vdim; the
+ *     read sees the token's own write).  S (slots, heads, dim, vdim) is continued and written back, from zero at position 0.
+ *     dim <= 512.  chunk as for nvx_mlstm_scan; ws takes n_seq * n_chunk_max * heads * dim * (vdim + 1) floats.
  * nvx_delta_scan:  x[t] holds q at q_off, k at k_off (kv_heads * dim) and v at v_off (heads * vdim); ab[t] = [a | b] (float32, heads
  *     each).  q, k <- unit length per head (x / sqrt(sum x^2 + 1e-6)), q also times dim^(-1/2);  g = exp(-exp(a_log) softplus(a +
  *     dt_bias)), beta = sigmoid(b);  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  out[t] = S^T q.  Head h reads q/k head
@@ -535,10 +546,15 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     turned over all of vdim by positions[t] * vfreq[m] in the same pair layout.  q_out[t], k_cache[slots[t]], v_cache[slots[t]]
  *     take the results; a negative slot stores no key or value.  vcs_out (n_tok, vdim) float32, if given with vfreq, receives every
  *     token's cos | sin (vdim / 2 each) of positions[t] * vfreq[m]: the table nvx_softcap_attn turns its read-out back with.
+ * nvx_tied_prep_store:  heads whose values are their keys as projected.  x[t] holds q at q_off (heads * dim) and k at k_off (kv_heads *
+ *     dim).  q_out[t] = q / rms(q) * q_w * k_w per head (q_w, k_w: dim entries shared by the heads); k_cache[slots[t]] = k as it is,
+ *     k_rn[slots[t]] (kv_heads float32) = 1 / rms(k) per head; a negative slot stores nothing.  nvx_softcap_attn with k_rn and the one
+ *     cache as keys and values then scores the normed keys and reads the raw ones.
  * nvx_softcap_attn:  token t of sequence b attends over the rows at slots kv_indices[kv_start[b] + j], j <= kv_len[b] - q_len[b] +
- *     (t - qo_indptr[b]) (and, with window > 0, only the last `window` of them: itself and the window - 1 before it):
- *     s_j = scale * q . k_j,  s_j <- cap tanh(s_j / cap) (cap > 0),  s_j <- s_j - r1[h] ln(1 + r2[h] (i - j)) (r1, r2 != null; i the
- *     query's position),  out = softmax(s) V; with vcs ((n_tok, vdim) float32: each query token's cos | sin, as nvx_attn_prep_store
+ *     (t - qo_indptr[b]) (and, with window > 0, only the last `window` of them: itself and the window - 1 before it; with
+ *     chunk > 0 only those of its own chunk of positions: i / chunk == j / chunk):
+ *     s_j = scale * q . k_j (k_rn != null, (slots, kv_heads) float32: times k_rn of the key's slot and head),  s_j <- cap tanh(s_j / cap) (cap > 0),  s_j <- s_j - r1[h] ln(1 + r2[h] (i - j)) (r1, r2 != null; i the
+ *     query's position),  s_j <- s_j - slopes[h] (i - j) (slopes != null),  out = softmax(s) V; with vcs ((n_tok, vdim) float32: each query token's cos | sin, as nvx_attn_prep_store
  *     hands them out) the pairs of out are turned back by those angles (the counterpart of rotated values), with gate out is multiplied by
  *     sigmoid(gate[t]) (same layout as out, or with gate_per_head one number per head: gate[t][h]).  With sink != 0 the softmax's sum
  *     has one more term exp(sink_score) that carries no value: p_j = exp(s_j) / (exp(sink_score) + sum exp(s)).  Query head h reads
@@ -586,8 +602,18 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     w_kv | key part turned the same way | zeros]; gate[t][h] = sigmoid(pre-activation), float32.
  * nvx_embed_scale:  x[t] = table[ids[t]] * scale (float32), h[t] the same in the table's format (h may be null).
  * nvx_tanh_cap:  out[i] = cap tanh(in[i] / cap) in float32 (cap <= 0: a copy).
- * nvx_skinny_proj:  out[t][n] = sum_k w[n][k] * f(x[t][k]) in float32, f = identity (in_act 0) or tanh (1); w float32 (n_out,
- *     k_in), x in the format `fmt`.  Meant for few outputs (gate and router logits) or few inputs (the second half of a low-rank
+ * nvx_residual_norm:  v = x_in[t] (+ y[t]) (+ y2[t]) (format `fmt`) (+ add[t]) (+ bias) (float32); x_out[t] = v (x_in may be x_out);
+ *     h null: no more; split 0: h[t] = v / rms(v) * w;  split 1: h[t] = [hi | lo] (2 * width), hi v rounded to the format and lo what
+ *     that lost.  width <= 15360.
+ * nvx_embed_sum:  x[t] = table[ids[t]] (+ pair[r]) (+ pos_table[positions[t]]) in float32, then h as for nvx_residual_norm.  r = (previous
+ *     id * mul_prev + id * mul_cur) mod buckets, and `buckets` (pair has buckets + 1 rows) for a sequence's first token.  prev_id (slots)
+ *     keeps a sequence's last id between steps (its bits in a float32 word); a row without a slot reads and writes none.
+ * nvx_moe_route_sigmoid:  score = sigmoid(logit), choice score = score + correction[e]; n_groups > 1: the experts form that many equal
+ *     groups of neighbours, a group counts as the sum of its two largest choice scores, and only experts of the keep_groups best
+ *     groups can be chosen; the `top` largest choice scores are taken (ties: the lower id), wts = score * w_scale.  n_exp <= 1024.
+ * nvx_gelu_glu:  y[r][j] = gelu_tanh(gu[r][j]) * gu[r][ff + j].
+ * nvx_skinny_proj:  out[t][n] = g(sum_k w[n][k] * f(x[t][k]) + bias[n]) in float32, f = identity (in_act 0) or tanh (1), g = identity
+ *     (out_act 0) or sigmoid(.)^power (1); w float32 (n_out, k_in), bias float32 or null, x in the format `fmt`.  Meant for few outputs (gate and router logits) or few inputs (the second half of a low-rank
  *     map); one fixed summation order, no workspace. */
 int nvx_gated_residual_norm(const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, const float* w_y,
                             const float* w_y2, const void* gate, int64_t gate_stride, const float* gate_bias, int fmt,
@@ -620,7 +646,11 @@ int nvx_mlstm_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int6
                    const float* gate_bias, float cap, float* S, const float* N_in, const float* M_in, float* N, float* M,
                    int64_t n_slots, const int32_t* qo_indptr,
                    const int64_t* pos0, const int32_t* state_slot, float* out, int64_t n_tok, int64_t n_seq, int64_t heads,
-                   int64_t dim, int64_t vdim, nvx_stream_t stream);
+                   int64_t dim, int64_t vdim, int64_t chunk, int64_t n_chunk_max, float* ws, nvx_stream_t stream);
+int nvx_gla_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, float q_mul, const float* alpha,
+                 float* S, int64_t n_slots, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* out,
+                 int64_t n_tok, int64_t n_seq, int64_t heads, int64_t dim, int64_t vdim, int64_t chunk, int64_t n_chunk_max, float* ws,
+                 nvx_stream_t stream);
 int nvx_delta_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, const float* ab,
                    const float* a_log, const float* dt_bias, float* S, int64_t n_slots, const int32_t* qo_indptr,
                    const int64_t* pos0, const int32_t* state_slot, float* out, int64_t n_tok, int64_t n_seq, int64_t heads,
@@ -636,9 +666,12 @@ int nvx_rope_vnorm_store(const void* x, int64_t x_stride, int fmt, const int64_t
 int nvx_softcap_attn(const void* q, const void* k_cache, const void* v_cache, int fmt, const int32_t* kv_indices,
                      const int64_t* kv_start, const int32_t* kv_len, const int32_t* qo_indptr, const int32_t* tok_seq,
                      float scale, float cap, void* out, int64_t n_tok, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
-                     int n_split, float* part, int64_t window, const float* r1, const float* r2, const float* vcs,
-                     int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
+                     int n_split, float* part, int64_t window, int64_t chunk, const float* r1, const float* r2, const float* slopes,
+                     const float* k_rn, const float* vcs, int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
                      int64_t n_seq, int matrix_cores, nvx_stream_t stream);
+int nvx_tied_prep_store(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, const float* q_w, const float* k_w, float eps,
+                        const int64_t* slots, void* q_out, void* k_cache, float* k_rn, int64_t n_slots, int64_t n_tok, int64_t heads,
+                        int64_t kv_heads, int64_t dim, nvx_stream_t stream);
 int nvx_softcap_attn_tile_fits(int fmt, int64_t dim, int64_t vdim, int turned_halves);
 int nvx_attn_prep_store(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off,
                         const int64_t* positions, const float* q_w, const float* k_w, int norm_mode, float eps, const double* freq,
@@ -670,8 +703,18 @@ int nvx_moe_glu(const void* gu, int fmt, float limit, float alpha, float shift, 
                 nvx_stream_t stream);
 int nvx_moe_gather_rows(const void* ys, int fmt, const int64_t* dst, const float* wts, int64_t top, void* out, int64_t n_tok,
                         int64_t width, nvx_stream_t stream);
-int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const float* w, int in_act, float* out, int64_t n_tok,
-                    int64_t n_out, int64_t k_in, nvx_stream_t stream);
+int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const float* w, int in_act, const float* bias, int out_act, float power,
+                    float* out, int64_t n_tok, int64_t n_out, int64_t k_in, nvx_stream_t stream);
+int nvx_residual_norm(const float* x_in, const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, const float* add,
+                      const float* bias, int fmt, float* x_out, const float* w, float eps, int split, void* h, int64_t n_tok, int64_t width,
+                      nvx_stream_t stream);
+int nvx_embed_sum(const int64_t* ids, const void* table, int fmt, int64_t vocab, const void* pair, int64_t buckets, int64_t mul_prev,
+                  int64_t mul_cur, float* prev_id, int64_t n_slots, const void* pos_table, int64_t n_pos, const int64_t* positions,
+                  const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* x, const float* w,
+                  float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width, nvx_stream_t stream);
+int nvx_moe_route_sigmoid(const float* logits, const float* correction, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups,
+                          int64_t keep_groups, float w_scale, int32_t* idx, float* wts, nvx_stream_t stream);
+int nvx_gelu_glu(const void* gu, int fmt, void* y, int64_t rows, int64_t ff, nvx_stream_t stream);
 
 #ifdef __cplusplus
 }

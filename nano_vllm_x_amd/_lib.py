@@ -100,17 +100,17 @@ SIGNATURES = {
     "nvx_token_shift_mix": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
                                      _c_i64, _c_vp]),
     "nvx_scan_column_blocks": (_c_i64, [_c_i64, _c_i64]),
-    "nvx_mlstm_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp,
-                                _c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_mlstm_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp,
+                                _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
     "nvx_delta_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp,
                                 _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_rwkv_scan": (_c_i32, [_c_vp, _c_vp, _c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64,
                                _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_rope_vnorm_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_f32, _c_i32, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
                                       _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
-    "nvx_softcap_attn": (_c_i32, [_c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64,
-                                  _c_i64, _c_i64, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_i64, _c_i32, _c_i32, _c_f32, _c_i64,
-                                  _c_i32, _c_vp]),
+    "nvx_softcap_attn": (_c_i32, [_c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64,
+                                  _c_i64, _c_i64, _c_i64, _c_i32, _c_vp, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i32, _c_vp,
+                                  _c_i64, _c_i32, _c_i32, _c_f32, _c_i64, _c_i32, _c_vp]),
     "nvx_softcap_attn_tile_fits": (_c_i32, [_c_i32, _c_i64, _c_i64, _c_i32]),
     "nvx_attn_prep_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_i32, _c_f32, _c_vp, _c_i32, _c_i32,
                                      _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
@@ -138,7 +138,17 @@ SIGNATURES = {
     "nvx_hyper_mix": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_i64,
                                _c_i64, _c_i64, _c_vp]),
     "nvx_moe_route_softmax": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_vp]),
-    "nvx_skinny_proj": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_gla_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp,
+                              _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
+    "nvx_tied_prep_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64,
+                                     _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_residual_norm": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_f32, _c_i32, _c_vp, _c_i64,
+                                   _c_i64, _c_vp]),
+    "nvx_embed_sum": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_i64, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp,
+                               _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_i32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_moe_route_sigmoid": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_vp]),
+    "nvx_gelu_glu": (_c_i32, [_c_vp, _c_i32, _c_vp, _c_i64, _c_i64, _c_vp]),
+    "nvx_skinny_proj": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
 }
 
 _lib = None

@@ -152,6 +152,9 @@ class Engine(EngineCore):
             kv_cache_size = self.model_runner.profile_kv_cache_size(gpu_memory_utilization)
         self.kv_cache_size = kv_cache_size
         self.model_runner.initialize_kv_cache(kv_cache_size)
+        positions = getattr(self.model_runner.hf_config, "max_positions", None)
+        if positions is not None:      # a table of learned positions ends somewhere: no sequence may run past it
+            context_len, stop_at_context_len = min(context_len, positions), True
         super().__init__(kv_cache_size=kv_cache_size, max_bs=max_bs, context_len=context_len, prefix_reuse=prefix_reuse,
                          max_prefill_tokens=max_prefill_tokens, stop_at_context_len=stop_at_context_len,
                          chunked_prefill=chunked_prefill, state_slots=self.model_runner.state_slots)

@@ -58,20 +58,24 @@ class KVCachePool:
 class LatentCachePool:
     """Cache of layers that keep rows per token outside the K/V pool: ONE latent vector (latent attention), or a key row and a
     value row of sizes of their own (attention whose key and value sizes differ from layer to layer).  `ranks`: name ->
-    elements per token; per name a tensor (tokens, rank) in the activations' format.  Slot ids are the same token slots the
+    elements per token, or (elements, dtype) for a row in a format of its own (numbers that stay float32); per name a tensor
+    (tokens, rank), in the activations' format otherwise.  Slot ids are the same token slots the
     allocator below hands out, so a sequence's slot list serves every layer, whatever its rank."""
 
     def __init__(self, dtype: torch.dtype, device: torch.device, num_tokens: int, ranks: dict):
         self.dtype, self.device, self.num_tokens = dtype, device, num_tokens
         # zero-filled for the same reason as the K/V pool: a masked key must not bring NaN from stale memory
-        self.latents = {layer: torch.zeros((num_tokens, rank), dtype=dtype, device=device) for layer, rank in ranks.items()}
+        self.latents = {}
+        for layer, rank in ranks.items():
+            n, own = rank if isinstance(rank, tuple) else (rank, dtype)
+            self.latents[layer] = torch.zeros((num_tokens, n), dtype=own, device=device)
 
     def get(self, layer: int) -> torch.Tensor:
         return self.latents[layer]
 
     @staticmethod
     def bytes_per_token(ranks: dict, dtype: torch.dtype) -> int:
-        return sum(ranks.values()) * dtype.itemsize
+        return sum(r[0] * r[1].itemsize if isinstance(r, tuple) else r * dtype.itemsize for r in ranks.values())
 
 
 class RecurrentStatePool:

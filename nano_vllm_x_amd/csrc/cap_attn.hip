@@ -5,8 +5,11 @@
 //   - nvx_rope_vnorm_store: after the fused q|k|v projection: rotate q and k, norm v, scatter k and v into the caches;
 //   - nvx_attn_prep_store: the same place for heads with a query/key RMS norm (per head, or over all heads of a row at once), a
 //     rotation in either pair layout, and values that are themselves rotated by their position before they are cached;
+//   - nvx_tied_prep_store: the same place for heads whose values ARE their keys as projected: the row is cached once, the key norm's
+//     reciprocal root mean square beside it, and the key norm's weight goes into the queries;
 //   - nvx_softcap_attn: the attention itself; scores, maxima, exponentials and sums are float32 in every format.  Optional: a
-//     sliding window, a logarithmic distance penalty per head, a sink (one more term in the softmax's sum, with a score of its
+//     sliding window or chunks of positions (a token sees its own chunk only), a logarithmic or a linear distance penalty per head, keys
+//     that are cached as projected and normed as they are scored (tied keys and values: one row per token serves as both), a sink (one more term in the softmax's sum, with a score of its
 //     own and no value), the read-out turned back by the query's position (the counterpart of rotated values) and multiplied by
 //     a sigmoid gate (one per element, or one per head).
 #include "fmt_dev.h"
@@ -158,6 +161,42 @@ __global__ __launch_bounds__(256) void attn_prep_store_kernel(const A* __restric
     }
 }
 
+// One wave per (token, head), query heads first.  x[t] holds q at q_off (heads * dim) and k at k_off (kv_heads * dim).
+//   queries: q / rms(q) * q_w * k_w -> q_out;   keys: cached as they are in k_cache[slot], 1 / rms(k) in k_rn[slot] (kv_heads per slot).
+// A score q_hat . (k / rms(k) * k_w) is then (q_hat * k_w) . k times k_rn, and the cached row is the value too.
+template <typename A>
+__global__ __launch_bounds__(256) void tied_prep_store_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off,
+                                                             const float* __restrict__ q_w, const float* __restrict__ k_w, float eps,
+                                                             const int64_t* __restrict__ slots, A* __restrict__ q_out, A* __restrict__ k_cache,
+                                                             float* __restrict__ k_rn, int64_t n_rows, int heads, int kv_heads, int dim) {
+    const int64_t idx = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (idx >= n_rows) return;
+    const int lane = threadIdx.x & 63, per = heads + kv_heads;
+    const int64_t t = idx / per;
+    const int hd = (int)(idx % per);
+    const bool is_q = hd < heads;
+    const A* r = x + t * x_stride + (is_q ? q_off + hd * dim : k_off + (hd - heads) * dim);
+    float ss = 0.f;
+    for (int d = lane; d < dim; d += 64) { const float v = ld_f(r, d); ss += v * v; }
+    const float rn = 1.0f / sqrtf(wave_sum(ss) / (float)dim + eps);
+    if (is_q) {
+        A* o = q_out + (t * heads + hd) * dim;
+        for (int d = lane; d < dim; d += 64) st_f(o, d, ld_f(r, d) * rn * q_w[d] * k_w[d]);
+    } else {
+        const int64_t slot = slots[t];
+        if (slot < 0) return;
+        A* o = k_cache + (slot * kv_heads + (hd - heads)) * dim;
+        for (int d = lane; d < dim; d += 64) o[d] = r[d];
+        if (lane == 0) k_rn[slot * kv_heads + (hd - heads)] = rn;
+    }
+}
+
+// What limits the keys a token at `pos` sees from below: a window of `window` keys, chunks of `chunk` positions counted from 0 (neither: 0)
+__device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
+    if (window > 0) return pos - window + 1 > 0 ? pos - window + 1 : 0;
+    return chunk > 0 ? pos - pos % chunk : 0;
+}
+
 // The end of an attention read-out for one (token, head): `so` holds its vdim values in LDS (every thread of the workgroup has
 // passed a barrier since they were written).  With `turn` (the query token's cos | sin row, vdim / 2 each, as nvx_attn_prep_store
 // hands it out) the pairs are turned BACK by those angles (values were cached turned by their own positions, so the weighted sum
@@ -197,8 +236,9 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
                                                           const int32_t* __restrict__ kv_len, const int32_t* __restrict__ qo_indptr,
                                                           const int32_t* __restrict__ tok_seq, float scale, float cap, A* __restrict__ out,
                                                           int heads, int kv_heads, int dim, int vdim, int vec_v_ok, int n_split,
-                                                          float* __restrict__ part, int window, const float* __restrict__ r1,
-                                                          const float* __restrict__ r2, const float* __restrict__ vcs, int v_inter,
+                                                          float* __restrict__ part, int window, int chunk, const float* __restrict__ r1,
+                                                          const float* __restrict__ r2, const float* __restrict__ slopes,
+                                                          const float* __restrict__ k_rn, const float* __restrict__ vcs, int v_inter,
                                                           const A* __restrict__ gate, int64_t gate_stride, int gate_one, int sink,
                                                           float sink_score) {
     extern __shared__ float sm[];
@@ -211,9 +251,8 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
     const int64_t q0 = qo_indptr ? qo_indptr[b] : b;
     const int64_t q_n = qo_indptr ? qo_indptr[b + 1] - q0 : 1;
     const int visible = kv_len[b] - (int)(q_n - 1 - (t - q0));
-    // a window of w keys: the token itself and the w - 1 before it
-    const int first = (window > 0 && visible > window) ? visible - window : 0;
-    const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f;
+    const int first = first_seen(visible - 1, window, chunk);
+    const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f, slope = slopes ? slopes[hd] : 0.f;
     const int kvh = hd / (heads / kv_heads);
     const int32_t* slots = kv_indices + kv_start[b];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -247,7 +286,9 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
                 for (int d = 0; d < dim; ++d) dot += sq[d] * ld_f(kr, d);
             }
             s = dot * scale;
+            if (k_rn) s *= k_rn[slot * kv_heads + kvh];
             if (cap > 0.f) s = cap * tanhf(s / cap);
+            if (slopes) s -= slope * (float)(visible - 1 - j);
             if (r1) s -= pen_a * log1pf(pen_b * (float)(visible - 1 - j));      // the penalty grows with the distance to the query
         }
         const float m_new = fmaxf(m, wave_max(s));
@@ -371,11 +412,13 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
                                                                const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
                                                                const int32_t* __restrict__ kv_len, const int32_t* __restrict__ qo_indptr, int n_seq,
                                                                float scale, float cap, A* __restrict__ out, int heads, int kv_heads, int window,
-                                                               const float* __restrict__ r1, const float* __restrict__ r2,
+                                                               int chunk, const float* __restrict__ r1, const float* __restrict__ r2,
+                                                               const float* __restrict__ slopes, const float* __restrict__ k_rn,
                                                                const float* __restrict__ vcs, int v_inter, const A* __restrict__ gate,
                                                                int64_t gate_stride, int gate_one, int sink, float sink_score) {
     constexpr int dim = DS * 32, vdim = VT * 16;
     __shared__ A vt_lds[vdim * VT_ROW];
+    __shared__ __align__(16) float rn_lds[TILE_K];
     __shared__ int where[2];
     if (threadIdx.x == 0) {          // which sequence and which block of its tokens: sequences take ceil(tokens / 64) workgroups each
         // Workgroups start in the order of their numbers, and a block late in a portion has the most keys to walk: the count runs
@@ -398,14 +441,14 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     const int rows_here = q_n - qs < TILE_Q ? q_n - qs : TILE_Q;
     const int pos_first = kv_len[b] - q_n + qs;                 // position of the block's first query
     const int hi = pos_first + rows_here;                       // keys [lo, hi) are seen by some query of the block
-    const int lo = window > 0 && pos_first - window + 1 > 0 ? pos_first - window + 1 : 0;
+    const int lo = first_seen(pos_first, window, chunk);
     const int32_t* slots = kv_indices + kv_start[b];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
     const int row = wave * 16 + c;
     const bool row_on = row < rows_here;
     const int pos = pos_first + row;
     const int w_hi = pos_first + wave * 16 + 16 < hi ? pos_first + wave * 16 + 16 : hi;      // this wave's queries see [w_lo, w_hi)
-    const int w_lo = window > 0 && pos_first + wave * 16 - window + 1 > 0 ? pos_first + wave * 16 - window + 1 : 0;
+    const int w_lo = first_seen(pos_first + wave * 16, window, chunk), my_lo = first_seen(pos, window, chunk);
     const bool wave_on = wave * 16 < rows_here;
     const int64_t k_row = (int64_t)kv_heads * dim, v_row = (int64_t)kv_heads * vdim;
     nvx_u32x4 qb[DS];
@@ -414,7 +457,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
 #pragma unroll
         for (int s = 0; s < DS; ++s) qb[s] = *reinterpret_cast<const nvx_u32x4*>(qr + 32 * s);
     }
-    const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f;
+    const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f, slope2 = slopes ? slopes[hd] * 1.4426950408889634f : 0.f;
     nvx_f32x4 acc[VT];
 #pragma unroll
     for (int t = 0; t < VT; ++t) acc[t] = nvx_f32x4{0.f, 0.f, 0.f, 0.f};
@@ -428,6 +471,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     nvx_u32x4 kf[2][DS];
     vec8 vf[VPT];
     int k_slot[2], v_slot[VPT];
+    float rn_next = 1.f;                                             // (threads 0 .. 31: of the key whose value piece 0 they fetch)
     auto fetch_slots = [&](int j0) {                                 // (a key past the end reads a real row and is masked)
 #pragma unroll
         for (int hh = 0; hh < 2; ++hh) { const int j = j0 + hh * 16 + c; k_slot[hh] = slots[j < hi ? j : hi - 1]; }
@@ -443,6 +487,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
         }
     };
     auto fetch_value_rows = [&]() {
+        if (k_rn && threadIdx.x < TILE_K) rn_next = k_rn[(int64_t)v_slot[0] * kv_heads + kvh];
 #pragma unroll
         for (int u = 0; u < VPT; ++u) {
             const int i = threadIdx.x + 256 * u;
@@ -451,7 +496,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     };
     // Scores live in the log2 domain (the hardware's exponential and logarithm are base 2): s2 = log2(e) * score.
     //   no cap:  s2 = acc * (scale log2 e);   cap:  tanh(x) = 1 - 2 / (e^(2x) + 1), so s2 = (cap log2 e) (1 - 2 / (2^(acc * 2 scale log2 e / cap) + 1));
-    //   penalty: s2 -= r1 log2(1 + r2 distance).
+    //   penalty: s2 -= r1 log2(1 + r2 distance);   linear penalty: s2 -= (slope log2 e) distance;   keys normed here: acc times the key's 1 / rms.
     constexpr float LOG2E = 1.4426950408889634f;
     const float k_lin = cap > 0.f ? 2.0f * scale * LOG2E / cap : scale * LOG2E, k_cap = cap * LOG2E;
     const int j_begin = lo & ~(TILE_K - 1);
@@ -464,6 +509,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     const bool rows_full = wave * 16 + 16 <= rows_here;
     for (int j0 = j_begin; j0 < hi; j0 += TILE_K) {
         __syncthreads();                                             // the tile before has been read by all waves
+        if (k_rn && threadIdx.x < TILE_K) rn_lds[threadIdx.x] = rn_next;
 #pragma unroll
         for (int u = 0; u < VPT; ++u) {
             const int i = threadIdx.x + 256 * u;
@@ -495,17 +541,19 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
         if (j0 + 2 * TILE_K < hi) fetch_slots(j0 + 2 * TILE_K);
         if (!seen) continue;
         // every query of the wave sees every key of the tile (most tiles): no mask to work out
-        const bool full = rows_full && j0 + TILE_K - 1 <= q_lo && (window <= 0 || j0 > q_hi - window);
+        const bool full = rows_full && j0 + TILE_K - 1 <= q_lo && j0 >= first_seen(q_hi, window, chunk);
         float sv[8], mx = -INFINITY;
 #pragma unroll
         for (int hh = 0; hh < 2; ++hh) {
+            if (k_rn) sacc[hh] *= *reinterpret_cast<const nvx_f32x4*>(rn_lds + hh * 16 + 4 * g);
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
                 const int j = j0 + hh * 16 + 4 * g + r;
                 float sc = sacc[hh][r] * k_lin;
                 if (cap > 0.f) sc = k_cap - 2.0f * k_cap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc) + 1.0f);
                 if (r1) sc -= pen_a * __builtin_amdgcn_logf(1.0f + pen_b * (float)(pos - j));
-                if (!full && !(row_on && j <= pos && (window <= 0 || j > pos - window))) sc = -INFINITY;
+                if (slopes) sc -= slope2 * (float)(pos - j);
+                if (!full && !(row_on && j <= pos && j >= my_lo)) sc = -INFINITY;
                 sv[hh * 4 + r] = sc;
                 mx = fmaxf(mx, sc);
             }
@@ -689,11 +737,28 @@ extern "C" int nvx_attn_prep_store(const void* x, int64_t x_stride, int fmt, int
     return nvx_check_launch("nvx_attn_prep_store");
 }
 
+extern "C" int nvx_tied_prep_store(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, const float* q_w, const float* k_w,
+                                   float eps, const int64_t* slots, void* q_out, void* k_cache, float* k_rn, int64_t n_slots, int64_t n_tok,
+                                   int64_t heads, int64_t kv_heads, int64_t dim, nvx_stream_t stream) {
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_tied_prep_store: fmt must be 0, 1 or 2");
+    NVX_REQUIRE(n_tok >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && n_slots >= 0 && (heads + kv_heads) * dim < (1 << 30) &&
+                    n_tok * (heads + kv_heads) < (1ll << 32), NVX_EINVAL, "nvx_tied_prep_store: bad sizes");
+    NVX_REQUIRE(q_off >= 0 && k_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + kv_heads * dim, NVX_EINVAL,
+                "nvx_tied_prep_store: q or k lies outside a row");
+    if (n_tok == 0) return NVX_OK;
+    NVX_REQUIRE(x && q_w && k_w && slots && q_out && k_cache && k_rn, NVX_EINVAL, "nvx_tied_prep_store: null pointer");
+    const int64_t rows = n_tok * (heads + kv_heads);
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(tied_prep_store_kernel<A_>, dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, (hipStream_t)stream, (const A_*)x,
+                                         x_stride, (int)q_off, (int)k_off, q_w, k_w, eps, slots, (A_*)q_out, (A_*)k_cache, k_rn, rows, (int)heads,
+                                         (int)kv_heads, (int)dim));
+    return nvx_check_launch("nvx_tied_prep_store");
+}
+
 extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* v_cache, int fmt, const int32_t* kv_indices,
                                 const int64_t* kv_start, const int32_t* kv_len, const int32_t* qo_indptr, const int32_t* tok_seq,
                                 float scale, float cap, void* out, int64_t n_tok, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
-                                int n_split, float* part, int64_t window, const float* r1, const float* r2, const float* vcs,
-                                int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
+                                int n_split, float* part, int64_t window, int64_t chunk, const float* r1, const float* r2, const float* slopes,
+                                const float* k_rn, const float* vcs, int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
                                 int64_t n_seq, int matrix_cores, nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_softcap_attn: fmt must be 0, 1 or 2");
     NVX_REQUIRE(n_tok >= 0 && n_tok <= 65535 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && dim <= 4096 && vdim > 0 && vdim <= 512,
@@ -702,7 +767,8 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     NVX_REQUIRE(q && k_cache && v_cache && kv_indices && kv_start && kv_len && out, NVX_EINVAL, "nvx_softcap_attn: null pointer");
     NVX_REQUIRE((tok_seq != nullptr) == (qo_indptr != nullptr), NVX_EINVAL, "nvx_softcap_attn: tok_seq and qo_indptr go together");
     NVX_REQUIRE((r1 != nullptr) == (r2 != nullptr), NVX_EINVAL, "nvx_softcap_attn: the distance penalty takes both of its numbers per head");
-    NVX_REQUIRE(window >= 0 && window < (1ll << 31), NVX_EINVAL, "nvx_softcap_attn: bad window");
+    NVX_REQUIRE(window >= 0 && window < (1ll << 31) && chunk >= 0 && chunk < (1ll << 31) && (window == 0 || chunk == 0), NVX_EINVAL,
+                "nvx_softcap_attn: bad window or chunk (one of them at most)");
     NVX_REQUIRE(!vcs || (vdim % 2 == 0 && nvx_aligned16(vcs)), NVX_EINVAL, "nvx_softcap_attn: a read-out that is turned back has an even size");
     NVX_REQUIRE(!gate || gate_stride >= (gate_per_head ? heads : heads * vdim), NVX_EINVAL, "nvx_softcap_attn: row stride of the gate");
     // steps of many tokens in a 16-bit format, sizes the tile kernel is built for, 8-byte rows of the gate: the matrix cores
@@ -715,7 +781,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((softcap_attn_tile_kernel<typename tile_fmt<A_>::type, DS, VT>), tgrid, dim3(256), 0, (hipStream_t)stream, \
                                          (const typename tile_fmt<A_>::type*)q, (const typename tile_fmt<A_>::type*)k_cache,            \
                                          (const typename tile_fmt<A_>::type*)v_cache, kv_indices, kv_start, kv_len, qo_indptr, (int)n_seq, scale, \
-                                         cap, (typename tile_fmt<A_>::type*)out, (int)heads, (int)kv_heads, (int)window, r1, r2, vcs,    \
+                                         cap, (typename tile_fmt<A_>::type*)out, (int)heads, (int)kv_heads, (int)window, (int)chunk, r1, r2, slopes, k_rn, vcs, \
                                          v_interleaved, (const typename tile_fmt<A_>::type*)gate, gate_stride, gate_per_head, sink,   \
                                          sink_score))
 #define NVX_TILE_ATTN_V(DS)                                                       \
@@ -738,7 +804,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((softcap_attn_kernel<A_, EPL, VEC && sizeof(A_) == 2>), grid, dim3(256), lds, (hipStream_t)stream,     \
                                          (const A_*)q, (const A_*)k_cache, (const A_*)v_cache, kv_indices, kv_start, kv_len, qo_indptr,      \
                                          tok_seq, scale, cap, (A_*)out, (int)heads, (int)kv_heads, (int)dim, (int)vdim,       \
-                                         (int)nvx_aligned16(v_cache), n_split, part, (int)window, r1, r2, vcs, v_interleaved,   \
+                                         (int)nvx_aligned16(v_cache), n_split, part, (int)window, (int)chunk, r1, r2, slopes, k_rn, vcs, v_interleaved, \
                                          (const A_*)gate, gate_stride, gate_per_head, sink, sink_score))
 #define NVX_CAP_ATTN(EPL) do { if (vec) NVX_CAP_ATTN_V(EPL, true); else NVX_CAP_ATTN_V(EPL, false); } while (0)
     const bool vec = fmt != 2 && dim % 8 == 0 && nvx_aligned16(k_cache);

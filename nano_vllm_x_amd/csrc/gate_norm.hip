@@ -5,7 +5,10 @@
 //   - per-head RMS norm of a recurrence's or attention's read-out, times a weight, times an output gate;
 //   - stacks that norm a sublayer's OUTPUT instead of its input: the (weighted sum of one or two) results divided by its root
 //     mean square, times a weight (one number or one per channel), added to the stream, which the next sublayer reads as it is;
-//   - the two ends of such a stack: scaled embedding rows into the stream, and logits through cap * tanh(. / cap).
+//   - the two ends of such a stack: scaled embedding rows into the stream, and logits through cap * tanh(. / cap);
+//   - plain pre-normed stacks: one or two results (and further float32 terms) added to the stream and the next norm, in one launch,
+//     or the stream handed out as a hi + lo pair of 16-bit rows for a matrix product that must see more than 16 bits of it;
+//   - the embedding of such a stack: token row + row of a table of token pairs + learned position row, with that first norm.
 // Norms, gates and the stream are float32 in every activation format.
 #include "fmt_dev.h"
 
@@ -174,6 +177,126 @@ __global__ __launch_bounds__(256) void tanh_cap_kernel(const A* __restrict__ in,
     }
 }
 
+// The end of a row that waits in LDS (su, float32, written by this workgroup; a barrier lies in block256_sum, or is placed here):
+// nothing (h null), h = su / rms * w, or (split) h = [hi | lo], two rows of the activations' format whose sum is su to 16 bits and more.
+template <typename A>
+__device__ __forceinline__ void row_end(const float* su, float ss, float* red, const float* __restrict__ w, float eps, int split, A* __restrict__ h,
+                                        int64_t t, int width) {
+    if (!h) return;
+    if (split) {                                  // (every thread reads back the entries it wrote)
+        A* hr = h + t * 2 * (int64_t)width;
+        for (int c = threadIdx.x * 4; c < width; c += 1024) {
+            for (int i = c; i < c + 4 && i < width; ++i) {
+                const float v = su[i];
+                const A hi = (A)v;
+                hr[i] = hi;
+                hr[width + i] = (A)(v - (float)hi);
+            }
+        }
+        return;
+    }
+    const float rn = 1.0f / sqrtf(block256_sum(ss, red) / (float)width + eps);
+    A* hr = h + t * (int64_t)width;
+    for (int c = threadIdx.x * 4; c < width; c += 1024) {
+        if (c + 4 <= width && (width & 3) == 0) {
+            typedef A vec4 __attribute__((ext_vector_type(4)));
+            const nvx_f32x4 v = *reinterpret_cast<const nvx_f32x4*>(su + c), g = *reinterpret_cast<const nvx_f32x4*>(w + c);
+            vec4 o;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) o[i] = (A)(v[i] * rn * g[i]);
+            *reinterpret_cast<vec4*>(hr + c) = o;
+        } else {
+            for (int i = c; i < c + 4 && i < width; ++i) st_f(hr, i, su[i] * rn * w[i]);
+        }
+    }
+}
+
+// Per token t (one workgroup):  x_out[t] = x_in[t] (+ y[t]) (+ y2[t]) (+ add[t]) (+ bias);  then row_end of it.  V = 4: rows of all operands
+// start on borders of four elements and the width is a multiple of four.  x_in may be x_out.
+template <typename A, int V>
+__global__ __launch_bounds__(256) void residual_norm_kernel(const float* x_in, const A* __restrict__ y, int64_t y_stride, const A* __restrict__ y2,
+                                                           int64_t y2_stride, const float* __restrict__ add, const float* __restrict__ bias,
+                                                           float* x_out, const float* __restrict__ w, float eps, int split, A* __restrict__ h,
+                                                           int width) {
+    extern __shared__ __align__(16) float row_lds[];      // width
+    float* su = row_lds;
+    __shared__ float red[4];
+    typedef A veca __attribute__((ext_vector_type(V)));
+    typedef float vecf __attribute__((ext_vector_type(V)));
+    const int64_t t = blockIdx.x;
+    const int64_t row = t * (int64_t)width;
+    float ss = 0.f;
+    for (int c = threadIdx.x * V; c < width; c += 256 * V) {
+        vecf v = *reinterpret_cast<const vecf*>(x_in + row + c);
+        if (y) { const veca u = *reinterpret_cast<const veca*>(y + t * y_stride + c); for (int i = 0; i < V; ++i) v[i] += (float)u[i]; }
+        if (y2) { const veca u = *reinterpret_cast<const veca*>(y2 + t * y2_stride + c); for (int i = 0; i < V; ++i) v[i] += (float)u[i]; }
+        if (add) v += *reinterpret_cast<const vecf*>(add + row + c);
+        if (bias) v += *reinterpret_cast<const vecf*>(bias + c);
+        if (y || add || bias || x_out != x_in) *reinterpret_cast<vecf*>(x_out + row + c) = v;
+        *reinterpret_cast<vecf*>(su + c) = v;
+        for (int i = 0; i < V; ++i) ss += v[i] * v[i];
+    }
+    if (V == 1) __syncthreads();                  // (row_end takes four entries a thread)
+    row_end<A>(su, ss, red, w, eps, split, h, t, width);
+}
+
+// Per token t (one workgroup):  x[t] = table[ids[t]] (+ pair[r]) (+ pos_table[position]);  then row_end of it.
+//   r = (previous id * mul_prev + id * mul_cur) mod buckets, and the extra row `buckets` for a sequence's first token.  A token's
+//   predecessor is the step's own or, for the first token of a portion, the id that the sequence's state slot keeps (its bits in a
+//   float32 word).  The workgroup of a portion's first token reads that word before it replaces it by the portion's last id, and no
+//   other workgroup touches it.
+template <typename A>
+__global__ __launch_bounds__(256) void embed_sum_kernel(const int64_t* __restrict__ ids, const A* __restrict__ table, int64_t vocab,
+                                                       const A* __restrict__ pair, int64_t buckets, int64_t mul_prev, int64_t mul_cur,
+                                                       float* prev_id, const A* __restrict__ pos_table, int64_t n_pos,
+                                                       const int64_t* __restrict__ positions, const int32_t* __restrict__ tok_seq,
+                                                       const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
+                                                       const int32_t* __restrict__ state_slot, float* __restrict__ x, const float* __restrict__ w,
+                                                       float eps, int split, A* __restrict__ h, int width) {
+    extern __shared__ __align__(16) float row_lds[];      // width
+    float* su = row_lds;
+    __shared__ float red[4];
+    __shared__ int64_t pair_row;
+    const int64_t t = blockIdx.x;
+    int64_t id = ids[t];
+    id = id < 0 ? 0 : (id >= vocab ? vocab - 1 : id);
+    if (pair) {
+        if (threadIdx.x == 0) {
+            const int b = tok_seq ? tok_seq[t] : (int)t;
+            const SeqSpan s = seq_span(b, qo_indptr, pos0, state_slot);
+            int64_t prev = -1;                    // no predecessor: a sequence's first token (and a padding row)
+            if (t > s.q0) prev = ids[t - 1];
+            else if (s.slot >= 0) {
+                if (s.pos0 > 0) prev = __float_as_int(prev_id[s.slot]);
+                prev_id[s.slot] = __int_as_float((int)ids[s.q0 + s.n - 1]);
+            }
+            int64_t r = buckets;
+            if (prev >= 0) {
+                r = (prev * mul_prev + id * mul_cur) % buckets;
+                if (r < 0) r += buckets;
+            }
+            pair_row = r;
+        }
+        __syncthreads();
+    }
+    int64_t p = pos_table ? positions[t] : 0;
+    p = p < 0 ? 0 : (p >= n_pos ? n_pos - 1 : p);
+    const A* er = table + id * width;
+    const A* pr = pair ? pair + pair_row * width : nullptr;
+    const A* lr = pos_table ? pos_table + p * width : nullptr;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < width; c += 256) {
+        float v = ld_f(er, c);
+        if (pr) v += ld_f(pr, c);
+        if (lr) v += ld_f(lr, c);
+        x[t * (int64_t)width + c] = v;
+        su[c] = v;
+        ss += v * v;
+    }
+    __syncthreads();
+    row_end<A>(su, ss, red, w, eps, split, h, t, width);
+}
+
 // One wave per (token, head): out = o / rms(o) * w * gate, with gate = 1 (kind 0), sigmoid(z) (1) or z * sigmoid(z) (2) of
 // the gate pre-activations z (same layout as the output).  w has heads * vdim entries, or vdim shared by the heads.
 template <typename A>
@@ -201,14 +324,20 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
 
 
 // Projections onto FEW outputs or from FEW inputs, in float32: gate and router logits (outputs = heads or experts), the two
-// halves of a low-rank decay.  out[t][n] = sum_k W[n][k] * f(x[t][k]), f = identity or tanh; W float32 (n_out, k_in).  A
+// halves of a low-rank decay.  out[t][n] = g(sum_k W[n][k] * f(x[t][k]) + bias[n]), f = identity or tanh, g = identity or
+// sigmoid(.)^power (formed as exp(power * logsigmoid(.))); W float32 (n_out, k_in), bias float32 or null.  A
 // workgroup takes TOK tokens: their inputs wait in LDS as float32, every weight is read once for the TOK of them.  Wide
 // inputs: a wave per output, lanes over k.  Narrow inputs (k_in < 256): a thread per output.  No workspace, no atomics: the
 // sums have one order, and the launch can be captured.
+__device__ __forceinline__ float skinny_end(float z, const float* __restrict__ bias, int n, int out_act, float power) {
+    if (bias) z += bias[n];
+    return out_act == 1 ? expf(power * logsigmoid_f(z)) : z;
+}
+
 template <typename A, int TOK>
 __global__ __launch_bounds__(256) void skinny_proj_kernel(const A* __restrict__ x, int64_t x_stride, const float* __restrict__ w,
-                                                         int in_act, float* __restrict__ out, int64_t n_tok, int n_out, int k_in,
-                                                         int out_per_block) {
+                                                         int in_act, const float* __restrict__ bias, int out_act, float power,
+                                                         float* __restrict__ out, int64_t n_tok, int n_out, int k_in, int out_per_block) {
     extern __shared__ float xs[];      // TOK rows of k_in
     const int64_t t0 = (int64_t)blockIdx.x * TOK;
     const int nt = (int)(n_tok - t0 < TOK ? n_tok - t0 : TOK);
@@ -235,7 +364,7 @@ __global__ __launch_bounds__(256) void skinny_proj_kernel(const A* __restrict__ 
 #pragma unroll
             for (int tt = 0; tt < TOK; ++tt) {
                 const float sum = wave_sum(acc[tt]);
-                if (lane == 0 && tt < nt) out[(t0 + tt) * n_out + n] = sum;
+                if (lane == 0 && tt < nt) out[(t0 + tt) * n_out + n] = skinny_end(sum, bias, n, out_act, power);
             }
         }
     } else {
@@ -251,7 +380,7 @@ __global__ __launch_bounds__(256) void skinny_proj_kernel(const A* __restrict__ 
             }
 #pragma unroll
             for (int tt = 0; tt < TOK; ++tt)
-                if (tt < nt) out[(t0 + tt) * n_out + n] = acc[tt];
+                if (tt < nt) out[(t0 + tt) * n_out + n] = skinny_end(acc[tt], bias, n, out_act, power);
         }
     }
 }
@@ -260,9 +389,10 @@ __global__ __launch_bounds__(256) void skinny_proj_kernel(const A* __restrict__ 
 
 using namespace NVX_NS;
 
-extern "C" int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const float* w, int in_act, float* out, int64_t n_tok,
-                               int64_t n_out, int64_t k_in, nvx_stream_t stream) {
-    NVX_REQUIRE(fmt >= 0 && fmt <= 2 && (in_act == 0 || in_act == 1), NVX_EINVAL, "nvx_skinny_proj: fmt must be 0..2, in_act 0 or 1");
+extern "C" int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const float* w, int in_act, const float* bias, int out_act,
+                               float power, float* out, int64_t n_tok, int64_t n_out, int64_t k_in, nvx_stream_t stream) {
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2 && (in_act == 0 || in_act == 1) && (out_act == 0 || out_act == 1), NVX_EINVAL,
+                "nvx_skinny_proj: fmt must be 0..2, in_act and out_act 0 or 1");
     NVX_REQUIRE(n_tok >= 0 && n_out > 0 && n_out < (1 << 24) && k_in > 0 && k_in <= 12288 && x_stride >= k_in, NVX_EINVAL,
                 "nvx_skinny_proj: bad sizes (at most 12288 inputs)");
     if (n_tok == 0) return NVX_OK;
@@ -276,12 +406,12 @@ extern "C" int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const f
         const int64_t blocks = (n_tok + 3) / 4;
         NVX_REQUIRE(blocks < (1ll << 31), NVX_EINVAL, "nvx_skinny_proj: too many tokens");
         NVX_FMT_CALL(fmt, hipLaunchKernelGGL((skinny_proj_kernel<A_, 4>), dim3((unsigned)blocks, (unsigned)chunks), dim3(256),
-                                             (size_t)(4 * k_in) * sizeof(float), (hipStream_t)stream, (const A_*)x, x_stride, w, in_act, out, n_tok,
+                                             (size_t)(4 * k_in) * sizeof(float), (hipStream_t)stream, (const A_*)x, x_stride, w, in_act, bias, out_act, power, out, n_tok,
                                              (int)n_out, (int)k_in, opb));
     } else {
         NVX_REQUIRE(n_tok < (1ll << 31), NVX_EINVAL, "nvx_skinny_proj: too many tokens");
         NVX_FMT_CALL(fmt, hipLaunchKernelGGL((skinny_proj_kernel<A_, 1>), dim3((unsigned)n_tok, (unsigned)chunks), dim3(256),
-                                             (size_t)k_in * sizeof(float), (hipStream_t)stream, (const A_*)x, x_stride, w, in_act, out, n_tok,
+                                             (size_t)k_in * sizeof(float), (hipStream_t)stream, (const A_*)x, x_stride, w, in_act, bias, out_act, power, out, n_tok,
                                              (int)n_out, (int)k_in, opb));
     }
     return nvx_check_launch("nvx_skinny_proj");
@@ -370,6 +500,52 @@ extern "C" int nvx_embed_scale(const int64_t* ids, const void* table, int fmt, i
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL(embed_scale_kernel<A_>, dim3((unsigned)n_tok), dim3(256), 0, (hipStream_t)stream, ids, (const A_*)table, vocab,
                                          scale, x, (A_*)h, (int)width));
     return nvx_check_launch("nvx_embed_scale");
+}
+
+#define NVX_ROW_OK(name)                                                                                                               \
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, name ": fmt must be 0, 1 or 2");                                                     \
+    NVX_REQUIRE(n_tok >= 0 && n_tok < (1ll << 31) && width > 0, NVX_EINVAL, name ": bad sizes");                                       \
+    NVX_REQUIRE(width <= 15360, NVX_EUNSUPPORTED, name ": a row must fit LDS as float32 (width <= 15360)");                            \
+    NVX_REQUIRE(!h || split || w, NVX_EINVAL, name ": the norm needs its weight")
+
+extern "C" int nvx_residual_norm(const float* x_in, const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, const float* add,
+                                 const float* bias, int fmt, float* x_out, const float* w, float eps, int split, void* h, int64_t n_tok,
+                                 int64_t width, nvx_stream_t stream) {
+    NVX_ROW_OK("nvx_residual_norm");
+    if (n_tok == 0) return NVX_OK;
+    NVX_REQUIRE(x_in && x_out && (!y || y_stride >= width) && (!y2 || y2_stride >= width), NVX_EINVAL, "nvx_residual_norm: null pointer or row stride");
+    const size_t lds = (size_t)width * sizeof(float);
+    const auto ok4 = [&](const void* p, size_t item) { return (reinterpret_cast<uintptr_t>(p) & (4 * item - 1)) == 0; };
+    const size_t item = fmt == 2 ? 4 : 2;
+    const bool v4 = width % 4 == 0 && ok4(x_in, 4) && ok4(x_out, 4) && ok4(add, 4) && ok4(bias, 4) && ok4(w, 4) && ok4(y, item) && ok4(y2, item) &&
+                    ok4(h, item) && (!y || y_stride % 4 == 0) && (!y2 || y2_stride % 4 == 0);
+#define NVX_RESIDUAL_NORM(V)                                                                                                           \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((residual_norm_kernel<A_, V>), dim3((unsigned)n_tok), dim3(256), lds, (hipStream_t)stream, x_in, (const A_*)y, \
+                                         y_stride, (const A_*)y2, y2_stride, add, bias, x_out, w, eps, split, (A_*)h, (int)width))
+    if (v4) NVX_RESIDUAL_NORM(4);
+    else {
+        NVX_REQUIRE(width % 4 != 0, NVX_EINVAL, "nvx_residual_norm: rows of a width that is a multiple of four must start on such borders");
+        NVX_RESIDUAL_NORM(1);
+    }
+#undef NVX_RESIDUAL_NORM
+    return nvx_check_launch("nvx_residual_norm");
+}
+
+extern "C" int nvx_embed_sum(const int64_t* ids, const void* table, int fmt, int64_t vocab, const void* pair, int64_t buckets, int64_t mul_prev,
+                             int64_t mul_cur, float* prev_id, int64_t n_slots, const void* pos_table, int64_t n_pos, const int64_t* positions,
+                             const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* x,
+                             const float* w, float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width, nvx_stream_t stream) {
+    NVX_ROW_OK("nvx_embed_sum");
+    if (n_tok == 0) return NVX_OK;
+    NVX_REQUIRE(ids && table && vocab > 0 && vocab < (1ll << 31) && x, NVX_EINVAL, "nvx_embed_sum: bad table");
+    NVX_REQUIRE(!pair || (buckets > 0 && prev_id && n_slots > 0 && pos0 && state_slot && (tok_seq != nullptr) == (qo_indptr != nullptr) &&
+                          (qo_indptr || n_tok == n_seq)), NVX_EINVAL, "nvx_embed_sum: the pair table needs the step's layout and the predecessors' slots");
+    NVX_REQUIRE(!pos_table || (positions && n_pos > 0), NVX_EINVAL, "nvx_embed_sum: the position table needs positions");
+    NVX_REQUIRE(!h || width % 4 != 0 || nvx_aligned16(w), NVX_EINVAL, "nvx_embed_sum: the norm's weight must start on a 16-byte border");
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(embed_sum_kernel<A_>, dim3((unsigned)n_tok), dim3(256), (size_t)width * sizeof(float), (hipStream_t)stream, ids,
+                                         (const A_*)table, vocab, (const A_*)pair, buckets, mul_prev, mul_cur, prev_id, (const A_*)pos_table, n_pos,
+                                         positions, tok_seq, qo_indptr, pos0, state_slot, x, w, eps, split, (A_*)h, (int)width));
+    return nvx_check_launch("nvx_embed_sum");
 }
 
 extern "C" int nvx_tanh_cap(const void* in, int fmt, float cap, float* out, int64_t n, nvx_stream_t stream) {

@@ -2,13 +2,14 @@
 // OUTPUT (weight_out: fixed weights from a table).
 //   - nvx_moe_route: the `top` largest router logits of every token -> expert ids and sigmoid scores (float32);
 //   - nvx_moe_route_softmax: softmax scores, experts in groups of which only the best may be chosen, weights renormalised;
+//   - nvx_moe_route_sigmoid: sigmoid scores with a correction that enters the choice only, groups ranked by their two best experts;
 //   - nvx_moe_expert_rows: a token's experts evaluated row by row of their weights: the form for steps of few tokens, where
 //     every chosen expert's weights have to be streamed once per token anyway;
 //   - nvx_moe_order / nvx_moe_scatter_rows / nvx_moe_glu / nvx_moe_gather_rows: the pieces around per-expert matrix products
 //     for steps of many tokens (the expert order of the (token, choice) pairs and the experts' counts, scaled inputs gathered
 //     into that order, the gated activation, the tokens' results summed back).
 // Expert:  g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), y = g sigmoid(alpha g) (u + shift), out = W_down y
-// (limit = infinity, alpha = 1, shift = 0: silu(g) u).
+// (limit = infinity, alpha = 1, shift = 0: silu(g) u).  nvx_gelu_glu is the activation of plain gated layers, gelu_tanh(g) u.
 #include "fmt_dev.h"
 
 namespace NVX_NS {
@@ -78,6 +79,72 @@ __global__ __launch_bounds__(256) void moe_route_softmax_kernel(const float* __r
         sum += sc;
     }
     for (int k = 0; k < top; ++k) wts[t * top + k] /= (sum + norm_eps);
+}
+
+// Sigmoid router with groups: score = sigmoid(logit); the CHOICE score is score + correction[e] and may be negative.  The experts form
+// n_groups equal groups of neighbours, a group counts as the sum of its two largest choice scores (of its one, if it has one), and only
+// experts of the keep_groups best groups can be chosen (n_groups <= 1: all).  The `top` largest choice scores are taken (ties: the lower
+// id); a chosen expert's weight is its SCORE times w_scale.  A wave per token: its choice scores wait in LDS, a lane looks at every 64th
+// group and expert, and the winners are found by lane exchange.
+__device__ __forceinline__ void wave_best(float& v, int& i) {       // the largest v of the wave, the lowest i among equals (i < 0: none)
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) {
+        const float ov = __shfl_xor(v, m, 64);
+        const int oi = __shfl_xor(i, m, 64);
+        if (oi >= 0 && (i < 0 || ov > v || (ov == v && oi < i))) { v = ov; i = oi; }
+    }
+}
+__global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(const float* __restrict__ logits, const float* __restrict__ correction, int n_exp,
+                                                               int top, int n_groups, int keep_groups, float w_scale, int32_t* __restrict__ idx,
+                                                               float* __restrict__ wts, int64_t n_tok) {
+    extern __shared__ float sm[];                  // per wave: n_exp choice scores, n_groups group scores
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const bool grouped = n_groups > 1 && keep_groups < n_groups;
+    const int per = grouped ? n_exp / n_groups : n_exp;
+    float* choice = sm + wave * (n_exp + (grouped ? n_groups : 0));
+    float* gscore = choice + n_exp;
+    const int64_t t = (int64_t)blockIdx.x * 4 + wave;
+    const bool on = t < n_tok;
+    const float* z = logits + (on ? t : 0) * n_exp;
+    for (int e = lane; e < n_exp; e += 64) choice[e] = sigmoid_f(z[e]) + correction[e];
+    __syncthreads();
+    if (grouped) {
+        for (int g = lane; g < n_groups; g += 64) {
+            float a = choice[g * per], b = -INFINITY;          // the two largest
+            for (int e = 1; e < per; ++e) {
+                const float c = choice[g * per + e];
+                if (c > a) { b = a; a = c; }
+                else if (c > b) b = c;
+            }
+            gscore[g] = per > 1 ? a + b : a;
+        }
+        __syncthreads();
+        // the groups that stay are marked by an infinite score, the best first
+        for (int k = 0; k < keep_groups; ++k) {
+            float v = -INFINITY;
+            int i = -1;
+            for (int g = lane; g < n_groups; g += 64)
+                if (gscore[g] < INFINITY && (i < 0 || gscore[g] > v)) { v = gscore[g]; i = g; }
+            wave_best(v, i);
+            if (lane == 0 && i >= 0) gscore[i] = INFINITY;     // kept
+            __syncthreads();
+        }
+    }
+    for (int k = 0; k < top; ++k) {
+        float v = -INFINITY;
+        int i = -1;
+        for (int e = lane; e < n_exp; e += 64) {
+            const float c = choice[e];
+            if (c == -INFINITY || (grouped && gscore[e / per] != INFINITY)) continue;
+            if (i < 0 || c > v) { v = c; i = e; }
+        }
+        wave_best(v, i);
+        if (on && lane == 0) {
+            idx[t * top + k] = i < 0 ? 0 : i;
+            wts[t * top + k] = i < 0 ? 0.f : sigmoid_f(z[i]) * w_scale;
+        }
+        if (i >= 0 && lane == (i & 63)) choice[i] = -INFINITY;        // taken (only this lane reads entry i)
+    }
 }
 
 __device__ __forceinline__ float glu_act(float g, float u, float limit, float alpha, float shift) {
@@ -227,20 +294,26 @@ __global__ __launch_bounds__(256) void moe_scatter_rows_kernel(const A* __restri
     for (int c = threadIdx.x; c < width; c += 256) st_f(o, c, wt * ld_f(h, t * h_stride + c));
 }
 
-// y[r][j] = act(gu[r][j], gu[r][ff + j])
-template <typename A>
+// gelu_tanh(g) u
+__device__ __forceinline__ float gelu_glu_act(float g, float u) {
+    return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
+}
+
+// y[r][j] = act(gu[r][j], gu[r][ff + j]); GELU: gelu_tanh(g) u, the three constants are not read
+template <typename A, bool GELU>
 __global__ __launch_bounds__(256) void moe_glu_kernel(const A* __restrict__ gu, A* __restrict__ y, float limit, float alpha, float shift,
                                                      int64_t rows, int ff) {
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < rows * ff; i += (int64_t)gridDim.x * 256) {
         const int64_t r = i / ff;
         const int j = (int)(i % ff);
-        st_f(y, i, glu_act(ld_f(gu, r * 2 * ff + j), ld_f(gu, r * 2 * ff + ff + j), limit, alpha, shift));
+        const float g = ld_f(gu, r * 2 * ff + j), u = ld_f(gu, r * 2 * ff + ff + j);
+        st_f(y, i, GELU ? gelu_glu_act(g, u) : glu_act(g, u, limit, alpha, shift));
     }
 }
 
 // The same for 16-bit formats, eight neighbouring entries of a row per thread as one 16-byte load of each half and one store
 // (ff8 = ff / 8; rows start on 16-byte borders).
-template <typename A>
+template <typename A, bool GELU>
 __global__ __launch_bounds__(256) void moe_glu_vec8_kernel(const A* __restrict__ gu, A* __restrict__ y, float limit, float alpha, float shift,
                                                           int64_t rows, int ff8) {
     union Pack { uint4 v; A a[8]; };
@@ -253,7 +326,7 @@ __global__ __launch_bounds__(256) void moe_glu_vec8_kernel(const A* __restrict__
         g.v = *reinterpret_cast<const uint4*>(row + j);
         u.v = *reinterpret_cast<const uint4*>(row + (int64_t)ff8 * 8 + j);
 #pragma unroll
-        for (int k = 0; k < 8; ++k) o.a[k] = (A)glu_act((float)g.a[k], (float)u.a[k], limit, alpha, shift);
+        for (int k = 0; k < 8; ++k) o.a[k] = (A)(GELU ? gelu_glu_act((float)g.a[k], (float)u.a[k]) : glu_act((float)g.a[k], (float)u.a[k], limit, alpha, shift));
         *reinterpret_cast<uint4*>(y + i * 8) = o.v;
     }
 }
@@ -342,6 +415,20 @@ extern "C" int nvx_moe_route_softmax(const float* logits, int64_t n_tok, int64_t
     return nvx_check_launch("nvx_moe_route_softmax");
 }
 
+extern "C" int nvx_moe_route_sigmoid(const float* logits, const float* correction, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups,
+                                     int64_t keep_groups, float w_scale, int32_t* idx, float* wts, nvx_stream_t stream) {
+    NVX_REQUIRE(n_tok >= 0 && n_exp > 0 && n_exp <= 1024 && top > 0 && top <= n_exp, NVX_EINVAL, "nvx_moe_route_sigmoid: bad sizes (at most 1024 experts)");
+    NVX_REQUIRE(n_groups >= 0 && (n_groups <= 1 || (n_exp % n_groups == 0 && keep_groups >= 1 && keep_groups <= n_groups &&
+                                                   keep_groups * (n_exp / n_groups) >= top)),
+                NVX_EINVAL, "nvx_moe_route_sigmoid: groups must divide the experts and the kept groups must hold `top` experts");
+    if (n_tok == 0) return NVX_OK;
+    NVX_REQUIRE(logits && correction && idx && wts, NVX_EINVAL, "nvx_moe_route_sigmoid: null pointer");
+    const size_t lds = 4 * (size_t)(n_exp + (n_groups > 1 ? n_groups : 0)) * sizeof(float);
+    hipLaunchKernelGGL(moe_route_sigmoid_kernel, dim3((unsigned)((n_tok + 3) / 4)), dim3(256), lds, (hipStream_t)stream, logits, correction, (int)n_exp,
+                       (int)top, (int)n_groups, (int)keep_groups, w_scale, idx, wts, n_tok);
+    return nvx_check_launch("nvx_moe_route_sigmoid");
+}
+
 extern "C" int64_t nvx_moe_expert_rows_max_width(int64_t ff) {
     return ff > 0 && ff <= 12288 ? 12288 : 0;      // a row of either size waits in LDS as float32
 }
@@ -391,27 +478,39 @@ extern "C" int nvx_moe_scatter_rows(const void* h, int64_t h_stride, int fmt, co
     return nvx_check_launch("nvx_moe_scatter_rows");
 }
 
+template <bool GELU>
+static int launch_glu(const void* gu, int fmt, float limit, float alpha, float shift, void* y, int64_t rows, int64_t ff, hipStream_t s, const char* name) {
+    if (fmt != 2 && ff % 8 == 0 && nvx_aligned16(gu) && nvx_aligned16(y)) {
+        int64_t blocks = (rows * (ff / 8) + 255) / 256;
+        if (blocks > 256 * 64) blocks = 256 * 64;
+        if (fmt == 0)
+            hipLaunchKernelGGL((moe_glu_vec8_kernel<__bf16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const __bf16*)gu, (__bf16*)y, limit,
+                               alpha, shift, rows, (int)(ff / 8));
+        else
+            hipLaunchKernelGGL((moe_glu_vec8_kernel<_Float16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const _Float16*)gu, (_Float16*)y,
+                               limit, alpha, shift, rows, (int)(ff / 8));
+        return nvx_check_launch(name);
+    }
+    int64_t blocks = (rows * ff + 255) / 256;
+    if (blocks > 256 * 64) blocks = 256 * 64;
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((moe_glu_kernel<A_, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const A_*)gu, (A_*)y, limit, alpha, shift,
+                                         rows, (int)ff));
+    return nvx_check_launch(name);
+}
+
 extern "C" int nvx_moe_glu(const void* gu, int fmt, float limit, float alpha, float shift, void* y, int64_t rows, int64_t ff,
                            nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2 && rows >= 0 && ff > 0, NVX_EINVAL, "nvx_moe_glu: bad arguments");
     if (rows == 0) return NVX_OK;
     NVX_REQUIRE(gu && y, NVX_EINVAL, "nvx_moe_glu: null pointer");
-    if (fmt != 2 && ff % 8 == 0 && nvx_aligned16(gu) && nvx_aligned16(y)) {
-        int64_t blocks = (rows * (ff / 8) + 255) / 256;
-        if (blocks > 256 * 64) blocks = 256 * 64;
-        if (fmt == 0)
-            hipLaunchKernelGGL(moe_glu_vec8_kernel<__bf16>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const __bf16*)gu, (__bf16*)y,
-                               limit, alpha, shift, rows, (int)(ff / 8));
-        else
-            hipLaunchKernelGGL(moe_glu_vec8_kernel<_Float16>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const _Float16*)gu,
-                               (_Float16*)y, limit, alpha, shift, rows, (int)(ff / 8));
-        return nvx_check_launch("nvx_moe_glu");
-    }
-    int64_t blocks = (rows * ff + 255) / 256;
-    if (blocks > 256 * 64) blocks = 256 * 64;
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(moe_glu_kernel<A_>, dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream, (const A_*)gu, (A_*)y, limit,
-                                         alpha, shift, rows, (int)ff));
-    return nvx_check_launch("nvx_moe_glu");
+    return launch_glu<false>(gu, fmt, limit, alpha, shift, y, rows, ff, (hipStream_t)stream, "nvx_moe_glu");
+}
+
+extern "C" int nvx_gelu_glu(const void* gu, int fmt, void* y, int64_t rows, int64_t ff, nvx_stream_t stream) {
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2 && rows >= 0 && ff > 0, NVX_EINVAL, "nvx_gelu_glu: bad arguments");
+    if (rows == 0) return NVX_OK;
+    NVX_REQUIRE(gu && y, NVX_EINVAL, "nvx_gelu_glu: null pointer");
+    return launch_glu<true>(gu, fmt, 0.f, 0.f, 0.f, y, rows, ff, (hipStream_t)stream, "nvx_gelu_glu");
 }
 
 extern "C" int nvx_moe_gather_rows(const void* ys, int fmt, const int64_t* dst, const float* wts, int64_t top, void* out, int64_t n_tok,

@@ -1,11 +1,13 @@
 // Token mixers that carry a matrix per head from token to token, and the small steps in front of them:
 //   - short causal convolution over time per channel (optional bias, optional silu), its last inputs kept per sequence;
 //   - token shift: every token's row mixed with its predecessor's by per-channel weights, the last row kept per sequence;
-//   - three recurrences over a (key size x value size) memory per head:
+//   - recurrences over a (key size x value size) memory per head:
 //       mlstm   exponential input gate and sigmoid forget gate stabilised by a running maximum, normaliser vector;
 //       delta   per-head decay, then a rank-one correction of the memory towards the new value along the key;
 //       rwkv    per-key-channel decay, the current token read with a bonus before it is written;
-//       decay   one constant decay per head, the token written before it is read (linear attention with a fixed decay).
+//       decay   one constant decay per head, the token written before it is read (linear attention with a fixed decay);
+//       gla     a decay per key channel and token, the token written before it is read (gated linear attention).
+// Long portions of mlstm, decay and gla are cut into chunks that run side by side, in three phases (see decay).
 // One kernel per recurrence serves prompts, portions of prompts and single decoded tokens: a workgroup takes one head of
 // one sequence and a block of value columns, a thread keeps KR rows of one column in registers, P neighbouring lanes
 // share a column and add their partial read-outs by lane exchange.  The tokens' keys, queries and values are staged
@@ -145,14 +147,18 @@ __device__ __forceinline__ void unit_rows(float* dst, int nt, int dim, int p_lan
 // with q scaled by dim^(-1/2); m starts at 0.  S: (slots, heads, dim, vdim), n: (slots, heads, dim), m: (slots, heads).
 // Every column block of a head reads n and m (N_in, M_in) and the first one writes them (N, M): where a head has more than one
 // column block the caller hands in copies to read from, since a block that starts late must not see the new values.
-template <typename A>
+// PHASE 0: one workgroup walks a whole portion.  PHASE 1 and 3: chunks of `chunk` tokens side by side (blockIdx.z = sequence * n_chunk_max +
+// chunk).  Phase 1 builds a chunk's own memory from nothing (maximum -inf, so the chunk's maximum is that of its own terms) into ws and
+// also keeps its sum of forget gates; phase 3 starts from what the carry made of ws and writes the read-out only.
+struct MlstmChunks { float* S; float* N; float* M; float* F; int chunk; int n_max; };
+template <typename A, int PHASE>
 __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off, int v_off,
                                                         const float* __restrict__ gates, const float* __restrict__ gate_bias, float cap,
                                                         float* __restrict__ S, const float* __restrict__ N_in, const float* __restrict__ M_in,
                                                         float* __restrict__ N, float* __restrict__ M,
                                                         const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
                                                         const int32_t* __restrict__ state_slot, float* __restrict__ out, int heads, int dim,
-                                                        int vdim, int p_lanes) {
+                                                        int vdim, int p_lanes, MlstmChunks ck) {
     extern __shared__ float sm[];
     const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
     float* sq = sm;
@@ -161,15 +167,24 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
     float* si = sv + TB * cb;
     float* sf = si + TB;
     const int hd = blockIdx.y;
-    const SeqSpan sp = seq_span(blockIdx.z, qo_indptr, pos0, state_slot);
+    SeqSpan sp = seq_span(PHASE ? blockIdx.z / ck.n_max : blockIdx.z, qo_indptr, pos0, state_slot);
     if (sp.slot < 0 || sp.n <= 0) return;
+    if (PHASE) {
+        const int64_t first = (int64_t)(blockIdx.z % ck.n_max) * ck.chunk;
+        if (first >= sp.n) return;
+        sp.q0 += first;
+        sp.n = sp.n - first < ck.chunk ? sp.n - first : ck.chunk;
+    }
     const ScanThread th = scan_thread(p_lanes, vdim);
-    float* Sp = S + ((int64_t)sp.slot * heads + hd) * dim * vdim;
-    float* Np = N + ((int64_t)sp.slot * heads + hd) * dim;
-    const float* Np_in = N_in + ((int64_t)sp.slot * heads + hd) * dim;
+    const int64_t at = (int64_t)(PHASE ? (int)blockIdx.z : sp.slot) * heads + hd;
+    float* Sp = (PHASE ? ck.S : S) + at * dim * vdim;
+    float* Np = (PHASE ? ck.N : N) + at * dim;
+    const float* Np_in = PHASE ? Np : N_in + at * dim;
+    // phase 1 has no use for the normaliser but in the one wave that hands it on
+    const bool norm_here = PHASE != 1 || (blockIdx.x == 0 && threadIdx.x < 64);
     float s[KR], nn[KR];
-    float m = 0.f;
-    const bool cont = sp.pos0 > 0;
+    float m = PHASE == 1 ? -INFINITY : 0.f, f_sum = 0.f;
+    const bool cont = PHASE == 3 || (PHASE == 0 && sp.pos0 > 0);
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
@@ -177,13 +192,13 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
         s[r] = (in && th.active) ? Sp[(int64_t)row * vdim + th.e] : 0.f;
         nn[r] = in ? Np_in[row] : 0.f;
     }
-    if (cont) m = M_in[(int64_t)sp.slot * heads + hd];
+    if (cont) m = PHASE ? ck.M[at] : M_in[at];
     zero_rows(sq, 2 * TB * rs);
     const float q_mul = 1.0f / sqrtf((float)dim);
     for (int64_t t0 = 0; t0 < sp.n; t0 += TB) {
         const int nt = (int)(sp.n - t0 < TB ? sp.n - t0 : TB);
         __syncthreads();
-        stage_rows(sq, x, x_stride, sp.q0 + t0, nt, q_off + hd * dim, dim, p_lanes, q_mul);
+        if (PHASE != 1) stage_rows(sq, x, x_stride, sp.q0 + t0, nt, q_off + hd * dim, dim, p_lanes, q_mul);
         stage_rows(sk, x, x_stride, sp.q0 + t0, nt, k_off + hd * dim, dim, p_lanes, 1.0f);
         stage_cols(sv, x, x_stride, sp.q0 + t0, nt, v_off + hd * vdim, vdim, cb);
         if ((int)threadIdx.x < nt) {
@@ -197,9 +212,19 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
             const float m_new = fmaxf(gf + m, gi);
             const float keep = expf(gf + m - m_new), put = expf(gi - m_new);
             m = m_new;
+            if (PHASE == 1) f_sum += gf;
             const float v = sv[tt * cb + th.col];
             const float* kk = sk + tt * rs + th.p * KS;
             const float* qq = sq + tt * rs + th.p * KS;
+            if (PHASE == 1) {
+#pragma unroll
+                for (int r = 0; r < KR; ++r) s[r] = keep * s[r] + put * kk[r] * v;
+                if (norm_here) {
+#pragma unroll
+                    for (int r = 0; r < KR; ++r) nn[r] = keep * nn[r] + put * kk[r];
+                }
+                continue;
+            }
             float num = 0.f, nq = 0.f;
 #pragma unroll
             for (int r = 0; r < KR; ++r) {
@@ -215,14 +240,69 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
                 out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + th.e] = num / (fmaxf(fabsf(nq), expf(-m)) + 1e-6f);
         }
     }
+    if (PHASE == 3) return;
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
         if (row < dim && th.active) Sp[(int64_t)row * vdim + th.e] = s[r];
         if (row < dim && blockIdx.x == 0 && th.col == 0) Np[row] = nn[r];
     }
-    if (blockIdx.x == 0 && threadIdx.x == 0) M[(int64_t)sp.slot * heads + hd] = m;
+    if (blockIdx.x == 0 && threadIdx.x == 0) {
+        (PHASE ? ck.M : M)[at] = m;
+        if (PHASE) ck.F[at] = f_sum;
+    }
 }
+
+// Between the phases, the scalars: with F the sum of a chunk's forget gates and m_own its maximum, the maximum after the chunk is
+// max(F + m, m_own) (the same number as step by step), the memory in front is kept with e^(F + m - m') and the chunk's own enters with
+// e^(m_own - m').  M becomes the maximum at every chunk's start, F the factor `keep`, put the other; one thread per (sequence, head).
+__global__ __launch_bounds__(64) void mlstm_chunk_scalars_kernel(float* __restrict__ M_pool, float* __restrict__ M, float* __restrict__ F,
+                                                                float* __restrict__ put, const int32_t* __restrict__ qo_indptr,
+                                                                const int64_t* __restrict__ pos0, const int32_t* __restrict__ state_slot, int heads,
+                                                                int chunk, int n_chunk_max, int n_seq) {
+    const int i = blockIdx.x * 64 + threadIdx.x;
+    if (i >= n_seq * heads) return;
+    const int seq = i / heads, hd = i % heads;
+    const SeqSpan sp = seq_span(seq, qo_indptr, pos0, state_slot);
+    if (sp.slot < 0 || sp.n <= 0) return;
+    float run = sp.pos0 > 0 ? M_pool[(int64_t)sp.slot * heads + hd] : 0.f;
+    for (int ck = 0; (int64_t)ck * chunk < sp.n; ++ck) {
+        const int64_t at = ((int64_t)seq * n_chunk_max + ck) * heads + hd;
+        const float own = M[at], f = F[at], next = fmaxf(f + run, own);
+        M[at] = run;
+        F[at] = expf(f + run - next);
+        put[at] = expf(own - next);
+        run = next;
+    }
+    M_pool[(int64_t)sp.slot * heads + hd] = run;
+}
+
+// Between the phases, a memory of `rows` x `cols` per head: ws[sequence][chunk] holds every chunk's own contribution and is replaced by
+// the memory at the chunk's start; what is there after the last chunk goes to the pool.  One chunk further: keep * memory + put * own,
+// keep one number per head or (keep_rows) per head and row, put one per head or (null) 1.  One thread per element.
+__global__ __launch_bounds__(256) void chunk_carry_kernel(float* __restrict__ pool, float* __restrict__ ws, const float* __restrict__ keep, int keep_rows,
+                                                         const float* __restrict__ put, const int32_t* __restrict__ qo_indptr,
+                                                         const int64_t* __restrict__ pos0, const int32_t* __restrict__ state_slot, int heads, int rows,
+                                                         int cols, int chunk, int n_chunk_max) {
+    const SeqSpan sp = seq_span(blockIdx.y, qo_indptr, pos0, state_slot);
+    if (sp.slot < 0 || sp.n <= 0) return;
+    const int64_t per = (int64_t)heads * rows * cols, i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= per) return;
+    const int hd = (int)(i / ((int64_t)rows * cols)), row = (int)(i / cols % rows);
+    const int n_ck = (int)((sp.n + chunk - 1) / chunk);
+    float run = sp.pos0 > 0 ? pool[(int64_t)sp.slot * per + i] : 0.f;
+    float* w = ws + (int64_t)blockIdx.y * n_chunk_max * per + i;
+    const float* kp = keep + (int64_t)blockIdx.y * n_chunk_max * heads * (keep_rows ? rows : 1) + (keep_rows ? hd * rows + row : hd);
+    const float* pp = put ? put + (int64_t)blockIdx.y * n_chunk_max * heads + hd : nullptr;
+    const int64_t k_step = (int64_t)heads * (keep_rows ? rows : 1);
+    for (int ck = 0; ck < n_ck; ++ck) {
+        const float own = w[ck * per];
+        w[ck * per] = run;
+        run = kp[ck * k_step] * run + (pp ? pp[(int64_t)ck * heads] * own : own);
+    }
+    pool[(int64_t)sp.slot * per + i] = run;
+}
+
 
 // Gated delta rule.  x[t] holds q at q_off, k at k_off (kv_heads * dim each, after convolution and silu) and v at v_off (heads *
 // vdim); ab[t] = [a | b] pre-activations (heads each, float32).  q and k are scaled to unit length per head (q also by
@@ -478,7 +558,99 @@ __global__ __launch_bounds__(256) void decay_chunk_carry_kernel(const float* __r
     *Sp = run;
 }
 
-// launch geometry of the three recurrences: lanes per column (a power of two), threads per workgroup, value columns per
+// Gated linear attention.  x[t] holds q at q_off, k at k_off (heads * dim each) and v at v_off (heads * vdim); alpha (n_tok, heads * dim)
+// float32: the decay of every key channel at every token.
+//   S <- diag(alpha) S + k v^T;  o = S^T (q_mul q)  (the read sees the token's own write).          S: (slots, heads, dim, vdim).
+// Phases as in decay_scan_kernel; phase 1 also hands out, per key channel, the product of the chunk's decays (ws_keep), which is what the
+// carry multiplies the memory in front with.
+template <typename A, int PHASE>
+__global__ __launch_bounds__(256) void gla_scan_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off, int v_off, float q_mul,
+                                                      const float* __restrict__ alpha, float* __restrict__ S, const int32_t* __restrict__ qo_indptr,
+                                                      const int64_t* __restrict__ pos0, const int32_t* __restrict__ state_slot, float* __restrict__ out,
+                                                      int heads, int dim, int vdim, int p_lanes, int tb, int chunk, int n_chunk_max,
+                                                      float* __restrict__ ws, float* __restrict__ ws_keep) {
+    extern __shared__ float sm[];
+    const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
+    float* sq = sm;
+    float* sk = sq + tb * rs;
+    float* sa = sk + tb * rs;
+    float* sv = sa + tb * rs;
+    const int hd = blockIdx.y;
+    SeqSpan sp = seq_span(PHASE ? blockIdx.z / n_chunk_max : blockIdx.z, qo_indptr, pos0, state_slot);
+    if (sp.slot < 0 || sp.n <= 0) return;
+    if (PHASE) {
+        const int64_t first = (int64_t)(blockIdx.z % n_chunk_max) * chunk;
+        if (first >= sp.n) return;
+        sp.q0 += first;
+        sp.n = sp.n - first < chunk ? sp.n - first : chunk;
+    }
+    const ScanThread th = scan_thread(p_lanes, vdim);
+    const int64_t at = (int64_t)(PHASE ? (int)blockIdx.z : sp.slot) * heads + hd;
+    float* Sp = (PHASE ? ws : S) + at * dim * vdim;
+    float s[KR], pr[KR];
+    const bool cont = PHASE == 3 || (PHASE == 0 && sp.pos0 > 0);
+    const bool keep_here = PHASE == 1 && blockIdx.x == 0 && threadIdx.x < 64;       // the wave that multiplies the decays up
+#pragma unroll
+    for (int r = 0; r < KR; ++r) {
+        const int row = th.r0 + r;
+        s[r] = (cont && row < dim && th.active) ? Sp[(int64_t)row * vdim + th.e] : 0.f;
+        pr[r] = 1.f;
+    }
+    zero_rows(sq, 3 * tb * rs);
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, n_waves = blockDim.x >> 6;
+    for (int64_t t0 = 0; t0 < sp.n; t0 += tb) {
+        const int nt = (int)(sp.n - t0 < tb ? sp.n - t0 : tb);
+        __syncthreads();
+        for (int tt = wave; tt < nt; tt += n_waves) {
+            const int64_t tok = sp.q0 + t0 + tt;
+            const A* xr = x + tok * x_stride;
+            const float* ar = alpha + (tok * heads + hd) * dim;
+            for (int d = lane; d < dim; d += 64) {
+                const int o = tt * rs + lds_row(d);
+                if (PHASE != 1) sq[o] = ld_f(xr, q_off + hd * dim + d) * q_mul;
+                sk[o] = ld_f(xr, k_off + hd * dim + d);
+                sa[o] = ar[d];
+            }
+            for (int c = lane; c < cb; c += 64) {
+                const int e = blockIdx.x * cb + c;
+                sv[tt * cb + c] = e < vdim ? ld_f(xr, v_off + hd * vdim + e) : 0.f;
+            }
+        }
+        __syncthreads();
+        for (int tt = 0; tt < nt; ++tt) {
+            const float v = sv[tt * cb + th.col];
+            const float* kk = sk + tt * rs + th.p * KS;
+            const float* qq = sq + tt * rs + th.p * KS;
+            const float* aa = sa + tt * rs + th.p * KS;
+            if (PHASE == 1) {
+#pragma unroll
+                for (int r = 0; r < KR; ++r) s[r] = aa[r] * s[r] + kk[r] * v;
+                if (keep_here) {
+#pragma unroll
+                    for (int r = 0; r < KR; ++r) pr[r] *= aa[r];
+                }
+                continue;
+            }
+            float o = 0.f;
+#pragma unroll
+            for (int r = 0; r < KR; ++r) {
+                s[r] = aa[r] * s[r] + kk[r] * v;
+                o += s[r] * qq[r];
+            }
+            o = lanes_sum(o, p_lanes);
+            if (th.p == 0 && th.active) out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + th.e] = o;
+        }
+    }
+    if (PHASE == 3) return;
+#pragma unroll
+    for (int r = 0; r < KR; ++r) {
+        const int row = th.r0 + r;
+        if (row < dim && th.active) Sp[(int64_t)row * vdim + th.e] = s[r];
+        if (keep_here && th.col == 0 && row < dim) ws_keep[at * dim + row] = pr[r];
+    }
+}
+
+// launch geometry of the recurrences: lanes per column (a power of two), threads per workgroup, value columns per
 // workgroup
 struct ScanLaunch { int p_lanes, threads, cb; };
 static bool scan_launch(int64_t dim, int64_t vdim, ScanLaunch* g) {
@@ -558,7 +730,7 @@ extern "C" int nvx_mlstm_scan(const void* x, int64_t x_stride, int fmt, int64_t 
                               const float* gate_bias, float cap, float* S, const float* N_in, const float* M_in, float* N, float* M,
                               int64_t n_slots, const int32_t* qo_indptr,
                               const int64_t* pos0, const int32_t* state_slot, float* out, int64_t n_tok, int64_t n_seq, int64_t heads,
-                              int64_t dim, int64_t vdim, nvx_stream_t stream) {
+                              int64_t dim, int64_t vdim, int64_t chunk, int64_t n_chunk_max, float* ws, nvx_stream_t stream) {
     NVX_LAYOUT_OK("nvx_mlstm_scan");
     ScanLaunch g;
     NVX_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && vdim > 0 && vdim < (1 << 24) && n_slots >= 0 && cap > 0.f, NVX_EINVAL,
@@ -568,12 +740,33 @@ extern "C" int nvx_mlstm_scan(const void* x, int64_t x_stride, int fmt, int64_t 
     NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
                     x_stride >= v_off + heads * vdim, NVX_EINVAL, "nvx_mlstm_scan: q, k or v lies outside a row");
     const size_t lds = (size_t)(2 * TB * g.p_lanes * KS + TB * g.cb + 2 * TB) * sizeof(float);
-    const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)n_seq);
-    NVX_REQUIRE(grid.x == 1 || (N_in != N && M_in != M), NVX_EINVAL,
+    NVX_REQUIRE(chunk == 0 || (chunk > 0 && chunk < (1 << 30) && n_chunk_max > 0 && n_seq * n_chunk_max <= 65535 && ws && qo_indptr), NVX_EINVAL,
+                "nvx_mlstm_scan: chunks need a ragged step, their workspace, and at most 65535 of them");
+    const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
+    NVX_REQUIRE(chunk || grid.x == 1 || (N_in != N && M_in != M), NVX_EINVAL,
                 "nvx_mlstm_scan: a head with several column blocks reads its normaliser and maximum from copies");
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(mlstm_scan_kernel<A_>, grid, dim3(g.threads), lds, (hipStream_t)stream, (const A_*)x, x_stride, (int)q_off,
-                                         (int)k_off, (int)v_off, gates, gate_bias, cap, S, N_in, M_in, N, M, qo_indptr, pos0, state_slot, out, (int)heads,
-                                         (int)dim, (int)vdim, g.p_lanes));
+    // the workspace: memories, normalisers, maxima, forget sums / keep factors, put factors of all chunks
+    const int64_t n_ws = chunk ? n_seq * n_chunk_max * heads : 0;
+    MlstmChunks ck = {ws, ws + n_ws * dim * vdim, ws + n_ws * dim * (vdim + 1), ws + n_ws * (dim * (vdim + 1) + 1), (int)chunk, (int)n_chunk_max};
+    float* put = ws + n_ws * (dim * (vdim + 1) + 2);
+    const hipStream_t st = (hipStream_t)stream;
+#define NVX_MLSTM_SCAN(PHASE)                                                                                                                     \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((mlstm_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, st, (const A_*)x, x_stride, (int)q_off, (int)k_off, \
+                                         (int)v_off, gates, gate_bias, cap, S, N_in, M_in, N, M, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim, \
+                                         (int)vdim, g.p_lanes, ck))
+    if (!chunk) {
+        NVX_MLSTM_SCAN(0);
+    } else {
+        NVX_MLSTM_SCAN(1);
+        hipLaunchKernelGGL(mlstm_chunk_scalars_kernel, dim3((unsigned)((n_seq * heads + 63) / 64)), dim3(64), 0, st, M, ck.M, ck.F, put, qo_indptr, pos0,
+                           state_slot, (int)heads, (int)chunk, (int)n_chunk_max, (int)n_seq);
+        hipLaunchKernelGGL(chunk_carry_kernel, dim3((unsigned)((heads * dim * vdim + 255) / 256), (unsigned)n_seq), dim3(256), 0, st, S, ck.S,
+                           (const float*)ck.F, 0, (const float*)put, qo_indptr, pos0, state_slot, (int)heads, (int)dim, (int)vdim, (int)chunk, (int)n_chunk_max);
+        hipLaunchKernelGGL(chunk_carry_kernel, dim3((unsigned)((heads * dim + 255) / 256), (unsigned)n_seq), dim3(256), 0, st, N, ck.N,
+                           (const float*)ck.F, 0, (const float*)put, qo_indptr, pos0, state_slot, (int)heads, (int)dim, 1, (int)chunk, (int)n_chunk_max);
+        NVX_MLSTM_SCAN(3);
+    }
+#undef NVX_MLSTM_SCAN
     return nvx_check_launch("nvx_mlstm_scan");
 }
 
@@ -646,4 +839,39 @@ extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t 
     }
 #undef NVX_DECAY_SCAN
     return nvx_check_launch("nvx_decay_scan");
+}
+
+extern "C" int nvx_gla_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, float q_mul, const float* alpha,
+                            float* S, int64_t n_slots, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* out,
+                            int64_t n_tok, int64_t n_seq, int64_t heads, int64_t dim, int64_t vdim, int64_t chunk, int64_t n_chunk_max, float* ws,
+                            nvx_stream_t stream) {
+    NVX_LAYOUT_OK("nvx_gla_scan");
+    ScanLaunch g;
+    NVX_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && vdim > 0 && vdim < (1 << 24) && n_slots >= 0, NVX_EINVAL, "nvx_gla_scan: bad sizes");
+    NVX_REQUIRE(scan_launch(dim, vdim, &g), NVX_EUNSUPPORTED, "nvx_gla_scan: key size above 512");
+    NVX_REQUIRE(x && alpha && S && out, NVX_EINVAL, "nvx_gla_scan: null pointer");
+    NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
+                    x_stride >= v_off + heads * vdim, NVX_EINVAL, "nvx_gla_scan: q, k or v lies outside a row");
+    const int tb = g.p_lanes <= 2 ? 32 : (g.p_lanes == 4 ? 16 : (g.p_lanes == 8 ? 8 : 4));
+    const size_t lds = (size_t)(3 * tb * g.p_lanes * KS + tb * g.cb) * sizeof(float);
+    NVX_REQUIRE(chunk == 0 || (chunk > 0 && chunk < (1 << 30) && n_chunk_max > 0 && n_seq * n_chunk_max <= 65535 && ws && qo_indptr), NVX_EINVAL,
+                "nvx_gla_scan: chunks need a ragged step, their workspace, and at most 65535 of them");
+    const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
+    float* keep = chunk ? ws + n_seq * n_chunk_max * heads * dim * vdim : nullptr;      // behind the chunks' memories
+    const hipStream_t st = (hipStream_t)stream;
+#define NVX_GLA_SCAN(PHASE)                                                                                                                        \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((gla_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, st, (const A_*)x, x_stride, (int)q_off, (int)k_off, \
+                                         (int)v_off, q_mul, alpha, S, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim, (int)vdim, g.p_lanes, \
+                                         tb, (int)chunk, (int)n_chunk_max, ws, keep))
+    if (!chunk) {
+        NVX_GLA_SCAN(0);
+    } else {
+        NVX_GLA_SCAN(1);
+        hipLaunchKernelGGL(chunk_carry_kernel, dim3((unsigned)((heads * dim * vdim + 255) / 256), (unsigned)n_seq), dim3(256), 0, st, S, ws,
+                           (const float*)keep, 1, (const float*)nullptr, qo_indptr, pos0, state_slot, (int)heads, (int)dim, (int)vdim, (int)chunk,
+                           (int)n_chunk_max);
+        NVX_GLA_SCAN(3);
+    }
+#undef NVX_GLA_SCAN
+    return nvx_check_launch("nvx_gla_scan");
 }

@@ -31,7 +31,7 @@ from torch import nn
 from . import distributed as tpd
 from . import ops
 from .layers.cap_attention import NormedAttention
-from .layers.moe import TableMoE
+from .layers.moe import DenseGLU, TableMoE
 from .layers.recurrent import DecayLinearAttention
 
 MIXERS = ("attention", "parallel")
@@ -153,19 +153,6 @@ class ParallelMixer(nn.Module):
         self.in_proj = nn.Linear(width, self.left.proj_rows + self.right.proj_rows, bias=True)
         nn.init.zeros_(self.in_proj.bias)      # it stays zero where the design has no bias (the gates, the right branch)
         self.left_scale, self.right_scale = m["left_scale"], m["right_scale"]
-
-
-class DenseGLU(nn.Module):
-    """W_down (g sigmoid(alpha g) (u + 1)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit); gate and up are one product."""
-
-    def __init__(self, width: int, ff: int, limit: float, alpha: float):
-        super().__init__()
-        self.ff, self.limit, self.alpha = ff, float(limit), float(alpha)
-        self.gu_proj = nn.Linear(width, 2 * ff, bias=False)      # rows: gate | up
-        self.down = nn.Linear(ff, width, bias=False)
-
-    def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return self.down(ops.moe_glu(self.gu_proj(h), self.limit, self.alpha, 1.0))
 
 
 class GibavikLayer(nn.Module):

@@ -1,7 +1,7 @@
 """Causal attention with grouped key/value heads and separate key and value sizes over per-token key and value rows in the
 token cache: SoftcapAttention (rotary positions on a leading part of each head, unit-mean-square values, capped scores) and
 NormedAttention (query/key RMS norms, optional rotation of keys AND values, window, distance penalty, output gate, borrowed
-keys and values)."""
+keys and values), TiedAttention (one cached row per token and head is key and value, linear distance penalty, chunks of positions)."""
 from __future__ import annotations
 
 import torch
@@ -136,3 +136,50 @@ class NormedAttention(nn.Module):
 
     def forward(self, h: torch.Tensor, positions: torch.Tensor, md) -> torch.Tensor:
         return self.attend(self.in_proj(h), 0, positions, md)
+
+
+def geometric_slopes(heads: int, base: float = 8.0):
+    """One slope per head for a linear distance penalty: 2^(-base (h + 1) / heads), h = 0 .. heads - 1."""
+    return [2.0 ** (-base * (h + 1) / heads) for h in range(heads)]
+
+
+class TiedAttention(nn.Module):
+    """Grouped-head softmax attention whose VALUES ARE ITS KEYS as projected: q = W_q h, k = W_k h (optional biases); queries and keys are
+    scored after an RMS norm per head (weights of `dim` entries shared by the heads), the read-out sums the keys as they came out of the
+    projection.  score = scale * q . k - slopes[h] * (i - j) (slopes None: no penalty); `window` > 0: a token sees itself and the window
+    - 1 before it; `chunk` > 0: it sees the earlier tokens of its own chunk of positions, i // chunk == j // chunk.
+    The cache holds ONE row per token under `cache_name`, the raw key, and beside it one float32 number per key/value head, the
+    reciprocal root mean square of the key: the norm's weight goes into the queries, the number multiplies the score, and neither the
+    norm nor a second row costs cache or bandwidth.  The projections q | k are rows of one matrix product.
+    `at`: the name of another set of cache rows (a layer that runs several times over a sequence has one per run)."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, scale: float, eps: float, cache_name, slopes=None, window=None, chunk=None,
+                 bias: bool = False, o_bias: bool = False):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("query heads must be a multiple of key/value heads")
+        if window and chunk:
+            raise ValueError("a window or chunks, not both")
+        self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, dim
+        self.scale, self.eps, self.window, self.chunk, self.cache_name = float(scale), eps, int(window or 0), int(chunk or 0), cache_name
+        self.q_cols, self.k_cols = heads * dim, kv_heads * dim
+        self.in_proj = nn.Linear(width, self.q_cols + self.k_cols, bias=bias)      # rows: q | k
+        self.q_norm = nn.Parameter(torch.zeros(dim, dtype=torch.float32))
+        self.k_norm = nn.Parameter(torch.zeros(dim, dtype=torch.float32))
+        if slopes is not None and len(slopes) != heads:
+            raise ValueError(f"{heads} heads need {heads} slopes, got {len(slopes)}")
+        self.register_buffer("slopes", torch.tensor([float(s) for s in slopes], dtype=torch.float32) if slopes is not None else None, persistent=False)
+        self.o_proj = nn.Linear(heads * dim, width, bias=o_bias)
+
+    def cache_rows(self, at=None) -> dict:
+        n = self.cache_name if at is None else at
+        return {(n, "k"): self.kv_heads * self.dim, (n, "rn"): (self.kv_heads, torch.float32)}
+
+    def forward(self, h: torch.Tensor, md, at=None) -> torch.Tensor:
+        n = self.cache_name if at is None else at
+        rows, rn = md.cache.latent((n, "k")), md.cache.latent((n, "rn"))
+        q = ops.tied_prep_store(self.in_proj(h), (0, self.q_cols), self.q_norm, self.k_norm, self.eps, md.out_slots, rows, rn, self.heads,
+                                self.kv_heads, self.dim)
+        o = ops.softcap_attn(q, rows, rows, md.kv_indices, md.kv_start, md.kv_len, md.layout, self.scale, 0.0, self.heads, self.kv_heads, self.dim,
+                             self.dim, window=self.window, chunk=self.chunk, slopes=self.slopes, k_rn=rn)
+        return self.o_proj(o)

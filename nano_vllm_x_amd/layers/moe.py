@@ -1,6 +1,6 @@
-"""Mixtures of small gated feed-forward experts: behind a sigmoid router whose score scales an expert's input, behind a softmax
-router with groups whose renormalised scores weigh the experts' outputs, or chosen by a table of token ids with fixed weights on
-the experts' outputs."""
+"""Gated feed-forward layers, and mixtures of small ones: behind a sigmoid router whose score scales an expert's input, behind a softmax
+router with groups whose renormalised scores weigh the experts' outputs, behind a sigmoid router with groups and a correction that
+enters the choice only, or chosen by a table of token ids with fixed weights on the experts' outputs."""
 from __future__ import annotations
 
 import torch
@@ -8,6 +8,32 @@ import torch.nn.functional as F
 from torch import nn
 
 from .. import ops
+
+
+class DenseGLU(nn.Module):
+    """W_down (g sigmoid(alpha g) (u + 1)) with g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit); gate and up are one product."""
+
+    def __init__(self, width: int, ff: int, limit: float, alpha: float):
+        super().__init__()
+        self.ff, self.limit, self.alpha = ff, float(limit), float(alpha)
+        self.gu_proj = nn.Linear(width, 2 * ff, bias=False)      # rows: gate | up
+        self.down = nn.Linear(ff, width, bias=False)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return self.down(ops.moe_glu(self.gu_proj(h), self.limit, self.alpha, 1.0))
+
+
+class GeluGLU(nn.Module):
+    """W_down (gelu_tanh(W_gate h) * (W_up h)); gate and up are one product."""
+
+    def __init__(self, width: int, ff: int):
+        super().__init__()
+        self.ff = ff
+        self.gu_proj = nn.Linear(width, 2 * ff, bias=False)      # rows: gate | up
+        self.down = nn.Linear(ff, width, bias=False)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        return self.down(ops.gelu_glu(self.gu_proj(h)))
 
 
 class ExpertBank(nn.Module):
@@ -150,3 +176,26 @@ class GroupedSoftmaxMoE(ExpertBank):
     def forward(self, h: torch.Tensor, decode_step: bool = False) -> torch.Tensor:
         idx, wts = ops.moe_route_softmax(ops.skinny_proj(h, self.router), self.top, self.groups, self.keep, self.norm_eps)
         return self.run(h, idx, wts, decode_step, weight_out=True)
+
+
+class GroupedSigmoidMoE(ExpertBank):
+    """scores = sigmoid(W_router h) (float32), choice scores = scores + `correction` (one number per expert, which moves the choice and not
+    the weights).  The experts form `groups` equal groups of neighbours; a group counts as the sum of its two largest choice scores and only
+    experts of the `keep` best groups can be chosen (groups None or 1: no such limit).  Every token takes the `top` largest choice scores;
+    the weights are scale * score, not renormalised, and weigh the experts' OUTPUTS.  `shared`: a feed-forward that every token passes, whose
+    result comes beside the experts' sum.  Expert: g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), W_down (g * sigmoid(alpha *
+    g) * (u + shift)).  Returns (experts' sum, shared result or None): the two are added where they enter the float32 stream."""
+
+    def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, alpha: float, shift: float = 1.0, groups=None, keep=None,
+                 scale: float = 1.0, shared: nn.Module | None = None):
+        super().__init__(width, experts, top, ff, limit, alpha, shift)
+        self.groups, self.keep, self.scale = int(groups or 0), int(keep or 0), float(scale)
+        if self.groups > 1 and (experts % self.groups or not 1 <= self.keep <= self.groups or self.keep * (experts // self.groups) < top):
+            raise ValueError("groups must divide the experts and the kept groups must hold `top` experts")
+        self.router = nn.Parameter(torch.zeros(experts, width, dtype=torch.float32))
+        self.correction = nn.Parameter(torch.zeros(experts, dtype=torch.float32))
+        self.shared = shared
+
+    def forward(self, h: torch.Tensor, decode_step: bool = False):
+        idx, wts = ops.moe_route_sigmoid(ops.skinny_proj(h, self.router), self.correction, self.top, self.groups, self.keep, self.scale)
+        return self.run(h, idx, wts, decode_step, weight_out=True), self.shared(h) if self.shared is not None else None

@@ -39,7 +39,8 @@ class MLSTM(nn.Module):
     m' = max(f + m, i), S <- e^(f + m - m') S + e^(i - m') k v^T, n likewise with k alone,
     o = S^T q / (max(|n . q|, e^(-m')) + 1e-6) with q = W_q h / sqrt(dim).  Each head's o is divided by its root mean square,
     the heads times `norm` times sigmoid(W_g h), then W_o.  q, k, v and the output gate are one matrix product; the two
-    gate projections are float32 and so are S, n and m, which live in the state pool under (state_name, "S" | "n" | "m")."""
+    gate projections are float32 and so are S, n and m, which live in the state pool under (state_name, "S" | "n" | "m") -- or under
+    the name `at` (a layer that runs several times over a sequence has a state per run)."""
 
     def __init__(self, width: int, heads: int, dim: int, vdim: int, gate_cap: float, eps: float, state_name):
         super().__init__()
@@ -49,12 +50,12 @@ class MLSTM(nn.Module):
         self.norm = _f32(heads * vdim)
         self.o_proj = nn.Linear(heads * vdim, width, bias=False)
 
-    def state_shapes(self) -> dict:
-        n = self.state_name
+    def state_shapes(self, at=None) -> dict:
+        n = self.state_name if at is None else at
         return {(n, "S"): (self.heads, self.dim, self.vdim), (n, "n"): (self.heads, self.dim), (n, "m"): (self.heads,)}
 
-    def forward(self, h: torch.Tensor, md) -> torch.Tensor:
-        hd, he, n = self.heads * self.dim, self.heads * self.vdim, self.state_name
+    def forward(self, h: torch.Tensor, md, at=None) -> torch.Tensor:
+        hd, he, n = self.heads * self.dim, self.heads * self.vdim, self.state_name if at is None else at
         x = self.qkvg_proj(h)
         gates = ops.skinny_proj(h, self.gate_w)
         o = ops.mlstm_scan(x, (0, hd, 2 * hd), gates, self.gate_b, self.gate_cap, md.cache.state((n, "S")), md.cache.state((n, "n")),
@@ -211,3 +212,31 @@ class RGLRU(nn.Module):
         gates = torch.bmm(u.view(t, self.blocks, -1).transpose(0, 1), self.gate_w)      # (blocks, T, 2 * block width)
         s = ops.rglru_scan(yx[:, :self.inner], u, gates, self.gate_b, self.rate, md.cache.state((n, "S")), md.layout)
         return self.o_proj(s)
+
+
+class GatedLinearAttention(nn.Module):
+    """Linear attention with a decay per key channel and token: q = W_q h / sqrt(dim), k = W_k h (heads x dim), v = W_v h (heads x vdim),
+    alpha = sigmoid(W_a2 (W_a1 h) + b)^(1 / tau) (heads x dim); per head S <- diag(alpha) S + k v^T, o = S^T q (the read sees the
+    token's own write).  Each head's o is divided by its root mean square, times `norm` (vdim, shared by the heads), times silu(W_g h), then
+    W_o.  q, k, v and the output gate are one matrix product; the two small projections of the decay are float32 and so are alpha and S,
+    which lives in the state pool under (state_name, "S"), or under the name `at` (see MLSTM).  The inner size of the decay's projections
+    is that of the parameters a1 and a2 (a checkpoint's shapes set it)."""
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, tau: float, rank: int, eps: float, state_name):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.tau, self.eps, self.state_name = heads, dim, vdim, float(tau), eps, state_name
+        self.qkvg_proj = nn.Linear(width, 2 * heads * dim + 2 * heads * vdim, bias=False)     # rows: q | k | v | g
+        self.a1, self.a2, self.a2_b = _f32(rank, width), _f32(heads * dim, rank), _f32(heads * dim)
+        self.norm = _f32(vdim)
+        self.o_proj = nn.Linear(heads * vdim, width, bias=False)
+
+    def state_shapes(self, at=None) -> dict:
+        return {(self.state_name if at is None else at, "S"): (self.heads, self.dim, self.vdim)}
+
+    def forward(self, h: torch.Tensor, md, at=None) -> torch.Tensor:
+        hd, he, n = self.heads * self.dim, self.heads * self.vdim, self.state_name if at is None else at
+        x = self.qkvg_proj(h)
+        alpha = ops.skinny_proj(ops.skinny_proj(h, self.a1), self.a2, bias=self.a2_b, out_act="sigmoid_pow", power=1.0 / self.tau)
+        o = ops.gla_scan(x, (0, hd, 2 * hd), alpha, md.cache.state((n, "S")), md.layout, self.heads, self.dim, self.vdim, q_mul=self.dim ** -0.5)
+        y = ops.head_norm_gate(o, self.norm, self.eps, gate=x[:, 2 * hd + he:], kind="silu")
+        return self.o_proj(y)

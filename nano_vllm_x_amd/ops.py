@@ -967,10 +967,33 @@ def token_shift_mix(h, mu, state, layout: StepLayout):
     return out
 
 
-def mlstm_scan(x, offsets, gates, gate_bias, cap: float, mem, norm, peak, layout: StepLayout, heads: int, dim: int, vdim: int):
+SCAN_CHUNK_FROM = 256       # portions from this length on are cut into chunks that run side by side
+SCAN_CHUNKS = ((65536, 32), (131072, 64), (None, 128))      # (tokens x heads of a step up to ..., tokens of a chunk): short chunks while
+# the step is too small to fill the chip with long ones, long chunks (fewer carried states) from there on (4 x 1 024 tokens, 8
+# heads: 895 us in one walk, 301 in chunks of 128, 150 in chunks of 32; 16 x 1 024 tokens: 446 us at 128 and 64, 474 at 32)
+SCAN_WS_BYTES = 1 << 30     # the chunks' states may take this much; longer chunks otherwise
+
+
+def _scan_chunks(layout: StepLayout, heads: int, per_chunk: int, chunk: Optional[int]):
+    """(chunk, chunks of the longest portion) a recurrence over a matrix per head cuts a step's portions into (0, 0: not at all).
+    `per_chunk`: floats of workspace a chunk of one sequence takes; `chunk` None: by the step's shape."""
+    if chunk is None:
+        chunk = 0
+        if layout.qo_indptr is not None and layout.max_q >= SCAN_CHUNK_FROM:
+            chunk = next(c for upto, c in SCAN_CHUNKS if upto is None or layout.n_tok * heads <= upto)
+    if not chunk or layout.qo_indptr is None:
+        return 0, 0
+    while layout.n_seq * -(-layout.max_q // chunk) * per_chunk * 4 > SCAN_WS_BYTES or layout.n_seq * -(-layout.max_q // chunk) > 65535:
+        chunk *= 2
+    n_chunks = -(-layout.max_q // chunk)
+    return (chunk, n_chunks) if n_chunks > 1 else (0, 0)
+
+
+def mlstm_scan(x, offsets, gates, gate_bias, cap: float, mem, norm, peak, layout: StepLayout, heads: int, dim: int, vdim: int,
+               chunk: Optional[int] = None):
     """Matrix memory with a stabilised exponential input gate.  x (T, >= ...): q, k (heads * dim each) and v (heads * vdim) at the
     three column `offsets`; gates (T, 2 * heads) float32 = input | forget pre-activations, gate_bias (2 * heads); mem (slots,
-    heads, dim, vdim), norm (slots, heads, dim), peak (slots, heads) float32, continued and written back.
+    heads, dim, vdim), norm (slots, heads, dim), peak (slots, heads) float32, continued and written back.  `chunk` as for decay_scan.
     Returns the read-out (T, heads, vdim) float32."""
     _dev(x, gates, gate_bias, mem, norm, peak)
     _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[0] == layout.n_tok, "mlstm_scan: x must be (T, columns) with unit inner stride")
@@ -984,11 +1007,14 @@ def mlstm_scan(x, offsets, gates, gate_bias, cap: float, mem, norm, peak, layout
     lib = _lib.load()
     # a head whose value columns take several workgroups: all of them read the normaliser and the maximum, the first writes them
     # back, so they read from copies (a workgroup that starts late must not see the new values)
-    several = lib.nvx_scan_column_blocks(dim, vdim) != 1
+    per_chunk = heads * (dim * (vdim + 1) + 3)
+    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk)
+    ws = torch.empty((layout.n_seq * n_chunks * per_chunk,), dtype=F32, device=x.device) if chunk else None
+    several = not chunk and lib.nvx_scan_column_blocks(dim, vdim) != 1
     norm_in, peak_in = (norm.clone(), peak.clone()) if several else (norm, peak)
     _lib.check(lib.nvx_mlstm_scan(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], _ptr(gates), _ptr(gate_bias), float(cap),
                                   _ptr(mem), _ptr(norm_in), _ptr(peak_in), _ptr(norm), _ptr(peak), n_slots, *_layout_args(layout), _ptr(out), t, layout.n_seq, heads, dim, vdim,
-                                  _stream()), "nvx_mlstm_scan")
+                                  chunk, n_chunks, _ptr(ws), _stream()), "nvx_mlstm_scan")
     return out
 
 
@@ -1061,10 +1087,13 @@ SOFTCAP_SPLITS = 4
 
 def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: StepLayout, scale: float, cap: float, heads: int,
                  kv_heads: int, dim: int, vdim: int, n_split: Optional[int] = None, window: int = 0, r1=None, r2=None, v_turn=None,
-                 v_interleaved: bool = False, gate=None, matrix_cores: bool = True, sink_score: Optional[float] = None):
+                 v_interleaved: bool = False, gate=None, matrix_cores: bool = True, sink_score: Optional[float] = None, chunk: int = 0, slopes=None,
+                 k_rn=None):
     """Causal attention of q (T, heads * dim) over cached rows: sequence b's tokens are at slots kv_indices[kv_start[b] :
     kv_start[b] + kv_len[b]]; scores scale * q . k pass cap * tanh(. / cap) (cap <= 0: not) before the softmax.
-    `window` > 0: a token sees itself and the window - 1 tokens before it.  `r1`, `r2` (heads, float32): r1 ln(1 + r2 (i - j)) is
+    `window` > 0: a token sees itself and the window - 1 tokens before it; `chunk` > 0: those of its own chunk of positions (i // chunk
+    equal).  `slopes` (heads, float32): slopes[h] (i - j) is taken off the score.  `k_rn` (slots, kv_heads, float32), as tied_prep_store
+    fills it: a key's score is multiplied by its entry (k_cache and v_cache may then be the same tensor).  `r1`, `r2` (heads, float32): r1 ln(1 + r2 (i - j)) is
     taken off the score of key j for the query at position i.  `v_turn` (T, vdim) float32, every query token's cos | sin as
     attn_prep_store returns them: the read-out's pairs ((m, m + vdim / 2), or (2m, 2m + 1) if `v_interleaved`) are turned back by
     those angles, undoing the turn attn_prep_store gave the values.  `gate`
@@ -1081,6 +1110,15 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
           "softcap_attn: v_turn must be float32 (T, vdim)")
     _need(gate is None or (gate.dim() == 2 and gate.shape[0] == q.shape[0] and gate.shape[1] in (heads, heads * vdim) and gate.stride(1) == 1 and
                            gate.dtype == q.dtype), "softcap_attn: gate shape / format")
+    _need(not (window and chunk), "softcap_attn: a window or chunks, not both")
+    if slopes is not None:
+        _dev(slopes)
+        _f32c(slopes, "softcap_attn: slopes")
+        _need(slopes.numel() == heads, "softcap_attn: slopes have one number per head")
+    if k_rn is not None:
+        _dev(k_rn)
+        _f32c(k_rn, "softcap_attn: k_rn")
+        _need(k_rn.shape == (k_cache.shape[0], kv_heads), "softcap_attn: k_rn must be (slots, kv_heads)")
     gate_per_head = gate is not None and gate.shape[1] == heads and vdim != 1
     t = q.shape[0]
     _need(q.shape == (t, heads * dim) and q.is_contiguous() and t == layout.n_tok, "softcap_attn: q must be contiguous (T, heads * dim)")
@@ -1099,7 +1137,8 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
     lib = _lib.load()
     _lib.check(lib.nvx_softcap_attn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _fmt(q), _ptr(kv_indices), _ptr(kv_start), _ptr(kv_len),
                                     _ptr(layout.qo_indptr), _ptr(layout.tok_seq), float(scale), float(cap), _ptr(out), t, heads, kv_heads, dim,
-                                    vdim, n_split, _ptr(part), int(window or 0), _ptr(r1), _ptr(r2), _ptr(v_turn), int(bool(v_interleaved)),
+                                    vdim, n_split, _ptr(part), int(window or 0), int(chunk or 0), _ptr(r1), _ptr(r2), _ptr(slopes), _ptr(k_rn), _ptr(v_turn),
+                                    int(bool(v_interleaved)),
                                     _ptr(gate), gate.stride(0) if gate is not None else 0, int(gate_per_head), int(sink_score is not None),
                                     float(sink_score or 0.0), layout.n_seq, int(bool(matrix_cores)), _stream()),
                "nvx_softcap_attn")
@@ -1146,13 +1185,6 @@ def attn_prep_store(x, offsets, positions, q_w, k_w, norm_mode: str, eps: float,
     return q, v_turn
 
 
-DECAY_SCAN_CHUNK_FROM = 256       # portions from this length on are cut into chunks that run side by side
-DECAY_SCAN_CHUNKS = ((65536, 32), (131072, 64), (None, 128))      # (tokens x heads of a step up to ..., tokens of a chunk): short chunks while
-# the step is too small to fill the chip with long ones, long chunks (fewer carried states) from there on (4 x 1 024 tokens, 8
-# heads: 895 us in one walk, 301 in chunks of 128, 150 in chunks of 32; 16 x 1 024 tokens: 446 us at 128 and 64, 474 at 32)
-DECAY_SCAN_WS_BYTES = 1 << 30     # the chunks' states may take this much; longer chunks otherwise
-
-
 def decay_scan(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int, vdim: int, act: str = "none", chunk: Optional[int] = None):
     """Linear attention with one constant decay per head.  x (T, columns): q, k (heads * dim each) and v (heads * vdim) at the
     three column `offsets`, passed through `act` ("none" or "silu") first; decay (heads) float32; mem (slots, heads, dim, vdim)
@@ -1167,20 +1199,8 @@ def decay_scan(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int,
     _need(decay.numel() == heads and mem.shape == (n_slots, heads, dim, vdim), "decay_scan: shapes")
     t = x.shape[0]
     out = torch.empty((t, heads, vdim), dtype=F32, device=x.device)
-    if chunk is None:
-        chunk = 0
-        if layout.qo_indptr is not None and layout.max_q >= DECAY_SCAN_CHUNK_FROM:
-            chunk = next(c for upto, c in DECAY_SCAN_CHUNKS if upto is None or t * heads <= upto)
-    n_chunks, ws = 0, None
-    if chunk and layout.qo_indptr is not None:
-        per = heads * dim * vdim * 4
-        while layout.n_seq * -(-layout.max_q // chunk) * per > DECAY_SCAN_WS_BYTES or layout.n_seq * -(-layout.max_q // chunk) > 65535:
-            chunk *= 2
-        n_chunks = -(-layout.max_q // chunk)
-        if n_chunks > 1:
-            ws = torch.empty((layout.n_seq * n_chunks, heads, dim, vdim), dtype=F32, device=x.device)
-    if ws is None:
-        chunk = n_chunks = 0
+    chunk, n_chunks = _scan_chunks(layout, heads, heads * dim * vdim, chunk)
+    ws = torch.empty((layout.n_seq * n_chunks, heads, dim, vdim), dtype=F32, device=x.device) if chunk else None
     lib = _lib.load()
     _lib.check(lib.nvx_decay_scan(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], {"none": 0, "silu": 1}[act], _ptr(decay),
                                   _ptr(mem), n_slots, *_layout_args(layout), _ptr(out), t, layout.n_seq, heads, dim, vdim, chunk, n_chunks,
@@ -1339,8 +1359,8 @@ def moe_gather_rows(ys, dst, wts=None):
     return out
 
 
-def skinny_proj(x, w, in_act: str = "none"):
-    """out = f(x) @ w.T in float32, f = identity or tanh: x (T, k_in) in any activation format (rows may be a slice of wider
+def skinny_proj(x, w, in_act: str = "none", bias=None, out_act: str = "none", power: float = 1.0):
+    """out = g(f(x) @ w.T + bias) in float32, f = identity or tanh, g = identity or ("sigmoid_pow") sigmoid(.)^power: x (T, k_in) in any activation format (rows may be a slice of wider
     rows), w (n_out, k_in) float32.  For few outputs (gate and router logits) or few inputs; one fixed summation order and
     no workspace, so a captured launch replays to the same bits."""
     _dev(x, w)
@@ -1348,8 +1368,12 @@ def skinny_proj(x, w, in_act: str = "none"):
     _need(x.dim() == 2 and x.stride(1) == 1 and w.dim() == 2 and w.shape[1] == x.shape[1], "skinny_proj: x must be (T, k_in), w (n_out, k_in)")
     out = torch.empty((x.shape[0], w.shape[0]), dtype=F32, device=x.device)
     lib = _lib.load()
-    _lib.check(lib.nvx_skinny_proj(_ptr(x), x.stride(0), _fmt(x), _ptr(w), {"none": 0, "tanh": 1}[in_act], _ptr(out), x.shape[0], w.shape[0],
-                                   x.shape[1], _stream()), "nvx_skinny_proj")
+    if bias is not None:
+        _dev(bias)
+        _f32c(bias, "skinny_proj: bias")
+        _need(bias.numel() == w.shape[0], "skinny_proj: bias size")
+    _lib.check(lib.nvx_skinny_proj(_ptr(x), x.stride(0), _fmt(x), _ptr(w), {"none": 0, "tanh": 1}[in_act], _ptr(bias), {"none": 0, "sigmoid_pow": 1}[out_act],
+                                   float(power), _ptr(out), x.shape[0], w.shape[0], x.shape[1], _stream()), "nvx_skinny_proj")
     return out
 
 
@@ -1479,3 +1503,147 @@ def moe_route_softmax(logits, top: int, n_groups: int = 0, keep_groups: int = 0,
     _lib.check(lib.nvx_moe_route_softmax(_ptr(logits), t, n_exp, top, int(n_groups or 0), int(keep_groups or 0), float(norm_eps), _ptr(idx),
                                          _ptr(wts), _stream()), "nvx_moe_route_softmax")
     return idx, wts
+
+
+# ---------------------------------------------------------------------------------------------
+# plain pre-normed stream with its embedding sum, tied keys and values, gated linear attention, the sigmoid router with groups
+# ---------------------------------------------------------------------------------------------
+def _row_end(t: int, width: int, w, split: bool, dtype, device, what: str):
+    """The row output of residual_norm and embed_sum: none, the normed row, or the [hi | lo] pair."""
+    if w is None and not split:
+        return None
+    if w is not None:
+        _dev(w)
+        _f32c(w, what + ": w")
+        _need(w.numel() == width and not split, what + ": w size (and no split beside a norm)")
+    return torch.empty((t, 2 * width if split else width), dtype=dtype, device=device)
+
+
+def residual_norm(x, y=None, y2=None, add=None, bias=None, w=None, eps: float = 0.0, split: bool = False, dtype=None, out=None):
+    """v = x (+ y) (+ y2) (+ add) (+ bias): x, add (T, width) and bias (width) float32, y and y2 (T, width) in the activations' format
+    `dtype` (default: y's).  v replaces x, or goes to `out`.  Returns v / rms(v) * w if `w` (width, float32) is given, [hi | lo] (T, 2 *
+    width) with hi = v rounded to `dtype` and lo = what that lost if `split`, else None."""
+    _dev(x, y, y2, add, bias, out)
+    _f32c(x, "residual_norm: x")
+    t, width = x.shape
+    for name, r in (("y", y), ("y2", y2)):
+        _need(r is None or (r.shape == (t, width) and r.stride(1) == 1), f"residual_norm: {name} must be (T, width) with unit inner stride")
+    for name, r, shape in (("add", add, (t, width)), ("bias", bias, (width,)), ("out", out, (t, width))):
+        if r is not None:
+            _f32c(r, "residual_norm: " + name)
+            _need(tuple(r.shape) == shape, f"residual_norm: {name} shape")
+    dtype = dtype or (y.dtype if y is not None else None)
+    _need(dtype in _FMT and all(r is None or r.dtype == dtype for r in (y, y2)), "residual_norm: y, y2 and the output share one format")
+    h = _row_end(t, width, w, split, dtype, x.device, "residual_norm")
+    lib = _lib.load()
+    _lib.check(lib.nvx_residual_norm(_ptr(x), _ptr(y), y.stride(0) if y is not None else 0, _ptr(y2), y2.stride(0) if y2 is not None else 0, _ptr(add),
+                                     _ptr(bias), _FMT[dtype], _ptr(x if out is None else out), _ptr(w), float(eps), int(split), _ptr(h), t, width,
+                                     _stream()), "nvx_residual_norm")
+    return h
+
+
+def embed_sum(ids, table, layout: Optional[StepLayout] = None, pair=None, mul_prev: int = 0, mul_cur: int = 0, prev_id=None, pos_table=None,
+              positions=None, w=None, eps: float = 0.0, split: bool = False):
+    """x = table[ids] (+ pair[r]) (+ pos_table[positions]) in float32, r = (previous id * mul_prev + id * mul_cur) mod buckets with buckets
+    = pair.shape[0] - 1, and the last row for a sequence's first token; prev_id (slots, 1) float32 carries every sequence's last id from
+    step to step.  Returns (x, h), h as residual_norm's result."""
+    _dev(ids, table, pair, prev_id, pos_table, positions)
+    t, width = ids.numel(), table.shape[1]
+    _need(ids.dtype == torch.int64 and ids.is_contiguous() and table.dim() == 2 and table.is_contiguous(), "embed_sum: ids must be int64, the table contiguous")
+    for name, tab in (("pair", pair), ("pos_table", pos_table)):
+        _need(tab is None or (tab.dtype == table.dtype and tab.is_contiguous() and tab.dim() == 2 and tab.shape[1] == width), f"embed_sum: {name} shape / format")
+    la = (None, None, None, None)
+    n_slots = 0
+    if pair is not None:
+        _need(pair.shape[0] >= 2 and layout is not None and layout.n_tok == t, "embed_sum: the pair table needs the step's layout")
+        _f32c(prev_id, "embed_sum: prev_id")
+        n_slots = prev_id.shape[0]
+        _need(prev_id.numel() == n_slots, "embed_sum: prev_id has one word per slot")
+        la = (_ptr(layout.tok_seq), *_layout_args(layout))
+    if pos_table is not None:
+        _need(positions is not None and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == t, "embed_sum: positions must be int64 (T)")
+    x = torch.empty((t, width), dtype=F32, device=ids.device)
+    h = _row_end(t, width, w, split, table.dtype, ids.device, "embed_sum")
+    lib = _lib.load()
+    _lib.check(lib.nvx_embed_sum(_ptr(ids), _ptr(table), _fmt(table), table.shape[0], _ptr(pair), pair.shape[0] - 1 if pair is not None else 0, int(mul_prev),
+                                 int(mul_cur), _ptr(prev_id), n_slots, _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0,
+                                 _ptr(positions) if pos_table is not None else None, *la, _ptr(x), _ptr(w), float(eps), int(split), _ptr(h), t,
+                                 layout.n_seq if layout is not None else t, width, _stream()), "nvx_embed_sum")
+    return x, h
+
+
+def tied_prep_store(x, offsets, q_w, k_w, eps: float, slots, k_cache, k_rn, heads: int, kv_heads: int, dim: int):
+    """After a fused projection x (T, columns) holding q and k at the two column `offsets`, for heads whose values are their keys as
+    projected: k_cache[slots] = k, k_rn[slots] = 1 / rms(k) per head (float32), and the queries RMS-normed per head times q_w * k_w (dim
+    entries each, shared by the heads).  softcap_attn(q, k_cache, k_cache, k_rn=k_rn) then scores normed keys and reads raw ones."""
+    _dev(x, q_w, k_w, slots, k_cache, k_rn)
+    t = x.shape[0]
+    _need(x.dim() == 2 and x.stride(1) == 1, "tied_prep_store: x must be (T, columns) with unit inner stride")
+    for name, w in (("q_w", q_w), ("k_w", k_w), ("k_rn", k_rn)):
+        _f32c(w, "tied_prep_store: " + name)
+    n_slots = k_cache.shape[0]
+    _need(q_w.numel() == dim and k_w.numel() == dim, "tied_prep_store: norm weights have dim entries")
+    _need(slots.dtype == torch.int64 and slots.is_contiguous() and slots.numel() == t, "tied_prep_store: slots must be int64 (T)")
+    _need(k_cache.dtype == x.dtype and k_cache.is_contiguous() and k_cache.shape == (n_slots, kv_heads * dim) and k_rn.shape == (n_slots, kv_heads),
+          "tied_prep_store: cache shapes")
+    q = torch.empty((t, heads * dim), dtype=x.dtype, device=x.device)
+    lib = _lib.load()
+    _lib.check(lib.nvx_tied_prep_store(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], _ptr(q_w), _ptr(k_w), float(eps), _ptr(slots), _ptr(q),
+                                       _ptr(k_cache), _ptr(k_rn), n_slots, t, heads, kv_heads, dim, _stream()), "nvx_tied_prep_store")
+    return q
+
+
+def gla_scan(x, offsets, alpha, mem, layout: StepLayout, heads: int, dim: int, vdim: int, q_mul: float = 1.0, chunk: Optional[int] = None):
+    """Gated linear attention.  x (T, columns): q, k (heads * dim each) and v (heads * vdim) at the three column `offsets`; alpha (T, heads
+    * dim) float32, the decay of every key channel; mem (slots, heads, dim, vdim) float32, continued and written back.
+    S <- diag(alpha) S + k v^T, read-out q_mul S^T q.  `chunk` as for decay_scan.  Returns (T, heads, vdim) float32."""
+    _dev(x, alpha, mem)
+    _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[0] == layout.n_tok, "gla_scan: x must be (T, columns) with unit inner stride")
+    t = x.shape[0]
+    _f32c(alpha, "gla_scan: alpha")
+    _f32c(mem, "gla_scan: mem")
+    n_slots = mem.shape[0]
+    _need(alpha.shape == (t, heads * dim) and mem.shape == (n_slots, heads, dim, vdim), "gla_scan: shapes")
+    out = torch.empty((t, heads, vdim), dtype=F32, device=x.device)
+    per_chunk = heads * dim * (vdim + 1)
+    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk)
+    ws = torch.empty((layout.n_seq * n_chunks * per_chunk,), dtype=F32, device=x.device) if chunk else None
+    lib = _lib.load()
+    _lib.check(lib.nvx_gla_scan(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], float(q_mul), _ptr(alpha), _ptr(mem), n_slots,
+                                *_layout_args(layout), _ptr(out), t, layout.n_seq, heads, dim, vdim, chunk, n_chunks, _ptr(ws), _stream()), "nvx_gla_scan")
+    return out
+
+
+def moe_route_sigmoid(logits, correction, top: int, n_groups: int = 0, keep_groups: int = 0, scale: float = 1.0):
+    """logits (T, experts) float32 -> (ids (T, top) int32, weights (T, top) float32).  Scores are sigmoids; choice scores are score +
+    correction (experts, float32).  With n_groups > 1 the experts form equal groups of neighbours, a group counts as the sum of its two
+    largest choice scores, and only experts of the keep_groups best groups can be chosen; the `top` largest choice scores are taken
+    (ties: the lower id).  A weight is the expert's score (without the correction) times `scale`."""
+    _dev(logits, correction)
+    _f32c(logits, "moe_route_sigmoid: logits")
+    _f32c(correction, "moe_route_sigmoid: correction")
+    t, n_exp = logits.shape
+    _need(correction.numel() == n_exp, "moe_route_sigmoid: one correction per expert")
+    idx = torch.empty((t, top), dtype=torch.int32, device=logits.device)
+    wts = torch.empty((t, top), dtype=F32, device=logits.device)
+    lib = _lib.load()
+    _lib.check(lib.nvx_moe_route_sigmoid(_ptr(logits), _ptr(correction), t, n_exp, top, int(n_groups or 0), int(keep_groups or 0), float(scale), _ptr(idx),
+                                         _ptr(wts), _stream()), "nvx_moe_route_sigmoid")
+    return idx, wts
+
+
+def gelu_glu(gu):
+    """gu (rows, 2 * ff) = gate | up pre-activations -> gelu_tanh(gate) * up."""
+    _dev(gu)
+    _need(gu.dim() == 2 and gu.is_contiguous() and gu.shape[1] % 2 == 0, "gelu_glu: gu must be contiguous (rows, 2 * ff)")
+    y = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
+    lib = _lib.load()
+    _lib.check(lib.nvx_gelu_glu(_ptr(gu), _fmt(gu), _ptr(y), gu.shape[0], gu.shape[1] // 2, _stream()), "nvx_gelu_glu")
+    return y
+
+
+def product_f32(x, w):
+    """x @ w.T as a library product that returns its float32 sums unrounded; x (T, k), w (n, k) in one format."""
+    if x.dtype == F32:
+        return torch.nn.functional.linear(x, w)
+    return torch.mm(x, w.t(), out_dtype=F32)

@@ -34,8 +34,14 @@ def _ladusun():
     return LadusunConfig.from_dict, LadusunForCausalLM
 
 
+def _zenedra():
+    from .zenedra import ZenedraConfig, ZenedraForCausalLM
+    return ZenedraConfig.from_dict, ZenedraForCausalLM
+
+
 # architecture name (config.json "architectures"[0] or "architecture") -> loader of (config reader, model class)
-ARCHITECTURES = {"Qwen3ForCausalLM": _qwen3, "Kabidra": _kabidra, "Meronex": _meronex, "Gibavik": _gibavik, "Ladusun": _ladusun}
+ARCHITECTURES = {"Qwen3ForCausalLM": _qwen3, "Kabidra": _kabidra, "Meronex": _meronex, "Gibavik": _gibavik, "Ladusun": _ladusun,
+                 "Zenedra": _zenedra}
 
 
 def architecture_of(config: dict) -> str:

@@ -85,7 +85,7 @@ _DEFS = {
     "softcap_attn": "(Tensor q, Tensor k_cache, Tensor v_cache, Tensor kv_indices, Tensor kv_start, Tensor kv_len, Tensor pos0, "
                     "Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq, float scale, float cap, int heads, int kv_heads, int dim, int vdim, "
                     "int window=0, Tensor? r1=None, Tensor? r2=None, Tensor? v_turn=None, bool v_interleaved=False, Tensor? gate=None, "
-                    "float? sink_score=None) -> Tensor",
+                    "float? sink_score=None, int chunk=0, Tensor? slopes=None, Tensor? k_rn=None) -> Tensor",
     # post-normed stream, query/key norms with rotated values, decayed linear attention, experts with weights on their outputs
     "attn_prep_store": "(Tensor x, int q_off, int k_off, int v_off, Tensor positions, Tensor? q_w, Tensor? k_w, str norm_mode, float eps, "
                        "Tensor? freq, int rot_dims, bool interleaved, Tensor? vfreq, Tensor? slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, "
@@ -102,7 +102,7 @@ _DEFS = {
     "moe_scatter_rows": "(Tensor h, Tensor? wts, Tensor dst) -> Tensor",
     "moe_glu": "(Tensor gu, float limit, float alpha, float shift=1.0) -> Tensor",
     "moe_gather_rows": "(Tensor ys, Tensor dst, Tensor? wts=None) -> Tensor",
-    "skinny_proj": "(Tensor x, Tensor w, str in_act) -> Tensor",
+    "skinny_proj": "(Tensor x, Tensor w, str in_act, Tensor? bias=None, str out_act='none', float power=1.0) -> Tensor",
     # several residual streams, the real-gated recurrence, a latent with a rotated key part, the softmax router with groups
     "hyper_mix": "(Tensor(a!) x, Tensor? y, Tensor? scale, Tensor? mix, Tensor? w_out, Tensor? w_in, Tensor? w_norm, float eps, ScalarType out_dtype) "
                  "-> Tensor",
@@ -114,6 +114,16 @@ _DEFS = {
     "latent_rope_prep": "(Tensor x, int q_off, int kv_off, int g_off, Tensor positions, Tensor? freq, float mag, Tensor w_kv, float eps, "
                         "Tensor slots, Tensor(a!) cache, int heads, int dim, int rot) -> (Tensor, Tensor)",
     "moe_route_softmax": "(Tensor logits, int top, int n_groups, int keep_groups, float norm_eps) -> (Tensor, Tensor)",
+    # plain pre-normed stream with its embedding sum, tied keys and values, gated linear attention, the sigmoid router with groups
+    "residual_norm": "(Tensor(a!) x, Tensor? y, Tensor? y2, Tensor? add, Tensor? bias, Tensor? w, float eps, bool split, ScalarType dtype) -> Tensor?",
+    "embed_sum": "(Tensor ids, Tensor table, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq, Tensor? pair, int mul_prev, int mul_cur, "
+                 "Tensor(a!)? prev_id, Tensor? pos_table, Tensor? positions, Tensor? w, float eps, bool split) -> (Tensor, Tensor?)",
+    "tied_prep_store": "(Tensor x, int q_off, int k_off, Tensor q_w, Tensor k_w, float eps, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_rn, "
+                       "int heads, int kv_heads, int dim) -> Tensor",
+    "gla_scan": "(Tensor x, int q_off, int k_off, int v_off, Tensor alpha, Tensor(a!) mem, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, "
+                "Tensor? tok_seq, int heads, int dim, int vdim, float q_mul) -> Tensor",
+    "moe_route_sigmoid": "(Tensor logits, Tensor correction, int top, int n_groups, int keep_groups, float scale) -> (Tensor, Tensor)",
+    "gelu_glu": "(Tensor gu) -> Tensor",
 }
 for _name, _sig in _DEFS.items():
     _LIB.define(_name + _sig)
@@ -308,10 +318,10 @@ def _rope_vnorm_store(qkv, positions, freq, mag, rot_dims, eps, slots, k_cache, 
 
 
 def _softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, pos0, state_slot, qo_indptr, tok_seq, scale, cap, heads, kv_heads, dim, vdim,
-                  window=0, r1=None, r2=None, v_turn=None, v_interleaved=False, gate=None, sink_score=None):
+                  window=0, r1=None, r2=None, v_turn=None, v_interleaved=False, gate=None, sink_score=None, chunk=0, slopes=None, k_rn=None):
     return ops.softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, _layout(q.shape[0], pos0, state_slot, qo_indptr, tok_seq), scale, cap,
                             heads, kv_heads, dim, vdim, window=window, r1=r1, r2=r2, v_turn=v_turn, v_interleaved=v_interleaved, gate=gate,
-                            sink_score=sink_score)
+                            sink_score=sink_score, chunk=chunk, slopes=slopes, k_rn=k_rn)
 
 
 def _attn_prep_store(x, q_off, k_off, v_off, positions, q_w, k_w, norm_mode, eps, freq, rot_dims, interleaved, vfreq, slots, k_cache, v_cache,
@@ -360,8 +370,8 @@ def _moe_gather_rows(ys, dst, wts=None):
     return ops.moe_gather_rows(ys, dst, wts)
 
 
-def _skinny_proj(x, w, in_act):
-    return ops.skinny_proj(x, w, in_act)
+def _skinny_proj(x, w, in_act, bias=None, out_act="none", power=1.0):
+    return ops.skinny_proj(x, w, in_act, bias=bias, out_act=out_act, power=power)
 
 
 def _hyper_mix(x, y, scale, mix, w_out, w_in, w_norm, eps, out_dtype):
@@ -386,6 +396,31 @@ def _latent_rope_prep(x, q_off, kv_off, g_off, positions, freq, mag, w_kv, eps, 
 
 def _moe_route_softmax(logits, top, n_groups, keep_groups, norm_eps):
     return ops.moe_route_softmax(logits, top, n_groups, keep_groups, norm_eps)
+
+
+def _residual_norm(x, y, y2, add, bias, w, eps, split, dtype):
+    return ops.residual_norm(x, y, y2, add=add, bias=bias, w=w, eps=eps, split=split, dtype=dtype)
+
+
+def _embed_sum(ids, table, pos0, state_slot, qo_indptr, tok_seq, pair, mul_prev, mul_cur, prev_id, pos_table, positions, w, eps, split):
+    return ops.embed_sum(ids, table, _layout(ids.numel(), pos0, state_slot, qo_indptr, tok_seq), pair=pair, mul_prev=mul_prev, mul_cur=mul_cur,
+                         prev_id=prev_id, pos_table=pos_table, positions=positions, w=w, eps=eps, split=split)
+
+
+def _tied_prep_store(x, q_off, k_off, q_w, k_w, eps, slots, k_cache, k_rn, heads, kv_heads, dim):
+    return ops.tied_prep_store(x, (q_off, k_off), q_w, k_w, eps, slots, k_cache, k_rn, heads, kv_heads, dim)
+
+
+def _gla_scan(x, q_off, k_off, v_off, alpha, mem, pos0, state_slot, qo_indptr, tok_seq, heads, dim, vdim, q_mul):
+    return ops.gla_scan(x, (q_off, k_off, v_off), alpha, mem, _layout(x.shape[0], pos0, state_slot, qo_indptr, tok_seq), heads, dim, vdim, q_mul=q_mul)
+
+
+def _moe_route_sigmoid(logits, correction, top, n_groups, keep_groups, scale):
+    return ops.moe_route_sigmoid(logits, correction, top, n_groups, keep_groups, scale)
+
+
+def _gelu_glu(gu):
+    return ops.gelu_glu(gu)
 
 
 for _name in _DEFS:
