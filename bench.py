@@ -972,10 +972,183 @@ def _ladusun_kernel_table(z, t_pre, n_dec, ctx, phases=("prefill", "decode")):
     return rows
 
 
+def _zenedra_config(z):
+    """Layers attention, mlstm, gla, attention with the middle two run twice (six layer runs; three layers run once where the other models
+    have three); heads of 128 with 8 key/value heads, chunks of 512 positions; recurrences with keys 64 and values 128 wide; the first
+    feed-forward dense, the others eight experts of ff / 4 in four groups, two a token, beside a shared one of ff / 2, so that a token's
+    feed-forward work equals the dense model's."""
+    w, hd = z["width"], z["width"] // 128
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"] // 4, "limit": 7.0}, "shared": {"ff": z["ff"] // 2, "limit": 7.0},
+           "router": {"experts": 8, "top": 2, "scale": 1.5, "groups": {"count": 4, "keep": 2}}}
+    att = {"type": "attention", "mixer": {"heads": z["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 512}}}
+    mls = {"type": "mlstm", "mixer": {"heads": hd, "dim": 64, "vdim": 128, "gate_cap": 15.0}}
+    gla = {"type": "gla", "mixer": {"heads": hd, "dim": 64, "vdim": 128, "tau": 16.0}}
+    if z["layers"] == 6:
+        kinds, loop = (att, mls, gla, att), {"start": 1, "stop": 3, "times": 2}
+    else:
+        kinds, loop = [(att, mls, gla)[i % 3] for i in range(z["layers"])], {"start": 0, "stop": z["layers"], "times": 1}
+    layers = [dict(k, mlp=dense if i == 0 else moe) for i, k in enumerate(kinds)]
+    return {"architecture": "Zenedra", "vocab": z["vocab"], "width": w, "norm": {"eps": 1e-5}, "max_positions": 8192,
+            "embedding": {"bigram": {"buckets": 32003, "mul_prev": 31, "mul_cur": 7}}, "loop": loop, "layers": layers}
+
+
+def _zenedra_kernel_table(z, t_pre, n_dec, ctx, phases=("prefill", "decode")):
+    """Each kernel of Zenedra beside the like kernel of Gibavik, Ladusun, Meronex or Qwen3 at the same shape: time, and the fraction of its
+    roofline (HBM bytes it must move at 8 TB/s; attention in prefill: its multiply-adds at the dense bf16 MFMA peak; the recurrences in
+    prefill: their multiply-adds at the float32 vector peak, since their states are float32)."""
+    from nano_vllm_x_amd import ops
+    dev, bf = torch.device("cuda"), torch.bfloat16
+    w, ff, h = z["width"], z["ff"], z["heads"]
+    hd, chunk = w // 128, 512
+    rows = []
+
+    def layout(n_seq, q_len, pos0):
+        p = torch.full((n_seq,), pos0, dtype=torch.int64, device=dev)
+        sl = torch.arange(n_seq, dtype=torch.int32, device=dev)
+        if q_len == 1:
+            return ops.StepLayout(n_seq, n_seq, p, sl)
+        qo = torch.arange(0, n_seq + 1, dtype=torch.int32, device=dev) * q_len
+        return ops.StepLayout(n_seq * q_len, n_seq, p, sl, qo, torch.arange(n_seq, dtype=torch.int32, device=dev).repeat_interleave(q_len), max_q=q_len)
+
+    def add(name, phase, us, bytes_=None, flops=None, like=None, peak=None):
+        if bytes_:
+            frac, bound = bytes_ / (us * 1e-6) / (HBM_PEAK_GBS * 1e9), "HBM"
+        else:
+            frac, bound = flops / (us * 1e-6) / ((peak or MFMA_BF16_PEAK_TFLOPS) * 1e12), "MFMA" if peak is None else "fp32 VALU"
+        rows.append({"kernel": name, "phase": phase, "us": round(us, 1), "of_roofline": round(frac, 3), "bound": bound, "like": like})
+
+    for phase, (n_seq, q_len, pos0) in (("prefill", (max(t_pre // 1024, 1), 1024, 0)), ("decode", (n_dec, 1, ctx))):
+        if phase not in phases:
+            continue
+        t = n_seq * q_len
+        dec = phase == "decode"
+        lay = layout(n_seq, q_len, pos0)
+        reps = 20 if dec else 5
+        y, y2, x = torch.randn(t, w, device=dev).to(bf), torch.randn(t, w, device=dev).to(bf), torch.randn(t, w, device=dev)
+        one, wv = torch.ones(1, device=dev), torch.ones(w, device=dev)
+        # both ends of the stack and the sublayer boundary: 2 B per result, 4 B of stream read and written, 2 B of the next sublayer's rows
+        table, pair, pos_table = (torch.randn(n, w, device=dev).to(bf) for n in (z["vocab"], 32004, 8192))
+        ids = torch.randint(0, z["vocab"], (t,), device=dev)
+        positions = (torch.arange(t, device=dev) % q_len + pos0).to(torch.int64)
+        prev = torch.zeros(n_seq + 1, 1, device=dev)
+        add("embed_sum (token + pair + position rows, [hi | lo])", phase,
+            _time_us(lambda: ops.embed_sum(ids, table, lay, pair=pair, mul_prev=31, mul_cur=7, prev_id=prev, pos_table=pos_table, positions=positions, split=True)),
+            bytes_=t * w * 14, like="embed_scale")
+        add("gibavik embed_scale", phase, _time_us(lambda: ops.embed_scale(ids, table, 8.0)), bytes_=t * w * 8)
+        add("residual_norm", phase, _time_us(lambda: ops.residual_norm(x, y, w=wv, eps=1e-5)), bytes_=t * w * 12, like="postnorm_residual")
+        add("residual_norm, two results", phase, _time_us(lambda: ops.residual_norm(x, y, y2, w=wv, eps=1e-5)), bytes_=t * w * 14, like="postnorm_residual, two results")
+        add("residual_norm, [hi | lo] rows", phase, _time_us(lambda: ops.residual_norm(x, y, split=True)), bytes_=t * w * 14, like="postnorm_residual")
+        x0 = torch.randn(t, w, device=dev)
+        add("residual_norm, head of a pass", phase, _time_us(lambda: ops.residual_norm(x, add=x0, bias=wv, w=wv, eps=1e-5, dtype=bf)), bytes_=t * w * 14,
+            like="postnorm_residual, two results")
+        add("gibavik postnorm_residual", phase, _time_us(lambda: ops.postnorm_residual(x, y=y, w_post=one, eps=1e-5)), bytes_=t * w * 12)
+        add("gibavik postnorm_residual, two results", phase, _time_us(lambda: ops.postnorm_residual(x, y=y, y2=y2, a=0.5, b=1.0, w_post=one, eps=1e-5)),
+            bytes_=t * w * 14)
+        hl, w2 = torch.randn(t, 2 * w, device=dev).to(bf), torch.randn(w, 2 * w, device=dev).to(bf)
+        add("join of a pass (library product, float32 sums)", phase, _time_us(lambda: ops.product_f32(hl, w2)), flops=4.0 * t * w * w,
+            like="the same product with bfloat16 results")
+        add("the same product with bfloat16 results", phase, _time_us(lambda: torch.nn.functional.linear(hl, w2)), flops=4.0 * t * w * w)
+        # activations and the router
+        gu = torch.randn(t, 2 * ff, device=dev).to(bf)
+        add("gelu_glu", phase, _time_us(lambda: ops.gelu_glu(gu)), bytes_=t * ff * 6, like="silu_mul")
+        add("qwen3 silu_mul", phase, _time_us(lambda: ops.silu_mul(gu)), bytes_=t * ff * 6)
+        z8, corr = torch.randn(t, 8, device=dev), torch.randn(8, device=dev)
+        add("moe_route_sigmoid (groups, correction)", phase, _time_us(lambda: ops.moe_route_sigmoid(z8, corr, 2, 4, 2, 1.5)), bytes_=t * (8 * 4 + 2 * 8),
+            like="moe_route_softmax")
+        add("ladusun moe_route_softmax (groups)", phase, _time_us(lambda: ops.moe_route_softmax(z8, 2, 4, 2, 1e-20)), bytes_=t * (8 * 4 + 2 * 8))
+        # gated linear attention: q | k | v and the channels' decays in float32, beside the memory with one constant decay per head
+        xr = torch.randn(t, 2 * hd * 64 + 2 * w, device=dev).to(bf)
+        mem = torch.zeros(n_seq + 1, hd, 64, 128, device=dev)
+        alpha, decay = torch.rand(t, hd * 64, device=dev) * 0.1 + 0.9, torch.full((hd,), 0.99, device=dev)
+        offs = (0, hd * 64, 2 * hd * 64)
+        us_gla = _time_us(lambda: ops.gla_scan(xr, offs, alpha, mem, lay, hd, 64, 128, q_mul=0.125), reps)
+        us_dec = _time_us(lambda: ops.decay_scan(xr, offs, decay, mem, lay, hd, 64, 128), reps)
+        gates, gb = torch.randn(t, 2 * hd, device=dev), torch.full((2 * hd,), 1.0, device=dev)
+        nrm, peak = torch.zeros(n_seq + 1, hd, 64, device=dev), torch.zeros(n_seq + 1, hd, device=dev)
+        us_ml = _time_us(lambda: ops.mlstm_scan(xr, offs, gates, gb, 15.0, mem, nrm, peak, lay, hd, 64, 128), reps)
+        io = t * (2 * hd * 64 + w) * 2 + t * w * 4
+        if dec:
+            add("gla_scan", phase, us_gla, bytes_=n_seq * hd * 64 * 128 * 8 + io + t * hd * 64 * 4, like="decay_scan")
+            add("mlstm_scan", phase, us_ml, bytes_=n_seq * hd * 64 * 129 * 8 + io, like="decay_scan")
+            add("gibavik decay_scan", phase, us_dec, bytes_=n_seq * hd * 64 * 128 * 8 + io)
+        else:
+            # per (row, column) of a memory and token: one multiply-add for the decay and the write each, one for the read
+            fl = t * hd * 64 * 128 * 6.0
+            add("gla_scan (chunks side by side)", phase, us_gla, flops=fl, like="decay_scan", peak=FP32_VALU_PEAK_TFLOPS)
+            add("mlstm_scan (chunks side by side)", phase, us_ml, flops=fl, like="decay_scan", peak=FP32_VALU_PEAK_TFLOPS)
+            add("gibavik decay_scan (chunks side by side)", phase, us_dec, flops=fl, peak=FP32_VALU_PEAK_TFLOPS)
+            us = _time_us(lambda: ops.mlstm_scan(xr, offs, gates, gb, 15.0, mem, nrm, peak, lay, hd, 64, 128, chunk=0), reps)
+            add("mlstm_scan (one walk per portion)", phase, us, flops=fl, peak=FP32_VALU_PEAK_TFLOPS)
+        a1, a2, ab = torch.randn(16, w, device=dev), torch.randn(hd * 64, 16, device=dev), torch.zeros(hd * 64, device=dev)
+        z1 = ops.skinny_proj(y, a1)
+        add("skinny_proj (decay, width -> 16)", phase, _time_us(lambda: ops.skinny_proj(y, a1)), bytes_=t * w * 2, like="skinny_proj of a router")
+        add("skinny_proj (decay, 16 -> channels, sigmoid^(1/tau))", phase,
+            _time_us(lambda: ops.skinny_proj(z1, a2, bias=ab, out_act="sigmoid_pow", power=1 / 16.0)), bytes_=t * hd * 64 * 4, like="skinny_proj of a router")
+        rt = torch.randn(8, w, device=dev)
+        add("ladusun skinny_proj of a router (width -> 8)", phase, _time_us(lambda: ops.skinny_proj(y, rt)), bytes_=t * w * 2)
+        o32, gate = torch.randn(t, hd, 128, device=dev), torch.randn(t, w, device=dev).to(bf)
+        add("head_norm_gate", phase, _time_us(lambda: ops.head_norm_gate(o32, wv[:128].contiguous(), 1e-5, gate=gate, kind="silu")), bytes_=t * w * 8)
+        # attention: one row per token is key and value, beside Gibavik's and Qwen3's two
+        kv_len = pos0 + q_len
+        n_rows = n_seq * kv_len
+        kc, vc = torch.randn(n_rows, 8 * 128, device=dev).to(bf), torch.randn(n_rows, 8 * 128, device=dev).to(bf)
+        rn = torch.rand(n_rows, 8, device=dev) + 0.5
+        idx = torch.arange(n_rows, dtype=torch.int32, device=dev)
+        kv_start = torch.arange(n_seq, dtype=torch.int64, device=dev) * kv_len
+        kvl = torch.full((n_seq,), kv_len, dtype=torch.int32, device=dev)
+        qkv = torch.randn(t, (h + 16) * 128, device=dev).to(bf)
+        slots = (torch.arange(t, device=dev) // q_len * kv_len + positions).to(torch.int64)
+        qn, kn = torch.ones(128, device=dev), torch.ones(128, device=dev)
+        add("tied_prep_store", phase, _time_us(lambda: ops.tied_prep_store(qkv, (0, h * 128), qn, kn, 1e-5, slots, kc, rn, h, 8, 128)),
+            bytes_=t * (h + 8) * 128 * 4, like="attn_prep_store")
+        add("gibavik attn_prep_store (head norms, no rotation)", phase,
+            _time_us(lambda: ops.attn_prep_store(qkv, (0, h * 128, (h + 8) * 128), positions, qn, kn, "head", 1e-5, None, 0, False, None, slots, kc, vc, h, 8, 128, 128)),
+            bytes_=t * (h + 16) * 128 * 4)
+        q128 = torch.randn(t, h * 128, device=dev).to(bf)
+        slopes = torch.rand(h, device=dev) * 0.1
+        r1, r2 = torch.full((h,), 0.5, device=dev), torch.full((h,), 0.1, device=dev)
+        us_tied = _time_us(lambda: ops.softcap_attn(q128, kc, kc, idx, kv_start, kvl, lay, 0.09, 0.0, h, 8, 128, 128, slopes=slopes, k_rn=rn), reps)
+        ck = chunk + 1 if dec else chunk           # (at decode shapes: the context's last token at the end of a chunk's 512th key)
+        us_chunk = _time_us(lambda: ops.softcap_attn(q128, kc, kc, idx, kv_start, kvl, lay, 0.09, 0.0, h, 8, 128, 128, slopes=slopes, k_rn=rn, chunk=ck), reps)
+        us_pen = _time_us(lambda: ops.softcap_attn(q128, kc, vc, idx, kv_start, kvl, lay, 0.09, 0.0, h, 8, 128, 128, r1=r1, r2=r2), reps)
+        kc4, vc4 = kc.view(n_rows, 8, 128), vc.view(n_rows, 8, 128)
+        if not dec:
+            pairs, pairs_c = n_seq * q_len * (q_len + 1) // 2, n_seq * (q_len // chunk) * chunk * (chunk + 1) // 2
+            add("softcap_attn (tied rows, slopes, all keys)", phase, us_tied, flops=4.0 * h * 128 * pairs, like="softcap_attn (distance penalty)")
+            add("softcap_attn (tied rows, slopes, chunks of 512)", phase, us_chunk, flops=4.0 * h * 128 * pairs_c, like="softcap_attn (distance penalty)")
+            add("gibavik softcap_attn (distance penalty)", phase, us_pen, flops=4.0 * h * 128 * pairs)
+            plan = ops.prefill_plan_ws(n_seq, dev)
+            kv_indptr = torch.arange(0, n_seq + 1, dtype=torch.int32, device=dev) * kv_len
+            ops.prefill_plan(lay.qo_indptr, plan)
+            us = _time_us(lambda: ops.paged_prefill(q128, kc4, vc4, lay.qo_indptr, kv_indptr, idx, plan, h, 8, 0.1), reps=5)
+            add("qwen3 paged_prefill", phase, us, flops=4.0 * h * 128 * pairs)
+        else:
+            io = 2 * t * h * 128 * 2
+            add("softcap_attn (tied rows, slopes, all keys)", phase, us_tied, bytes_=n_rows * 8 * (256 + 4) + io, like="softcap_attn (distance penalty)")
+            add("softcap_attn (tied rows, slopes, chunks of 512)", phase, us_chunk, bytes_=n_seq * ((kv_len - 1) % ck + 1) * 8 * (256 + 4) + io,
+                like="softcap_attn (distance penalty)")
+            add("gibavik softcap_attn (distance penalty)", phase, us_pen, bytes_=n_rows * 8 * 128 * 2 * 2 + io)
+            ws = ops.DecodeWorkspace(n_seq, h, 8, dev)
+            ops.decode_plan(kvl, kv_start, ws)
+            us = _time_us(lambda: ops.paged_decode(q128, kc4, vc4, idx, n_seq, ws, 0.1))
+            add("qwen3 paged_decode", phase, us, bytes_=n_rows * 8 * 128 * 2 * 2 + io)
+            # experts: eight of ff / 4, two a token, the weights on the outputs; beside them Gibavik's of ff / 2
+            hm = torch.randn(t, w, device=dev).to(bf)
+            eidx = torch.stack([torch.randperm(8, device=dev)[:2] for _ in range(t)]).to(torch.int32)
+            wts = torch.full((t, 2), 0.5, device=dev)
+            for name, f, like in (("moe_expert_rows (experts of ff / 4)", ff // 4, "gibavik moe_expert_rows"), ("gibavik moe_expert_rows (experts of ff / 2)", ff // 2, None)):
+                w_gu, w_d = torch.randn(8, 2 * f, w, device=dev).to(bf) * 0.02, torch.randn(8, w, f, device=dev).to(bf) * 0.02
+                us = _time_us(lambda: ops.moe_expert_rows(hm, eidx, wts, w_gu, w_d, 7.0, 1.702, 1.0, True))
+                add(name, phase, us, bytes_=min(t * 2, 8) * 3 * f * w * 2, like=like)
+    return rows
+
+
 ARCHS = {"kabidra": (lambda z: _kabidra_config(z), lambda *a, **k: _kernel_table(*a), "Kabidra"),
          "meronex": (lambda z: _meronex_config(z), lambda *a, **k: _meronex_kernel_table(*a, **k), "Meronex"),
          "gibavik": (lambda z: _gibavik_config(z), lambda *a, **k: _gibavik_kernel_table(*a, **k), "Gibavik"),
-         "ladusun": (lambda z: _ladusun_config(z), lambda *a, **k: _ladusun_kernel_table(*a, **k), "Ladusun")}
+         "ladusun": (lambda z: _ladusun_config(z), lambda *a, **k: _ladusun_kernel_table(*a, **k), "Ladusun"),
+         "zenedra": (lambda z: _zenedra_config(z), lambda *a, **k: _zenedra_kernel_table(*a, **k), "Zenedra")}
 
 
 def arch_compare(args):
@@ -998,7 +1171,7 @@ def arch_compare(args):
         entry = {"geometry": z}
         with tempfile.TemporaryDirectory() as tmp:
             engines = [(args.arch, make_config(z)), ("qwen3", _qwen3_config(z))]
-            if args.arch == "ladusun":          # its closest relative in this package (attention with borrowed keys beside a recurrence, experts)
+            if args.arch in ("ladusun", "zenedra"):     # the closest relative in this package (attention beside a matrix memory or recurrence, experts)
                 engines.insert(1, ("gibavik", _gibavik_config(z)))
             for model, cfg in engines if args.arch_serve else ():
                 d = os.path.join(tmp, model)
@@ -1014,7 +1187,7 @@ def arch_compare(args):
         print(f"[arch-compare] {name}: kernels one by one", file=sys.stderr, flush=True)
         with torch.inference_mode():
             t_pre = args.arch_seqs * args.arch_prompt
-            if args.arch in ("gibavik", "ladusun") and args.arch_portion:      # the kernels one by one at the size of the steps the engines ran
+            if args.arch in ("gibavik", "ladusun", "zenedra") and args.arch_portion:      # the kernels one by one at the size of the steps the engines ran
                 t_pre = min(t_pre, max(args.arch_portion, args.arch_prompt))
             entry["kernels"] = kernel_table(z, t_pre, args.arch_seqs, args.arch_prompt,
                                             phases=tuple(args.arch_phases.split(",")))

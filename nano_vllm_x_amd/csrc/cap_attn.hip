@@ -374,6 +374,140 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
     }
 }
 
+// ---- tied rows, for steps of few tokens ---------------------------------------------------------------------------------------
+// One workgroup of four waves per (NH query heads of one key/value head, token, split).  A cached row is key AND value, so it is read
+// once, by LPR neighbouring lanes of eight elements each (LPR: 8, 16, 32 or 64, the first that covers dim / 8), and stays in registers from the
+// score to the read-out, for all NH heads: a wave takes U keys per lane group at a time (their loads in flight together), sums the
+// products over the lane group, and adds the weighted rows to what the lane keeps of the read-out.  Every lane group has a running
+// maximum and sum of its own; groups, waves and splits are merged at the end.
+template <int LPR> __device__ __forceinline__ float group_sum(float v) {      // over LPR neighbouring lanes, in the vector ALU
+    v += dpp_move<0xB1>(v);                        // lane ^ 1
+    v += dpp_move<0x4E>(v);                        // lane ^ 2
+    v += dpp_move<0x141>(v);                       // the other quad of eight
+    if (LPR >= 16) v += dpp_move<0x140>(v);        // the other eight of sixteen
+    if (LPR >= 32) v += xor16(v);
+    if (LPR >= 64) v += xor32(v);
+    return v;
+}
+template <typename A, int NH, int U, int LPR>
+__global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict__ q, const A* __restrict__ rows, const float* __restrict__ k_rn,
+                                                            const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
+                                                            const int32_t* __restrict__ kv_len, const int32_t* __restrict__ qo_indptr,
+                                                            const int32_t* __restrict__ tok_seq, float scale, A* __restrict__ out, int heads,
+                                                            int kv_heads, int dim, int n_split, float* __restrict__ part, int window, int chunk,
+                                                            const float* __restrict__ slopes) {
+    extern __shared__ float sm[];
+    float* sacc = sm;                       // 4 waves x NH x dim
+    float* sml = sacc + 4 * NH * dim;       // 4 waves x NH maxima, then as many sums
+    const int per_kv = heads / kv_heads, blocks_per_kv = (per_kv + NH - 1) / NH;
+    const int kvh = blockIdx.x / blocks_per_kv, h0 = kvh * per_kv + (blockIdx.x % blocks_per_kv) * NH;
+    const int n_here = (kvh + 1) * per_kv - h0 < NH ? (kvh + 1) * per_kv - h0 : NH;       // heads of this block
+    const int64_t t = blockIdx.y;
+    const int b = tok_seq ? tok_seq[t] : (int)t;
+    const int64_t q0 = qo_indptr ? qo_indptr[b] : b;
+    const int64_t q_n = qo_indptr ? qo_indptr[b + 1] - q0 : 1;
+    const int visible = kv_len[b] - (int)(q_n - 1 - (t - q0));
+    const int first = first_seen(visible - 1, window, chunk);
+    const int32_t* slots = kv_indices + kv_start[b];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g = lane / LPR, l = lane % LPR;
+    constexpr int groups = 64 / LPR;
+    const bool on = l * 8 < dim;
+    typedef A vec8 __attribute__((ext_vector_type(8)));
+    float qv[NH][8], acc[NH][8], m[NH], sum[NH], slope[NH];
+#pragma unroll
+    for (int n = 0; n < NH; ++n) {
+        const int h = h0 + (n < n_here ? n : 0);
+        slope[n] = slopes ? slopes[h] : 0.f;
+        m[n] = -INFINITY;
+        sum[n] = 0.f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            qv[n][i] = on ? ld_f(q, (t * heads + h) * (int64_t)dim + l * 8 + i) * scale : 0.f;
+            acc[n][i] = 0.f;
+        }
+    }
+    const int step = U * groups;            // keys of a wave's turn
+    for (int j0 = first + ((int)blockIdx.z * 4 + wave) * step; j0 < visible; j0 += 4 * n_split * step) {
+        vec8 kv[U];
+        float rn[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {       // (a key past the end reads a real row and gets no weight)
+            const int j = j0 + u * groups + g;
+            const int64_t row = (int64_t)slots[j < visible ? j : first] * kv_heads + kvh;
+            rn[u] = k_rn[row];
+            kv[u] = *reinterpret_cast<const vec8*>(rows + row * dim + (on ? l * 8 : 0));
+        }
+#pragma unroll
+        for (int n = 0; n < NH; ++n) {
+            float s[U], mx = m[n];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                float d = 0.f;
+#pragma unroll
+                for (int i = 0; i < 8; ++i) d += qv[n][i] * (float)kv[u][i];
+                d = group_sum<LPR>(d);
+                const int j = j0 + u * groups + g;
+                s[u] = j < visible ? d * rn[u] - slope[n] * (float)(visible - 1 - j) : -INFINITY;
+                mx = fmaxf(mx, s[u]);
+            }
+            const float base = mx == -INFINITY ? 0.f : mx;                  // (nothing seen by this lane group yet)
+            const float corr = expf(m[n] - base);
+            m[n] = mx;
+            sum[n] *= corr;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) acc[n][i] *= corr;
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const float p = expf(s[u] - base);
+                sum[n] += p;
+#pragma unroll
+                for (int i = 0; i < 8; ++i) acc[n][i] += p * (float)kv[u][i];
+            }
+        }
+    }
+#pragma unroll
+    for (int n = 0; n < NH; ++n) {          // the wave's lane groups
+        float mx = m[n];
+        for (int k = LPR; k < 64; k <<= 1) mx = fmaxf(mx, __shfl_xor(mx, k, 64));
+        const float f = m[n] == -INFINITY ? 0.f : expf(m[n] - mx);
+        sum[n] *= f;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[n][i] *= f;
+        for (int k = LPR; k < 64; k <<= 1) {
+            sum[n] += __shfl_xor(sum[n], k, 64);
+#pragma unroll
+            for (int i = 0; i < 8; ++i) acc[n][i] += __shfl_xor(acc[n][i], k, 64);
+        }
+        if (g == 0 && on) {
+#pragma unroll
+            for (int i = 0; i < 8; ++i) sacc[(wave * NH + n) * dim + l * 8 + i] = acc[n][i];
+        }
+        if (lane == 0) { sml[wave * NH + n] = mx; sml[4 * NH + wave * NH + n] = sum[n]; }
+    }
+    __syncthreads();
+    for (int n = 0; n < n_here; ++n) {      // the four waves
+        float f[4], mm = -INFINITY, total = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) mm = fmaxf(mm, sml[w * NH + n]);
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float mw = sml[w * NH + n];
+            f[w] = mw == -INFINITY ? 0.f : expf(mw - mm);
+            total += sml[4 * NH + w * NH + n] * f[w];
+        }
+        const int64_t row = t * heads + h0 + n;
+        float* pr = n_split > 1 ? part + (row * n_split + blockIdx.z) * (dim + 2) : nullptr;
+        for (int e = threadIdx.x; e < dim; e += 256) {
+            float o = 0.f;
+#pragma unroll
+            for (int w = 0; w < 4; ++w) o += sacc[(w * NH + n) * dim + e] * f[w];
+            if (pr) pr[2 + e] = o;
+            else st_f(out, row * dim + e, o / total);
+        }
+        if (pr && threadIdx.x == 0) { pr[0] = mm; pr[1] = total; }
+    }
+}
+
 // ---- the same attention on the matrix cores, for steps of many tokens in a 16-bit format -------------------------------------
 // A workgroup takes 64 consecutive query tokens of ONE sequence and one query head; each of its four waves owns 16 of them.  Keys
 // are walked in tiles of 32.  Per tile and wave:
@@ -799,6 +933,33 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     }
     const size_t lds = (size_t)(dim + 4 * vdim + 8) * sizeof(float);
     NVX_REQUIRE(n_split >= 1 && n_split <= 64 && (n_split == 1 || part), NVX_EINVAL, "nvx_softcap_attn: a key split needs its workspace");
+    // tied rows without what that kernel does not do: a row is read once
+    if (k_rn && k_cache == v_cache && dim == vdim && dim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && !sink && nvx_aligned16(k_cache)) {
+        const int per_kv = (int)(heads / kv_heads), nh = per_kv >= 4 ? 4 : (per_kv >= 2 ? 2 : 1);
+        const dim3 tgrid((unsigned)(kv_heads * ((per_kv + nh - 1) / nh)), (unsigned)n_tok, (unsigned)n_split);
+        const size_t tlds = (size_t)(4 * nh * dim + 8 * nh) * sizeof(float);
+#define NVX_TIED_ROWS_L(NH, LPR)                                                                                                                \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((tied_rows_attn_kernel<A_, NH, sizeof(A_) == 2 ? 8 : 4, LPR>), tgrid, dim3(256), tlds, (hipStream_t)stream, \
+                                         (const A_*)q, (const A_*)k_cache, k_rn, kv_indices, kv_start, kv_len, qo_indptr, tok_seq, scale, (A_*)out,  \
+                                         (int)heads, (int)kv_heads, (int)dim, n_split, part, (int)window, (int)chunk, slopes))
+#define NVX_TIED_ROWS(NH)                            \
+    do {                                             \
+        if (dim <= 64) NVX_TIED_ROWS_L(NH, 8);       \
+        else if (dim <= 128) NVX_TIED_ROWS_L(NH, 16); \
+        else if (dim <= 256) NVX_TIED_ROWS_L(NH, 32); \
+        else NVX_TIED_ROWS_L(NH, 64);                \
+    } while (0)
+        if (nh == 4) NVX_TIED_ROWS(4);
+        else if (nh == 2) NVX_TIED_ROWS(2);
+        else NVX_TIED_ROWS(1);
+#undef NVX_TIED_ROWS_L
+#undef NVX_TIED_ROWS
+        if (n_split > 1)
+            NVX_FMT_CALL(fmt, hipLaunchKernelGGL(softcap_merge_kernel<A_>, dim3((unsigned)(n_tok * heads)), dim3(64), 0, (hipStream_t)stream,
+                                                 (const float*)part, n_split, (A_*)out, (int)vdim, (int)heads, vcs, v_interleaved, (const A_*)gate,
+                                                 gate_stride, gate_per_head, sink, sink_score));
+        return nvx_check_launch("nvx_softcap_attn");
+    }
     const dim3 grid((unsigned)heads, (unsigned)n_tok, (unsigned)n_split);
 #define NVX_CAP_ATTN_V(EPL, VEC)                                                                                                          \
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((softcap_attn_kernel<A_, EPL, VEC && sizeof(A_) == 2>), grid, dim3(256), lds, (hipStream_t)stream,     \
