@@ -385,6 +385,59 @@ __global__ __launch_bounds__(256) void skinny_proj_kernel(const A* __restrict__ 
     }
 }
 
+// The same for wide inputs whose rows start on borders of four elements (k_in >= 256 and a multiple of 4).  A workgroup takes SKW_TOK tokens
+// and SKW_OUT outputs; its four waves take the inputs 256 at a time, every fourth piece each, a lane four neighbouring inputs: all loads
+// of a piece are in flight together, every weight serves SKW_TOK tokens and every input SKW_OUT outputs from registers, and the sums of
+// lanes and waves have one order, whatever the batch.
+constexpr int SKW_TOK = 4, SKW_OUT = 8;
+template <typename A>
+__global__ __launch_bounds__(256) void skinny_wide_kernel(const A* __restrict__ x, int64_t x_stride, const float* __restrict__ w, int in_act,
+                                                         const float* __restrict__ bias, int out_act, float power, float* __restrict__ out, int64_t n_tok,
+                                                         int n_out, int k_in) {
+    typedef A veca __attribute__((ext_vector_type(4)));
+    __shared__ float part[4][SKW_TOK * SKW_OUT];
+    const int64_t t0 = (int64_t)blockIdx.x * SKW_TOK;
+    const int n0 = blockIdx.y * SKW_OUT, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    float acc[SKW_TOK][SKW_OUT];
+#pragma unroll
+    for (int t = 0; t < SKW_TOK; ++t)
+#pragma unroll
+        for (int n = 0; n < SKW_OUT; ++n) acc[t][n] = 0.f;
+    for (int k = wave * 256 + lane * 4; k < k_in; k += 1024) {
+        veca xv[SKW_TOK];
+        nvx_f32x4 wv[SKW_OUT];
+#pragma unroll
+        for (int t = 0; t < SKW_TOK; ++t) xv[t] = *reinterpret_cast<const veca*>(x + (t0 + t < n_tok ? t0 + t : n_tok - 1) * x_stride + k);
+#pragma unroll
+        for (int n = 0; n < SKW_OUT; ++n) wv[n] = *reinterpret_cast<const nvx_f32x4*>(w + (int64_t)(n0 + n < n_out ? n0 + n : n_out - 1) * k_in + k);
+#pragma unroll
+        for (int t = 0; t < SKW_TOK; ++t) {
+            float xf[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) { const float v = (float)xv[t][i]; xf[i] = in_act == 1 ? tanhf(v) : v; }
+#pragma unroll
+            for (int n = 0; n < SKW_OUT; ++n)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) acc[t][n] += xf[i] * wv[n][i];
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < SKW_TOK; ++t)
+#pragma unroll
+        for (int n = 0; n < SKW_OUT; ++n) {
+            float v = quarter_sum(acc[t][n]);
+            v += xor16(v);
+            v += xor32(v);
+            if (lane == 0) part[wave][t * SKW_OUT + n] = v;
+        }
+    __syncthreads();
+    if (threadIdx.x < SKW_TOK * SKW_OUT) {
+        const int t = threadIdx.x / SKW_OUT, n = threadIdx.x % SKW_OUT;
+        const float v = part[0][threadIdx.x] + part[1][threadIdx.x] + part[2][threadIdx.x] + part[3][threadIdx.x];
+        if (t0 + t < n_tok && n0 + n < n_out) out[(t0 + t) * n_out + n0 + n] = skinny_end(v, bias, n0 + n, out_act, power);
+    }
+}
+
 }  // namespace NVX_NS
 
 using namespace NVX_NS;
@@ -402,6 +455,14 @@ extern "C" int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const f
     const int opb = k_in >= 256 ? 8 : 256;
     const int64_t chunks = (n_out + opb - 1) / opb;
     NVX_REQUIRE(chunks <= 65535, NVX_EINVAL, "nvx_skinny_proj: too many outputs");
+    const uintptr_t x_border = fmt == 2 ? 15u : 7u;
+    if (k_in >= 256 && k_in % 4 == 0 && x_stride % 4 == 0 && (reinterpret_cast<uintptr_t>(x) & x_border) == 0 && nvx_aligned16(w)) {
+        NVX_REQUIRE((n_tok + SKW_TOK - 1) / SKW_TOK < (1ll << 31), NVX_EINVAL, "nvx_skinny_proj: too many tokens");
+        NVX_FMT_CALL(fmt, hipLaunchKernelGGL(skinny_wide_kernel<A_>, dim3((unsigned)((n_tok + SKW_TOK - 1) / SKW_TOK), (unsigned)((n_out + SKW_OUT - 1) / SKW_OUT)),
+                                             dim3(256), 0, (hipStream_t)stream, (const A_*)x, x_stride, w, in_act, bias, out_act, power, out, n_tok, (int)n_out,
+                                             (int)k_in));
+        return nvx_check_launch("nvx_skinny_proj");
+    }
     if (k_in <= 3072) {
         const int64_t blocks = (n_tok + 3) / 4;
         NVX_REQUIRE(blocks < (1ll << 31), NVX_EINVAL, "nvx_skinny_proj: too many tokens");

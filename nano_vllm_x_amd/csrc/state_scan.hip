@@ -126,6 +126,50 @@ __device__ __forceinline__ void stage_cols(float* dst, const A* x, int64_t x_str
         dst[i] = e < vdim ? ld_f(x, (tok0 + tt) * x_stride + off + e) : 0.f;
     }
 }
+// The same for the chunked recurrences, `V` neighbouring elements of a row at a time (V = 4: dim, off and the rows' stride are multiples
+// of four and x starts on such a border) and STAGE_U pieces of a thread in flight together before the first is written: a stage is one
+// or two memory round trips instead of one per piece.  act 1: silu; times mul.
+constexpr int STAGE_U = 8;
+__device__ __forceinline__ float scan_act(float z, int act) { return act == 1 ? z * sigmoid_f(z) : z; }
+template <typename A, int V, bool ROWS>
+__device__ __forceinline__ void stage_pieces(float* dst, int rs, const A* __restrict__ x, int64_t x_stride, int nt, int n, int n_zero, int act, float mul) {
+    typedef A veca __attribute__((ext_vector_type(V)));
+    typedef float vecf __attribute__((ext_vector_type(V)));
+    const int per = n_zero / V, pieces = nt * per;            // n elements of a row are there, those up to n_zero are zeros
+    for (int i0 = threadIdx.x; i0 < pieces; i0 += blockDim.x * STAGE_U) {
+        veca v[STAGE_U];
+#pragma unroll
+        for (int u = 0; u < STAGE_U; ++u) {
+            const int i = i0 + u * (int)blockDim.x, tt = i / per, d = (i - tt * per) * V;
+            if (i < pieces && d < n) v[u] = *reinterpret_cast<const veca*>(x + tt * x_stride + d);
+        }
+#pragma unroll
+        for (int u = 0; u < STAGE_U; ++u) {
+            const int i = i0 + u * (int)blockDim.x, tt = i / per, d = (i - tt * per) * V;
+            if (i >= pieces) continue;
+            vecf f;
+#pragma unroll
+            for (int k = 0; k < V; ++k) f[k] = d < n ? scan_act((float)v[u][k], act) * mul : 0.f;
+            *reinterpret_cast<vecf*>(dst + tt * rs + (ROWS ? lds_row(d) : d)) = f;
+        }
+    }
+}
+// key rows (dst: rs floats a token, lds_row inside), and value columns (dst: `width` floats a token, of which `n` are within the head)
+template <typename A>
+__device__ __forceinline__ void stage_key_rows(float* dst, int rs, const A* x, int64_t x_stride, int nt, int dim, bool vec, int act = 0, float mul = 1.0f) {
+    if (vec) stage_pieces<A, 4, true>(dst, rs, x, x_stride, nt, dim, dim, act, mul);
+    else stage_pieces<A, 1, true>(dst, rs, x, x_stride, nt, dim, dim, act, mul);
+}
+template <typename A>
+__device__ __forceinline__ void stage_value_cols(float* dst, int width, const A* x, int64_t x_stride, int nt, int n, bool vec, int act = 0) {
+    if (vec) stage_pieces<A, 4, false>(dst, width, x, x_stride, nt, n < width ? n : width, width, act, 1.0f);
+    else stage_pieces<A, 1, false>(dst, width, x, x_stride, nt, n < width ? n : width, width, act, 1.0f);
+}
+// whether a launch may stage four elements at a time
+template <typename A>
+static bool stage_vec_ok(const void* x, int64_t x_stride, int64_t q_off, int64_t k_off, int64_t v_off, int64_t dim, int64_t vdim, int64_t cols) {
+    return (reinterpret_cast<uintptr_t>(x) & (4 * sizeof(A) - 1)) == 0 && ((x_stride | q_off | k_off | v_off | dim | vdim | cols) & 3) == 0;
+}
 __device__ __forceinline__ void zero_rows(float* dst, int n) {
     for (int i = threadIdx.x; i < n; i += blockDim.x) dst[i] = 0.f;
 }
@@ -158,14 +202,14 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
                                                         float* __restrict__ N, float* __restrict__ M,
                                                         const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
                                                         const int32_t* __restrict__ state_slot, float* __restrict__ out, int heads, int dim,
-                                                        int vdim, int p_lanes, MlstmChunks ck) {
+                                                        int vdim, int p_lanes, int tb, int vec, MlstmChunks ck) {
     extern __shared__ float sm[];
     const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
     float* sq = sm;
-    float* sk = sq + TB * rs;
-    float* sv = sk + TB * rs;
-    float* si = sv + TB * cb;
-    float* sf = si + TB;
+    float* sk = sq + tb * rs;
+    float* sv = sk + tb * rs;
+    float* si = sv + tb * cb;
+    float* sf = si + tb;
     const int hd = blockIdx.y;
     SeqSpan sp = seq_span(PHASE ? blockIdx.z / ck.n_max : blockIdx.z, qo_indptr, pos0, state_slot);
     if (sp.slot < 0 || sp.n <= 0) return;
@@ -193,14 +237,15 @@ __global__ __launch_bounds__(256) void mlstm_scan_kernel(const A* __restrict__ x
         nn[r] = in ? Np_in[row] : 0.f;
     }
     if (cont) m = PHASE ? ck.M[at] : M_in[at];
-    zero_rows(sq, 2 * TB * rs);
+    zero_rows(sq, 2 * tb * rs);
     const float q_mul = 1.0f / sqrtf((float)dim);
-    for (int64_t t0 = 0; t0 < sp.n; t0 += TB) {
-        const int nt = (int)(sp.n - t0 < TB ? sp.n - t0 : TB);
+    for (int64_t t0 = 0; t0 < sp.n; t0 += tb) {
+        const int nt = (int)(sp.n - t0 < tb ? sp.n - t0 : tb);
         __syncthreads();
-        if (PHASE != 1) stage_rows(sq, x, x_stride, sp.q0 + t0, nt, q_off + hd * dim, dim, p_lanes, q_mul);
-        stage_rows(sk, x, x_stride, sp.q0 + t0, nt, k_off + hd * dim, dim, p_lanes, 1.0f);
-        stage_cols(sv, x, x_stride, sp.q0 + t0, nt, v_off + hd * vdim, vdim, cb);
+        const A* xr = x + (sp.q0 + t0) * x_stride;
+        if (PHASE != 1) stage_key_rows(sq, rs, xr + q_off + hd * dim, x_stride, nt, dim, vec, 0, q_mul);
+        stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec);
+        stage_value_cols(sv, cb, xr + v_off + hd * vdim + blockIdx.x * cb, x_stride, nt, vdim - (int)blockIdx.x * cb, vec);
         if ((int)threadIdx.x < nt) {
             const float* g = gates + (sp.q0 + t0 + threadIdx.x) * 2 * heads;
             si[threadIdx.x] = cap * tanhf((g[hd] + gate_bias[hd]) / cap);
@@ -453,7 +498,6 @@ __global__ __launch_bounds__(256) void rwkv_scan_kernel(const A* __restrict__ rx
 // the state at every chunk's start (and writes the sequence's final state), phase 3 walks every chunk from there with the read-out.
 // Because the decay is a constant, the carry over a chunk of n tokens is decay^n S + (the chunk's own contribution).  phase 0: one
 // workgroup walks the whole portion (single tokens, short portions).
-__device__ __forceinline__ float scan_act(float z, int act) { return act == 1 ? z * sigmoid_f(z) : z; }
 // `tb` tokens are staged at a time: 32 where the key size leaves LDS for them (more than the other recurrences take: an activation
 // is applied as they are staged, and fewer, longer stages hide more of the loads), fewer for wide keys.
 template <typename A, int PHASE>
@@ -461,7 +505,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
                                                         const float* __restrict__ decay, float* __restrict__ S,
                                                         const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
                                                         const int32_t* __restrict__ state_slot, float* __restrict__ out, int heads, int dim,
-                                                        int vdim, int p_lanes, int tb, int chunk, int n_chunk_max, float* __restrict__ ws) {
+                                                        int vdim, int p_lanes, int tb, int vec, int chunk, int n_chunk_max, float* __restrict__ ws) {
     constexpr int phase = PHASE;
     extern __shared__ float sm[];
     const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
@@ -493,17 +537,10 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
     for (int64_t t0 = 0; t0 < sp.n; t0 += tb) {
         const int nt = (int)(sp.n - t0 < tb ? sp.n - t0 : tb);
         __syncthreads();
-        for (int i = threadIdx.x; i < nt * dim; i += blockDim.x) {
-            const int tt = i / dim, d = i % dim;
-            const int64_t r = (sp.q0 + t0 + tt) * x_stride + hd * dim + d;
-            if (phase != 1) sq[tt * rs + lds_row(d)] = scan_act(ld_f(x, r + q_off), act);      // (phase 1 wants the state only)
-            sk[tt * rs + lds_row(d)] = scan_act(ld_f(x, r + k_off), act);
-        }
-        for (int i = threadIdx.x; i < nt * cb; i += blockDim.x) {
-            const int tt = i / cb, c = i % cb;
-            const int e = blockIdx.x * cb + c;
-            sv[i] = e < vdim ? scan_act(ld_f(x, (sp.q0 + t0 + tt) * x_stride + v_off + hd * vdim + e), act) : 0.f;
-        }
+        const A* xr = x + (sp.q0 + t0) * x_stride;
+        if (phase != 1) stage_key_rows(sq, rs, xr + q_off + hd * dim, x_stride, nt, dim, vec, act);      // (phase 1 wants the state only)
+        stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec, act);
+        stage_value_cols(sv, cb, xr + v_off + hd * vdim + blockIdx.x * cb, x_stride, nt, vdim - (int)blockIdx.x * cb, vec, act);
         __syncthreads();
         for (int tt = 0; tt < nt; ++tt) {
             const float v = sv[tt * cb + th.col];
@@ -562,12 +599,12 @@ __global__ __launch_bounds__(256) void decay_chunk_carry_kernel(const float* __r
 // float32: the decay of every key channel at every token.
 //   S <- diag(alpha) S + k v^T;  o = S^T (q_mul q)  (the read sees the token's own write).          S: (slots, heads, dim, vdim).
 // Phases as in decay_scan_kernel; phase 1 also hands out, per key channel, the product of the chunk's decays (ws_keep), which is what the
-// carry multiplies the memory in front with.
-template <typename A, int PHASE>
+// carry multiplies the memory in front with.  A thread keeps NC columns: the rows it reads from LDS then serve NC of them.
+template <typename A, int PHASE, int NC>
 __global__ __launch_bounds__(256) void gla_scan_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off, int v_off, float q_mul,
                                                       const float* __restrict__ alpha, float* __restrict__ S, const int32_t* __restrict__ qo_indptr,
                                                       const int64_t* __restrict__ pos0, const int32_t* __restrict__ state_slot, float* __restrict__ out,
-                                                      int heads, int dim, int vdim, int p_lanes, int tb, int chunk, int n_chunk_max,
+                                                      int heads, int dim, int vdim, int p_lanes, int tb, int vec, int chunk, int n_chunk_max,
                                                       float* __restrict__ ws, float* __restrict__ ws_keep) {
     extern __shared__ float sm[];
     const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
@@ -585,67 +622,68 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(const A* __restrict__ x, 
         sp.n = sp.n - first < chunk ? sp.n - first : chunk;
     }
     const ScanThread th = scan_thread(p_lanes, vdim);
+    const int e0 = blockIdx.x * cb * NC + th.col;              // this thread's value columns: e0, e0 + cb, ...
     const int64_t at = (int64_t)(PHASE ? (int)blockIdx.z : sp.slot) * heads + hd;
     float* Sp = (PHASE ? ws : S) + at * dim * vdim;
-    float s[KR], pr[KR];
+    float s[NC][KR], pr[KR];
     const bool cont = PHASE == 3 || (PHASE == 0 && sp.pos0 > 0);
     const bool keep_here = PHASE == 1 && blockIdx.x == 0 && threadIdx.x < 64;       // the wave that multiplies the decays up
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
-        s[r] = (cont && row < dim && th.active) ? Sp[(int64_t)row * vdim + th.e] : 0.f;
+#pragma unroll
+        for (int n = 0; n < NC; ++n) s[n][r] = (cont && row < dim && e0 + n * cb < vdim) ? Sp[(int64_t)row * vdim + e0 + n * cb] : 0.f;
         pr[r] = 1.f;
     }
     zero_rows(sq, 3 * tb * rs);
-    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, n_waves = blockDim.x >> 6;
     for (int64_t t0 = 0; t0 < sp.n; t0 += tb) {
         const int nt = (int)(sp.n - t0 < tb ? sp.n - t0 : tb);
         __syncthreads();
-        for (int tt = wave; tt < nt; tt += n_waves) {
-            const int64_t tok = sp.q0 + t0 + tt;
-            const A* xr = x + tok * x_stride;
-            const float* ar = alpha + (tok * heads + hd) * dim;
-            for (int d = lane; d < dim; d += 64) {
-                const int o = tt * rs + lds_row(d);
-                if (PHASE != 1) sq[o] = ld_f(xr, q_off + hd * dim + d) * q_mul;
-                sk[o] = ld_f(xr, k_off + hd * dim + d);
-                sa[o] = ar[d];
-            }
-            for (int c = lane; c < cb; c += 64) {
-                const int e = blockIdx.x * cb + c;
-                sv[tt * cb + c] = e < vdim ? ld_f(xr, v_off + hd * vdim + e) : 0.f;
-            }
-        }
+        const A* xr = x + (sp.q0 + t0) * x_stride;
+        if (PHASE != 1) stage_key_rows(sq, rs, xr + q_off + hd * dim, x_stride, nt, dim, vec, 0, q_mul);
+        stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec);
+        stage_key_rows(sa, rs, alpha + ((sp.q0 + t0) * heads + hd) * dim, (int64_t)heads * dim, nt, dim, vec);
+        stage_value_cols(sv, cb * NC, xr + v_off + hd * vdim + blockIdx.x * cb * NC, x_stride, nt, vdim - (int)blockIdx.x * cb * NC, vec);
         __syncthreads();
         for (int tt = 0; tt < nt; ++tt) {
-            const float v = sv[tt * cb + th.col];
+            float v[NC], o[NC];
+#pragma unroll
+            for (int n = 0; n < NC; ++n) { v[n] = sv[(tt * NC + n) * cb + th.col]; o[n] = 0.f; }
             const float* kk = sk + tt * rs + th.p * KS;
             const float* qq = sq + tt * rs + th.p * KS;
             const float* aa = sa + tt * rs + th.p * KS;
             if (PHASE == 1) {
 #pragma unroll
-                for (int r = 0; r < KR; ++r) s[r] = aa[r] * s[r] + kk[r] * v;
+                for (int r = 0; r < KR; ++r)
+#pragma unroll
+                    for (int n = 0; n < NC; ++n) s[n][r] = aa[r] * s[n][r] + kk[r] * v[n];
                 if (keep_here) {
 #pragma unroll
                     for (int r = 0; r < KR; ++r) pr[r] *= aa[r];
                 }
                 continue;
             }
-            float o = 0.f;
 #pragma unroll
-            for (int r = 0; r < KR; ++r) {
-                s[r] = aa[r] * s[r] + kk[r] * v;
-                o += s[r] * qq[r];
+            for (int r = 0; r < KR; ++r)
+#pragma unroll
+                for (int n = 0; n < NC; ++n) {
+                    s[n][r] = aa[r] * s[n][r] + kk[r] * v[n];
+                    o[n] += s[n][r] * qq[r];
+                }
+#pragma unroll
+            for (int n = 0; n < NC; ++n) {
+                const float sum = lanes_sum(o[n], p_lanes);
+                if (th.p == 0 && e0 + n * cb < vdim) out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + e0 + n * cb] = sum;
             }
-            o = lanes_sum(o, p_lanes);
-            if (th.p == 0 && th.active) out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + th.e] = o;
         }
     }
     if (PHASE == 3) return;
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
-        if (row < dim && th.active) Sp[(int64_t)row * vdim + th.e] = s[r];
+#pragma unroll
+        for (int n = 0; n < NC; ++n)
+            if (row < dim && e0 + n * cb < vdim) Sp[(int64_t)row * vdim + e0 + n * cb] = s[n][r];
         if (keep_here && th.col == 0 && row < dim) ws_keep[at * dim + row] = pr[r];
     }
 }
@@ -653,7 +691,7 @@ __global__ __launch_bounds__(256) void gla_scan_kernel(const A* __restrict__ x, 
 // launch geometry of the recurrences: lanes per column (a power of two), threads per workgroup, value columns per
 // workgroup
 struct ScanLaunch { int p_lanes, threads, cb; };
-static bool scan_launch(int64_t dim, int64_t vdim, ScanLaunch* g) {
+static bool scan_launch(int64_t dim, int64_t vdim, ScanLaunch* g) {      // (a thread that keeps several columns: pass vdim over their number)
     int p = 1;
     while ((int64_t)p * KR < dim) p <<= 1;
     if (p > 16) return false;                       // dim <= 512: two staged operands of TB tokens fit the default LDS window
@@ -739,7 +777,8 @@ extern "C" int nvx_mlstm_scan(const void* x, int64_t x_stride, int fmt, int64_t 
     NVX_REQUIRE(x && gates && gate_bias && S && N && M && N_in && M_in && out, NVX_EINVAL, "nvx_mlstm_scan: null pointer");
     NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
                     x_stride >= v_off + heads * vdim, NVX_EINVAL, "nvx_mlstm_scan: q, k or v lies outside a row");
-    const size_t lds = (size_t)(2 * TB * g.p_lanes * KS + TB * g.cb + 2 * TB) * sizeof(float);
+    const int tb = g.p_lanes <= 4 ? 32 : (g.p_lanes == 8 ? 16 : TB);
+    const size_t lds = (size_t)(2 * tb * g.p_lanes * KS + tb * g.cb + 2 * tb) * sizeof(float);
     NVX_REQUIRE(chunk == 0 || (chunk > 0 && chunk < (1 << 30) && n_chunk_max > 0 && n_seq * n_chunk_max <= 65535 && ws && qo_indptr), NVX_EINVAL,
                 "nvx_mlstm_scan: chunks need a ragged step, their workspace, and at most 65535 of them");
     const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
@@ -753,7 +792,7 @@ extern "C" int nvx_mlstm_scan(const void* x, int64_t x_stride, int fmt, int64_t 
 #define NVX_MLSTM_SCAN(PHASE)                                                                                                                     \
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((mlstm_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, st, (const A_*)x, x_stride, (int)q_off, (int)k_off, \
                                          (int)v_off, gates, gate_bias, cap, S, N_in, M_in, N, M, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim, \
-                                         (int)vdim, g.p_lanes, ck))
+                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb), ck))
     if (!chunk) {
         NVX_MLSTM_SCAN(0);
     } else {
@@ -827,7 +866,7 @@ extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t 
 #define NVX_DECAY_SCAN(PHASE)                                                                                                                      \
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((decay_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, (hipStream_t)stream, (const A_*)x, x_stride,   \
                                          (int)q_off, (int)k_off, (int)v_off, act, decay, S, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim,  \
-                                         (int)vdim, g.p_lanes, tb, (int)chunk, (int)n_chunk_max, ws))
+                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb), (int)chunk, (int)n_chunk_max, ws))
     if (!chunk) {
         NVX_DECAY_SCAN(0);
     } else {
@@ -852,25 +891,29 @@ extern "C" int nvx_gla_scan(const void* x, int64_t x_stride, int fmt, int64_t q_
     NVX_REQUIRE(x && alpha && S && out, NVX_EINVAL, "nvx_gla_scan: null pointer");
     NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
                     x_stride >= v_off + heads * vdim, NVX_EINVAL, "nvx_gla_scan: q, k or v lies outside a row");
-    const int tb = g.p_lanes <= 2 ? 32 : (g.p_lanes == 4 ? 16 : (g.p_lanes == 8 ? 8 : 4));
-    const size_t lds = (size_t)(3 * tb * g.p_lanes * KS + tb * g.cb) * sizeof(float);
+    const int nc = chunk && vdim > 1 ? 2 : 1;      // value columns per thread: a staged row then serves two of them
+    NVX_REQUIRE(scan_launch(dim, (vdim + nc - 1) / nc, &g), NVX_EUNSUPPORTED, "nvx_gla_scan: key size above 512");
+    const int tb = g.p_lanes <= 2 && nc == 1 ? 32 : (g.p_lanes <= 4 ? 16 : (g.p_lanes == 8 ? 8 : 4));
+    const size_t lds = (size_t)(3 * tb * g.p_lanes * KS + tb * g.cb * nc) * sizeof(float);
     NVX_REQUIRE(chunk == 0 || (chunk > 0 && chunk < (1 << 30) && n_chunk_max > 0 && n_seq * n_chunk_max <= 65535 && ws && qo_indptr), NVX_EINVAL,
                 "nvx_gla_scan: chunks need a ragged step, their workspace, and at most 65535 of them");
-    const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
+    const dim3 grid((unsigned)((vdim + g.cb * nc - 1) / (g.cb * nc)), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
     float* keep = chunk ? ws + n_seq * n_chunk_max * heads * dim * vdim : nullptr;      // behind the chunks' memories
     const hipStream_t st = (hipStream_t)stream;
-#define NVX_GLA_SCAN(PHASE)                                                                                                                        \
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((gla_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, st, (const A_*)x, x_stride, (int)q_off, (int)k_off, \
+#define NVX_GLA_SCAN(PHASE, NC)                                                                                                                        \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((gla_scan_kernel<A_, PHASE, NC>), grid, dim3(g.threads), lds, st, (const A_*)x, x_stride, (int)q_off, (int)k_off, \
                                          (int)v_off, q_mul, alpha, S, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim, (int)vdim, g.p_lanes, \
-                                         tb, (int)chunk, (int)n_chunk_max, ws, keep))
+                                         tb, (int)(stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb * nc) && nvx_aligned16(alpha)), (int)chunk, (int)n_chunk_max, ws, keep))
     if (!chunk) {
-        NVX_GLA_SCAN(0);
+        NVX_GLA_SCAN(0, 1);
     } else {
-        NVX_GLA_SCAN(1);
+        if (nc == 2) NVX_GLA_SCAN(1, 2);
+        else NVX_GLA_SCAN(1, 1);
         hipLaunchKernelGGL(chunk_carry_kernel, dim3((unsigned)((heads * dim * vdim + 255) / 256), (unsigned)n_seq), dim3(256), 0, st, S, ws,
                            (const float*)keep, 1, (const float*)nullptr, qo_indptr, pos0, state_slot, (int)heads, (int)dim, (int)vdim, (int)chunk,
                            (int)n_chunk_max);
-        NVX_GLA_SCAN(3);
+        if (nc == 2) NVX_GLA_SCAN(3, 2);
+        else NVX_GLA_SCAN(3, 1);
     }
 #undef NVX_GLA_SCAN
     return nvx_check_launch("nvx_gla_scan");

@@ -971,16 +971,18 @@ SCAN_CHUNK_FROM = 256       # portions from this length on are cut into chunks t
 SCAN_CHUNKS = ((65536, 32), (131072, 64), (None, 128))      # (tokens x heads of a step up to ..., tokens of a chunk): short chunks while
 # the step is too small to fill the chip with long ones, long chunks (fewer carried states) from there on (4 x 1 024 tokens, 8
 # heads: 895 us in one walk, 301 in chunks of 128, 150 in chunks of 32; 16 x 1 024 tokens: 446 us at 128 and 64, 474 at 32)
+GLA_SCAN_CHUNKS = ((32768, 32), (None, 64))       # (4 x 1 024 tokens: 8 heads 116 us at 32, 164 at 64; 16 heads 222 and 178)
+MLSTM_SCAN_CHUNKS = ((None, 64),)                 # (the same: 191 and 167; 312 and 291; one walk per portion: 1 420)
 SCAN_WS_BYTES = 1 << 30     # the chunks' states may take this much; longer chunks otherwise
 
 
-def _scan_chunks(layout: StepLayout, heads: int, per_chunk: int, chunk: Optional[int]):
+def _scan_chunks(layout: StepLayout, heads: int, per_chunk: int, chunk: Optional[int], table=SCAN_CHUNKS):
     """(chunk, chunks of the longest portion) a recurrence over a matrix per head cuts a step's portions into (0, 0: not at all).
-    `per_chunk`: floats of workspace a chunk of one sequence takes; `chunk` None: by the step's shape."""
+    `per_chunk`: floats of workspace a chunk of one sequence takes; `chunk` None: by the step's shape, from `table`."""
     if chunk is None:
         chunk = 0
         if layout.qo_indptr is not None and layout.max_q >= SCAN_CHUNK_FROM:
-            chunk = next(c for upto, c in SCAN_CHUNKS if upto is None or layout.n_tok * heads <= upto)
+            chunk = next(c for upto, c in table if upto is None or layout.n_tok * heads <= upto)
     if not chunk or layout.qo_indptr is None:
         return 0, 0
     while layout.n_seq * -(-layout.max_q // chunk) * per_chunk * 4 > SCAN_WS_BYTES or layout.n_seq * -(-layout.max_q // chunk) > 65535:
@@ -1008,7 +1010,7 @@ def mlstm_scan(x, offsets, gates, gate_bias, cap: float, mem, norm, peak, layout
     # a head whose value columns take several workgroups: all of them read the normaliser and the maximum, the first writes them
     # back, so they read from copies (a workgroup that starts late must not see the new values)
     per_chunk = heads * (dim * (vdim + 1) + 3)
-    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk)
+    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk, MLSTM_SCAN_CHUNKS)
     ws = torch.empty((layout.n_seq * n_chunks * per_chunk,), dtype=F32, device=x.device) if chunk else None
     several = not chunk and lib.nvx_scan_column_blocks(dim, vdim) != 1
     norm_in, peak_in = (norm.clone(), peak.clone()) if several else (norm, peak)
@@ -1606,7 +1608,7 @@ def gla_scan(x, offsets, alpha, mem, layout: StepLayout, heads: int, dim: int, v
     _need(alpha.shape == (t, heads * dim) and mem.shape == (n_slots, heads, dim, vdim), "gla_scan: shapes")
     out = torch.empty((t, heads, vdim), dtype=F32, device=x.device)
     per_chunk = heads * dim * (vdim + 1)
-    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk)
+    chunk, n_chunks = _scan_chunks(layout, heads, per_chunk, chunk, GLA_SCAN_CHUNKS)
     ws = torch.empty((layout.n_seq * n_chunks * per_chunk,), dtype=F32, device=x.device) if chunk else None
     lib = _lib.load()
     _lib.check(lib.nvx_gla_scan(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], float(q_mul), _ptr(alpha), _ptr(mem), n_slots,
