@@ -191,6 +191,52 @@ __global__ __launch_bounds__(256) void tied_prep_store_kernel(const A* __restric
     }
 }
 
+template <int LPR> __device__ __forceinline__ float group_sum(float v) {      // over LPR neighbouring lanes, in the vector ALU
+    v += dpp_move<0xB1>(v);                        // lane ^ 1
+    v += dpp_move<0x4E>(v);                        // lane ^ 2
+    v += dpp_move<0x141>(v);                       // the other quad of eight
+    if (LPR >= 16) v += dpp_move<0x140>(v);        // the other eight of sixteen
+    if (LPR >= 32) v += xor16(v);
+    if (LPR >= 64) v += xor32(v);
+    return v;
+}
+
+// The same with a head per LPR neighbouring lanes of eight elements each (16-byte loads and stores in 16-bit formats; dim a multiple of
+// eight up to 8 * LPR, rows on such borders): 64 / LPR heads a wave.
+template <typename A, int LPR>
+__global__ __launch_bounds__(256) void tied_prep_store_vec_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off,
+                                                                 const float* __restrict__ q_w, const float* __restrict__ k_w, float eps,
+                                                                 const int64_t* __restrict__ slots, A* __restrict__ q_out, A* __restrict__ k_cache,
+                                                                 float* __restrict__ k_rn, int64_t n_rows, int heads, int kv_heads, int dim) {
+    typedef A vec8 __attribute__((ext_vector_type(8)));
+    const int64_t idx = ((int64_t)blockIdx.x * 256 + threadIdx.x) / LPR;
+    const int l = threadIdx.x % LPR, per = heads + kv_heads;
+    const bool row_on = idx < n_rows, on = row_on && l * 8 < dim;
+    const int64_t t = row_on ? idx / per : 0;
+    const int hd = row_on ? (int)(idx % per) : 0;
+    const bool is_q = hd < heads;
+    vec8 v;
+    float ss = 0.f;
+    if (on) {
+        v = *reinterpret_cast<const vec8*>(x + t * x_stride + (is_q ? q_off + hd * dim : k_off + (hd - heads) * dim) + l * 8);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += (float)v[i] * (float)v[i];
+    }
+    const float rn = 1.0f / sqrtf(group_sum<LPR>(ss) / (float)dim + eps);
+    if (!on) return;
+    if (is_q) {
+        vec8 o;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = (A)((float)v[i] * rn * q_w[l * 8 + i] * k_w[l * 8 + i]);
+        *reinterpret_cast<vec8*>(q_out + (t * heads + hd) * dim + l * 8) = o;
+    } else {
+        const int64_t slot = slots[t];
+        if (slot < 0) return;
+        *reinterpret_cast<vec8*>(k_cache + (slot * kv_heads + (hd - heads)) * dim + l * 8) = v;
+        if (l == 0) k_rn[slot * kv_heads + (hd - heads)] = rn;
+    }
+}
+
 // What limits the keys a token at `pos` sees from below: a window of `window` keys, chunks of `chunk` positions counted from 0 (neither: 0)
 __device__ __forceinline__ int first_seen(int pos, int window, int chunk) {
     if (window > 0) return pos - window + 1 > 0 ? pos - window + 1 : 0;
@@ -380,15 +426,6 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
 // score to the read-out, for all NH heads: a wave takes U keys per lane group at a time (their loads in flight together), sums the
 // products over the lane group, and adds the weighted rows to what the lane keeps of the read-out.  Every lane group has a running
 // maximum and sum of its own; groups, waves and splits are merged at the end.
-template <int LPR> __device__ __forceinline__ float group_sum(float v) {      // over LPR neighbouring lanes, in the vector ALU
-    v += dpp_move<0xB1>(v);                        // lane ^ 1
-    v += dpp_move<0x4E>(v);                        // lane ^ 2
-    v += dpp_move<0x141>(v);                       // the other quad of eight
-    if (LPR >= 16) v += dpp_move<0x140>(v);        // the other eight of sixteen
-    if (LPR >= 32) v += xor16(v);
-    if (LPR >= 64) v += xor32(v);
-    return v;
-}
 template <typename A, int NH, int U, int LPR>
 __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict__ q, const A* __restrict__ rows, const float* __restrict__ k_rn,
                                                             const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
@@ -876,12 +913,25 @@ extern "C" int nvx_tied_prep_store(const void* x, int64_t x_stride, int fmt, int
                                    int64_t heads, int64_t kv_heads, int64_t dim, nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_tied_prep_store: fmt must be 0, 1 or 2");
     NVX_REQUIRE(n_tok >= 0 && heads > 0 && kv_heads > 0 && dim > 0 && n_slots >= 0 && (heads + kv_heads) * dim < (1 << 30) &&
-                    n_tok * (heads + kv_heads) < (1ll << 32), NVX_EINVAL, "nvx_tied_prep_store: bad sizes");
+                    n_tok * (heads + kv_heads) < (1ll << 30), NVX_EINVAL, "nvx_tied_prep_store: bad sizes");
     NVX_REQUIRE(q_off >= 0 && k_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + kv_heads * dim, NVX_EINVAL,
                 "nvx_tied_prep_store: q or k lies outside a row");
     if (n_tok == 0) return NVX_OK;
     NVX_REQUIRE(x && q_w && k_w && slots && q_out && k_cache && k_rn, NVX_EINVAL, "nvx_tied_prep_store: null pointer");
     const int64_t rows = n_tok * (heads + kv_heads);
+    if (dim % 8 == 0 && dim <= 512 && x_stride % 8 == 0 && q_off % 8 == 0 && k_off % 8 == 0 && nvx_aligned16(x) && nvx_aligned16(q_out) &&
+        nvx_aligned16(k_cache)) {
+#define NVX_TIED_PREP(LPR)                                                                                                                            \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((tied_prep_store_vec_kernel<A_, LPR>), dim3((unsigned)((rows * LPR + 255) / 256)), dim3(256), 0, (hipStream_t)stream, \
+                                         (const A_*)x, x_stride, (int)q_off, (int)k_off, q_w, k_w, eps, slots, (A_*)q_out, (A_*)k_cache, k_rn, rows, (int)heads, \
+                                         (int)kv_heads, (int)dim))
+        if (dim <= 64) NVX_TIED_PREP(8);
+        else if (dim <= 128) NVX_TIED_PREP(16);
+        else if (dim <= 256) NVX_TIED_PREP(32);
+        else NVX_TIED_PREP(64);
+#undef NVX_TIED_PREP
+        return nvx_check_launch("nvx_tied_prep_store");
+    }
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL(tied_prep_store_kernel<A_>, dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, (hipStream_t)stream, (const A_*)x,
                                          x_stride, (int)q_off, (int)k_off, q_w, k_w, eps, slots, (A_*)q_out, (A_*)k_cache, k_rn, rows, (int)heads,
                                          (int)kv_heads, (int)dim));

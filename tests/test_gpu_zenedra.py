@@ -160,20 +160,22 @@ def test_sublayer_boundary(fmt, width):
 
 
 @pytest.mark.parametrize("fmt", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("heads,kv_heads,dim", [(6, 2, 24), (3, 3, 7), (4, 1, 96), (2, 2, 1)])
-def test_queries_are_normed_and_raw_keys_stored_with_their_reciprocal_norm(fmt, heads, kv_heads, dim):
+@pytest.mark.parametrize("heads,kv_heads,dim,at", [(6, 2, 24, 3), (3, 3, 7, 3), (4, 1, 96, 8), (2, 2, 1, 5), (6, 2, 24, 8), (5, 1, 64, 16), (2, 1, 200, 8), (3, 1, 512, 0)])
+def test_queries_are_normed_and_raw_keys_stored_with_their_reciprocal_norm(fmt, heads, kv_heads, dim, at):
+    """The parts are slices of a wider projection, at columns that fit 16-byte loads and at columns that do not."""
     from nano_vllm_x_amd import ops
     g = torch.Generator().manual_seed(dim)
     t, eps = 6, 1e-2
     nq, nk = heads * dim, kv_heads * dim
-    x = torch.randn(t, 3 + nq + 2 + nk, generator=g).to(fmt)
+    gap = 8 if at % 8 == 0 else 2
+    x = torch.randn(t, at + nq + gap + nk, generator=g).to(fmt)
     qw, kw = torch.randn(dim, generator=g), torch.randn(dim, generator=g)
     slots = torch.tensor([4, 0, -1, 7, 2, 5], dtype=torch.int64)
     cache, rn = torch.full((8, nk), 9.0).to(fmt).cuda(), torch.full((8, kv_heads), 9.0).cuda()
-    q = ops.tied_prep_store(x.cuda(), (3, 3 + nq + 2), qw.cuda(), kw.cuda(), eps, slots.cuda(), cache, rn, heads, kv_heads, dim)
-    want_q = zo.rms(x[:, 3:3 + nq].double().view(t, heads, dim), eps) * qw.double() * kw.double()
+    q = ops.tied_prep_store(x.cuda(), (at, at + nq + gap), qw.cuda(), kw.cuda(), eps, slots.cuda(), cache, rn, heads, kv_heads, dim)
+    want_q = zo.rms(x[:, at:at + nq].double().view(t, heads, dim), eps) * qw.double() * kw.double()
     close(q.float().cpu(), want_q.reshape(t, nq), 1e-5 if fmt == torch.float32 else 4e-2, "queries")
-    k = x[:, 5 + nq:]
+    k = x[:, at + nq + gap:]
     keep = slots >= 0
     assert torch.equal(cache.cpu()[slots[keep]], k[keep])
     want_rn = 1.0 / torch.sqrt((k.double().view(t, kv_heads, dim) ** 2).mean(-1) + eps)
