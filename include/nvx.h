@@ -50,8 +50,12 @@ typedef void* nvx_stream_t;
  *  18: keys and values tied in one cached row (`nvx_tied_prep_store`), chunks of positions, a linear distance penalty and keys normed as
  *      they are scored in nvx_softcap_attn; gated linear attention (`nvx_gla_scan`); nvx_mlstm_scan takes long portions in chunks; the
  *      sigmoid router with groups (`nvx_moe_route_sigmoid`), `nvx_gelu_glu`, `nvx_residual_norm`, `nvx_embed_sum`; nvx_skinny_proj has a bias
- *      and an output activation. */
-#define NVX_ABI_VERSION 18
+ *      and an output activation.
+ *  19: queries, keys and values convolved over time ahead of the cache (`nvx_conv_attn_prep`), a step's table of rotations
+ *      (`nvx_turn_table`), a sink per head and kept first tokens in nvx_softcap_attn, rotated queries and keys in nvx_decay_scan, its form for
+ *      single tokens (`nvx_decay_step`), layer norms in nvx_residual_norm and nvx_embed_sum, row strides and a gate per row in nvx_moe_glu;
+ *      nvx_softcap_attn and nvx_head_norm_gate write rows of a wider buffer, times a constant. */
+#define NVX_ABI_VERSION 19
 
 /* Library identification and diagnostics. */
 int nvx_abi_version(void);
@@ -507,8 +511,9 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     r = y[t], or with y2: r = (y[t] / rms(y[t]) * w_y + y2[t] / rms(y2[t]) * w_y2) / 2      (rms over the whole row, with eps)
  *     gate != NULL: r *= sigmoid(gate[t] + gate_bias)   (gate_bias may be NULL);   x[t] += mult * r   (y == NULL: x unchanged)
  *     w_norm != NULL: h_out[t] = x[t] with each of `groups` consecutive slices divided by sqrt(mean(slice^2) + eps), times w_norm.
- * nvx_head_norm_gate:  out[t][h] = o[t][h] / rms(o[t][h]) * w * G   per head of vdim values; w has heads * vdim entries, or vdim
- *     shared by the heads (w_shared); kind 0: G = 1, 1: G = sigmoid(gate), 2: G = gate * sigmoid(gate)  (gate laid out as out).
+ * nvx_head_norm_gate:  out[t][h] = mul * o[t][h] / rms(o[t][h]) * w * G   per head of vdim values; w has heads * vdim entries, or vdim
+ *     shared by the heads (w_shared), or is null (ones); kind 0: G = 1, 1: G = sigmoid(gate), 2: G = gate * sigmoid(gate)  (gate and out:
+ *     rows of heads * vdim at their own strides).
  * nvx_short_conv_silu:  out[t][c] = silu(sum_j w[j][c] * x[t - (taps_n - 1) + j][c]) over t's own sequence (w: taps_n rows of
  *     `channels`); inputs before this step come from state[slot] (taps_n - 1 rows, oldest first), which is then replaced by the
  *     sequence's last taps_n - 1 inputs; inputs before the sequence's start are zero.
@@ -557,7 +562,9 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     query's position),  s_j <- s_j - slopes[h] (i - j) (slopes != null),  out = softmax(s) V; with vcs ((n_tok, vdim) float32: each query token's cos | sin, as nvx_attn_prep_store
  *     hands them out) the pairs of out are turned back by those angles (the counterpart of rotated values), with gate out is multiplied by
  *     sigmoid(gate[t]) (same layout as out, or with gate_per_head one number per head: gate[t][h]).  With sink != 0 the softmax's sum
- *     has one more term exp(sink_score) that carries no value: p_j = exp(s_j) / (exp(sink_score) + sum exp(s)).  Query head h reads
+ *     has one more term exp(sink_score) that carries no value: p_j = exp(s_j) / (exp(sink_score) + sum exp(s)); sinks != null: exp(sinks[h])
+ *     instead, a number per head.  keep_first > 0 (with a window): the sequence's first keep_first tokens stay visible to every later one.
+ *     out[t] (rows out_stride apart) is the result times out_mul.  Query head h reads
  *     key/value head h / (heads / kv_heads).  q (n_tok, heads * dim), k_cache (slots, kv_heads * dim), v_cache (slots, kv_heads *
  *     vdim), out (n_tok, heads * vdim).  n_split > 1 (for steps of few tokens): a (token, head)'s keys are dealt out over n_split
  *     workgroups whose partial results go to `part` (n_tok * heads * n_split * (vdim + 2) floats) and are merged by a second launch.
@@ -566,7 +573,7 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  *     keys in tiles of 32, weights as hi + lo 16-bit halves); scores and the softmax stay float32.
  * nvx_moe_route:  idx[t][k], wts[t][k] = the expert with the k-th largest logit of token t (ties: the lower id) and the sigmoid
  *     of that logit.
- * nvx_moe_route_softmax:  scores = softmax(logits[t]) over all n_exp experts; with n_groups > 1 the experts form n_groups equal
+ * nvx_moe_route_softmax:  (rows of logits logits_stride apart)  scores = softmax(logits[t]) over all n_exp experts; with n_groups > 1 the experts form n_groups equal
  *     groups of neighbours, a group counts as its largest score and only experts of the keep_groups best groups can be chosen; idx[t]
  *     = the `top` largest scores among those (ties: the lower id), wts[t][k] = score / (sum of the chosen scores + norm_eps).
  * Expert e:  g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), y = g sigmoid(alpha g) (u + shift), result W_down y, with
@@ -578,12 +585,25 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  * nvx_moe_order:  dst[r] = place of pair r (= token * top + choice) when the n pairs are put in expert order, pairs of one expert
  *     keeping their order; counts[e] = pairs of expert e.  n_exp <= nvx_moe_order_max_experts().
  * nvx_moe_scatter_rows:  xs[dst[r]] = wts[r] * h[r / top] for every (token, choice) pair r (wts == null: ones).
- * nvx_moe_glu:  y[r][j] = the expert's activation of (gu[r][j], gu[r][ff + j]).
+ * nvx_moe_glu:  y[r][j] = the expert's activation of (gu[r][j], gu[r][ff + j]), times sigmoid(row_gate[r * row_gate_stride]) if row_gate is
+ *     given; rows of gu and y at their own strides.
  * nvx_moe_gather_rows:  out[t] = sum_k wts[t * top + k] * ys[dst[t * top + k]] (wts == null: ones).
  * nvx_decay_scan:  x[t] holds q at q_off, k at k_off (heads * dim each) and v at v_off (heads * vdim); act 1: silu of all three first.
  *     S <- decay[h] S + k v^T;  out[t] = S^T q.   S (slots, heads, dim, vdim), decay (heads) float32.  dim <= 512.  chunk > 0 (ragged
  *     steps): portions are cut into chunks of that many tokens which run side by side, the states at their starts carried through
  *     ws (n_seq * n_chunk_max * heads * dim * vdim floats; n_chunk_max >= the chunks of the longest portion); chunk 0: one walk.
+ *     rot_dims > 0: pairs (m, m + rot_dims / 2) of every q and k head are first rotated, (u, v) -> (u c - v s, v c + u s) with c =
+ *     turn[t * turn_stride + m] and s = turn[t * turn_stride + turn_sin_off + m] (float32, as nvx_turn_table writes them); k is multiplied
+ *     by k_mul.
+ * nvx_decay_step:  nvx_decay_scan for a step of one token per sequence, with the end of nvx_head_norm_gate (w null): out[b][h] = mul * o /
+ *     rms(o) * G, G from the columns of x at g_off by `kind`; rows of out out_stride apart, in the format `fmt`.  A sequence without a slot
+ *     gets zeros.  vdim <= nvx_decay_step_max_vdim() (256 where it is not a multiple of four).
+ * nvx_turn_table:  out[t] = [cos(positions[t] * freq[m]) for m < n | sin(.) for m < n], angles formed and reduced in double precision.
+ * nvx_conv_attn_prep:  x[t] = [q (heads * dim) | k (kv_heads * dim) | v (kv_heads * vdim)], rows x_stride apart, all of them channels of a
+ *     causal convolution over the sequence: u[t][c] = sum_j w[j][c] x[t - (taps_n - 1) + j][c] (w: taps_n rows of that many channels; inputs
+ *     before this step from state[slot] (taps_n - 1 rows, oldest first), which then takes the last ones; zeros before the sequence's
+ *     start).  Every q and k head of u is then rotated (rot_dims, turn: as for nvx_decay_scan) and with `norm` divided by its root mean square;
+ *     q_out[t], k_cache[slots[t]], v_cache[slots[t]] take the results (a negative slot: no key or value).  Float32 up to what is stored.
  * nvx_postnorm_residual:  r = a y[t] (+ b y2[t]);  x[t] += r / rms(r) * w_post (w_post_n = 1: one number, = width: per channel);
  *     h_out[t] = x[t] / rms(x[t]) * w_next (w_next != null) or x[t] itself, in the format `fmt`.  rms(z) = sqrt(mean z^2 + eps).
  * nvx_hyper_mix:  n_streams residual streams per token, x_out (n_tok, n_streams, width) float32.  With a result y (format `fmt`):
@@ -603,7 +623,7 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  * nvx_embed_scale:  x[t] = table[ids[t]] * scale (float32), h[t] the same in the table's format (h may be null).
  * nvx_tanh_cap:  out[i] = cap tanh(in[i] / cap) in float32 (cap <= 0: a copy).
  * nvx_residual_norm:  v = x_in[t] (+ y[t]) (+ y2[t]) (format `fmt`) (+ add[t]) (+ bias) (float32); x_out[t] = v (x_in may be x_out);
- *     h null: no more; split 0: h[t] = v / rms(v) * w;  split 1: h[t] = [hi | lo] (2 * width), hi v rounded to the format and lo what
+ *     h null: no more; split 0: h[t] = v / rms(v) * w, or with w_bias the layer norm (v - mean) / sqrt(variance + eps) * w + w_bias;  split 1: h[t] = [hi | lo] (2 * width), hi v rounded to the format and lo what
  *     that lost.  width <= 15360.
  * nvx_embed_sum:  x[t] = table[ids[t]] (+ pair[r]) (+ pos_table[positions[t]]) in float32, then h as for nvx_residual_norm.  r = (previous
  *     id * mul_prev + id * mul_cur) mod buckets, and `buckets` (pair has buckets + 1 rows) for a sequence's first token.  prev_id (slots)
@@ -620,7 +640,7 @@ int nvx_gated_residual_norm(const void* y, int64_t y_stride, const void* y2, int
                             float mult, float* x, const float* w_norm, int groups, float eps, void* h_out, int64_t n_tok,
                             int64_t width, nvx_stream_t stream);
 int nvx_head_norm_gate(const float* o, const float* w, int w_shared, const void* gate, int64_t gate_stride, int kind, int fmt,
-                       float eps, void* out, int64_t n_tok, int64_t heads, int64_t vdim, nvx_stream_t stream);
+                       float eps, float mul, void* out, int64_t out_stride, int64_t n_tok, int64_t heads, int64_t vdim, nvx_stream_t stream);
 int nvx_short_conv_silu(const void* x, int64_t x_stride, int fmt, const float* w, int taps_n, float* state, int64_t n_slots,
                         const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot,
                         void* out, int64_t n_tok, int64_t n_seq, int64_t channels, nvx_stream_t stream);
@@ -668,7 +688,7 @@ int nvx_softcap_attn(const void* q, const void* k_cache, const void* v_cache, in
                      float scale, float cap, void* out, int64_t n_tok, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
                      int n_split, float* part, int64_t window, int64_t chunk, const float* r1, const float* r2, const float* slopes,
                      const float* k_rn, const float* vcs, int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
-                     int64_t n_seq, int matrix_cores, nvx_stream_t stream);
+                     const float* sinks, int64_t keep_first, float out_mul, int64_t out_stride, int64_t n_seq, int matrix_cores, nvx_stream_t stream);
 int nvx_tied_prep_store(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, const float* q_w, const float* k_w, float eps,
                         const int64_t* slots, void* q_out, void* k_cache, float* k_rn, int64_t n_slots, int64_t n_tok, int64_t heads,
                         int64_t kv_heads, int64_t dim, nvx_stream_t stream);
@@ -681,7 +701,18 @@ int nvx_attn_prep_store(const void* x, int64_t x_stride, int fmt, int64_t q_off,
 int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, int act,
                    const float* decay, float* S, int64_t n_slots, const int32_t* qo_indptr, const int64_t* pos0,
                    const int32_t* state_slot, float* out, int64_t n_tok, int64_t n_seq, int64_t heads, int64_t dim, int64_t vdim,
-                   int64_t chunk, int64_t n_chunk_max, float* ws, nvx_stream_t stream);
+                   int64_t chunk, int64_t n_chunk_max, float* ws, const float* turn, int64_t turn_stride, int64_t turn_sin_off, int rot_dims,
+                   float k_mul, nvx_stream_t stream);
+int64_t nvx_decay_step_max_vdim(void);
+int nvx_decay_step(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, int act, const float* decay, float* S,
+                   int64_t n_slots, const int64_t* pos0, const int32_t* state_slot, int64_t n_seq, int64_t heads, int64_t dim, int64_t vdim,
+                   const float* turn, int64_t turn_stride, int64_t turn_sin_off, int rot_dims, float k_mul, float eps, int64_t g_off, int kind,
+                   float mul, void* out, int64_t out_stride, nvx_stream_t stream);
+int nvx_turn_table(const int64_t* positions, const double* freq, int64_t n, float* out, int64_t n_tok, nvx_stream_t stream);
+int nvx_conv_attn_prep(const void* x, int64_t x_stride, int fmt, const float* w, int taps_n, float* state, int64_t n_slots, const int32_t* tok_seq,
+                       const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, const float* turn, int64_t turn_stride,
+                       int64_t turn_sin_off, int rot_dims, int norm, float eps, const int64_t* slots, void* q_out, void* k_cache, void* v_cache,
+                       int64_t n_tok, int64_t n_seq, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim, nvx_stream_t stream);
 int nvx_postnorm_residual(const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, float a, float b, const float* w_post,
                           int64_t w_post_n, int fmt, float* x, const float* w_next, int64_t w_next_n, float eps, void* h_out,
                           int64_t n_tok, int64_t width, nvx_stream_t stream);
@@ -689,7 +720,7 @@ int nvx_embed_scale(const int64_t* ids, const void* table, int fmt, int64_t voca
                     int64_t width, nvx_stream_t stream);
 int nvx_tanh_cap(const void* in, int fmt, float cap, float* out, int64_t n, nvx_stream_t stream);
 int nvx_moe_route(const float* logits, int64_t n_tok, int64_t n_exp, int64_t top, int32_t* idx, float* wts, nvx_stream_t stream);
-int nvx_moe_route_softmax(const float* logits, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups, int64_t keep_groups,
+int nvx_moe_route_softmax(const float* logits, int64_t logits_stride, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups, int64_t keep_groups,
                           float norm_eps, int32_t* idx, float* wts, nvx_stream_t stream);
 int64_t nvx_moe_expert_rows_max_width(int64_t ff);
 int nvx_moe_expert_rows(const void* h, int64_t h_stride, int fmt, const int32_t* idx, const float* wts, int64_t top,
@@ -699,19 +730,19 @@ int64_t nvx_moe_order_max_experts(void);
 int nvx_moe_order(const int32_t* idx, int64_t n, int64_t n_exp, int64_t* dst, int32_t* counts, nvx_stream_t stream);
 int nvx_moe_scatter_rows(const void* h, int64_t h_stride, int fmt, const float* wts, const int64_t* dst, int64_t top, void* xs,
                          int64_t n_tok, int64_t width, nvx_stream_t stream);
-int nvx_moe_glu(const void* gu, int fmt, float limit, float alpha, float shift, void* y, int64_t rows, int64_t ff,
-                nvx_stream_t stream);
+int nvx_moe_glu(const void* gu, int64_t gu_stride, int fmt, float limit, float alpha, float shift, const float* row_gate, int64_t row_gate_stride,
+                void* y, int64_t y_stride, int64_t rows, int64_t ff, nvx_stream_t stream);
 int nvx_moe_gather_rows(const void* ys, int fmt, const int64_t* dst, const float* wts, int64_t top, void* out, int64_t n_tok,
                         int64_t width, nvx_stream_t stream);
 int nvx_skinny_proj(const void* x, int64_t x_stride, int fmt, const float* w, int in_act, const float* bias, int out_act, float power,
                     float* out, int64_t n_tok, int64_t n_out, int64_t k_in, nvx_stream_t stream);
 int nvx_residual_norm(const float* x_in, const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, const float* add,
-                      const float* bias, int fmt, float* x_out, const float* w, float eps, int split, void* h, int64_t n_tok, int64_t width,
-                      nvx_stream_t stream);
+                      const float* bias, int fmt, float* x_out, const float* w, const float* w_bias, float eps, int split, void* h, int64_t n_tok,
+                      int64_t width, nvx_stream_t stream);
 int nvx_embed_sum(const int64_t* ids, const void* table, int fmt, int64_t vocab, const void* pair, int64_t buckets, int64_t mul_prev,
                   int64_t mul_cur, float* prev_id, int64_t n_slots, const void* pos_table, int64_t n_pos, const int64_t* positions,
                   const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* x, const float* w,
-                  float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width, nvx_stream_t stream);
+                  const float* w_bias, float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width, nvx_stream_t stream);
 int nvx_moe_route_sigmoid(const float* logits, const float* correction, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups,
                           int64_t keep_groups, float w_scale, int32_t* idx, float* wts, nvx_stream_t stream);
 int nvx_gelu_glu(const void* gu, int fmt, void* y, int64_t rows, int64_t ff, nvx_stream_t stream);

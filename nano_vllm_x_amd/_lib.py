@@ -94,7 +94,8 @@ SIGNATURES = {
                                  _c_vp]),
     "nvx_gated_residual_norm": (_c_i32, [_c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_i64, _c_vp, _c_i32, _c_f32, _c_vp, _c_vp, _c_i32,
                                          _c_f32, _c_vp, _c_i64, _c_i64, _c_vp]),
-    "nvx_head_norm_gate": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_vp, _c_i64, _c_i32, _c_i32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_head_norm_gate": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_vp, _c_i64, _c_i32, _c_i32, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64,
+                                    _c_vp]),
     "nvx_short_conv_silu": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
                                      _c_i64, _c_vp]),
     "nvx_token_shift_mix": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
@@ -108,14 +109,14 @@ SIGNATURES = {
                                _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_rope_vnorm_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_f32, _c_i32, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
                                       _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
-    "nvx_softcap_attn": (_c_i32, [_c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64,
-                                  _c_i64, _c_i64, _c_i64, _c_i32, _c_vp, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i32, _c_vp,
-                                  _c_i64, _c_i32, _c_i32, _c_f32, _c_i64, _c_i32, _c_vp]),
+    "nvx_softcap_attn": (_c_i32, [_c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64,
+                                  _c_i64, _c_i64, _c_i32, _c_vp, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i32, _c_vp, _c_i64,
+                                  _c_i32, _c_i32, _c_f32, _c_vp, _c_i64, _c_f32, _c_i64, _c_i64, _c_i32, _c_vp]),
     "nvx_softcap_attn_tile_fits": (_c_i32, [_c_i32, _c_i64, _c_i64, _c_i32]),
     "nvx_attn_prep_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp, _c_i32, _c_f32, _c_vp, _c_i32, _c_i32,
                                      _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
-    "nvx_decay_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_i32, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp,
-                                _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
+    "nvx_decay_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_i32, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64,
+                                _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp, _c_i64, _c_i64, _c_i32, _c_f32, _c_vp]),
     "nvx_postnorm_residual": (_c_i32, [_c_vp, _c_i64, _c_vp, _c_i64, _c_f32, _c_f32, _c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_i64, _c_f32, _c_vp,
                                        _c_i64, _c_i64, _c_vp]),
     "nvx_embed_scale": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_i64, _c_f32, _c_vp, _c_vp, _c_i64, _c_i64, _c_vp]),
@@ -127,7 +128,7 @@ SIGNATURES = {
     "nvx_moe_order_max_experts": (_c_i64, []),
     "nvx_moe_order": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_vp, _c_vp, _c_vp]),
     "nvx_moe_scatter_rows": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_i64, _c_vp]),
-    "nvx_moe_glu": (_c_i32, [_c_vp, _c_i32, _c_f32, _c_f32, _c_f32, _c_vp, _c_i64, _c_i64, _c_vp]),
+    "nvx_moe_glu": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_f32, _c_f32, _c_f32, _c_vp, _c_i64, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_moe_gather_rows": (_c_i32, [_c_vp, _c_i32, _c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_i64, _c_vp]),
     "nvx_short_conv": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_i32, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64,
                                 _c_i64, _c_i64, _c_vp]),
@@ -137,17 +138,23 @@ SIGNATURES = {
                                       _c_i64, _c_i64, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_hyper_mix": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_vp, _c_i64, _c_i32, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_i64,
                                _c_i64, _c_i64, _c_vp]),
-    "nvx_moe_route_softmax": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_vp]),
+    "nvx_moe_route_softmax": (_c_i32, [_c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_vp]),
     "nvx_gla_scan": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp,
                               _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp, _c_vp]),
     "nvx_tied_prep_store": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_vp, _c_vp, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64,
                                      _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
-    "nvx_residual_norm": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_f32, _c_i32, _c_vp, _c_i64,
+    "nvx_residual_norm": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp, _c_i32, _c_vp, _c_vp, _c_vp, _c_f32, _c_i32, _c_vp, _c_i64,
                                    _c_i64, _c_vp]),
-    "nvx_embed_sum": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_i64, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp,
+    "nvx_embed_sum": (_c_i32, [_c_vp, _c_vp, _c_i32, _c_i64, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp,
                                _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_f32, _c_i32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
     "nvx_moe_route_sigmoid": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_f32, _c_vp, _c_vp, _c_vp]),
     "nvx_gelu_glu": (_c_i32, [_c_vp, _c_i32, _c_vp, _c_i64, _c_i64, _c_vp]),
+    "nvx_turn_table": (_c_i32, [_c_vp, _c_vp, _c_i64, _c_vp, _c_i64, _c_vp]),
+    "nvx_conv_attn_prep": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i64, _c_vp, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64,
+                                    _c_i32, _c_i32, _c_f32, _c_vp, _c_vp, _c_vp, _c_vp, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_i64, _c_vp]),
+    "nvx_decay_step_max_vdim": (_c_i64, []),
+    "nvx_decay_step": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_i64, _c_i64, _c_i64, _c_i32, _c_vp, _c_vp, _c_i64, _c_vp, _c_vp, _c_i64, _c_i64,
+                                _c_i64, _c_i64, _c_vp, _c_i64, _c_i64, _c_i32, _c_f32, _c_f32, _c_i64, _c_i32, _c_f32, _c_vp, _c_i64, _c_vp]),
     "nvx_skinny_proj": (_c_i32, [_c_vp, _c_i64, _c_i32, _c_vp, _c_i32, _c_vp, _c_i32, _c_f32, _c_vp, _c_i64, _c_i64, _c_i64, _c_vp]),
 }
 

@@ -10,7 +10,7 @@
 //   - nvx_softcap_attn: the attention itself; scores, maxima, exponentials and sums are float32 in every format.  Optional: a
 //     sliding window or chunks of positions (a token sees its own chunk only), a logarithmic or a linear distance penalty per head, keys
 //     that are cached as projected and normed as they are scored (tied keys and values: one row per token serves as both), a sink (one more term in the softmax's sum, with a score of its
-//     own and no value), the read-out turned back by the query's position (the counterpart of rotated values) and multiplied by
+//     own -- one number, or one per head -- and no value), the first tokens of a sequence kept visible behind the window, the read-out turned back by the query's position (the counterpart of rotated values) and multiplied by
 //     a sigmoid gate (one per element, or one per head).
 #include "fmt_dev.h"
 
@@ -58,15 +58,6 @@ __global__ __launch_bounds__(256) void rope_vnorm_store_kernel(const A* __restri
     }
 }
 
-
-// cos and sin of an angle given in double precision (position * frequency, exact to the table's accuracy at any position): the
-// angle is brought into [-pi, pi] in double precision, where its float32 value is off by at most 2e-7, and the float32 functions
-// take it from there.
-__device__ __forceinline__ void turn_of(double a, float& c, float& s) {
-    const double two_pi = 6.283185307179586476925286766559;
-    const float r = (float)(a - two_pi * rint(a / two_pi));
-    sincosf(r, &s, &c);
-}
 
 // One workgroup per token.  q, k and v are heads * dim, kv_heads * dim and kv_heads * vdim elements of row t of x, at q_off, k_off
 // and v_off (kv_heads == 0: a layer that borrows another layer's keys and values prepares its queries only).
@@ -191,16 +182,6 @@ __global__ __launch_bounds__(256) void tied_prep_store_kernel(const A* __restric
     }
 }
 
-template <int LPR> __device__ __forceinline__ float group_sum(float v) {      // over LPR neighbouring lanes, in the vector ALU
-    v += dpp_move<0xB1>(v);                        // lane ^ 1
-    v += dpp_move<0x4E>(v);                        // lane ^ 2
-    v += dpp_move<0x141>(v);                       // the other quad of eight
-    if (LPR >= 16) v += dpp_move<0x140>(v);        // the other eight of sixteen
-    if (LPR >= 32) v += xor16(v);
-    if (LPR >= 64) v += xor32(v);
-    return v;
-}
-
 // The same with a head per LPR neighbouring lanes of eight elements each (16-byte loads and stores in 16-bit formats; dim a multiple of
 // eight up to 8 * LPR, rows on such borders): 64 / LPR heads a wave.
 template <typename A, int LPR>
@@ -276,6 +257,8 @@ __device__ __forceinline__ float lane_value(float v, int lane) {      // `lane` 
 // One workgroup of four waves per (head, token).  The waves take the visible keys in tiles of 64, every fourth tile each: a
 // lane scores one key (the query waits in LDS), the wave keeps a running maximum and sum, then each lane accumulates the
 // weighted values of EPL of the head's value columns over the tile's keys.  The four partial results are merged through LDS.
+// With `keep` > 0 the first keys of the sequence stay visible when the window has moved past them: the walk goes over those keys and
+// then over the window's, as one list.
 template <typename A, int EPL, bool VEC>
 __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__ q, const A* __restrict__ k_cache, const A* __restrict__ v_cache,
                                                           const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
@@ -286,7 +269,8 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
                                                           const float* __restrict__ r2, const float* __restrict__ slopes,
                                                           const float* __restrict__ k_rn, const float* __restrict__ vcs, int v_inter,
                                                           const A* __restrict__ gate, int64_t gate_stride, int gate_one, int sink,
-                                                          float sink_score) {
+                                                          float sink_score, const float* __restrict__ sinks, int keep, float out_mul,
+                                                          int64_t out_stride) {
     extern __shared__ float sm[];
     float* sq = sm;                   // dim
     float* sacc = sq + dim;           // 4 * vdim
@@ -298,7 +282,9 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
     const int64_t q_n = qo_indptr ? qo_indptr[b + 1] - q0 : 1;
     const int visible = kv_len[b] - (int)(q_n - 1 - (t - q0));
     const int first = first_seen(visible - 1, window, chunk);
+    const int kept = keep < first ? keep : first, n_keys = kept + visible - first;      // the walk: keys 0 .. kept - 1, then first .. visible - 1
     const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f, slope = slopes ? slopes[hd] : 0.f;
+    if (sinks) sink_score = sinks[hd];
     const int kvh = hd / (heads / kv_heads);
     const int32_t* slots = kv_indices + kv_start[b];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -313,9 +299,9 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
     // value rows by 16-byte loads: vdim = 8 * (a power of two up to 64), rows 16-byte aligned (the caller checks the base)
     const bool vec_values = VEC && (vdim & 7) == 0 && ((vdim >> 3) & ((vdim >> 3) - 1)) == 0 && (vdim >> 3) <= 64 && vec_v_ok;
     // with n_split > 1 (steps of few tokens) the key tiles are dealt out over n_split workgroups as well as over the four waves
-    for (int j0 = first + (blockIdx.z * 4 + wave) * 64; j0 < visible; j0 += 256 * n_split) {
-        const int j = j0 + lane;
-        const bool valid = j < visible;
+    for (int i0 = (blockIdx.z * 4 + wave) * 64; i0 < n_keys; i0 += 256 * n_split) {
+        const bool valid = i0 + lane < n_keys;
+        const int j = i0 + lane < kept ? i0 + lane : first + (i0 + lane - kept);
         const int slot = valid ? slots[j] : 0;
         float s = -INFINITY;
         if (valid) {
@@ -344,7 +330,7 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
         m = m_new;
 #pragma unroll
         for (int c = 0; c < EPL; ++c) acc[c] *= corr;
-        const int n_here = visible - j0 < 64 ? visible - j0 : 64;
+        const int n_here = n_keys - i0 < 64 ? n_keys - i0 : 64;
         if constexpr (VEC) {
             // a value row is vdim / 8 lanes of eight elements (16-byte loads), so 64 / (vdim / 8) keys are taken at a time
             if (vec_values) {
@@ -408,15 +394,15 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
 #pragma unroll
         for (int w = 0; w < 4; ++w) o += sacc[w * vdim + e] * f[w];
         if (pr) pr[2 + e] = o;
-        else if (vcs || gate) sacc[e] = o / total;            // (this thread alone reads column e of the four partial sums)
-        else st_f(out, t * (int64_t)heads * vdim + (int64_t)hd * vdim + e, o / total);
+        else if (vcs || gate) sacc[e] = o / total * out_mul;  // (this thread alone reads column e of the four partial sums)
+        else st_f(out, t * out_stride + (int64_t)hd * vdim + e, o / total * out_mul);
     }
     if (pr && threadIdx.x == 0) { pr[0] = mm; pr[1] = total; }
     if (!pr && (vcs || gate)) {
         __syncthreads();
         attn_readout_end<A>(sacc, vdim, vcs ? vcs + t * (int64_t)vdim : nullptr, v_inter,
                             gate ? gate + t * gate_stride + (gate_one ? (int64_t)hd : (int64_t)hd * vdim) : nullptr, gate_one != 0,
-                            out + t * (int64_t)heads * vdim + (int64_t)hd * vdim, 256);
+                            out + t * out_stride + (int64_t)hd * vdim, 256);
     }
 }
 
@@ -559,6 +545,9 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
 //       order; the tile is written transposed by the whole workgroup, once for its four waves.
 // At the end a lane holds, for its query, value columns 16 * tile + 4 * quarter + r: both partners of a pair that is turned back
 // (halves: tiles vt and vt + VT / 2; side by side: r and r + 1) are in the lane, so the read-out's end needs no exchange.
+// PAD: key and value sizes that are multiples of eight below the tile's 32 * DS and 16 * VT; what is missing of a key counts as zeros, and
+// products of tiles that lie wholly outside are left out.
+// With `keep` > 0 the tiles of the sequence's first keys come before those of the window.
 typedef __attribute__((ext_vector_type(8))) __bf16 ca_bf16x8;
 typedef __attribute__((ext_vector_type(8))) _Float16 ca_f16x8;
 template <typename A> __device__ __forceinline__ nvx_f32x4 ca_mfma32(nvx_u32x4 a, nvx_u32x4 b, nvx_f32x4 c) {
@@ -578,7 +567,7 @@ constexpr int TILE_Q = 64;       // query tokens per workgroup
 constexpr int TILE_K = 32;       // keys per step
 constexpr int VT_ROW = 40;       // elements per row of the V^T tile in LDS: 32 keys and a pad that spreads the rows over the banks
 
-template <typename A, int DS, int VT>
+template <typename A, int DS, int VT, bool PAD>
 __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restrict__ q, const A* __restrict__ k_cache, const A* __restrict__ v_cache,
                                                                const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
                                                                const int32_t* __restrict__ kv_len, const int32_t* __restrict__ qo_indptr, int n_seq,
@@ -586,9 +575,11 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
                                                                int chunk, const float* __restrict__ r1, const float* __restrict__ r2,
                                                                const float* __restrict__ slopes, const float* __restrict__ k_rn,
                                                                const float* __restrict__ vcs, int v_inter, const A* __restrict__ gate,
-                                                               int64_t gate_stride, int gate_one, int sink, float sink_score) {
-    constexpr int dim = DS * 32, vdim = VT * 16;
-    __shared__ A vt_lds[vdim * VT_ROW];
+                                                               int64_t gate_stride, int gate_one, int sink, float sink_score,
+                                                               const float* __restrict__ sinks, int keep, float out_mul, int64_t out_stride,
+                                                               int dim_rt, int vdim_rt) {
+    const int dim = PAD ? dim_rt : DS * 32, vdim = PAD ? vdim_rt : VT * 16;
+    __shared__ A vt_lds[VT * 16 * VT_ROW];
     __shared__ __align__(16) float rn_lds[TILE_K];
     __shared__ int where[2];
     if (threadIdx.x == 0) {          // which sequence and which block of its tokens: sequences take ceil(tokens / 64) workgroups each
@@ -626,8 +617,12 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     {
         const A* qr = q + ((int64_t)q0 + qs + (row_on ? row : rows_here - 1)) * heads * dim + (int64_t)hd * dim + 8 * g;
 #pragma unroll
-        for (int s = 0; s < DS; ++s) qb[s] = *reinterpret_cast<const nvx_u32x4*>(qr + 32 * s);
+        for (int s = 0; s < DS; ++s) {
+            if (!PAD || 8 * g + 32 * s < dim) qb[s] = *reinterpret_cast<const nvx_u32x4*>(qr + 32 * s);
+            else qb[s] = nvx_u32x4{0u, 0u, 0u, 0u};
+        }
     }
+    if (sinks) sink_score = sinks[hd];
     const float pen_a = r1 ? r1[hd] : 0.f, pen_b = r1 ? r2[hd] : 0.f, slope2 = slopes ? slopes[hd] * 1.4426950408889634f : 0.f;
     nvx_f32x4 acc[VT];
 #pragma unroll
@@ -636,8 +631,8 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     // Rows hang on slot ids, which hang on the slot list: two memory round trips in a row.  The ids are read two tiles ahead and the
     // rows one tile ahead (keys into the registers the products read, values into registers that the next step writes to LDS),
     // so that neither wait stands in front of a tile's products.
-    constexpr int VCH = TILE_K * (vdim / 8);                         // 16-byte pieces of a tile of values
-    constexpr int VPT = (VCH + 255) / 256;                           // ... per thread
+    const int VCH = TILE_K * (vdim / 8);                             // 16-byte pieces of a tile of values
+    constexpr int VPT = (TILE_K * VT * 2 + 255) / 256;               // ... per thread
     typedef A vec8 __attribute__((ext_vector_type(8)));
     nvx_u32x4 kf[2][DS];
     vec8 vf[VPT];
@@ -654,7 +649,10 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
         for (int hh = 0; hh < 2; ++hh) {
             const A* kr = k_cache + (int64_t)k_slot[hh] * k_row + (int64_t)kvh * dim + 8 * g;
 #pragma unroll
-            for (int s = 0; s < DS; ++s) kf[hh][s] = *reinterpret_cast<const nvx_u32x4*>(kr + 32 * s);
+            for (int s = 0; s < DS; ++s) {
+                if (!PAD || 8 * g + 32 * s < dim) kf[hh][s] = *reinterpret_cast<const nvx_u32x4*>(kr + 32 * s);
+                else kf[hh][s] = nvx_u32x4{0u, 0u, 0u, 0u};
+            }
         }
     };
     auto fetch_value_rows = [&]() {
@@ -671,14 +669,18 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
     constexpr float LOG2E = 1.4426950408889634f;
     const float k_lin = cap > 0.f ? 2.0f * scale * LOG2E / cap : scale * LOG2E, k_cap = cap * LOG2E;
     const int j_begin = lo & ~(TILE_K - 1);
-    fetch_slots(j_begin);
+    // tiles of kept keys that lie in front of the window's first tile, then the window's
+    const int kept_tiles = ((keep < j_begin ? keep : j_begin) + TILE_K - 1) / TILE_K, n_tiles = kept_tiles + (hi - j_begin + TILE_K - 1) / TILE_K;
+    auto tile_at = [&](int i) { return i < kept_tiles ? i * TILE_K : j_begin + (i - kept_tiles) * TILE_K; };
+    fetch_slots(tile_at(0));
     if (wave_on) fetch_key_rows();
     fetch_value_rows();
-    if (j_begin + TILE_K < hi) fetch_slots(j_begin + TILE_K);
+    if (1 < n_tiles) fetch_slots(tile_at(1));
     const int q_lo = pos_first + wave * 16;                          // positions of this wave's first and last query
     const int q_hi = q_lo + 15;
     const bool rows_full = wave * 16 + 16 <= rows_here;
-    for (int j0 = j_begin; j0 < hi; j0 += TILE_K) {
+    for (int it = 0; it < n_tiles; ++it) {
+        const int j0 = tile_at(it);
         __syncthreads();                                             // the tile before has been read by all waves
         if (k_rn && threadIdx.x < TILE_K) rn_lds[threadIdx.x] = rn_next;
 #pragma unroll
@@ -693,26 +695,27 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
         __syncthreads();
         // issued behind the barrier (which waits for every load before it): the next tile's rows and the ids of the one after
         // travel while this tile's products run; the key rows as soon as this tile's have been multiplied
-        const bool more = j0 + TILE_K < hi;
+        const bool more = it + 1 < n_tiles;
         if (more) fetch_value_rows();                                // (with the ids read one step ago)
         if (!wave_on) {
-            if (j0 + 2 * TILE_K < hi) fetch_slots(j0 + 2 * TILE_K);
+            if (it + 2 < n_tiles) fetch_slots(tile_at(it + 2));
             continue;
         }
-        const bool seen = j0 < w_hi && j0 + TILE_K > w_lo;           // some query of this wave sees some key of the tile
+        const bool seen = j0 < w_hi && (j0 + TILE_K > w_lo || j0 < keep);      // some query of this wave sees some key of the tile
         nvx_f32x4 sacc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
         if (seen) {
 #pragma unroll
             for (int s = 0; s < DS; ++s) {
+                if (PAD && 32 * s >= dim) continue;
                 sacc[0] = ca_mfma32<A>(kf[0][s], qb[s], sacc[0]);
                 sacc[1] = ca_mfma32<A>(kf[1][s], qb[s], sacc[1]);
             }
         }
         if (more) fetch_key_rows();
-        if (j0 + 2 * TILE_K < hi) fetch_slots(j0 + 2 * TILE_K);
+        if (it + 2 < n_tiles) fetch_slots(tile_at(it + 2));
         if (!seen) continue;
         // every query of the wave sees every key of the tile (most tiles): no mask to work out
-        const bool full = rows_full && j0 + TILE_K - 1 <= q_lo && j0 >= first_seen(q_hi, window, chunk);
+        const bool full = rows_full && j0 + TILE_K - 1 <= q_lo && (j0 >= first_seen(q_hi, window, chunk) || j0 + TILE_K <= keep);
         float sv[8], mx = -INFINITY;
 #pragma unroll
         for (int hh = 0; hh < 2; ++hh) {
@@ -724,7 +727,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
                 if (cap > 0.f) sc = k_cap - 2.0f * k_cap * __builtin_amdgcn_rcpf(__builtin_amdgcn_exp2f(sc) + 1.0f);
                 if (r1) sc -= pen_a * __builtin_amdgcn_logf(1.0f + pen_b * (float)(pos - j));
                 if (slopes) sc -= slope2 * (float)(pos - j);
-                if (!full && !(row_on && j <= pos && j >= my_lo)) sc = -INFINITY;
+                if (!full && !(row_on && j <= pos && (j >= my_lo || j < keep))) sc = -INFINITY;
                 sv[hh * 4 + r] = sc;
                 mx = fmaxf(mx, sc);
             }
@@ -752,6 +755,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
         }
 #pragma unroll
         for (int t = 0; t < VT; ++t) {
+            if (PAD && 16 * t >= vdim) continue;
             // row (value column) 16 t + c of V^T, keys 4 g .. 4 g + 3 of both halves: the order of the lane's weights
             const A* vr = vt_lds + (t * 16 + c) * VT_ROW + 4 * g;
             const uint2 a0 = *reinterpret_cast<const uint2*>(vr), a1 = *reinterpret_cast<const uint2*>(vr + 16);
@@ -771,7 +775,7 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
 #pragma unroll
         for (int t = 0; t < VT; ++t) acc[t] *= alpha;
     }
-    const float inv = 1.0f / l_run;
+    const float inv = out_mul / l_run;
 #pragma unroll
     for (int t = 0; t < VT; ++t) acc[t] *= inv;
     const int64_t tok = (int64_t)q0 + qs + row;
@@ -800,11 +804,12 @@ __global__ __launch_bounds__(256) void softcap_attn_tile_kernel(const A* __restr
             }
         }
     }
-    A* orow = out + tok * heads * vdim + (int64_t)hd * vdim + 4 * g;
+    A* orow = out + tok * out_stride + (int64_t)hd * vdim + 4 * g;
     const A* grow = gate && !gate_one ? gate + tok * gate_stride + (int64_t)hd * vdim + 4 * g : nullptr;
     const float g_head = gate && gate_one ? sigmoid_f((float)gate[tok * gate_stride + hd]) : 1.0f;      // one gate for the whole head
 #pragma unroll
     for (int t = 0; t < VT; ++t) {
+        if (PAD && t * 16 + 4 * g >= vdim) continue;
         float o[4] = {acc[t][0] * g_head, acc[t][1] * g_head, acc[t][2] * g_head, acc[t][3] * g_head};
         if (grow) {
             typedef A vec4 __attribute__((ext_vector_type(4)));
@@ -821,9 +826,10 @@ template <typename A>
 __global__ __launch_bounds__(64) void softcap_merge_kernel(const float* __restrict__ part, int n_split, A* __restrict__ out, int vdim,
                                                           int heads, const float* __restrict__ vcs, int v_inter,
                                                           const A* __restrict__ gate, int64_t gate_stride, int gate_one, int sink,
-                                                          float sink_score) {
+                                                          float sink_score, const float* __restrict__ sinks, float out_mul, int64_t out_stride) {
     __shared__ float so[512];
-    const int64_t row = blockIdx.x;
+    const int64_t row = blockIdx.x, t = row / heads, hd = row % heads;
+    if (sinks) sink_score = sinks[hd];
     const float* pr = part + row * n_split * (vdim + 2);
     float mm = sink ? sink_score : -INFINITY;
     for (int s = 0; s < n_split; ++s) mm = fmaxf(mm, pr[s * (vdim + 2)]);
@@ -838,15 +844,14 @@ __global__ __launch_bounds__(64) void softcap_merge_kernel(const float* __restri
             const float m = pr[s * (vdim + 2)];
             if (m != -INFINITY) o += pr[s * (vdim + 2) + 2 + e] * expf(m - mm);
         }
-        if (vcs || gate) so[e] = o / total;
-        else st_f(out, row * vdim + e, o / total);
+        if (vcs || gate) so[e] = o / total * out_mul;
+        else st_f(out, t * out_stride + hd * vdim + e, o / total * out_mul);
     }
     if (vcs || gate) {
-        const int64_t t = row / heads;
         __syncthreads();
         attn_readout_end<A>(so, vdim, vcs ? vcs + t * (int64_t)vdim : nullptr, v_inter,
-                            gate ? gate + t * gate_stride + (gate_one ? row % heads : (row % heads) * vdim) : nullptr, gate_one != 0,
-                            out + row * vdim, 64);
+                            gate ? gate + t * gate_stride + (gate_one ? hd : hd * vdim) : nullptr, gate_one != 0,
+                            out + t * out_stride + hd * vdim, 64);
     }
 }
 
@@ -858,11 +863,14 @@ using namespace NVX_NS;
 template <typename T> struct tile_fmt { typedef T type; };
 template <> struct tile_fmt<float> { typedef __bf16 type; };
 
-// Whether nvx_softcap_attn has a matrix-core form for these sizes: 16-bit formats, key and value sizes of 64, 96 or 128; a read-out
-// that is turned back in the halves layout needs both halves in whole column tiles.
+// Whether nvx_softcap_attn has a matrix-core form for these sizes: 16-bit formats, key and value sizes that are multiples of eight up to
+// 128; a read-out that is turned back in the halves layout needs both halves in whole column tiles (key and value sizes of 64, 96 or 128).
+static bool whole_tiles(int64_t dim, int64_t vdim) {
+    return (dim == 64 || dim == 96 || dim == 128) && (vdim == 64 || vdim == 96 || vdim == 128);
+}
 extern "C" int nvx_softcap_attn_tile_fits(int fmt, int64_t dim, int64_t vdim, int turned_halves) {
-    const bool sizes = (dim == 64 || dim == 96 || dim == 128) && (vdim == 64 || vdim == 96 || vdim == 128);
-    return (fmt == 0 || fmt == 1) && sizes && (!turned_halves || (vdim / 16) % 2 == 0);
+    const bool sizes = dim > 0 && vdim > 0 && dim % 8 == 0 && vdim % 8 == 0 && dim <= 128 && vdim <= 128;
+    return (fmt == 0 || fmt == 1) && sizes && (!turned_halves || whole_tiles(dim, vdim));
 }
 
 extern "C" int nvx_rope_vnorm_store(const void* x, int64_t x_stride, int fmt, const int64_t* positions, const double* freq, float mag,
@@ -943,7 +951,8 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
                                 float scale, float cap, void* out, int64_t n_tok, int64_t heads, int64_t kv_heads, int64_t dim, int64_t vdim,
                                 int n_split, float* part, int64_t window, int64_t chunk, const float* r1, const float* r2, const float* slopes,
                                 const float* k_rn, const float* vcs, int v_interleaved, const void* gate, int64_t gate_stride, int gate_per_head, int sink, float sink_score,
-                                int64_t n_seq, int matrix_cores, nvx_stream_t stream) {
+                                const float* sinks, int64_t keep_first, float out_mul, int64_t out_stride, int64_t n_seq, int matrix_cores,
+                                nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_softcap_attn: fmt must be 0, 1 or 2");
     NVX_REQUIRE(n_tok >= 0 && n_tok <= 65535 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && dim <= 4096 && vdim > 0 && vdim <= 512,
                 NVX_EINVAL, "nvx_softcap_attn: bad sizes (at most 65535 tokens a step, key size <= 4096, value size <= 512)");
@@ -953,28 +962,36 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     NVX_REQUIRE((r1 != nullptr) == (r2 != nullptr), NVX_EINVAL, "nvx_softcap_attn: the distance penalty takes both of its numbers per head");
     NVX_REQUIRE(window >= 0 && window < (1ll << 31) && chunk >= 0 && chunk < (1ll << 31) && (window == 0 || chunk == 0), NVX_EINVAL,
                 "nvx_softcap_attn: bad window or chunk (one of them at most)");
+    NVX_REQUIRE(keep_first >= 0 && keep_first < (1ll << 31) && out_stride >= heads * vdim, NVX_EINVAL, "nvx_softcap_attn: kept tokens or row stride of the output");
+    if (window == 0) keep_first = 0;      // (everything is kept)
+    sink = sink || sinks;
     NVX_REQUIRE(!vcs || (vdim % 2 == 0 && nvx_aligned16(vcs)), NVX_EINVAL, "nvx_softcap_attn: a read-out that is turned back has an even size");
     NVX_REQUIRE(!gate || gate_stride >= (gate_per_head ? heads : heads * vdim), NVX_EINVAL, "nvx_softcap_attn: row stride of the gate");
     // steps of many tokens in a 16-bit format, sizes the tile kernel is built for, 8-byte rows of the gate: the matrix cores
     if (matrix_cores && nvx_softcap_attn_tile_fits(fmt, dim, vdim, vcs != nullptr && !v_interleaved) && qo_indptr && n_split == 1 && n_seq > 0 &&
-        nvx_aligned16(q) && nvx_aligned16(k_cache) && nvx_aligned16(v_cache) && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 &&
+        nvx_aligned16(q) && nvx_aligned16(k_cache) && nvx_aligned16(v_cache) && (reinterpret_cast<uintptr_t>(out) & 7u) == 0 && out_stride % 4 == 0 &&
         (!gate || gate_per_head || ((reinterpret_cast<uintptr_t>(gate) & 7u) == 0 && gate_stride % 4 == 0))) {
         NVX_REQUIRE((n_tok + TILE_Q - 1) / TILE_Q + n_seq <= 65535, NVX_EINVAL, "nvx_softcap_attn: too many tokens or sequences in one step");
         const dim3 tgrid((unsigned)heads, (unsigned)((n_tok + TILE_Q - 1) / TILE_Q + n_seq));
-#define NVX_TILE_ATTN(DS, VT)                                                                                                            \
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((softcap_attn_tile_kernel<typename tile_fmt<A_>::type, DS, VT>), tgrid, dim3(256), 0, (hipStream_t)stream, \
+#define NVX_TILE_ATTN(DS, VT, PAD)                                                                                                            \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((softcap_attn_tile_kernel<typename tile_fmt<A_>::type, DS, VT, PAD>), tgrid, dim3(256), 0, (hipStream_t)stream, \
                                          (const typename tile_fmt<A_>::type*)q, (const typename tile_fmt<A_>::type*)k_cache,            \
                                          (const typename tile_fmt<A_>::type*)v_cache, kv_indices, kv_start, kv_len, qo_indptr, (int)n_seq, scale, \
                                          cap, (typename tile_fmt<A_>::type*)out, (int)heads, (int)kv_heads, (int)window, (int)chunk, r1, r2, slopes, k_rn, vcs, \
                                          v_interleaved, (const typename tile_fmt<A_>::type*)gate, gate_stride, gate_per_head, sink,   \
-                                         sink_score))
+                                         sink_score, sinks, (int)keep_first, out_mul, out_stride, (int)dim, (int)vdim))
 #define NVX_TILE_ATTN_V(DS)                                                       \
     do {                                                                          \
-        if (vdim == 64) NVX_TILE_ATTN(DS, 4);                                     \
-        else if (vdim == 96) NVX_TILE_ATTN(DS, 6);                                \
-        else NVX_TILE_ATTN(DS, 8);                                                \
+        if (vdim == 64) NVX_TILE_ATTN(DS, 4, false);                              \
+        else if (vdim == 96) NVX_TILE_ATTN(DS, 6, false);                         \
+        else NVX_TILE_ATTN(DS, 8, false);                                         \
     } while (0)
-        if (dim == 64) NVX_TILE_ATTN_V(2);
+        if (!whole_tiles(dim, vdim)) {
+            if (dim <= 64 && vdim <= 64) NVX_TILE_ATTN(2, 4, true);
+            else if (dim <= 64) NVX_TILE_ATTN(2, 8, true);
+            else if (vdim <= 64) NVX_TILE_ATTN(4, 4, true);
+            else NVX_TILE_ATTN(4, 8, true);
+        } else if (dim == 64) NVX_TILE_ATTN_V(2);
         else if (dim == 96) NVX_TILE_ATTN_V(3);
         else NVX_TILE_ATTN_V(4);
 #undef NVX_TILE_ATTN_V
@@ -984,7 +1001,8 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     const size_t lds = (size_t)(dim + 4 * vdim + 8) * sizeof(float);
     NVX_REQUIRE(n_split >= 1 && n_split <= 64 && (n_split == 1 || part), NVX_EINVAL, "nvx_softcap_attn: a key split needs its workspace");
     // tied rows without what that kernel does not do: a row is read once
-    if (k_rn && k_cache == v_cache && dim == vdim && dim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && !sink && nvx_aligned16(k_cache)) {
+    if (k_rn && k_cache == v_cache && dim == vdim && dim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && !sink && keep_first == 0 &&
+        out_mul == 1.0f && out_stride == heads * vdim && nvx_aligned16(k_cache)) {
         const int per_kv = (int)(heads / kv_heads), nh = per_kv >= 4 ? 4 : (per_kv >= 2 ? 2 : 1);
         const dim3 tgrid((unsigned)(kv_heads * ((per_kv + nh - 1) / nh)), (unsigned)n_tok, (unsigned)n_split);
         const size_t tlds = (size_t)(4 * nh * dim + 8 * nh) * sizeof(float);
@@ -1007,7 +1025,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
         if (n_split > 1)
             NVX_FMT_CALL(fmt, hipLaunchKernelGGL(softcap_merge_kernel<A_>, dim3((unsigned)(n_tok * heads)), dim3(64), 0, (hipStream_t)stream,
                                                  (const float*)part, n_split, (A_*)out, (int)vdim, (int)heads, vcs, v_interleaved, (const A_*)gate,
-                                                 gate_stride, gate_per_head, sink, sink_score));
+                                                 gate_stride, gate_per_head, sink, sink_score, sinks, out_mul, out_stride));
         return nvx_check_launch("nvx_softcap_attn");
     }
     const dim3 grid((unsigned)heads, (unsigned)n_tok, (unsigned)n_split);
@@ -1016,7 +1034,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
                                          (const A_*)q, (const A_*)k_cache, (const A_*)v_cache, kv_indices, kv_start, kv_len, qo_indptr,      \
                                          tok_seq, scale, cap, (A_*)out, (int)heads, (int)kv_heads, (int)dim, (int)vdim,       \
                                          (int)nvx_aligned16(v_cache), n_split, part, (int)window, (int)chunk, r1, r2, slopes, k_rn, vcs, v_interleaved, \
-                                         (const A_*)gate, gate_stride, gate_per_head, sink, sink_score))
+                                         (const A_*)gate, gate_stride, gate_per_head, sink, sink_score, sinks, (int)keep_first, out_mul, out_stride))
 #define NVX_CAP_ATTN(EPL) do { if (vec) NVX_CAP_ATTN_V(EPL, true); else NVX_CAP_ATTN_V(EPL, false); } while (0)
     const bool vec = fmt != 2 && dim % 8 == 0 && nvx_aligned16(k_cache);
     if (vdim <= 64) NVX_CAP_ATTN(1);
@@ -1027,7 +1045,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     if (n_split > 1)
         NVX_FMT_CALL(fmt, hipLaunchKernelGGL(softcap_merge_kernel<A_>, dim3((unsigned)(n_tok * heads)), dim3(64), 0, (hipStream_t)stream,
                                              (const float*)part, n_split, (A_*)out, (int)vdim, (int)heads, vcs, v_interleaved, (const A_*)gate,
-                                             gate_stride, gate_per_head, sink, sink_score));
+                                             gate_stride, gate_per_head, sink, sink_score, sinks, out_mul, out_stride));
 #undef NVX_CAP_ATTN
     return nvx_check_launch("nvx_softcap_attn");
 }

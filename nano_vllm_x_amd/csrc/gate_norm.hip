@@ -178,10 +178,11 @@ __global__ __launch_bounds__(256) void tanh_cap_kernel(const A* __restrict__ in,
 }
 
 // The end of a row that waits in LDS (su, float32, written by this workgroup; a barrier lies in block256_sum, or is placed here):
-// nothing (h null), h = su / rms * w, or (split) h = [hi | lo], two rows of the activations' format whose sum is su to 16 bits and more.
+// nothing (h null), h = su / rms * w, with `b` the layer norm h = (su - mean) / sqrt(variance + eps) * w + b (variance: the mean of the
+// squared deviations), or (split) h = [hi | lo], two rows of the activations' format whose sum is su to 16 bits and more.
 template <typename A>
-__device__ __forceinline__ void row_end(const float* su, float ss, float* red, const float* __restrict__ w, float eps, int split, A* __restrict__ h,
-                                        int64_t t, int width) {
+__device__ __forceinline__ void row_end(const float* su, float ss, float* red, const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                        int split, A* __restrict__ h, int64_t t, int width) {
     if (!h) return;
     if (split) {                                  // (every thread reads back the entries it wrote)
         A* hr = h + t * 2 * (int64_t)width;
@@ -195,18 +196,38 @@ __device__ __forceinline__ void row_end(const float* su, float ss, float* red, c
         }
         return;
     }
+    float mean = 0.f;
+    if (b) {                                      // (a thread reads entries that the whole workgroup can see, or that it wrote itself)
+        auto over_row = [&](auto f) {
+            for (int c = threadIdx.x * 4; c < width; c += 1024) {
+                if ((width & 3) == 0) {
+                    const nvx_f32x4 v = *reinterpret_cast<const nvx_f32x4*>(su + c);
+                    f(v[0]); f(v[1]); f(v[2]); f(v[3]);
+                } else {
+                    for (int i = c; i < c + 4 && i < width; ++i) f(su[i]);
+                }
+            }
+        };
+        float s1 = 0.f;
+        over_row([&](float v) { s1 += v; });
+        mean = block256_sum(s1, red) / (float)width;
+        ss = 0.f;
+        over_row([&](float v) { const float d = v - mean; ss += d * d; });
+    }
     const float rn = 1.0f / sqrtf(block256_sum(ss, red) / (float)width + eps);
     A* hr = h + t * (int64_t)width;
     for (int c = threadIdx.x * 4; c < width; c += 1024) {
         if (c + 4 <= width && (width & 3) == 0) {
             typedef A vec4 __attribute__((ext_vector_type(4)));
             const nvx_f32x4 v = *reinterpret_cast<const nvx_f32x4*>(su + c), g = *reinterpret_cast<const nvx_f32x4*>(w + c);
+            nvx_f32x4 add = {0.f, 0.f, 0.f, 0.f};
+            if (b) add = *reinterpret_cast<const nvx_f32x4*>(b + c);
             vec4 o;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) o[i] = (A)(v[i] * rn * g[i]);
+            for (int i = 0; i < 4; ++i) o[i] = (A)((v[i] - mean) * rn * g[i] + add[i]);
             *reinterpret_cast<vec4*>(hr + c) = o;
         } else {
-            for (int i = c; i < c + 4 && i < width; ++i) st_f(hr, i, su[i] * rn * w[i]);
+            for (int i = c; i < c + 4 && i < width; ++i) st_f(hr, i, (su[i] - mean) * rn * w[i] + (b ? b[i] : 0.f));
         }
     }
 }
@@ -216,8 +237,8 @@ __device__ __forceinline__ void row_end(const float* su, float ss, float* red, c
 template <typename A, int V>
 __global__ __launch_bounds__(256) void residual_norm_kernel(const float* x_in, const A* __restrict__ y, int64_t y_stride, const A* __restrict__ y2,
                                                            int64_t y2_stride, const float* __restrict__ add, const float* __restrict__ bias,
-                                                           float* x_out, const float* __restrict__ w, float eps, int split, A* __restrict__ h,
-                                                           int width) {
+                                                           float* x_out, const float* __restrict__ w, const float* __restrict__ b, float eps,
+                                                           int split, A* __restrict__ h, int width) {
     extern __shared__ __align__(16) float row_lds[];      // width
     float* su = row_lds;
     __shared__ float red[4];
@@ -237,7 +258,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const float* x_in, c
         for (int i = 0; i < V; ++i) ss += v[i] * v[i];
     }
     if (V == 1) __syncthreads();                  // (row_end takes four entries a thread)
-    row_end<A>(su, ss, red, w, eps, split, h, t, width);
+    row_end<A>(su, ss, red, w, b, eps, split, h, t, width);
 }
 
 // Per token t (one workgroup):  x[t] = table[ids[t]] (+ pair[r]) (+ pos_table[position]);  then row_end of it.
@@ -252,7 +273,7 @@ __global__ __launch_bounds__(256) void embed_sum_kernel(const int64_t* __restric
                                                        const int64_t* __restrict__ positions, const int32_t* __restrict__ tok_seq,
                                                        const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
                                                        const int32_t* __restrict__ state_slot, float* __restrict__ x, const float* __restrict__ w,
-                                                       float eps, int split, A* __restrict__ h, int width) {
+                                                       const float* __restrict__ b, float eps, int split, A* __restrict__ h, int width) {
     extern __shared__ __align__(16) float row_lds[];      // width
     float* su = row_lds;
     __shared__ float red[4];
@@ -294,15 +315,16 @@ __global__ __launch_bounds__(256) void embed_sum_kernel(const int64_t* __restric
         ss += v * v;
     }
     __syncthreads();
-    row_end<A>(su, ss, red, w, eps, split, h, t, width);
+    row_end<A>(su, ss, red, w, b, eps, split, h, t, width);
 }
 
-// One wave per (token, head): out = o / rms(o) * w * gate, with gate = 1 (kind 0), sigmoid(z) (1) or z * sigmoid(z) (2) of
-// the gate pre-activations z (same layout as the output).  w has heads * vdim entries, or vdim shared by the heads.
+// One wave per (token, head): out = mul * o / rms(o) * w * gate, with gate = 1 (kind 0), sigmoid(z) (1) or z * sigmoid(z) (2) of
+// the gate pre-activations z (rows of heads * vdim).  w has heads * vdim entries, or vdim shared by the heads, or is null (ones).
 template <typename A>
 __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, int w_shared,
                                                             const A* __restrict__ gate, int64_t gate_stride, int kind, float eps,
-                                                            A* __restrict__ out, int64_t n_rows, int heads, int vdim) {
+                                                            float mul, A* __restrict__ out, int64_t out_stride, int64_t n_rows, int heads,
+                                                            int vdim) {
     const int64_t idx = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
     if (idx >= n_rows) return;
     const int lane = threadIdx.x & 63;
@@ -311,14 +333,15 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
     const int64_t base = t * (int64_t)heads * vdim + (int64_t)hd * vdim;
     float ss = 0.f;
     for (int e = lane; e < vdim; e += 64) { const float v = o[base + e]; ss += v * v; }
-    const float rn = 1.0f / sqrtf(wave_sum(ss) / (float)vdim + eps);
+    const float rn = mul / sqrtf(wave_sum(ss) / (float)vdim + eps);
     for (int e = lane; e < vdim; e += 64) {
-        float v = o[base + e] * rn * w[w_shared ? e : hd * vdim + e];
+        float v = o[base + e] * rn;
+        if (w) v *= w[w_shared ? e : hd * vdim + e];
         if (kind) {
             const float z = ld_f(gate, t * gate_stride + (int64_t)hd * vdim + e);
             v *= kind == 1 ? sigmoid_f(z) : z * sigmoid_f(z);
         }
-        st_f(out, base + e, v);
+        st_f(out, t * out_stride + (int64_t)hd * vdim + e, v);
     }
 }
 
@@ -498,15 +521,17 @@ extern "C" int nvx_gated_residual_norm(const void* y, int64_t y_stride, const vo
 }
 
 extern "C" int nvx_head_norm_gate(const float* o, const float* w, int w_shared, const void* gate, int64_t gate_stride, int kind, int fmt,
-                                  float eps, void* out, int64_t n_tok, int64_t heads, int64_t vdim, nvx_stream_t stream) {
+                                  float eps, float mul, void* out, int64_t out_stride, int64_t n_tok, int64_t heads, int64_t vdim,
+                                  nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2 && kind >= 0 && kind <= 2, NVX_EINVAL, "nvx_head_norm_gate: fmt must be 0..2, kind 0..2");
     NVX_REQUIRE(n_tok >= 0 && heads > 0 && vdim > 0 && heads * vdim < (1 << 30), NVX_EINVAL, "nvx_head_norm_gate: bad sizes");
     if (n_tok == 0) return NVX_OK;
-    NVX_REQUIRE(o && w && out && (kind == 0 || (gate && gate_stride >= heads * vdim)), NVX_EINVAL, "nvx_head_norm_gate: null pointer");
+    NVX_REQUIRE(o && out && out_stride >= heads * vdim && (kind == 0 || (gate && gate_stride >= heads * vdim)), NVX_EINVAL,
+                "nvx_head_norm_gate: null pointer or row stride");
     const int64_t rows = n_tok * heads;
     NVX_REQUIRE((rows + 3) / 4 < (1ll << 31), NVX_EINVAL, "nvx_head_norm_gate: too many rows");
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL(head_norm_gate_kernel<A_>, dim3((unsigned)((rows + 3) / 4)), dim3(256), 0, (hipStream_t)stream, o, w,
-                                         w_shared, (const A_*)gate, gate_stride, kind, eps, (A_*)out, rows, (int)heads, (int)vdim));
+                                         w_shared, (const A_*)gate, gate_stride, kind, eps, mul, (A_*)out, out_stride, rows, (int)heads, (int)vdim));
     return nvx_check_launch("nvx_head_norm_gate");
 }
 
@@ -567,22 +592,23 @@ extern "C" int nvx_embed_scale(const int64_t* ids, const void* table, int fmt, i
     NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, name ": fmt must be 0, 1 or 2");                                                     \
     NVX_REQUIRE(n_tok >= 0 && n_tok < (1ll << 31) && width > 0, NVX_EINVAL, name ": bad sizes");                                       \
     NVX_REQUIRE(width <= 15360, NVX_EUNSUPPORTED, name ": a row must fit LDS as float32 (width <= 15360)");                            \
-    NVX_REQUIRE(!h || split || w, NVX_EINVAL, name ": the norm needs its weight")
+    NVX_REQUIRE(!h || split || w, NVX_EINVAL, name ": the norm needs its weight");                                                     \
+    NVX_REQUIRE(!w_bias || (w && !split), NVX_EINVAL, name ": the layer norm's bias goes with its weight")
 
 extern "C" int nvx_residual_norm(const float* x_in, const void* y, int64_t y_stride, const void* y2, int64_t y2_stride, const float* add,
-                                 const float* bias, int fmt, float* x_out, const float* w, float eps, int split, void* h, int64_t n_tok,
-                                 int64_t width, nvx_stream_t stream) {
+                                 const float* bias, int fmt, float* x_out, const float* w, const float* w_bias, float eps, int split, void* h,
+                                 int64_t n_tok, int64_t width, nvx_stream_t stream) {
     NVX_ROW_OK("nvx_residual_norm");
     if (n_tok == 0) return NVX_OK;
     NVX_REQUIRE(x_in && x_out && (!y || y_stride >= width) && (!y2 || y2_stride >= width), NVX_EINVAL, "nvx_residual_norm: null pointer or row stride");
     const size_t lds = (size_t)width * sizeof(float);
     const auto ok4 = [&](const void* p, size_t item) { return (reinterpret_cast<uintptr_t>(p) & (4 * item - 1)) == 0; };
     const size_t item = fmt == 2 ? 4 : 2;
-    const bool v4 = width % 4 == 0 && ok4(x_in, 4) && ok4(x_out, 4) && ok4(add, 4) && ok4(bias, 4) && ok4(w, 4) && ok4(y, item) && ok4(y2, item) &&
+    const bool v4 = width % 4 == 0 && ok4(x_in, 4) && ok4(x_out, 4) && ok4(add, 4) && ok4(bias, 4) && ok4(w, 4) && ok4(w_bias, 4) && ok4(y, item) && ok4(y2, item) &&
                     ok4(h, item) && (!y || y_stride % 4 == 0) && (!y2 || y2_stride % 4 == 0);
 #define NVX_RESIDUAL_NORM(V)                                                                                                           \
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((residual_norm_kernel<A_, V>), dim3((unsigned)n_tok), dim3(256), lds, (hipStream_t)stream, x_in, (const A_*)y, \
-                                         y_stride, (const A_*)y2, y2_stride, add, bias, x_out, w, eps, split, (A_*)h, (int)width))
+                                         y_stride, (const A_*)y2, y2_stride, add, bias, x_out, w, w_bias, eps, split, (A_*)h, (int)width))
     if (v4) NVX_RESIDUAL_NORM(4);
     else {
         NVX_REQUIRE(width % 4 != 0, NVX_EINVAL, "nvx_residual_norm: rows of a width that is a multiple of four must start on such borders");
@@ -595,17 +621,19 @@ extern "C" int nvx_residual_norm(const float* x_in, const void* y, int64_t y_str
 extern "C" int nvx_embed_sum(const int64_t* ids, const void* table, int fmt, int64_t vocab, const void* pair, int64_t buckets, int64_t mul_prev,
                              int64_t mul_cur, float* prev_id, int64_t n_slots, const void* pos_table, int64_t n_pos, const int64_t* positions,
                              const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0, const int32_t* state_slot, float* x,
-                             const float* w, float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width, nvx_stream_t stream) {
+                             const float* w, const float* w_bias, float eps, int split, void* h, int64_t n_tok, int64_t n_seq, int64_t width,
+                             nvx_stream_t stream) {
     NVX_ROW_OK("nvx_embed_sum");
     if (n_tok == 0) return NVX_OK;
     NVX_REQUIRE(ids && table && vocab > 0 && vocab < (1ll << 31) && x, NVX_EINVAL, "nvx_embed_sum: bad table");
     NVX_REQUIRE(!pair || (buckets > 0 && prev_id && n_slots > 0 && pos0 && state_slot && (tok_seq != nullptr) == (qo_indptr != nullptr) &&
                           (qo_indptr || n_tok == n_seq)), NVX_EINVAL, "nvx_embed_sum: the pair table needs the step's layout and the predecessors' slots");
     NVX_REQUIRE(!pos_table || (positions && n_pos > 0), NVX_EINVAL, "nvx_embed_sum: the position table needs positions");
-    NVX_REQUIRE(!h || width % 4 != 0 || nvx_aligned16(w), NVX_EINVAL, "nvx_embed_sum: the norm's weight must start on a 16-byte border");
+    NVX_REQUIRE(!h || width % 4 != 0 || (nvx_aligned16(w) && nvx_aligned16(w_bias)), NVX_EINVAL,
+                "nvx_embed_sum: the norm's weight and bias must start on a 16-byte border");
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL(embed_sum_kernel<A_>, dim3((unsigned)n_tok), dim3(256), (size_t)width * sizeof(float), (hipStream_t)stream, ids,
                                          (const A_*)table, vocab, (const A_*)pair, buckets, mul_prev, mul_cur, prev_id, (const A_*)pos_table, n_pos,
-                                         positions, tok_seq, qo_indptr, pos0, state_slot, x, w, eps, split, (A_*)h, (int)width));
+                                         positions, tok_seq, qo_indptr, pos0, state_slot, x, w, w_bias, eps, split, (A_*)h, (int)width));
     return nvx_check_launch("nvx_embed_sum");
 }
 

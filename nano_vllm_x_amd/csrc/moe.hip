@@ -36,12 +36,12 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
 // group counts as its best score, and only experts of the keep_groups best groups can be chosen (n_groups <= 1: all of them);
 // the `top` largest scores among those are chosen (ties: the lower id) and their scores, divided by their sum + norm_eps, are the
 // weights.  One thread per token; everything float32.
-__global__ __launch_bounds__(256) void moe_route_softmax_kernel(const float* __restrict__ logits, int n_exp, int top, int n_groups,
+__global__ __launch_bounds__(256) void moe_route_softmax_kernel(const float* __restrict__ logits, int64_t logits_stride, int n_exp, int top, int n_groups,
                                                                int keep_groups, float norm_eps, int32_t* __restrict__ idx,
                                                                float* __restrict__ wts, int64_t n_tok) {
     const int64_t t = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (t >= n_tok) return;
-    const float* z = logits + t * n_exp;
+    const float* z = logits + t * logits_stride;
     float zmax = -INFINITY;
     for (int e = 0; e < n_exp; ++e) zmax = fmaxf(zmax, z[e]);
     float denom = 0.f;
@@ -299,35 +299,40 @@ __device__ __forceinline__ float gelu_glu_act(float g, float u) {
     return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g))) * u;
 }
 
-// y[r][j] = act(gu[r][j], gu[r][ff + j]); GELU: gelu_tanh(g) u, the three constants are not read
+// y[r][j] = act(gu[r][j], gu[r][ff + j]) (times sigmoid(row_gate[r]) if given); GELU: gelu_tanh(g) u, the three constants are not read
 template <typename A, bool GELU>
-__global__ __launch_bounds__(256) void moe_glu_kernel(const A* __restrict__ gu, A* __restrict__ y, float limit, float alpha, float shift,
+__global__ __launch_bounds__(256) void moe_glu_kernel(const A* __restrict__ gu, int64_t gu_stride, A* __restrict__ y, int64_t y_stride, float limit,
+                                                     float alpha, float shift, const float* __restrict__ row_gate, int64_t row_gate_stride,
                                                      int64_t rows, int ff) {
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < rows * ff; i += (int64_t)gridDim.x * 256) {
         const int64_t r = i / ff;
         const int j = (int)(i % ff);
-        const float g = ld_f(gu, r * 2 * ff + j), u = ld_f(gu, r * 2 * ff + ff + j);
-        st_f(y, i, GELU ? gelu_glu_act(g, u) : glu_act(g, u, limit, alpha, shift));
+        const float g = ld_f(gu, r * gu_stride + j), u = ld_f(gu, r * gu_stride + ff + j);
+        const float v = GELU ? gelu_glu_act(g, u) : glu_act(g, u, limit, alpha, shift);
+        st_f(y, r * y_stride + j, row_gate ? v * sigmoid_f(row_gate[r * row_gate_stride]) : v);
     }
 }
 
 // The same for 16-bit formats, eight neighbouring entries of a row per thread as one 16-byte load of each half and one store
 // (ff8 = ff / 8; rows start on 16-byte borders).
 template <typename A, bool GELU>
-__global__ __launch_bounds__(256) void moe_glu_vec8_kernel(const A* __restrict__ gu, A* __restrict__ y, float limit, float alpha, float shift,
-                                                          int64_t rows, int ff8) {
+__global__ __launch_bounds__(256) void moe_glu_vec8_kernel(const A* __restrict__ gu, int64_t gu_stride, A* __restrict__ y, int64_t y_stride,
+                                                          float limit, float alpha, float shift, const float* __restrict__ row_gate,
+                                                          int64_t row_gate_stride, int64_t rows, int ff8) {
     union Pack { uint4 v; A a[8]; };
     const int64_t n = rows * ff8;
     for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
         const int64_t r = i / ff8;
         const int64_t j = (i - r * ff8) * 8;
-        const A* row = gu + r * 16 * ff8;
+        const A* row = gu + r * gu_stride;
+        const float rg = row_gate ? sigmoid_f(row_gate[r * row_gate_stride]) : 1.0f;
         Pack g, u, o;
         g.v = *reinterpret_cast<const uint4*>(row + j);
         u.v = *reinterpret_cast<const uint4*>(row + (int64_t)ff8 * 8 + j);
 #pragma unroll
-        for (int k = 0; k < 8; ++k) o.a[k] = (A)(GELU ? gelu_glu_act((float)g.a[k], (float)u.a[k]) : glu_act((float)g.a[k], (float)u.a[k], limit, alpha, shift));
-        *reinterpret_cast<uint4*>(y + i * 8) = o.v;
+        for (int k = 0; k < 8; ++k)
+            o.a[k] = (A)(rg * (GELU ? gelu_glu_act((float)g.a[k], (float)u.a[k]) : glu_act((float)g.a[k], (float)u.a[k], limit, alpha, shift)));
+        *reinterpret_cast<uint4*>(y + r * y_stride + j) = o.v;
     }
 }
 
@@ -402,15 +407,15 @@ extern "C" int nvx_moe_route(const float* logits, int64_t n_tok, int64_t n_exp, 
     return nvx_check_launch("nvx_moe_route");
 }
 
-extern "C" int nvx_moe_route_softmax(const float* logits, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups, int64_t keep_groups,
+extern "C" int nvx_moe_route_softmax(const float* logits, int64_t logits_stride, int64_t n_tok, int64_t n_exp, int64_t top, int64_t n_groups, int64_t keep_groups,
                                      float norm_eps, int32_t* idx, float* wts, nvx_stream_t stream) {
     NVX_REQUIRE(n_tok >= 0 && n_exp > 0 && n_exp < (1 << 20) && top > 0 && top <= n_exp, NVX_EINVAL, "nvx_moe_route_softmax: bad sizes");
     NVX_REQUIRE(n_groups >= 0 && n_groups <= 256 && (n_groups <= 1 || (n_exp % n_groups == 0 && keep_groups >= 1 && keep_groups <= n_groups &&
                                                                       keep_groups * (n_exp / n_groups) >= top)),
                 NVX_EINVAL, "nvx_moe_route_softmax: groups must divide the experts (at most 256 groups) and the kept groups must hold `top` experts");
     if (n_tok == 0) return NVX_OK;
-    NVX_REQUIRE(logits && idx && wts, NVX_EINVAL, "nvx_moe_route_softmax: null pointer");
-    hipLaunchKernelGGL(moe_route_softmax_kernel, dim3((unsigned)((n_tok + 255) / 256)), dim3(256), 0, (hipStream_t)stream, logits, (int)n_exp,
+    NVX_REQUIRE(logits && idx && wts && logits_stride >= n_exp, NVX_EINVAL, "nvx_moe_route_softmax: null pointer or row stride");
+    hipLaunchKernelGGL(moe_route_softmax_kernel, dim3((unsigned)((n_tok + 255) / 256)), dim3(256), 0, (hipStream_t)stream, logits, logits_stride, (int)n_exp,
                        (int)top, (int)n_groups, (int)keep_groups, norm_eps, idx, wts, n_tok);
     return nvx_check_launch("nvx_moe_route_softmax");
 }
@@ -478,39 +483,42 @@ extern "C" int nvx_moe_scatter_rows(const void* h, int64_t h_stride, int fmt, co
     return nvx_check_launch("nvx_moe_scatter_rows");
 }
 
+// gu rows of [gate | up] gu_stride apart, y rows y_stride apart; row_gate: one logit per row, rows row_gate_stride apart (null: no gate)
 template <bool GELU>
-static int launch_glu(const void* gu, int fmt, float limit, float alpha, float shift, void* y, int64_t rows, int64_t ff, hipStream_t s, const char* name) {
-    if (fmt != 2 && ff % 8 == 0 && nvx_aligned16(gu) && nvx_aligned16(y)) {
+static int launch_glu(const void* gu, int64_t gu_stride, int fmt, float limit, float alpha, float shift, const float* row_gate, int64_t row_gate_stride,
+                      void* y, int64_t y_stride, int64_t rows, int64_t ff, hipStream_t s, const char* name) {
+    if (fmt != 2 && ff % 8 == 0 && gu_stride % 8 == 0 && y_stride % 8 == 0 && nvx_aligned16(gu) && nvx_aligned16(y)) {
         int64_t blocks = (rows * (ff / 8) + 255) / 256;
         if (blocks > 256 * 64) blocks = 256 * 64;
         if (fmt == 0)
-            hipLaunchKernelGGL((moe_glu_vec8_kernel<__bf16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const __bf16*)gu, (__bf16*)y, limit,
-                               alpha, shift, rows, (int)(ff / 8));
+            hipLaunchKernelGGL((moe_glu_vec8_kernel<__bf16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const __bf16*)gu, gu_stride, (__bf16*)y,
+                               y_stride, limit, alpha, shift, row_gate, row_gate_stride, rows, (int)(ff / 8));
         else
-            hipLaunchKernelGGL((moe_glu_vec8_kernel<_Float16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const _Float16*)gu, (_Float16*)y,
-                               limit, alpha, shift, rows, (int)(ff / 8));
+            hipLaunchKernelGGL((moe_glu_vec8_kernel<_Float16, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const _Float16*)gu, gu_stride,
+                               (_Float16*)y, y_stride, limit, alpha, shift, row_gate, row_gate_stride, rows, (int)(ff / 8));
         return nvx_check_launch(name);
     }
     int64_t blocks = (rows * ff + 255) / 256;
     if (blocks > 256 * 64) blocks = 256 * 64;
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((moe_glu_kernel<A_, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const A_*)gu, (A_*)y, limit, alpha, shift,
-                                         rows, (int)ff));
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((moe_glu_kernel<A_, GELU>), dim3((unsigned)blocks), dim3(256), 0, s, (const A_*)gu, gu_stride, (A_*)y, y_stride,
+                                         limit, alpha, shift, row_gate, row_gate_stride, rows, (int)ff));
     return nvx_check_launch(name);
 }
 
-extern "C" int nvx_moe_glu(const void* gu, int fmt, float limit, float alpha, float shift, void* y, int64_t rows, int64_t ff,
-                           nvx_stream_t stream) {
-    NVX_REQUIRE(fmt >= 0 && fmt <= 2 && rows >= 0 && ff > 0, NVX_EINVAL, "nvx_moe_glu: bad arguments");
+extern "C" int nvx_moe_glu(const void* gu, int64_t gu_stride, int fmt, float limit, float alpha, float shift, const float* row_gate,
+                           int64_t row_gate_stride, void* y, int64_t y_stride, int64_t rows, int64_t ff, nvx_stream_t stream) {
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2 && rows >= 0 && ff > 0 && gu_stride >= 2 * ff && y_stride >= ff && (!row_gate || row_gate_stride >= 1), NVX_EINVAL,
+                "nvx_moe_glu: bad arguments");
     if (rows == 0) return NVX_OK;
     NVX_REQUIRE(gu && y, NVX_EINVAL, "nvx_moe_glu: null pointer");
-    return launch_glu<false>(gu, fmt, limit, alpha, shift, y, rows, ff, (hipStream_t)stream, "nvx_moe_glu");
+    return launch_glu<false>(gu, gu_stride, fmt, limit, alpha, shift, row_gate, row_gate_stride, y, y_stride, rows, ff, (hipStream_t)stream, "nvx_moe_glu");
 }
 
 extern "C" int nvx_gelu_glu(const void* gu, int fmt, void* y, int64_t rows, int64_t ff, nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2 && rows >= 0 && ff > 0, NVX_EINVAL, "nvx_gelu_glu: bad arguments");
     if (rows == 0) return NVX_OK;
     NVX_REQUIRE(gu && y, NVX_EINVAL, "nvx_gelu_glu: null pointer");
-    return launch_glu<true>(gu, fmt, 0.f, 0.f, 0.f, y, rows, ff, (hipStream_t)stream, "nvx_gelu_glu");
+    return launch_glu<true>(gu, 2 * ff, fmt, 0.f, 0.f, 0.f, nullptr, 0, y, ff, rows, ff, (hipStream_t)stream, "nvx_gelu_glu");
 }
 
 extern "C" int nvx_moe_gather_rows(const void* ys, int fmt, const int64_t* dst, const float* wts, int64_t top, void* out, int64_t n_tok,

@@ -5,7 +5,9 @@
 //       mlstm   exponential input gate and sigmoid forget gate stabilised by a running maximum, normaliser vector;
 //       delta   per-head decay, then a rank-one correction of the memory towards the new value along the key;
 //       rwkv    per-key-channel decay, the current token read with a bonus before it is written;
-//       decay   one constant decay per head, the token written before it is read (linear attention with a fixed decay);
+//       decay   one constant decay per head, the token written before it is read (linear attention with a fixed decay; queries and keys may
+//               be rotated by position as they are staged: retention); steps of one token per sequence have a form of their own that
+//               walks the memory once and ends in the norm and gate of the read-out;
 //       gla     a decay per key channel and token, the token written before it is read (gated linear attention).
 // Long portions of mlstm, decay and gla are cut into chunks that run side by side, in three phases (see decay).
 // One kernel per recurrence serves prompts, portions of prompts and single decoded tokens: a workgroup takes one head of
@@ -498,6 +500,8 @@ __global__ __launch_bounds__(256) void rwkv_scan_kernel(const A* __restrict__ rx
 // the state at every chunk's start (and writes the sequence's final state), phase 3 walks every chunk from there with the read-out.
 // Because the decay is a constant, the carry over a chunk of n tokens is decay^n S + (the chunk's own contribution).  phase 0: one
 // workgroup walks the whole portion (single tokens, short portions).
+// With `half` > 0 the pairs (m, m + half) of every staged query and key are rotated by the token's angles (turn), in float32, and keys are
+// multiplied by k_mul.
 // `tb` tokens are staged at a time: 32 where the key size leaves LDS for them (more than the other recurrences take: an activation
 // is applied as they are staged, and fewer, longer stages hide more of the loads), fewer for wide keys.
 template <typename A, int PHASE>
@@ -505,7 +509,8 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
                                                         const float* __restrict__ decay, float* __restrict__ S,
                                                         const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
                                                         const int32_t* __restrict__ state_slot, float* __restrict__ out, int heads, int dim,
-                                                        int vdim, int p_lanes, int tb, int vec, int chunk, int n_chunk_max, float* __restrict__ ws) {
+                                                        int vdim, int p_lanes, int tb, int vec, int chunk, int n_chunk_max, float* __restrict__ ws,
+                                                        TurnRows turn, int half, float k_mul) {
     constexpr int phase = PHASE;
     extern __shared__ float sm[];
     const int cb = blockDim.x / p_lanes, rs = p_lanes * KS;
@@ -539,9 +544,27 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
         __syncthreads();
         const A* xr = x + (sp.q0 + t0) * x_stride;
         if (phase != 1) stage_key_rows(sq, rs, xr + q_off + hd * dim, x_stride, nt, dim, vec, act);      // (phase 1 wants the state only)
-        stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec, act);
+        stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec, act, k_mul);
         stage_value_cols(sv, cb, xr + v_off + hd * vdim + blockIdx.x * cb, x_stride, nt, vdim - (int)blockIdx.x * cb, vec, act);
         __syncthreads();
+        if (half) {
+            for (int i = threadIdx.x; i < nt * half; i += blockDim.x) {
+                const int tt = i / half, m = i - tt * half, d0 = lds_row(m), d1 = lds_row(m + half);
+                const float* tr = turn.cos + (sp.q0 + t0 + tt) * turn.stride + m;
+                const float c = tr[0], sn = tr[turn.sin_off];
+                float* kr = sk + tt * rs;
+                const float u = kr[d0], v = kr[d1];
+                kr[d0] = u * c - v * sn;
+                kr[d1] = v * c + u * sn;
+                if (phase != 1) {
+                    float* qr = sq + tt * rs;
+                    const float a = qr[d0], b = qr[d1];
+                    qr[d0] = a * c - b * sn;
+                    qr[d1] = b * c + a * sn;
+                }
+            }
+            __syncthreads();
+        }
         for (int tt = 0; tt < nt; ++tt) {
             const float v = sv[tt * cb + th.col];
             const float* kk = sk + tt * rs + th.p * KS;
@@ -566,6 +589,102 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
         if (row < dim && th.active) Sp[(int64_t)row * vdim + th.e] = s[r];
+    }
+}
+
+// The same recurrence for steps of one token per sequence.  A workgroup takes one head of one sequence: the rotated query and key and the
+// value wait in LDS, thread (group, column piece) walks every n_groups-th row of the memory V columns at a time (U rows' loads in flight
+// together; the memory is read and written once), and the groups' partial read-outs are added through LDS.  The end is that of
+// head_norm_gate: the read-out divided by its root mean square, times mul, times the gate (kind 0: none, 1: sigmoid, 2: silu).
+template <typename A, int V>
+__global__ __launch_bounds__(256) void decay_step_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off, int v_off, int act,
+                                                        const float* __restrict__ decay, float* __restrict__ S, const int64_t* __restrict__ pos0,
+                                                        const int32_t* __restrict__ state_slot, int heads, int dim, int vdim, TurnRows turn, int half,
+                                                        float k_mul, float eps, int g_off, int kind, float mul, A* __restrict__ out,
+                                                        int64_t out_stride) {
+    extern __shared__ __align__(16) float sm[];
+    float* sq = sm;                        // dim
+    float* sk = sq + dim;                  // dim
+    float* part = sk + dim;                // n_groups x cols (cols: vdim rounded up to a multiple of V, in pieces)
+    __shared__ float red[4];
+    typedef float vecf __attribute__((ext_vector_type(V)));
+    const int hd = blockIdx.x;
+    const int64_t b = blockIdx.y;
+    const int slot = state_slot[b];
+    const A* xr = x + b * x_stride;
+    A* orow = out + b * out_stride + (int64_t)hd * vdim;
+    if (slot < 0) {                        // a padding row: its output is read by the products behind it, nothing else
+        for (int e = threadIdx.x; e < vdim; e += 256) st_f(orow, e, 0.f);
+        return;
+    }
+    for (int d = threadIdx.x; d < dim; d += 256) {
+        float qv = scan_act(ld_f(xr, q_off + hd * dim + d), act), kv = scan_act(ld_f(xr, k_off + hd * dim + d), act);
+        if (d < 2 * half) {
+            const int o = d < half ? d + half : d - half;
+            const float qo = scan_act(ld_f(xr, q_off + hd * dim + o), act), ko = scan_act(ld_f(xr, k_off + hd * dim + o), act);
+            const float* tr = turn.cos + b * turn.stride + (d < half ? d : o);
+            const float c = tr[0], sn = d < half ? -tr[turn.sin_off] : tr[turn.sin_off];
+            qv = qv * c + qo * sn;
+            kv = kv * c + ko * sn;
+        }
+        sq[d] = qv;
+        sk[d] = kv * k_mul;
+    }
+    const int pieces = (vdim + V - 1) / V, n_groups = 256 / pieces;      // (the host keeps pieces <= 256)
+    const int grp = threadIdx.x / pieces, e0 = (threadIdx.x % pieces) * V;
+    const bool on = grp < n_groups;
+    const float g = decay[hd];
+    const bool cont = pos0[b] > 0;
+    float* Sp = S + ((int64_t)slot * heads + hd) * dim * vdim;
+    vecf val, acc;
+#pragma unroll
+    for (int i = 0; i < V; ++i) { val[i] = on ? scan_act(ld_f(xr, v_off + hd * vdim + e0 + i), act) : 0.f; acc[i] = 0.f; }
+    __syncthreads();
+    if (on) {
+        constexpr int U = 8;
+        for (int r0 = grp; r0 < dim; r0 += n_groups * U) {
+            vecf s[U];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int r = r0 + u * n_groups;
+                if (cont && r < dim) s[u] = *reinterpret_cast<const vecf*>(Sp + (int64_t)r * vdim + e0);
+                else {
+#pragma unroll
+                    for (int i = 0; i < V; ++i) s[u][i] = 0.f;
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int r = r0 + u * n_groups;
+                if (r >= dim) continue;
+                const float kr = sk[r], qr = sq[r];
+#pragma unroll
+                for (int i = 0; i < V; ++i) {
+                    s[u][i] = g * s[u][i] + kr * val[i];
+                    acc[i] += qr * s[u][i];
+                }
+                *reinterpret_cast<vecf*>(Sp + (int64_t)r * vdim + e0) = s[u];
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < V; ++i) part[grp * pieces * V + e0 + i] = acc[i];
+    }
+    __syncthreads();
+    float ss = 0.f;
+    for (int e = threadIdx.x; e < vdim; e += 256) {        // (a thread alone reads and writes its columns)
+        float o = 0.f;
+        for (int k = 0; k < n_groups; ++k) o += part[k * pieces * V + e];
+        part[e] = o;
+        ss += o * o;
+    }
+    const float rn = mul / sqrtf(block256_sum(ss, red) / (float)vdim + eps);
+    for (int e = threadIdx.x; e < vdim; e += 256) {
+        float v = part[e] * rn;
+        if (kind) {
+            const float z = ld_f(xr, g_off + hd * vdim + e);
+            v *= kind == 1 ? sigmoid_f(z) : z * sigmoid_f(z);
+        }
+        st_f(orow, e, v);
     }
 }
 
@@ -714,6 +833,13 @@ using namespace NVX_NS;
     NVX_REQUIRE(pos0 && state_slot, NVX_EINVAL, name ": null layout");                                                              \
     NVX_REQUIRE(qo_indptr || n_tok == n_seq, NVX_EINVAL, name ": without qo_indptr every sequence has one token")
 
+void nvx_launch_tail_rows(const void* x, int64_t x_stride, int fmt, int taps_n, float* state, const int32_t* qo_indptr, const int64_t* pos0,
+                          const int32_t* state_slot, int64_t n_seq, int64_t channels, hipStream_t stream) {
+    const unsigned cx = (unsigned)((channels + 255) / 256);
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(tail_rows_kernel<A_>, dim3(cx, (unsigned)n_seq), dim3(256), 0, stream, (const A_*)x, x_stride, taps_n - 1, state,
+                                         qo_indptr, pos0, state_slot, (int)channels));
+}
+
 extern "C" int nvx_short_conv(const void* x, int64_t x_stride, int fmt, const float* w, const float* bias, int act, int taps_n, float* state,
                               int64_t n_slots, const int32_t* tok_seq, const int32_t* qo_indptr, const int64_t* pos0,
                               const int32_t* state_slot, void* out, int64_t n_tok, int64_t n_seq, int64_t channels, nvx_stream_t stream) {
@@ -849,9 +975,13 @@ extern "C" int nvx_rwkv_scan(const void* r, const void* k, const void* v, int64_
 extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, int act,
                               const float* decay, float* S, int64_t n_slots, const int32_t* qo_indptr, const int64_t* pos0,
                               const int32_t* state_slot, float* out, int64_t n_tok, int64_t n_seq, int64_t heads, int64_t dim, int64_t vdim,
-                              int64_t chunk, int64_t n_chunk_max, float* ws, nvx_stream_t stream) {
+                              int64_t chunk, int64_t n_chunk_max, float* ws, const float* turn, int64_t turn_stride, int64_t turn_sin_off,
+                              int rot_dims, float k_mul, nvx_stream_t stream) {
     NVX_LAYOUT_OK("nvx_decay_scan");
     ScanLaunch g;
+    NVX_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || (turn && turn_stride >= turn_sin_off + rot_dims / 2)), NVX_EINVAL,
+                "nvx_decay_scan: the rotated part must be even and within a head, and needs its table");
+    const TurnRows tr{turn, turn_stride, turn_sin_off};
     NVX_REQUIRE(heads > 0 && heads <= 65535 && dim > 0 && vdim > 0 && vdim < (1 << 24) && n_slots >= 0 && (act == 0 || act == 1), NVX_EINVAL,
                 "nvx_decay_scan: bad sizes");
     NVX_REQUIRE(scan_launch(dim, vdim, &g), NVX_EUNSUPPORTED, "nvx_decay_scan: key size above 512");
@@ -866,7 +996,8 @@ extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t 
 #define NVX_DECAY_SCAN(PHASE)                                                                                                                      \
     NVX_FMT_CALL(fmt, hipLaunchKernelGGL((decay_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, (hipStream_t)stream, (const A_*)x, x_stride,   \
                                          (int)q_off, (int)k_off, (int)v_off, act, decay, S, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim,  \
-                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb), (int)chunk, (int)n_chunk_max, ws))
+                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb), (int)chunk, (int)n_chunk_max, ws, tr, \
+                                         rot_dims / 2, k_mul))
     if (!chunk) {
         NVX_DECAY_SCAN(0);
     } else {
@@ -878,6 +1009,37 @@ extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t 
     }
 #undef NVX_DECAY_SCAN
     return nvx_check_launch("nvx_decay_scan");
+}
+
+extern "C" int64_t nvx_decay_step_max_vdim() { return 1024; }      // (256 threads of four columns; not a multiple of four: 256)
+
+extern "C" int nvx_decay_step(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, int act, const float* decay,
+                              float* S, int64_t n_slots, const int64_t* pos0, const int32_t* state_slot, int64_t n_seq, int64_t heads, int64_t dim,
+                              int64_t vdim, const float* turn, int64_t turn_stride, int64_t turn_sin_off, int rot_dims, float k_mul, float eps,
+                              int64_t g_off, int kind, float mul, void* out, int64_t out_stride, nvx_stream_t stream) {
+    NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_decay_step: fmt must be 0, 1 or 2");
+    NVX_REQUIRE(n_seq >= 0 && n_seq <= 65535 && heads > 0 && dim > 0 && dim <= 4096 && vdim > 0 && n_slots >= 0 && (act == 0 || act == 1) && kind >= 0 && kind <= 2,
+                NVX_EINVAL, "nvx_decay_step: bad sizes");
+    const int v = vdim % 4 == 0 && nvx_aligned16(S) ? 4 : 1;
+    NVX_REQUIRE(vdim <= 256 * v, NVX_EUNSUPPORTED, "nvx_decay_step: value size above 1024 (256 where it is not a multiple of four)");
+    if (n_seq == 0) return NVX_OK;
+    NVX_REQUIRE(x && decay && S && pos0 && state_slot && out && out_stride >= heads * vdim, NVX_EINVAL, "nvx_decay_step: null pointer or row stride");
+    NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && g_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
+                    x_stride >= v_off + heads * vdim && (kind == 0 || x_stride >= g_off + heads * vdim), NVX_EINVAL,
+                "nvx_decay_step: q, k, v or the gate lies outside a row");
+    NVX_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || (turn && turn_stride >= turn_sin_off + rot_dims / 2)), NVX_EINVAL,
+                "nvx_decay_step: the rotated part must be even and within a head, and needs its table");
+    const TurnRows tr{turn, turn_stride, turn_sin_off};
+    const int64_t pieces = (vdim + v - 1) / v;
+    const size_t lds = (size_t)(2 * dim + (256 / pieces) * pieces * v) * sizeof(float);
+#define NVX_DECAY_STEP(V)                                                                                                                          \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((decay_step_kernel<A_, V>), dim3((unsigned)heads, (unsigned)n_seq), dim3(256), lds, (hipStream_t)stream,    \
+                                         (const A_*)x, x_stride, (int)q_off, (int)k_off, (int)v_off, act, decay, S, pos0, state_slot, (int)heads, (int)dim, \
+                                         (int)vdim, tr, rot_dims / 2, k_mul, eps, (int)g_off, kind, mul, (A_*)out, out_stride))
+    if (v == 4) NVX_DECAY_STEP(4);
+    else NVX_DECAY_STEP(1);
+#undef NVX_DECAY_STEP
+    return nvx_check_launch("nvx_decay_step");
 }
 
 extern "C" int nvx_gla_scan(const void* x, int64_t x_stride, int fmt, int64_t q_off, int64_t k_off, int64_t v_off, float q_mul, const float* alpha,

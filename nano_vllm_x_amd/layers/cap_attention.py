@@ -1,7 +1,8 @@
 """Causal attention with grouped key/value heads and separate key and value sizes over per-token key and value rows in the
 token cache: SoftcapAttention (rotary positions on a leading part of each head, unit-mean-square values, capped scores) and
 NormedAttention (query/key RMS norms, optional rotation of keys AND values, window, distance penalty, output gate, borrowed
-keys and values), TiedAttention (one cached row per token and head is key and value, linear distance penalty, chunks of positions)."""
+keys and values), TiedAttention (one cached row per token and head is key and value, linear distance penalty, chunks of positions),
+ConvAttention (a short convolution over time ahead of rotation and norm, a sink per head, a window behind which the first tokens stay)."""
 from __future__ import annotations
 
 import torch
@@ -183,3 +184,47 @@ class TiedAttention(nn.Module):
         o = ops.softcap_attn(q, rows, rows, md.kv_indices, md.kv_start, md.kv_len, md.layout, self.scale, 0.0, self.heads, self.kv_heads, self.dim,
                              self.dim, window=self.window, chunk=self.chunk, slopes=self.slopes, k_rn=rn)
         return self.o_proj(o)
+
+
+class ConvAttention(nn.Module):
+    """Grouped-head softmax attention whose queries, keys and values pass a short causal convolution per channel between their projection
+    and everything else: u_t = sum_j w[j] x_(t - taps + 1 + j), zeros before the sequence's start.  Then queries and keys are rotated by
+    position (the first rot dims of each head, halves layout) and divided by their root mean square per head (no weight).
+      window      a token sees itself and the window - 1 before it (None: all before it), and the sequence's first `keep_first` tokens
+      sinks       True: the softmax's sum has one more term exp(sink_h) without a value, a learned number per head
+      out_mul     the read-out is multiplied by this number before the output projection
+    The module is a block of a layer that shares its matrix products between several mechanisms: `attend` reads q | k | v from `col0` of the
+    layer's input product on and writes its heads into `out`, the columns of the layer's output product that belong to it.  The rotation
+    comes from the step's table (see TurnTables).  State: the convolution's last taps - 1 inputs (float32), under (state_name, "conv")."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, scale: float, eps: float, cache_names, state_name, rot_key=None,
+                 rot_dims: int = 0, window=None, keep_first: int = 0, sinks: bool = True, out_mul: float = 1.0):
+        super().__init__()
+        if heads % kv_heads:
+            raise ValueError("query heads must be a multiple of key/value heads")
+        if taps < 1:
+            raise ValueError("a convolution has at least one tap")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError("the rotated part of a head must be even and within the head")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.taps = heads, kv_heads, dim, vdim, taps
+        self.scale, self.eps, self.out_mul, self.rot_key = float(scale), eps, float(out_mul), rot_key
+        self.window, self.keep_first = int(window or 0), int(keep_first or 0) if window else 0
+        self.k_name, self.v_name = cache_names
+        self.state_name = state_name
+        self.q_cols, self.k_cols, self.v_cols = heads * dim, kv_heads * dim, kv_heads * vdim
+        self.proj_rows, self.out_cols = self.q_cols + self.k_cols + self.v_cols, heads * vdim
+        self.conv_w = nn.Parameter(torch.zeros(taps, self.proj_rows, dtype=torch.float32))      # row j: the tap taps - 1 - j tokens back
+        self.sinks = nn.Parameter(torch.zeros(heads, dtype=torch.float32)) if sinks else None
+
+    def cache_rows(self) -> dict:
+        return {self.k_name: self.k_cols, self.v_name: self.v_cols}
+
+    def state_shapes(self) -> dict:
+        return {(self.state_name, "conv"): (self.taps - 1, self.proj_rows)} if self.taps > 1 else {}
+
+    def attend(self, x: torch.Tensor, col0: int, turn, md, out: torch.Tensor):
+        k_cache, v_cache = md.cache.latent(self.k_name), md.cache.latent(self.v_name)
+        q = ops.conv_attn_prep(x[:, col0:col0 + self.proj_rows], self.conv_w, md.cache.state((self.state_name, "conv")) if self.taps > 1 else None, md.layout,
+                               turn, self.eps, md.out_slots, k_cache, v_cache, self.heads, self.kv_heads, self.dim, self.vdim)
+        ops.softcap_attn(q, k_cache, v_cache, md.kv_indices, md.kv_start, md.kv_len, md.layout, self.scale, 0.0, self.heads, self.kv_heads, self.dim,
+                         self.vdim, window=self.window, keep_first=self.keep_first, sinks=self.sinks, out_mul=self.out_mul, out=out)

@@ -1,6 +1,6 @@
 """Gated feed-forward layers, and mixtures of small ones: behind a sigmoid router whose score scales an expert's input, behind a softmax
 router with groups whose renormalised scores weigh the experts' outputs, behind a sigmoid router with groups and a correction that
-enters the choice only, or chosen by a table of token ids with fixed weights on the experts' outputs."""
+enters the choice only, or chosen by a table of token ids with fixed weights on the experts' outputs; a shared expert behind a gate."""
 from __future__ import annotations
 
 import torch
@@ -160,8 +160,8 @@ class TableMoE(ExpertBank):
 class GroupedSoftmaxMoE(ExpertBank):
     """scores = softmax(W_router h) over all experts (float32).  The experts form `groups` equal groups of neighbours; a group counts
     as its best score and only experts of the `keep` best groups can be chosen (groups None or 1: no such limit).  Every token takes
-    the `top` largest scores among those, the weights are these scores divided by their sum + norm_eps, and they weigh the experts'
-    OUTPUTS.  Expert: g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), W_down (g * sigmoid(alpha * g) * (u + shift))."""
+    the `top` largest scores among those, the weights are these scores divided by their sum + norm_eps (0.0: the softmax over the chosen
+    logits), and they weigh the experts' OUTPUTS.  Expert: g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), W_down (g * sigmoid(alpha * g) * (u + shift))."""
 
     def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, alpha: float, shift: float = 1.0, groups=None, keep=None,
                  norm_eps: float = 1e-20):
@@ -173,9 +173,24 @@ class GroupedSoftmaxMoE(ExpertBank):
         self.norm_eps = float(norm_eps)
         self.router = nn.Parameter(torch.zeros(experts, width, dtype=torch.float32))
 
-    def forward(self, h: torch.Tensor, decode_step: bool = False) -> torch.Tensor:
-        idx, wts = ops.moe_route_softmax(ops.skinny_proj(h, self.router), self.top, self.groups, self.keep, self.norm_eps)
+    def forward(self, h: torch.Tensor, decode_step: bool = False, logits=None) -> torch.Tensor:
+        """`logits` (T, experts): the router's, where the caller has made them beside other numbers per token."""
+        idx, wts = ops.moe_route_softmax(ops.skinny_proj(h, self.router) if logits is None else logits, self.top, self.groups, self.keep, self.norm_eps)
         return self.run(h, idx, wts, decode_step, weight_out=True)
+
+
+class GatedSharedExpert(nn.Module):
+    """A feed-forward that every token passes beside the chosen experts, times a gate of one number per token: sigmoid(z) W_down (silu(W_gate
+    h) * (W_up h)).  A block of a layer's shared products: `hidden` reads gate | up from `col0` of the layer's input product on and writes
+    the gated hidden row into `out`, the columns of the layer's output product that belong to W_down (the gate is one number per row, so it
+    passes through the product)."""
+
+    def __init__(self, ff: int):
+        super().__init__()
+        self.ff, self.proj_rows, self.out_cols = ff, 2 * ff, ff
+
+    def hidden(self, x: torch.Tensor, col0: int, gate: torch.Tensor, out: torch.Tensor):
+        ops.moe_glu(x[:, col0:col0 + self.proj_rows], float("inf"), 1.0, 0.0, row_gate=gate, out=out)
 
 
 class GroupedSigmoidMoE(ExpertBank):

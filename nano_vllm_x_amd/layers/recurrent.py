@@ -240,3 +240,38 @@ class GatedLinearAttention(nn.Module):
         o = ops.gla_scan(x, (0, hd, 2 * hd), alpha, md.cache.state((n, "S")), md.layout, self.heads, self.dim, self.vdim, q_mul=self.dim ** -0.5)
         y = ops.head_norm_gate(o, self.norm, self.eps, gate=x[:, 2 * hd + he:], kind="silu")
         return self.o_proj(y)
+
+
+class Retention(nn.Module):
+    """Linear attention with one constant decay per head whose queries and keys are rotated by position (Y. Sun, L. Dong et al., "Retentive
+    Network: A Successor to Transformer for Large Language Models"): q = W_q h, k = W_k h (heads x dim; the first rot dims of each head
+    rotated, halves layout), v = W_v h (heads x vdim); per head S <- decay_h S + dim^(-1/2) k v^T, o = S^T q (the read sees the token's own
+    write).  Each head's o is divided by its root mean square (no weight), times `out_mul`, times silu(W_g h).  State: S (float32), zero at a
+    sequence's start, under (state_name, "S").
+    As ConvAttention a block of a layer's shared products: `mix` reads q | k | v | g from `col0` on and writes its heads into `out`.  The
+    rotation is applied in float32 as the recurrence stages its rows.  Steps of one token per sequence are one launch (ops.decay_step)."""
+
+    def __init__(self, heads: int, dim: int, vdim: int, decay, eps: float, state_name, rot_key=None, rot_dims: int = 0, out_mul: float = 1.0):
+        super().__init__()
+        decay = [float(d) for d in decay]
+        if len(decay) != heads:
+            raise ValueError(f"{heads} heads need {heads} decays, got {len(decay)}")
+        if rot_dims % 2 or rot_dims > dim:
+            raise ValueError("the rotated part of a head must be even and within the head")
+        self.heads, self.dim, self.vdim, self.eps, self.state_name = heads, dim, vdim, eps, state_name
+        self.rot_key, self.out_mul = rot_key, float(out_mul)
+        self.register_buffer("decay", torch.tensor(decay, dtype=torch.float32), persistent=False)
+        self.proj_rows, self.out_cols = 2 * heads * dim + 2 * heads * vdim, heads * vdim
+
+    def state_shapes(self) -> dict:
+        return {(self.state_name, "S"): (self.heads, self.dim, self.vdim)}
+
+    def mix(self, x: torch.Tensor, col0: int, turn, md, out: torch.Tensor):
+        hd, he = self.heads * self.dim, self.heads * self.vdim
+        at, g0, mem, k_mul = (col0, col0 + hd, col0 + 2 * hd), col0 + 2 * hd + he, md.cache.state((self.state_name, "S")), self.dim ** -0.5
+        if ops.decay_step_fits(md.layout, self.dim, self.vdim):
+            ops.decay_step(x, at, self.decay, mem, md.layout, self.heads, self.dim, self.vdim, self.eps, turn=turn, k_mul=k_mul, gate_off=g0,
+                           gate_kind="silu", mul=self.out_mul, out=out)
+            return
+        o = ops.decay_scan(x, at, self.decay, mem, md.layout, self.heads, self.dim, self.vdim, turn=turn, k_mul=k_mul)
+        ops.head_norm_gate(o, None, self.eps, gate=x[:, g0:g0 + he], kind="silu", mul=self.out_mul, out=out)

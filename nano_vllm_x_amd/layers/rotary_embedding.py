@@ -74,3 +74,41 @@ def rotary_frequencies(dims: int, base: float, scaling: dict | None = None):
     hi = min(math.ceil(index_of(float(scaling["slow"]))), dims - 1)
     ramp = ((idx - lo) / max(hi - lo, 0.001)).clamp_(0.0, 1.0)
     return freq / factor * ramp + freq * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
+
+
+class TurnTables:
+    """The rotations a model's layers use, each distinct one once: `add` names a rotation and says where its angles will stand, `step`
+    makes a step's table of cosines and sines for all of them in one launch, `at` picks one out of it.  Register `freq` (float64) after the
+    last `add`."""
+
+    def __init__(self):
+        self._where, self._freqs = {}, []
+
+    def add(self, rot: dict | None):
+        """`rot` = {dims, base, scaling | None} (see rotary_frequencies); a scaling that changes the magnitude is refused.  Returns the key for
+        `at` (None: no rotation)."""
+        if not rot or not int(rot["dims"]):
+            return None
+        dims = int(rot["dims"])
+        if dims % 2:
+            raise ValueError("the rotated part of a head must be even")
+        scaling = rot.get("scaling")
+        key = (dims, float(rot["base"]), tuple(sorted((k, float(v)) for k, v in scaling.items())) if scaling else None)
+        if key not in self._where:
+            freq, mag = rotary_frequencies(dims, rot["base"], scaling)
+            if mag != 1.0:
+                raise NotImplementedError("a frequency scaling that changes the rotation's magnitude is not built for these layers")
+            self._where[key] = sum(f.numel() for f in self._freqs)
+            self._freqs.append(freq.to(torch.float64))
+        return key
+
+    def freq(self):
+        """Every rotation's frequencies side by side, float64 (None: no layer rotates)."""
+        return torch.cat(self._freqs) if self._freqs else None
+
+    @staticmethod
+    def step(positions: torch.Tensor, freq):
+        return None if freq is None else ops.turn_table(positions, freq)
+
+    def at(self, table, key):
+        return None if key is None else ops.Turn(table, self._where[key], key[0])

@@ -900,25 +900,36 @@ def gated_residual_norm(x, y=None, gate=None, gate_bias=None, mult: float = 1.0,
     return h
 
 
-def head_norm_gate(o, w, eps: float, gate=None, kind: str = "none", dtype=None):
-    """o (T, heads, vdim) float32: every head's row divided by its root mean square, times w ((heads, vdim), or (vdim,) shared
-    by the heads), times the output gate: kind "sigmoid" or "silu" of `gate` (T, heads * vdim).  Returns (T, heads * vdim)."""
+def _out_rows(out, t: int, width: int, dtype, device, what: str):
+    """`out` (T, width) in `dtype`, rows possibly slices of a wider buffer's; made here where the caller gave none."""
+    if out is None:
+        return torch.empty((t, width), dtype=dtype, device=device)
+    _dev(out)
+    _need(out.shape == (t, width) and out.stride(1) == 1 and out.dtype == dtype, what + ": out must be (T, columns) with unit inner stride, in the result's format")
+    return out
+
+
+def head_norm_gate(o, w, eps: float, gate=None, kind: str = "none", dtype=None, mul: float = 1.0, out=None):
+    """o (T, heads, vdim) float32: every head's row divided by its root mean square, times w ((heads, vdim), (vdim,) shared
+    by the heads, or None: ones) and `mul`, times the output gate: kind "sigmoid" or "silu" of `gate` (T, heads * vdim).  Returns (T,
+    heads * vdim): `out` where it is given (rows may be slices of a wider buffer's)."""
     _dev(o, w, gate)
     _f32c(o, "head_norm_gate: o")
-    _f32c(w, "head_norm_gate: w")
     _need(o.dim() == 3, "head_norm_gate: o must be (T, heads, vdim)")
     t, heads, vdim = o.shape
-    _need(w.numel() in (vdim, heads * vdim), "head_norm_gate: w size")
+    if w is not None:
+        _f32c(w, "head_norm_gate: w")
+        _need(w.numel() in (vdim, heads * vdim), "head_norm_gate: w size")
     k = {"none": 0, "sigmoid": 1, "silu": 2}[kind]
     if k:
         _need(gate is not None and gate.shape == (t, heads * vdim) and gate.stride(1) == 1, "head_norm_gate: gate shape")
         dtype = dtype or gate.dtype
         _need(gate.dtype == dtype, "head_norm_gate: gate format")
     _need(dtype in _FMT, "head_norm_gate: output format")
-    out = torch.empty((t, heads * vdim), dtype=dtype, device=o.device)
+    out = _out_rows(out, t, heads * vdim, dtype, o.device, "head_norm_gate")
     lib = _lib.load()
-    _lib.check(lib.nvx_head_norm_gate(_ptr(o), _ptr(w), int(w.numel() == vdim), _ptr(gate) if k else None,
-                                      gate.stride(0) if k else 0, k, _FMT[dtype], float(eps), _ptr(out), t, heads, vdim, _stream()),
+    _lib.check(lib.nvx_head_norm_gate(_ptr(o), _ptr(w), int(w is not None and w.numel() == vdim), _ptr(gate) if k else None,
+                                      gate.stride(0) if k else 0, k, _FMT[dtype], float(eps), float(mul), _ptr(out), out.stride(0), t, heads, vdim, _stream()),
                "nvx_head_norm_gate")
     return out
 
@@ -1085,12 +1096,13 @@ def rope_vnorm_store(qkv, positions, freq, mag: float, rot_dims: int, eps: float
 
 SOFTCAP_SPLIT_BELOW = 1024      # (token, head) pairs of a step below which the keys are split over workgroups too
 SOFTCAP_SPLITS = 4
+SOFTCAP_NARROW = 256            # keys a token sees at most
 
 
 def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: StepLayout, scale: float, cap: float, heads: int,
                  kv_heads: int, dim: int, vdim: int, n_split: Optional[int] = None, window: int = 0, r1=None, r2=None, v_turn=None,
                  v_interleaved: bool = False, gate=None, matrix_cores: bool = True, sink_score: Optional[float] = None, chunk: int = 0, slopes=None,
-                 k_rn=None):
+                 k_rn=None, sinks=None, keep_first: int = 0, out_mul: float = 1.0, out=None):
     """Causal attention of q (T, heads * dim) over cached rows: sequence b's tokens are at slots kv_indices[kv_start[b] :
     kv_start[b] + kv_len[b]]; scores scale * q . k pass cap * tanh(. / cap) (cap <= 0: not) before the softmax.
     `window` > 0: a token sees itself and the window - 1 tokens before it; `chunk` > 0: those of its own chunk of positions (i // chunk
@@ -1100,8 +1112,10 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
     attn_prep_store returns them: the read-out's pairs ((m, m + vdim / 2), or (2m, 2m + 1) if `v_interleaved`) are turned back by
     those angles, undoing the turn attn_prep_store gave the values.  `gate`
     (T, heads * vdim), or (T, heads) with one number per head: the read-out times sigmoid(gate).  `sink_score`: the softmax's sum has
-    one more term exp(sink_score) that carries no value (0.0: one is added to the denominator).  Steps of many tokens in a 16-bit format, with key and value sizes of 64,
-    96 or 128, run on the matrix cores unless `matrix_cores` is False.  Returns (T, heads * vdim) in q's format."""
+    one more term exp(sink_score) that carries no value (0.0: one is added to the denominator); `sinks` (heads, float32): exp(sinks[h])
+    instead.  `keep_first`: with a window, the sequence's first `keep_first` tokens stay visible.  Steps of many tokens in a 16-bit format,
+    with key and value sizes that are multiples of eight up to 128, run on the matrix cores unless `matrix_cores` is False.  Returns the
+    result times `out_mul`, (T, heads * vdim) in q's format: `out` where it is given (rows may be slices of a wider buffer's)."""
     _dev(q, k_cache, v_cache, kv_indices, kv_start, kv_len, r1, r2, v_turn, gate)
     _need((r1 is None) == (r2 is None), "softcap_attn: r1 and r2 go together")
     for a in (r1, r2):
@@ -1121,6 +1135,11 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
         _dev(k_rn)
         _f32c(k_rn, "softcap_attn: k_rn")
         _need(k_rn.shape == (k_cache.shape[0], kv_heads), "softcap_attn: k_rn must be (slots, kv_heads)")
+    if sinks is not None:
+        _dev(sinks)
+        _f32c(sinks, "softcap_attn: sinks")
+        _need(sinks.numel() == heads and sink_score is None, "softcap_attn: sinks have one number per head (and stand in for sink_score)")
+    _need(keep_first >= 0 and not (keep_first and chunk), "softcap_attn: kept first tokens go with a window")
     gate_per_head = gate is not None and gate.shape[1] == heads and vdim != 1
     t = q.shape[0]
     _need(q.shape == (t, heads * dim) and q.is_contiguous() and t == layout.n_tok, "softcap_attn: q must be contiguous (T, heads * dim)")
@@ -1130,11 +1149,13 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
     _need(kv_indices.dtype == torch.int32 and kv_indices.is_contiguous(), "softcap_attn: kv_indices must be int32")
     _need(kv_start.dtype == torch.int64 and kv_start.numel() >= layout.n_seq, "softcap_attn: kv_start must be int64 (B)")
     _need(kv_len.dtype == torch.int32 and kv_len.numel() >= layout.n_seq, "softcap_attn: kv_len must be int32 (B)")
-    out = torch.empty((t, heads * vdim), dtype=q.dtype, device=q.device)
+    out = _out_rows(out, t, heads * vdim, q.dtype, q.device, "softcap_attn")
     # a step of few tokens is few workgroups, each walking all of its sequence's keys: their keys are dealt out over several
-    # workgroups whose partial results a second launch merges (the choice depends on the step's shape only, never on its data)
+    # workgroups whose partial results a second launch merges (the choice depends on the step's shape only, never on its data); not
+    # where a window leaves a workgroup's four waves a tile of 64 keys each
     if n_split is None:
-        n_split = SOFTCAP_SPLITS if t * heads < SOFTCAP_SPLIT_BELOW else 1
+        narrow = window and window + keep_first <= SOFTCAP_NARROW
+        n_split = SOFTCAP_SPLITS if t * heads < SOFTCAP_SPLIT_BELOW and not narrow else 1
     part = torch.empty((t * heads * n_split * (vdim + 2),), dtype=F32, device=q.device) if n_split > 1 else None
     lib = _lib.load()
     _lib.check(lib.nvx_softcap_attn(_ptr(q), _ptr(k_cache), _ptr(v_cache), _fmt(q), _ptr(kv_indices), _ptr(kv_start), _ptr(kv_len),
@@ -1142,8 +1163,8 @@ def softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, layout: Step
                                     vdim, n_split, _ptr(part), int(window or 0), int(chunk or 0), _ptr(r1), _ptr(r2), _ptr(slopes), _ptr(k_rn), _ptr(v_turn),
                                     int(bool(v_interleaved)),
                                     _ptr(gate), gate.stride(0) if gate is not None else 0, int(gate_per_head), int(sink_score is not None),
-                                    float(sink_score or 0.0), layout.n_seq, int(bool(matrix_cores)), _stream()),
-               "nvx_softcap_attn")
+                                    float(sink_score or 0.0), _ptr(sinks), int(keep_first), float(out_mul), out.stride(0), layout.n_seq,
+                                    int(bool(matrix_cores)), _stream()), "nvx_softcap_attn")
     return out
 
 
@@ -1187,10 +1208,104 @@ def attn_prep_store(x, offsets, positions, q_w, k_w, norm_mode: str, eps: float,
     return q, v_turn
 
 
-def decay_scan(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int, vdim: int, act: str = "none", chunk: Optional[int] = None):
+class Turn:
+    """A rotation of the first `dims` entries of a head in pairs (m, m + dims / 2): its angles stand in columns first .. first + dims / 2 - 1
+    (cos) of a step's `table` (T, 2 n) as turn_table makes it, and n columns further on (sin)."""
+
+    __slots__ = ("table", "first", "dims")
+
+    def __init__(self, table, first: int, dims: int):
+        self.table, self.first, self.dims = table, int(first), int(dims)
+
+
+def _turn_args(turn: Optional[Turn], t: int, dim: int, what: str):
+    """(cos pointer, row stride, distance to the sin entries, rotated dims) of a launch."""
+    if turn is None or not turn.dims:
+        return None, 0, 0, 0
+    tab = turn.table
+    _dev(tab)
+    _f32c(tab, what + ": turn table")
+    n = tab.shape[1] // 2
+    _need(tab.shape == (t, 2 * n) and turn.dims % 2 == 0 and turn.dims <= dim and 0 <= turn.first and turn.first + turn.dims // 2 <= n,
+          what + ": the rotation lies outside its table, or is longer than a head")
+    return tab.data_ptr() + 4 * turn.first, 2 * n, n, turn.dims
+
+
+def turn_table(positions, freq):
+    """(T, 2 n) float32: cos | sin of positions[t] * freq[m] (freq: n float64), formed and reduced in double precision.  One launch a step
+    serves every layer (and every rotation: freq may be several tables side by side)."""
+    _dev(positions, freq)
+    _need(positions.dtype == torch.int64 and positions.is_contiguous() and positions.dim() == 1, "turn_table: positions must be int64 (T)")
+    _need(freq.dtype == torch.float64 and freq.is_contiguous() and freq.dim() == 1 and freq.numel() > 0, "turn_table: freq must be float64")
+    t, n = positions.numel(), freq.numel()
+    out = torch.empty((t, 2 * n), dtype=F32, device=positions.device)
+    lib = _lib.load()
+    _lib.check(lib.nvx_turn_table(_ptr(positions), _ptr(freq), n, _ptr(out), t, _stream()), "nvx_turn_table")
+    return out
+
+
+def conv_attn_prep(x, w, state, layout: StepLayout, turn: Optional[Turn], eps: float, slots, k_cache, v_cache, heads: int, kv_heads: int, dim: int,
+                   vdim: int, norm: bool = True):
+    """x (T, heads * dim + kv_heads * (dim + vdim)) = q | k | v as projected (rows may be slices of wider rows).  Every channel passes a causal
+    convolution over its sequence (w (taps, channels) float32, row j multiplying the input taps - 1 - j tokens back; state (slots, taps - 1,
+    channels) float32, read for the inputs before this step and replaced by each sequence's last ones; None with one tap), every query and
+    key head is rotated by its token's angles (`turn`, None: not) and, with `norm`, divided by its root mean square; keys and values go to
+    k_cache[slots] / v_cache[slots].  Float32 up to what is stored.  Returns the queries (T, heads * dim) in x's format."""
+    _dev(x, w, state, slots, k_cache, v_cache)
+    _need(x.dim() == 2 and x.stride(1) == 1, "conv_attn_prep: x must be (T, channels) with unit inner stride")
+    t, ch = x.shape
+    _f32c(w, "conv_attn_prep: w")
+    taps = w.shape[0]
+    _need(ch == heads * dim + kv_heads * (dim + vdim) and w.dim() == 2 and w.shape[1] == ch and t == layout.n_tok, "conv_attn_prep: shapes")
+    n_slots = 0
+    if taps > 1:
+        _f32c(state, "conv_attn_prep: state")
+        _need(state.dim() == 3 and state.shape[1:] == (taps - 1, ch), "conv_attn_prep: state shape")
+        n_slots = state.shape[0]
+    _need(slots.dtype == torch.int64 and slots.is_contiguous() and slots.numel() == t, "conv_attn_prep: slots must be int64 (T)")
+    rows = k_cache.shape[0]
+    _need(k_cache.dtype == x.dtype and v_cache.dtype == x.dtype and k_cache.is_contiguous() and v_cache.is_contiguous() and
+          k_cache.shape == (rows, kv_heads * dim) and v_cache.shape == (rows, kv_heads * vdim), "conv_attn_prep: cache shapes")
+    q = torch.empty((t, heads * dim), dtype=x.dtype, device=x.device)
+    lib = _lib.load()
+    _lib.check(lib.nvx_conv_attn_prep(_ptr(x), x.stride(0), _fmt(x), _ptr(w), taps, _ptr(state) if taps > 1 else None, n_slots, _ptr(layout.tok_seq),
+                                      *_layout_args(layout), *_turn_args(turn, t, dim, "conv_attn_prep"), int(bool(norm)), float(eps), _ptr(slots), _ptr(q),
+                                      _ptr(k_cache), _ptr(v_cache), t, layout.n_seq, heads, kv_heads, dim, vdim, _stream()), "nvx_conv_attn_prep")
+    return q
+
+
+def decay_step_fits(layout: StepLayout, dim: int, vdim: int) -> bool:
+    """Whether decay_step serves this step: one token per sequence, and heads it is built for."""
+    return layout.qo_indptr is None and dim <= 4096 and vdim <= (_lib.load().nvx_decay_step_max_vdim() if vdim % 4 == 0 else 256)
+
+
+def decay_step(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int, vdim: int, eps: float, act: str = "none", turn: Optional[Turn] = None,
+               k_mul: float = 1.0, gate_off: Optional[int] = None, gate_kind: str = "none", mul: float = 1.0, out=None):
+    """decay_scan and head_norm_gate (without a weight) in one launch, for a step of one token per sequence: the memory is read and written
+    once and the read-out leaves normed and gated.  The gate's pre-activations are the heads * vdim columns of x at `gate_off`.  Returns (T,
+    heads * vdim) in x's format: `out` where it is given (rows may be slices of a wider buffer's)."""
+    _dev(x, decay, mem)
+    _need(x.dim() == 2 and x.stride(1) == 1 and x.shape[0] == layout.n_tok and layout.qo_indptr is None, "decay_step: x must be (T, columns), one token per sequence")
+    _f32c(decay, "decay_step: decay")
+    _f32c(mem, "decay_step: mem")
+    n_slots, t = mem.shape[0], x.shape[0]
+    _need(decay.numel() == heads and mem.shape == (n_slots, heads, dim, vdim), "decay_step: shapes")
+    kind = {"none": 0, "sigmoid": 1, "silu": 2}[gate_kind]
+    _need(kind == 0 or gate_off is not None, "decay_step: a gate needs its columns")
+    out = _out_rows(out, t, heads * vdim, x.dtype, x.device, "decay_step")
+    lib = _lib.load()
+    _lib.check(lib.nvx_decay_step(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], {"none": 0, "silu": 1}[act], _ptr(decay), _ptr(mem),
+                                  n_slots, _ptr(layout.pos0), _ptr(layout.state_slot), t, heads, dim, vdim, *_turn_args(turn, t, dim, "decay_step"),
+                                  float(k_mul), float(eps), int(gate_off or 0), kind, float(mul), _ptr(out), out.stride(0), _stream()), "nvx_decay_step")
+    return out
+
+
+def decay_scan(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int, vdim: int, act: str = "none", chunk: Optional[int] = None,
+               turn=None, k_mul: float = 1.0):
     """Linear attention with one constant decay per head.  x (T, columns): q, k (heads * dim each) and v (heads * vdim) at the
     three column `offsets`, passed through `act` ("none" or "silu") first; decay (heads) float32; mem (slots, heads, dim, vdim)
     float32, continued and written back.  S <- decay S + k v^T, read-out S^T q.  Returns (T, heads, vdim) float32.
+    `turn` (a Turn): queries and keys are rotated by their tokens' angles as they are staged; keys are multiplied by `k_mul`.
     Ragged steps with long portions are cut into chunks of `chunk` tokens (default: by the step's shape; 0: never) that run side by
     side: the result is the same up to the rounding of decay^n against n multiplications."""
     _dev(x, decay, mem)
@@ -1206,7 +1321,7 @@ def decay_scan(x, offsets, decay, mem, layout: StepLayout, heads: int, dim: int,
     lib = _lib.load()
     _lib.check(lib.nvx_decay_scan(_ptr(x), x.stride(0), _fmt(x), offsets[0], offsets[1], offsets[2], {"none": 0, "silu": 1}[act], _ptr(decay),
                                   _ptr(mem), n_slots, *_layout_args(layout), _ptr(out), t, layout.n_seq, heads, dim, vdim, chunk, n_chunks,
-                                  _ptr(ws), _stream()), "nvx_decay_scan")
+                                  _ptr(ws), *_turn_args(turn, t, dim, "decay_scan"), float(k_mul), _stream()), "nvx_decay_scan")
     return out
 
 
@@ -1337,16 +1452,20 @@ def moe_scatter_rows(h, wts, dst, spare_rows: int = 0):
     return xs
 
 
-def moe_glu(gu, limit: float, alpha: float, shift: float = 1.0):
+def moe_glu(gu, limit: float, alpha: float, shift: float = 1.0, row_gate=None, out=None):
     """gu (rows, 2 * ff) = gate | up pre-activations -> min(g, limit) * sigmoid(alpha * min(g, limit)) * (clamp(u, +-limit) + shift)
-    (limit = inf, alpha = 1, shift = 0: silu(g) * u)."""
-    _dev(gu)
-    _need(gu.dim() == 2 and gu.is_contiguous() and gu.shape[1] % 2 == 0, "moe_glu: gu must be contiguous (rows, 2 * ff)")
-    y = torch.empty((gu.shape[0], gu.shape[1] // 2), dtype=gu.dtype, device=gu.device)
+    (limit = inf, alpha = 1, shift = 0: silu(g) * u), times sigmoid(row_gate[r]) if `row_gate` (rows, float32, any stride) is given.  Rows of
+    gu and of `out` may be slices of wider rows."""
+    _dev(gu, row_gate)
+    _need(gu.dim() == 2 and gu.stride(1) == 1 and gu.shape[1] % 2 == 0, "moe_glu: gu must be (rows, 2 * ff) with unit inner stride")
+    rows, ff = gu.shape[0], gu.shape[1] // 2
+    _need(row_gate is None or (row_gate.dtype == F32 and row_gate.shape == (rows,)), "moe_glu: row_gate must be float32 (rows)")
+    out = _out_rows(out, rows, ff, gu.dtype, gu.device, "moe_glu")
     lib = _lib.load()
-    _lib.check(lib.nvx_moe_glu(_ptr(gu), _fmt(gu), float(limit), float(alpha), float(shift), _ptr(y), gu.shape[0], gu.shape[1] // 2, _stream()),
-               "nvx_moe_glu")
-    return y
+    # (torch leaves the stride of a dimension of one entry free: it is not read where there is one row)
+    _lib.check(lib.nvx_moe_glu(_ptr(gu), max(gu.stride(0), 2 * ff), _fmt(gu), float(limit), float(alpha), float(shift), _ptr(row_gate),
+                               max(row_gate.stride(0), 1) if row_gate is not None else 0, _ptr(out), max(out.stride(0), ff), rows, ff, _stream()), "nvx_moe_glu")
+    return out
 
 
 def moe_gather_rows(ys, dst, wts=None):
@@ -1493,16 +1612,16 @@ def latent_rope_prep(x, offsets, positions, freq, mag: float, w_kv, eps: float, 
 
 
 def moe_route_softmax(logits, top: int, n_groups: int = 0, keep_groups: int = 0, norm_eps: float = 0.0):
-    """logits (T, experts) float32 -> (ids (T, top) int32, weights (T, top) float32).  Scores are the softmax over all experts; with
+    """logits (T, experts) float32 (rows may be slices of wider rows) -> (ids (T, top) int32, weights (T, top) float32).  Scores are the softmax over all experts; with
     n_groups > 1 the experts form equal groups of neighbours, a group counts as its best score, and only experts of the keep_groups
     best groups can be chosen; the `top` largest scores are taken (ties: the lower id) and divided by their sum + norm_eps."""
     _dev(logits)
-    _f32c(logits, "moe_route_softmax: logits")
+    _need(logits.dtype == F32 and logits.dim() == 2 and logits.stride(1) == 1, "moe_route_softmax: logits must be float32 with unit inner stride")
     t, n_exp = logits.shape
     idx = torch.empty((t, top), dtype=torch.int32, device=logits.device)
     wts = torch.empty((t, top), dtype=F32, device=logits.device)
     lib = _lib.load()
-    _lib.check(lib.nvx_moe_route_softmax(_ptr(logits), t, n_exp, top, int(n_groups or 0), int(keep_groups or 0), float(norm_eps), _ptr(idx),
+    _lib.check(lib.nvx_moe_route_softmax(_ptr(logits), max(logits.stride(0), n_exp), t, n_exp, top, int(n_groups or 0), int(keep_groups or 0), float(norm_eps), _ptr(idx),
                                          _ptr(wts), _stream()), "nvx_moe_route_softmax")
     return idx, wts
 
@@ -1510,8 +1629,12 @@ def moe_route_softmax(logits, top: int, n_groups: int = 0, keep_groups: int = 0,
 # ---------------------------------------------------------------------------------------------
 # plain pre-normed stream with its embedding sum, tied keys and values, gated linear attention, the sigmoid router with groups
 # ---------------------------------------------------------------------------------------------
-def _row_end(t: int, width: int, w, split: bool, dtype, device, what: str):
+def _row_end(t: int, width: int, w, split: bool, dtype, device, what: str, w_bias=None):
     """The row output of residual_norm and embed_sum: none, the normed row, or the [hi | lo] pair."""
+    if w_bias is not None:
+        _dev(w_bias)
+        _f32c(w_bias, what + ": w_bias")
+        _need(w is not None and w_bias.numel() == width, what + ": the layer norm's bias goes with its weight")
     if w is None and not split:
         return None
     if w is not None:
@@ -1521,9 +1644,10 @@ def _row_end(t: int, width: int, w, split: bool, dtype, device, what: str):
     return torch.empty((t, 2 * width if split else width), dtype=dtype, device=device)
 
 
-def residual_norm(x, y=None, y2=None, add=None, bias=None, w=None, eps: float = 0.0, split: bool = False, dtype=None, out=None):
+def residual_norm(x, y=None, y2=None, add=None, bias=None, w=None, eps: float = 0.0, split: bool = False, dtype=None, out=None, w_bias=None):
     """v = x (+ y) (+ y2) (+ add) (+ bias): x, add (T, width) and bias (width) float32, y and y2 (T, width) in the activations' format
-    `dtype` (default: y's).  v replaces x, or goes to `out`.  Returns v / rms(v) * w if `w` (width, float32) is given, [hi | lo] (T, 2 *
+    `dtype` (default: y's).  v replaces x, or goes to `out`.  Returns v / rms(v) * w if `w` (width, float32) is given (with `w_bias` too: the
+    layer norm (v - mean) / sqrt(variance + eps) * w + w_bias), [hi | lo] (T, 2 *
     width) with hi = v rounded to `dtype` and lo = what that lost if `split`, else None."""
     _dev(x, y, y2, add, bias, out)
     _f32c(x, "residual_norm: x")
@@ -1536,16 +1660,16 @@ def residual_norm(x, y=None, y2=None, add=None, bias=None, w=None, eps: float = 
             _need(tuple(r.shape) == shape, f"residual_norm: {name} shape")
     dtype = dtype or (y.dtype if y is not None else None)
     _need(dtype in _FMT and all(r is None or r.dtype == dtype for r in (y, y2)), "residual_norm: y, y2 and the output share one format")
-    h = _row_end(t, width, w, split, dtype, x.device, "residual_norm")
+    h = _row_end(t, width, w, split, dtype, x.device, "residual_norm", w_bias)
     lib = _lib.load()
     _lib.check(lib.nvx_residual_norm(_ptr(x), _ptr(y), y.stride(0) if y is not None else 0, _ptr(y2), y2.stride(0) if y2 is not None else 0, _ptr(add),
-                                     _ptr(bias), _FMT[dtype], _ptr(x if out is None else out), _ptr(w), float(eps), int(split), _ptr(h), t, width,
-                                     _stream()), "nvx_residual_norm")
+                                     _ptr(bias), _FMT[dtype], _ptr(x if out is None else out), _ptr(w), _ptr(w_bias), float(eps), int(split), _ptr(h), t,
+                                     width, _stream()), "nvx_residual_norm")
     return h
 
 
 def embed_sum(ids, table, layout: Optional[StepLayout] = None, pair=None, mul_prev: int = 0, mul_cur: int = 0, prev_id=None, pos_table=None,
-              positions=None, w=None, eps: float = 0.0, split: bool = False):
+              positions=None, w=None, eps: float = 0.0, split: bool = False, w_bias=None):
     """x = table[ids] (+ pair[r]) (+ pos_table[positions]) in float32, r = (previous id * mul_prev + id * mul_cur) mod buckets with buckets
     = pair.shape[0] - 1, and the last row for a sequence's first token; prev_id (slots, 1) float32 carries every sequence's last id from
     step to step.  Returns (x, h), h as residual_norm's result."""
@@ -1565,11 +1689,11 @@ def embed_sum(ids, table, layout: Optional[StepLayout] = None, pair=None, mul_pr
     if pos_table is not None:
         _need(positions is not None and positions.dtype == torch.int64 and positions.is_contiguous() and positions.numel() == t, "embed_sum: positions must be int64 (T)")
     x = torch.empty((t, width), dtype=F32, device=ids.device)
-    h = _row_end(t, width, w, split, table.dtype, ids.device, "embed_sum")
+    h = _row_end(t, width, w, split, table.dtype, ids.device, "embed_sum", w_bias)
     lib = _lib.load()
     _lib.check(lib.nvx_embed_sum(_ptr(ids), _ptr(table), _fmt(table), table.shape[0], _ptr(pair), pair.shape[0] - 1 if pair is not None else 0, int(mul_prev),
                                  int(mul_cur), _ptr(prev_id), n_slots, _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0,
-                                 _ptr(positions) if pos_table is not None else None, *la, _ptr(x), _ptr(w), float(eps), int(split), _ptr(h), t,
+                                 _ptr(positions) if pos_table is not None else None, *la, _ptr(x), _ptr(w), _ptr(w_bias), float(eps), int(split), _ptr(h), t,
                                  layout.n_seq if layout is not None else t, width, _stream()), "nvx_embed_sum")
     return x, h
 

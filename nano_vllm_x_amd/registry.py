@@ -39,9 +39,14 @@ def _zenedra():
     return ZenedraConfig.from_dict, ZenedraForCausalLM
 
 
+def _fikotar():
+    from .fikotar import FikotarConfig, FikotarForCausalLM
+    return FikotarConfig.from_dict, FikotarForCausalLM
+
+
 # architecture name (config.json "architectures"[0] or "architecture") -> loader of (config reader, model class)
 ARCHITECTURES = {"Qwen3ForCausalLM": _qwen3, "Kabidra": _kabidra, "Meronex": _meronex, "Gibavik": _gibavik, "Ladusun": _ladusun,
-                 "Zenedra": _zenedra}
+                 "Zenedra": _zenedra, "Fikotar": _fikotar}
 
 
 def architecture_of(config: dict) -> str:

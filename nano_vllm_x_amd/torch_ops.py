@@ -71,7 +71,7 @@ _DEFS = {
     # gated residuals with grouped norms, matrix-memory recurrences, capped attention, mixtures of experts
     "gated_residual_norm": "(Tensor(a!) x, Tensor? y, Tensor? gate, Tensor? gate_bias, float mult, Tensor? w_norm, int groups, float eps, "
                            "Tensor? y2, Tensor? w_y, Tensor? w_y2, ScalarType dtype) -> Tensor?",
-    "head_norm_gate": "(Tensor o, Tensor w, float eps, Tensor? gate, str kind, ScalarType dtype) -> Tensor",
+    "head_norm_gate": "(Tensor o, Tensor? w, float eps, Tensor? gate, str kind, ScalarType dtype, float mul=1.0) -> Tensor",
     "short_conv_silu": "(Tensor x, Tensor w, Tensor(a!)? state, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq) -> Tensor",
     "token_shift_mix": "(Tensor h, Tensor mu, Tensor(a!) state, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq) -> Tensor",
     "mlstm_scan": "(Tensor x, int q_off, int k_off, int v_off, Tensor gates, Tensor gate_bias, float cap, Tensor(a!) mem, Tensor(b!) norm, "
@@ -85,13 +85,13 @@ _DEFS = {
     "softcap_attn": "(Tensor q, Tensor k_cache, Tensor v_cache, Tensor kv_indices, Tensor kv_start, Tensor kv_len, Tensor pos0, "
                     "Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq, float scale, float cap, int heads, int kv_heads, int dim, int vdim, "
                     "int window=0, Tensor? r1=None, Tensor? r2=None, Tensor? v_turn=None, bool v_interleaved=False, Tensor? gate=None, "
-                    "float? sink_score=None, int chunk=0, Tensor? slopes=None, Tensor? k_rn=None) -> Tensor",
+                    "float? sink_score=None, int chunk=0, Tensor? slopes=None, Tensor? k_rn=None, Tensor? sinks=None, int keep_first=0, float out_mul=1.0) -> Tensor",
     # post-normed stream, query/key norms with rotated values, decayed linear attention, experts with weights on their outputs
     "attn_prep_store": "(Tensor x, int q_off, int k_off, int v_off, Tensor positions, Tensor? q_w, Tensor? k_w, str norm_mode, float eps, "
                        "Tensor? freq, int rot_dims, bool interleaved, Tensor? vfreq, Tensor? slots, Tensor(a!)? k_cache, Tensor(b!)? v_cache, "
                        "int heads, int kv_heads, int dim, int vdim) -> (Tensor, Tensor?)",
     "decay_scan": "(Tensor x, int q_off, int k_off, int v_off, Tensor decay, Tensor(a!) mem, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, "
-                  "Tensor? tok_seq, int heads, int dim, int vdim, str act) -> Tensor",
+                  "Tensor? tok_seq, int heads, int dim, int vdim, str act, Tensor? turn_table=None, int turn_first=0, int rot_dims=0, float k_mul=1.0) -> Tensor",
     "postnorm_residual": "(Tensor(a!) x, Tensor? y, Tensor? w_post, float eps, Tensor? y2, float a, float b, Tensor? w_next, ScalarType dtype) -> Tensor",
     "embed_scale": "(Tensor ids, Tensor table, float scale) -> (Tensor, Tensor)",
     "tanh_cap": "(Tensor z, float cap) -> Tensor",
@@ -100,7 +100,7 @@ _DEFS = {
                        "bool weight_out=False) -> Tensor",
     "moe_order": "(Tensor idx, int n_exp) -> (Tensor, Tensor)",
     "moe_scatter_rows": "(Tensor h, Tensor? wts, Tensor dst) -> Tensor",
-    "moe_glu": "(Tensor gu, float limit, float alpha, float shift=1.0) -> Tensor",
+    "moe_glu": "(Tensor gu, float limit, float alpha, float shift=1.0, Tensor? row_gate=None) -> Tensor",
     "moe_gather_rows": "(Tensor ys, Tensor dst, Tensor? wts=None) -> Tensor",
     "skinny_proj": "(Tensor x, Tensor w, str in_act, Tensor? bias=None, str out_act='none', float power=1.0) -> Tensor",
     # several residual streams, the real-gated recurrence, a latent with a rotated key part, the softmax router with groups
@@ -115,15 +115,22 @@ _DEFS = {
                         "Tensor slots, Tensor(a!) cache, int heads, int dim, int rot) -> (Tensor, Tensor)",
     "moe_route_softmax": "(Tensor logits, int top, int n_groups, int keep_groups, float norm_eps) -> (Tensor, Tensor)",
     # plain pre-normed stream with its embedding sum, tied keys and values, gated linear attention, the sigmoid router with groups
-    "residual_norm": "(Tensor(a!) x, Tensor? y, Tensor? y2, Tensor? add, Tensor? bias, Tensor? w, float eps, bool split, ScalarType dtype) -> Tensor?",
+    "residual_norm": "(Tensor(a!) x, Tensor? y, Tensor? y2, Tensor? add, Tensor? bias, Tensor? w, float eps, bool split, ScalarType dtype, Tensor? w_bias=None) -> Tensor?",
     "embed_sum": "(Tensor ids, Tensor table, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq, Tensor? pair, int mul_prev, int mul_cur, "
-                 "Tensor(a!)? prev_id, Tensor? pos_table, Tensor? positions, Tensor? w, float eps, bool split) -> (Tensor, Tensor?)",
+                 "Tensor(a!)? prev_id, Tensor? pos_table, Tensor? positions, Tensor? w, float eps, bool split, Tensor? w_bias=None) -> (Tensor, Tensor?)",
     "tied_prep_store": "(Tensor x, int q_off, int k_off, Tensor q_w, Tensor k_w, float eps, Tensor slots, Tensor(a!) k_cache, Tensor(b!) k_rn, "
                        "int heads, int kv_heads, int dim) -> Tensor",
     "gla_scan": "(Tensor x, int q_off, int k_off, int v_off, Tensor alpha, Tensor(a!) mem, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, "
                 "Tensor? tok_seq, int heads, int dim, int vdim, float q_mul) -> Tensor",
     "moe_route_sigmoid": "(Tensor logits, Tensor correction, int top, int n_groups, int keep_groups, float scale) -> (Tensor, Tensor)",
     "gelu_glu": "(Tensor gu) -> Tensor",
+    # convolved queries, keys and values, a step's table of rotations, the decayed memory for single tokens
+    "turn_table": "(Tensor positions, Tensor freq) -> Tensor",
+    "conv_attn_prep": "(Tensor x, Tensor w, Tensor(a!)? state, Tensor pos0, Tensor state_slot, Tensor? qo_indptr, Tensor? tok_seq, Tensor? turn_table, "
+                      "int turn_first, int rot_dims, float eps, Tensor slots, Tensor(b!) k_cache, Tensor(c!) v_cache, int heads, int kv_heads, int dim, "
+                      "int vdim, bool norm=True) -> Tensor",
+    "decay_step": "(Tensor x, int q_off, int k_off, int v_off, Tensor decay, Tensor(a!) mem, Tensor pos0, Tensor state_slot, int heads, int dim, int vdim, "
+                  "float eps, str act, Tensor? turn_table, int turn_first, int rot_dims, float k_mul, int gate_off, str gate_kind, float mul=1.0) -> Tensor",
 }
 for _name, _sig in _DEFS.items():
     _LIB.define(_name + _sig)
@@ -287,8 +294,8 @@ def _gated_residual_norm(x, y, gate, gate_bias, mult, w_norm, groups, eps, y2, w
                                    w_y2=w_y2, dtype=dtype)
 
 
-def _head_norm_gate(o, w, eps, gate, kind, dtype):
-    return ops.head_norm_gate(o, w, eps, gate=gate, kind=kind, dtype=dtype)
+def _head_norm_gate(o, w, eps, gate, kind, dtype, mul=1.0):
+    return ops.head_norm_gate(o, w, eps, gate=gate, kind=kind, dtype=dtype, mul=mul)
 
 
 def _short_conv_silu(x, w, state, pos0, state_slot, qo_indptr, tok_seq):
@@ -318,10 +325,11 @@ def _rope_vnorm_store(qkv, positions, freq, mag, rot_dims, eps, slots, k_cache, 
 
 
 def _softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, pos0, state_slot, qo_indptr, tok_seq, scale, cap, heads, kv_heads, dim, vdim,
-                  window=0, r1=None, r2=None, v_turn=None, v_interleaved=False, gate=None, sink_score=None, chunk=0, slopes=None, k_rn=None):
+                  window=0, r1=None, r2=None, v_turn=None, v_interleaved=False, gate=None, sink_score=None, chunk=0, slopes=None, k_rn=None, sinks=None,
+                  keep_first=0, out_mul=1.0):
     return ops.softcap_attn(q, k_cache, v_cache, kv_indices, kv_start, kv_len, _layout(q.shape[0], pos0, state_slot, qo_indptr, tok_seq), scale, cap,
                             heads, kv_heads, dim, vdim, window=window, r1=r1, r2=r2, v_turn=v_turn, v_interleaved=v_interleaved, gate=gate,
-                            sink_score=sink_score, chunk=chunk, slopes=slopes, k_rn=k_rn)
+                            sink_score=sink_score, chunk=chunk, slopes=slopes, k_rn=k_rn, sinks=sinks, keep_first=keep_first, out_mul=out_mul)
 
 
 def _attn_prep_store(x, q_off, k_off, v_off, positions, q_w, k_w, norm_mode, eps, freq, rot_dims, interleaved, vfreq, slots, k_cache, v_cache,
@@ -330,8 +338,10 @@ def _attn_prep_store(x, q_off, k_off, v_off, positions, q_w, k_w, norm_mode, eps
                                v_cache, heads, kv_heads, dim, vdim)
 
 
-def _decay_scan(x, q_off, k_off, v_off, decay, mem, pos0, state_slot, qo_indptr, tok_seq, heads, dim, vdim, act):
-    return ops.decay_scan(x, (q_off, k_off, v_off), decay, mem, _layout(x.shape[0], pos0, state_slot, qo_indptr, tok_seq), heads, dim, vdim, act=act)
+def _decay_scan(x, q_off, k_off, v_off, decay, mem, pos0, state_slot, qo_indptr, tok_seq, heads, dim, vdim, act, turn_table=None,
+                turn_first=0, rot_dims=0, k_mul=1.0):
+    return ops.decay_scan(x, (q_off, k_off, v_off), decay, mem, _layout(x.shape[0], pos0, state_slot, qo_indptr, tok_seq), heads, dim, vdim, act=act,
+                          turn=_turn(turn_table, turn_first, rot_dims), k_mul=k_mul)
 
 
 def _postnorm_residual(x, y, w_post, eps, y2, a, b, w_next, dtype):
@@ -362,8 +372,8 @@ def _moe_scatter_rows(h, wts, dst):
     return ops.moe_scatter_rows(h, wts, dst)
 
 
-def _moe_glu(gu, limit, alpha, shift=1.0):
-    return ops.moe_glu(gu, limit, alpha, shift)
+def _moe_glu(gu, limit, alpha, shift=1.0, row_gate=None):
+    return ops.moe_glu(gu, limit, alpha, shift, row_gate=row_gate)
 
 
 def _moe_gather_rows(ys, dst, wts=None):
@@ -398,13 +408,13 @@ def _moe_route_softmax(logits, top, n_groups, keep_groups, norm_eps):
     return ops.moe_route_softmax(logits, top, n_groups, keep_groups, norm_eps)
 
 
-def _residual_norm(x, y, y2, add, bias, w, eps, split, dtype):
-    return ops.residual_norm(x, y, y2, add=add, bias=bias, w=w, eps=eps, split=split, dtype=dtype)
+def _residual_norm(x, y, y2, add, bias, w, eps, split, dtype, w_bias=None):
+    return ops.residual_norm(x, y, y2, add=add, bias=bias, w=w, eps=eps, split=split, dtype=dtype, w_bias=w_bias)
 
 
-def _embed_sum(ids, table, pos0, state_slot, qo_indptr, tok_seq, pair, mul_prev, mul_cur, prev_id, pos_table, positions, w, eps, split):
+def _embed_sum(ids, table, pos0, state_slot, qo_indptr, tok_seq, pair, mul_prev, mul_cur, prev_id, pos_table, positions, w, eps, split, w_bias=None):
     return ops.embed_sum(ids, table, _layout(ids.numel(), pos0, state_slot, qo_indptr, tok_seq), pair=pair, mul_prev=mul_prev, mul_cur=mul_cur,
-                         prev_id=prev_id, pos_table=pos_table, positions=positions, w=w, eps=eps, split=split)
+                         prev_id=prev_id, pos_table=pos_table, positions=positions, w=w, eps=eps, split=split, w_bias=w_bias)
 
 
 def _tied_prep_store(x, q_off, k_off, q_w, k_w, eps, slots, k_cache, k_rn, heads, kv_heads, dim):
@@ -421,6 +431,26 @@ def _moe_route_sigmoid(logits, correction, top, n_groups, keep_groups, scale):
 
 def _gelu_glu(gu):
     return ops.gelu_glu(gu)
+
+
+def _turn(table, first, dims):
+    return None if table is None else ops.Turn(table, first, dims)
+
+
+def _turn_table(positions, freq):
+    return ops.turn_table(positions, freq)
+
+
+def _conv_attn_prep(x, w, state, pos0, state_slot, qo_indptr, tok_seq, turn_table, turn_first, rot_dims, eps, slots, k_cache, v_cache, heads, kv_heads,
+                    dim, vdim, norm=True):
+    return ops.conv_attn_prep(x, w, state, _layout(x.shape[0], pos0, state_slot, qo_indptr, tok_seq), _turn(turn_table, turn_first, rot_dims), eps, slots,
+                              k_cache, v_cache, heads, kv_heads, dim, vdim, norm=norm)
+
+
+def _decay_step(x, q_off, k_off, v_off, decay, mem, pos0, state_slot, heads, dim, vdim, eps, act, turn_table, turn_first, rot_dims, k_mul, gate_off,
+                gate_kind, mul=1.0):
+    return ops.decay_step(x, (q_off, k_off, v_off), decay, mem, _layout(x.shape[0], pos0, state_slot, None, None), heads, dim, vdim, eps, act=act,
+                          turn=_turn(turn_table, turn_first, rot_dims), k_mul=k_mul, gate_off=gate_off, gate_kind=gate_kind, mul=mul)
 
 
 for _name in _DEFS:
