@@ -1144,11 +1144,178 @@ def _zenedra_kernel_table(z, t_pre, n_dec, ctx, phases=("prefill", "decode")):
     return rows
 
 
+def _fikotar_config(z):
+    """Every layer attention and retention side by side on one norm: heads of 128 with 8 key/value heads behind four taps, a window of 512 keys
+    and four kept tokens, 64 rotated dimensions; retention heads with keys 64 and values 128 wide; eight experts of ff / 4, two a token,
+    beside a shared one of ff / 2, so that a token's feed-forward work equals the dense model's."""
+    hd = z["width"] // 128
+    left = {"heads": z["heads"], "kv_heads": 8, "dim": 128, "vdim": 128, "conv": 4, "scale": 0.125, "mask": {"size": 512, "keep_first": 4},
+            "rot": {"dims": 64, "base": 5e5, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    right = {"heads": hd, "dim": 64, "vdim": 128, "decay": [1.0 - 2.0 ** -(3 + j % 8) for j in range(hd)], "rot": {"dims": 64, "base": 1e4}}
+    moe = {"kind": "moe", "expert": {"ff": z["ff"] // 4}, "router": {"experts": 8, "top": 2}, "shared": {"ff": z["ff"] // 2}}
+    one = {"type": "parallel", "mixer": {"left": left, "right": right, "left_scale": 0.5, "right_scale": 1.0}, "mlp": moe}
+    return {"architecture": "Fikotar", "vocab": z["vocab"], "width": z["width"], "norm": {"eps": 1e-5}, "logit_scale": 0.25,
+            "layers": [json.loads(json.dumps(one)) for _ in range(z["layers"])]}
+
+
+def _graph_us(fn, calls=20, reps=5):
+    """Device time of one call: `calls` of them in a captured graph, so that the host's launches are no part of it."""
+    fn()
+    torch.cuda.synchronize()
+    g = torch.cuda.CUDAGraph()
+    with torch.cuda.graph(g):
+        for _ in range(calls):
+            fn()
+    g.replay()
+    torch.cuda.synchronize()
+    a, b = torch.cuda.Event(enable_timing=True), torch.cuda.Event(enable_timing=True)
+    a.record()
+    for _ in range(reps):
+        g.replay()
+    b.record()
+    b.synchronize()
+    return a.elapsed_time(b) * 1e3 / (calls * reps)
+
+
+def _fikotar_kernel_table(z, t_pre, n_dec, ctx, phases=("prefill", "decode")):
+    """Each kernel of Fikotar beside the like kernel of Gibavik, Zenedra, Ladusun or Qwen3 at the same shape: device time in a captured graph
+    (both sides), and the fraction of its roofline (HBM bytes it must move at 8 TB/s; attention and products in prefill: their multiply-adds
+    at the dense bf16 MFMA peak; the memories in prefill: their multiply-adds at the float32 vector peak, since their states are float32).
+    At decode shapes operands that a kernel reads over and over may stay in the caches: such fractions can pass one."""
+    from nano_vllm_x_amd import ops
+    dev, bf = torch.device("cuda"), torch.bfloat16
+    w, ff, h = z["width"], z["ff"], z["heads"]
+    hd, window, keep, taps = w // 128, 512, 4, 4
+    rows = []
+
+    def layout(n_seq, q_len, pos0):
+        p = torch.full((n_seq,), pos0, dtype=torch.int64, device=dev)
+        sl = torch.arange(n_seq, dtype=torch.int32, device=dev)
+        if q_len == 1:
+            return ops.StepLayout(n_seq, n_seq, p, sl)
+        qo = torch.arange(0, n_seq + 1, dtype=torch.int32, device=dev) * q_len
+        return ops.StepLayout(n_seq * q_len, n_seq, p, sl, qo, torch.arange(n_seq, dtype=torch.int32, device=dev).repeat_interleave(q_len), max_q=q_len)
+
+    def add(name, phase, fn, bytes_=None, flops=None, like=None, peak=None):
+        print(f"[arch-compare]   {phase} {name}", file=sys.stderr, flush=True)
+        us = _graph_us(fn)
+        if bytes_:
+            frac, bound = bytes_ / (us * 1e-6) / (HBM_PEAK_GBS * 1e9), "HBM"
+        else:
+            frac, bound = flops / (us * 1e-6) / ((peak or MFMA_BF16_PEAK_TFLOPS) * 1e12), "MFMA" if peak is None else "fp32 VALU"
+        rows.append({"kernel": name, "phase": phase, "us": round(us, 1), "of_roofline": round(frac, 3), "bound": bound, "like": like})
+
+    for phase, (n_seq, q_len, pos0) in (("prefill", (max(t_pre // 1024, 1), 1024, 0)), ("decode", (n_dec, 1, ctx))):
+        if phase not in phases:
+            continue
+        t = n_seq * q_len
+        dec = phase == "decode"
+        lay = layout(n_seq, q_len, pos0)
+        y, y2, x = torch.randn(t, w, device=dev).to(bf), torch.randn(t, w, device=dev).to(bf), torch.randn(t, w, device=dev)
+        one, wv = torch.ones(1, device=dev), torch.ones(w, device=dev)
+        zx = torch.zeros(t, w, device=dev)
+        # both ends of a layer: 2 B per result, 4 B of stream read and written, 2 B of the next layer's rows
+        add("residual_norm, two results, layer norm", phase, lambda: ops.residual_norm(zx, y, y2, w=wv, w_bias=wv, eps=1e-5), bytes_=t * w * 14, like="residual_norm, two results")
+        add("zenedra residual_norm, two results", phase, lambda: ops.residual_norm(zx, y, y2, w=wv, eps=1e-5), bytes_=t * w * 14)
+        add("gibavik postnorm_residual, two results", phase, lambda: ops.postnorm_residual(zx, y=y, y2=y2, a=0.5, b=1.0, w_post=one, eps=1e-5), bytes_=t * w * 14)
+        table = torch.randn(z["vocab"], w, device=dev).to(bf)
+        ids = torch.randint(0, z["vocab"], (t,), device=dev)
+        add("embed_sum, layer norm", phase, lambda: ops.embed_sum(ids, table, w=wv, w_bias=wv, eps=1e-5), bytes_=t * w * 8, like="embed_scale")
+        add("gibavik embed_scale", phase, lambda: ops.embed_scale(ids, table, 8.0), bytes_=t * w * 8)
+        pos = (torch.arange(t, device=dev) % q_len + pos0).to(torch.int64)
+        freq = torch.rand(64, device=dev, dtype=torch.float64)
+        add("turn_table (two rotations, once a step)", phase, lambda: ops.turn_table(pos, freq), bytes_=t * 128 * 4, like="(none)")
+        tab = ops.turn_table(pos, freq)
+        left_turn, right_turn = ops.Turn(tab, 0, 64), ops.Turn(tab, 32, 64)
+        # one product for everything a layer projects, one over everything it reads out
+        n_left, n_right = (h + 16) * 128, hd * (2 * 64 + 2 * 128)
+        k_out = h * 128 + hd * 128 + ff // 2
+        w_in, w_out = torch.randn(n_left + n_right + ff, w, device=dev).to(bf) * 0.02, torch.randn(w, k_out, device=dev).to(bf) * 0.02
+        o = torch.randn(t, k_out, device=dev).to(bf)
+        xp = torch.nn.functional.linear(y, w_in)
+        prod = lambda a, b: dict(bytes_=(a.numel() + b.numel() + t * b.shape[0]) * 2) if dec else dict(flops=2.0 * t * b.numel())
+        add("input product of a layer (library)", phase, lambda: torch.nn.functional.linear(y, w_in), **prod(y, w_in), like="(library)")
+        add("output product of a layer (library)", phase, lambda: torch.nn.functional.linear(o, w_out), **prod(o, w_out), like="(library)")
+        kv_len = pos0 + q_len
+        n_rows = n_seq * kv_len
+        kc, vc = torch.randn(n_rows, 8 * 128, device=dev).to(bf), torch.randn(n_rows, 8 * 128, device=dev).to(bf)
+        idx = torch.arange(n_rows, dtype=torch.int32, device=dev)
+        kv_start = torch.arange(n_seq, dtype=torch.int64, device=dev) * kv_len
+        kvl = torch.full((n_seq,), kv_len, dtype=torch.int32, device=dev)
+        slots = (torch.arange(t, device=dev) // q_len * kv_len + pos).to(torch.int64)
+        cw, cst = torch.randn(taps, n_left, device=dev), torch.zeros(n_seq + 1, taps - 1, n_left, device=dev)
+        add("conv_attn_prep (four taps, rotation, head norms)", phase, lambda: ops.conv_attn_prep(xp[:, :n_left], cw, cst, lay, left_turn, 1e-5, slots, kc, vc, h, 8, 128, 128),
+            bytes_=t * n_left * 4 + n_seq * (taps - 1) * n_left * (8 if dec else 4), like="attn_prep_store")
+        qn = torch.ones(128, device=dev)
+        add("gibavik attn_prep_store (head norms, rotation)", phase, lambda: ops.attn_prep_store(xp, (0, h * 128, (h + 8) * 128), pos, qn, qn, "head", 1e-5, freq[:32].contiguous(), 64,
+            False, None, slots, kc, vc, h, 8, 128, 128), bytes_=t * n_left * 4)
+        q128 = torch.randn(t, h * 128, device=dev).to(bf)
+        sinks = torch.zeros(h, device=dev)
+        g128 = torch.randn(t, h * 128, device=dev).to(bf)
+        vturn = torch.randn(t, 128, device=dev)
+        att = lambda **kw: ops.softcap_attn(q128, kc, vc, idx, kv_start, kvl, lay, 0.125, 0.0, h, 8, 128, 128, **kw)
+        if dec:
+            seen, io = n_seq * min(kv_len, window) * 8 * 128 * 4, 2 * t * h * 128 * 2
+            cost = lambda keys, gate=0: dict(bytes_=keys + io + gate)
+            all_keys = n_rows * 8 * 128 * 4
+        else:
+            pairs, pairs_w = n_seq * q_len * (q_len + 1) // 2, n_seq * sum(min(i + 1, window) for i in range(q_len))
+            seen, all_keys = 4.0 * h * 128 * pairs_w, 4.0 * h * 128 * pairs
+            cost = lambda f, gate=0: dict(flops=f)
+        add("softcap_attn (window, kept tokens, sinks)", phase, lambda: att(window=window, keep_first=keep, sinks=sinks, out_mul=0.5, out=o[:, :h * 128]), **cost(seen),
+            like="softcap_attn (window, gate)")
+        add("gibavik softcap_attn (window, capped, turned back, gate)", phase, lambda: ops.softcap_attn(q128, kc, vc, idx, kv_start, kvl, lay, 0.125, 30.0, h, 8, 128, 128,
+            window=window, v_turn=vturn, gate=g128), **cost(seen, t * h * 128 * 2))
+        add("softcap_attn (sinks, all keys)", phase, lambda: att(sinks=sinks), **cost(all_keys), like="softcap_attn (plain)")
+        add("meronex softcap_attn (capped scores, all keys)", phase, lambda: ops.softcap_attn(q128, kc, vc, idx, kv_start, kvl, lay, 0.125, 30.0, h, 8, 128, 128), **cost(all_keys))
+        # retention: keys 64, values 128 wide
+        decay = torch.full((hd,), 0.99, device=dev)
+        mem = torch.zeros(n_seq + 1, hd, 64, 128, device=dev)
+        at = (n_left, n_left + hd * 64, n_left + 2 * hd * 64)
+        g0 = at[2] + hd * 128
+        if dec:
+            b = n_seq * hd * 64 * 128 * 8 + t * (2 * hd * 64 + hd * 128) * 2
+            add("decay_step (rotation, head norms, gate)", phase, lambda: ops.decay_step(xp, at, decay, mem, lay, hd, 64, 128, 1e-5, turn=right_turn, k_mul=0.125, gate_off=g0,
+                gate_kind="silu", out=o[:, h * 128:h * 128 + hd * 128]), bytes_=b + t * hd * 128 * 4, like="decay_scan + head_norm_gate")
+            add("gibavik decay_scan", phase, lambda: ops.decay_scan(xp, at, decay, mem, lay, hd, 64, 128, act="silu"), bytes_=b + t * hd * 128 * 4)
+        else:
+            f = 4.0 * t * hd * 64 * 128
+            add("decay_scan (rotation, chunks side by side)", phase, lambda: ops.decay_scan(xp, at, decay, mem, lay, hd, 64, 128, turn=right_turn, k_mul=0.125), flops=f,
+                peak=FP32_VALU_PEAK_TFLOPS, like="decay_scan")
+            add("gibavik decay_scan (silu, chunks side by side)", phase, lambda: ops.decay_scan(xp, at, decay, mem, lay, hd, 64, 128, act="silu"), flops=f, peak=FP32_VALU_PEAK_TFLOPS)
+        o32 = torch.randn(t, hd, 128, device=dev)
+        add("head_norm_gate (into the layer's read-outs)", phase, lambda: ops.head_norm_gate(o32, None, 1e-5, gate=xp[:, g0:g0 + hd * 128], kind="silu",
+            out=o[:, h * 128:h * 128 + hd * 128]), bytes_=t * hd * 128 * 8, like="head_norm_gate")
+        gate = torch.randn(t, hd * 128, device=dev).to(bf)
+        add("zenedra head_norm_gate", phase, lambda: ops.head_norm_gate(o32, qn, 1e-5, gate=gate, kind="silu"), bytes_=t * hd * 128 * 8)
+        # feed-forward: router and shared gate in one float32 projection, shared hidden rows, experts
+        rw, rw8 = torch.randn(9, w, device=dev), torch.randn(8, w, device=dev)
+        add("skinny_proj (router and shared gate: width -> 9)", phase, lambda: ops.skinny_proj(y, rw), bytes_=t * w * 2 + 9 * w * 4 + t * 36, like="skinny_proj of a router")
+        add("ladusun skinny_proj of a router (width -> 8)", phase, lambda: ops.skinny_proj(y, rw8), bytes_=t * w * 2 + 8 * w * 4 + t * 32)
+        zl = torch.randn(t, 9, device=dev)
+        add("moe_route_softmax (rows of nine)", phase, lambda: ops.moe_route_softmax(zl[:, :8], 2), bytes_=t * 52, like="moe_route_softmax")
+        zl8 = zl[:, :8].contiguous()
+        add("ladusun moe_route_softmax (groups)", phase, lambda: ops.moe_route_softmax(zl8, 2, 4, 2, 1e-20), bytes_=t * 48)
+        f2 = ff // 2
+        add("moe_glu (shared rows behind their gate)", phase, lambda: ops.moe_glu(xp[:, n_left + n_right:], float("inf"), 1.0, 0.0, row_gate=zl[:, 8], out=o[:, k_out - f2:]),
+            bytes_=t * f2 * 6, like="silu_mul")
+        gu = torch.randn(t, 2 * f2, device=dev).to(bf)
+        add("qwen3 silu_mul", phase, lambda: ops.silu_mul(gu), bytes_=t * f2 * 6)
+        if dec:
+            eidx = torch.stack([torch.randperm(8, device=dev)[:2] for _ in range(t)]).to(torch.int32)
+            wts = torch.full((t, 2), 0.5, device=dev)
+            for name, f, like in (("moe_expert_rows (experts of ff / 4)", ff // 4, "gibavik moe_expert_rows"), ("gibavik moe_expert_rows (experts of ff / 2)", ff // 2, None)):
+                w_gu, w_d = torch.randn(8, 2 * f, w, device=dev).to(bf) * 0.02, torch.randn(8, w, f, device=dev).to(bf) * 0.02
+                add(name, phase, lambda: ops.moe_expert_rows(y, eidx, wts, w_gu, w_d, float("inf"), 1.0, 0.0, True), bytes_=min(t * 2, 8) * 3 * f * w * 2, like=like)
+    return rows
+
+
 ARCHS = {"kabidra": (lambda z: _kabidra_config(z), lambda *a, **k: _kernel_table(*a), "Kabidra"),
          "meronex": (lambda z: _meronex_config(z), lambda *a, **k: _meronex_kernel_table(*a, **k), "Meronex"),
          "gibavik": (lambda z: _gibavik_config(z), lambda *a, **k: _gibavik_kernel_table(*a, **k), "Gibavik"),
          "ladusun": (lambda z: _ladusun_config(z), lambda *a, **k: _ladusun_kernel_table(*a, **k), "Ladusun"),
-         "zenedra": (lambda z: _zenedra_config(z), lambda *a, **k: _zenedra_kernel_table(*a, **k), "Zenedra")}
+         "zenedra": (lambda z: _zenedra_config(z), lambda *a, **k: _zenedra_kernel_table(*a, **k), "Zenedra"),
+         "fikotar": (lambda z: _fikotar_config(z), lambda *a, **k: _fikotar_kernel_table(*a, **k), "Fikotar")}
 
 
 def arch_compare(args):
@@ -1171,7 +1338,7 @@ def arch_compare(args):
         entry = {"geometry": z}
         with tempfile.TemporaryDirectory() as tmp:
             engines = [(args.arch, make_config(z)), ("qwen3", _qwen3_config(z))]
-            if args.arch in ("ladusun", "zenedra"):     # the closest relative in this package (attention beside a matrix memory or recurrence, experts)
+            if args.arch in ("ladusun", "zenedra", "fikotar"):     # the closest relative in this package (attention beside a matrix memory or recurrence, experts)
                 engines.insert(1, ("gibavik", _gibavik_config(z)))
             for model, cfg in engines if args.arch_serve else ():
                 d = os.path.join(tmp, model)
@@ -1187,7 +1354,7 @@ def arch_compare(args):
         print(f"[arch-compare] {name}: kernels one by one", file=sys.stderr, flush=True)
         with torch.inference_mode():
             t_pre = args.arch_seqs * args.arch_prompt
-            if args.arch in ("gibavik", "ladusun", "zenedra") and args.arch_portion:      # the kernels one by one at the size of the steps the engines ran
+            if args.arch in ("gibavik", "ladusun", "zenedra", "fikotar") and args.arch_portion:      # the kernels one by one at the size of the steps the engines ran
                 t_pre = min(t_pre, max(args.arch_portion, args.arch_prompt))
             entry["kernels"] = kernel_table(z, t_pre, args.arch_seqs, args.arch_prompt,
                                             phases=tuple(args.arch_phases.split(",")))

@@ -88,7 +88,9 @@ def sink_softmax_readout(q, k, v, mask, scale, sink):
 def prepared(h, w, p, m, eps):
     """(queries (T, H, D), keys (T, G, D), values (T, G, E)) of a window attention: projected, convolved, turned, queries and keys normed."""
     t, pos = h.shape[0], torch.arange(h.shape[0])
-    q, k, v = (causal_conv(h @ w[p + n].T, w[p + n + ".conv"]) for n in "qkv")
+    q, k, v = (h @ w[p + n].T for n in "qkv")
+    if m.get("conv"):
+        q, k, v = (causal_conv(u, w[p + n + ".conv"]) for u, n in ((q, "q"), (k, "k"), (v, "v")))
     q, k = q.view(t, m["heads"], m["dim"]), k.view(t, m["kv_heads"], m["dim"])
     return unit_rms(turned(q, pos, m.get("rot")), eps), unit_rms(turned(k, pos, m.get("rot")), eps), v.view(t, m["kv_heads"], m["vdim"])
 
