@@ -579,9 +579,9 @@ int nvx_latent_attn(const void* q, const void* cache, int fmt, const int32_t* kv
  * Expert e:  g = min(W_gate x, limit), u = clamp(W_up x, -limit, limit), y = g sigmoid(alpha g) (u + shift), result W_down y, with
  *     w_gu (experts, 2 ff, width) = rows [gate | up] and w_d (experts, width, ff).  (limit = infinity, alpha = 1, shift = 0: silu(g) u.)
  * nvx_moe_expert_rows:  out[t] = sum_k expert_idx[t][k](wts[t][k] * h[t]), or sum_k wts[t][k] * expert_idx[t][k](h[t]) if
- *     weight_out; the experts' rows streamed per (token, choice) pair by
- *     workgroups of a few dozen rows; ws: n_tok * top * ff floats (the hidden activations between its two launches); width <=
- *     nvx_moe_expert_rows_max_width(ff).
+ *     weight_out; 16-bit formats with width and ff multiples of eight: an expert's rows read once for up to 16 of its (token, choice) pairs,
+ *     on the matrix cores; else streamed per pair by workgroups of a few dozen rows.  ws: n_tok * top * (ff + width) floats (hidden
+ *     activations and output rows between its launches); width <= nvx_moe_expert_rows_max_width(ff).
  * nvx_moe_order:  dst[r] = place of pair r (= token * top + choice) when the n pairs are put in expert order, pairs of one expert
  *     keeping their order; counts[e] = pairs of expert e.  n_exp <= nvx_moe_order_max_experts().
  * nvx_moe_scatter_rows:  xs[dst[r]] = wts[r] * h[r / top] for every (token, choice) pair r (wts == null: ones).

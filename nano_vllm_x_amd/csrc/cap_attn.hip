@@ -406,22 +406,24 @@ __global__ __launch_bounds__(256) void softcap_attn_kernel(const A* __restrict__
     }
 }
 
-// ---- tied rows, for steps of few tokens ---------------------------------------------------------------------------------------
-// One workgroup of four waves per (NH query heads of one key/value head, token, split).  A cached row is key AND value, so it is read
-// once, by LPR neighbouring lanes of eight elements each (LPR: 8, 16, 32 or 64, the first that covers dim / 8), and stays in registers from the
+// ---- a row read once for all the heads it serves, for steps of few tokens -----------------------------------------------------
+// One workgroup of four waves per (NH query heads of one key/value head, token, split).  A cached row is read once, by LPR neighbouring
+// lanes of eight elements each (LPR: 8, 16, 32 or 64, the first that covers the longer of key and value), and stays in registers from the
 // score to the read-out, for all NH heads: a wave takes U keys per lane group at a time (their loads in flight together), sums the
 // products over the lane group, and adds the weighted rows to what the lane keeps of the read-out.  Every lane group has a running
-// maximum and sum of its own; groups, waves and splits are merged at the end.
-template <typename A, int NH, int U, int LPR>
-__global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict__ q, const A* __restrict__ rows, const float* __restrict__ k_rn,
-                                                            const int32_t* __restrict__ kv_indices, const int64_t* __restrict__ kv_start,
-                                                            const int32_t* __restrict__ kv_len, const int32_t* __restrict__ qo_indptr,
-                                                            const int32_t* __restrict__ tok_seq, float scale, A* __restrict__ out, int heads,
-                                                            int kv_heads, int dim, int n_split, float* __restrict__ part, int window, int chunk,
-                                                            const float* __restrict__ slopes) {
+// maximum and sum of its own; groups, waves and splits are merged at the end.  TIED: a cached row is key AND value, and k_rn norms its
+// score; otherwise values have rows of their own.
+template <typename A, int NH, int U, int LPR, bool TIED>
+__global__ __launch_bounds__(256) void rows_attn_kernel(const A* __restrict__ q, const A* __restrict__ rows, const A* __restrict__ v_rows,
+                                                       const float* __restrict__ k_rn, const int32_t* __restrict__ kv_indices,
+                                                       const int64_t* __restrict__ kv_start, const int32_t* __restrict__ kv_len,
+                                                       const int32_t* __restrict__ qo_indptr, const int32_t* __restrict__ tok_seq, float scale,
+                                                       A* __restrict__ out, int heads, int kv_heads, int dim, int vdim, int n_split,
+                                                       float* __restrict__ part, int window, int chunk, const float* __restrict__ slopes, int sink,
+                                                       float sink_score, const float* __restrict__ sinks, int keep, float out_mul, int64_t out_stride) {
     extern __shared__ float sm[];
-    float* sacc = sm;                       // 4 waves x NH x dim
-    float* sml = sacc + 4 * NH * dim;       // 4 waves x NH maxima, then as many sums
+    float* sacc = sm;                       // 4 waves x NH x vdim
+    float* sml = sacc + 4 * NH * vdim;      // 4 waves x NH maxima, then as many sums
     const int per_kv = heads / kv_heads, blocks_per_kv = (per_kv + NH - 1) / NH;
     const int kvh = blockIdx.x / blocks_per_kv, h0 = kvh * per_kv + (blockIdx.x % blocks_per_kv) * NH;
     const int n_here = (kvh + 1) * per_kv - h0 < NH ? (kvh + 1) * per_kv - h0 : NH;       // heads of this block
@@ -431,10 +433,11 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
     const int64_t q_n = qo_indptr ? qo_indptr[b + 1] - q0 : 1;
     const int visible = kv_len[b] - (int)(q_n - 1 - (t - q0));
     const int first = first_seen(visible - 1, window, chunk);
+    const int kept = keep < first ? keep : first, n_keys = kept + visible - first;      // the walk: keys 0 .. kept - 1, then first .. visible - 1
     const int32_t* slots = kv_indices + kv_start[b];
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, g = lane / LPR, l = lane % LPR;
     constexpr int groups = 64 / LPR;
-    const bool on = l * 8 < dim;
+    const bool on = l * 8 < dim, on_v = l * 8 < vdim;
     typedef A vec8 __attribute__((ext_vector_type(8)));
     float qv[NH][8], acc[NH][8], m[NH], sum[NH], slope[NH];
 #pragma unroll
@@ -450,15 +453,16 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
         }
     }
     const int step = U * groups;            // keys of a wave's turn
-    for (int j0 = first + ((int)blockIdx.z * 4 + wave) * step; j0 < visible; j0 += 4 * n_split * step) {
-        vec8 kv[U];
+    for (int i0 = ((int)blockIdx.z * 4 + wave) * step; i0 < n_keys; i0 += 4 * n_split * step) {
+        vec8 kv[U], vv[TIED ? 1 : U];
         float rn[U];
 #pragma unroll
         for (int u = 0; u < U; ++u) {       // (a key past the end reads a real row and gets no weight)
-            const int j = j0 + u * groups + g;
-            const int64_t row = (int64_t)slots[j < visible ? j : first] * kv_heads + kvh;
-            rn[u] = k_rn[row];
+            const int i = i0 + u * groups + g < n_keys ? i0 + u * groups + g : n_keys - 1;
+            const int64_t row = (int64_t)slots[i < kept ? i : first + i - kept] * kv_heads + kvh;
             kv[u] = *reinterpret_cast<const vec8*>(rows + row * dim + (on ? l * 8 : 0));
+            if constexpr (TIED) rn[u] = k_rn[row];
+            else vv[u] = *reinterpret_cast<const vec8*>(v_rows + row * vdim + (on_v ? l * 8 : 0));
         }
 #pragma unroll
         for (int n = 0; n < NH; ++n) {
@@ -469,8 +473,9 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
 #pragma unroll
                 for (int i = 0; i < 8; ++i) d += qv[n][i] * (float)kv[u][i];
                 d = group_sum<LPR>(d);
-                const int j = j0 + u * groups + g;
-                s[u] = j < visible ? d * rn[u] - slope[n] * (float)(visible - 1 - j) : -INFINITY;
+                const int i = i0 + u * groups + g, j = i < kept ? i : first + i - kept;
+                if constexpr (TIED) d *= rn[u];
+                s[u] = i < n_keys ? d - slope[n] * (float)(visible - 1 - j) : -INFINITY;
                 mx = fmaxf(mx, s[u]);
             }
             const float base = mx == -INFINITY ? 0.f : mx;                  // (nothing seen by this lane group yet)
@@ -484,7 +489,7 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
                 const float p = expf(s[u] - base);
                 sum[n] += p;
 #pragma unroll
-                for (int i = 0; i < 8; ++i) acc[n][i] += p * (float)kv[u][i];
+                for (int i = 0; i < 8; ++i) acc[n][i] += p * (float)(TIED ? kv[u][i] : vv[TIED ? 0 : u][i]);
             }
         }
     }
@@ -501,17 +506,21 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
 #pragma unroll
             for (int i = 0; i < 8; ++i) acc[n][i] += __shfl_xor(acc[n][i], k, 64);
         }
-        if (g == 0 && on) {
+        if (g == 0 && on_v) {
 #pragma unroll
-            for (int i = 0; i < 8; ++i) sacc[(wave * NH + n) * dim + l * 8 + i] = acc[n][i];
+            for (int i = 0; i < 8; ++i) sacc[(wave * NH + n) * vdim + l * 8 + i] = acc[n][i];
         }
         if (lane == 0) { sml[wave * NH + n] = mx; sml[4 * NH + wave * NH + n] = sum[n]; }
     }
     __syncthreads();
     for (int n = 0; n < n_here; ++n) {      // the four waves
-        float f[4], mm = -INFINITY, total = 0.f;
+        // a sink is one more term of the softmax's sum (a split's parts get it where they are merged)
+        const bool sunk = sink && n_split == 1;
+        const float sink_n = sunk ? (sinks ? sinks[h0 + n] : sink_score) : -INFINITY;
+        float f[4], mm = sink_n;
 #pragma unroll
         for (int w = 0; w < 4; ++w) mm = fmaxf(mm, sml[w * NH + n]);
+        float total = sunk ? expf(sink_n - mm) : 0.f;
 #pragma unroll
         for (int w = 0; w < 4; ++w) {
             const float mw = sml[w * NH + n];
@@ -519,13 +528,13 @@ __global__ __launch_bounds__(256) void tied_rows_attn_kernel(const A* __restrict
             total += sml[4 * NH + w * NH + n] * f[w];
         }
         const int64_t row = t * heads + h0 + n;
-        float* pr = n_split > 1 ? part + (row * n_split + blockIdx.z) * (dim + 2) : nullptr;
-        for (int e = threadIdx.x; e < dim; e += 256) {
+        float* pr = n_split > 1 ? part + (row * n_split + blockIdx.z) * (vdim + 2) : nullptr;
+        for (int e = threadIdx.x; e < vdim; e += 256) {
             float o = 0.f;
 #pragma unroll
-            for (int w = 0; w < 4; ++w) o += sacc[(w * NH + n) * dim + e] * f[w];
+            for (int w = 0; w < 4; ++w) o += sacc[(w * NH + n) * vdim + e] * f[w];
             if (pr) pr[2 + e] = o;
-            else st_f(out, row * dim + e, o / total);
+            else st_f(out, t * out_stride + (int64_t)(h0 + n) * vdim + e, o / total * out_mul);
         }
         if (pr && threadIdx.x == 0) { pr[0] = mm; pr[1] = total; }
     }
@@ -1000,28 +1009,32 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     }
     const size_t lds = (size_t)(dim + 4 * vdim + 8) * sizeof(float);
     NVX_REQUIRE(n_split >= 1 && n_split <= 64 && (n_split == 1 || part), NVX_EINVAL, "nvx_softcap_attn: a key split needs its workspace");
-    // tied rows without what that kernel does not do: a row is read once
-    if (k_rn && k_cache == v_cache && dim == vdim && dim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && !sink && keep_first == 0 &&
-        out_mul == 1.0f && out_stride == heads * vdim && nvx_aligned16(k_cache)) {
+    // without what the kernel does not do: a row is read once for up to four heads
+    const bool tied = k_rn && k_cache == v_cache && dim == vdim;
+    if ((tied || !k_rn) && dim % 8 == 0 && vdim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && nvx_aligned16(k_cache) && nvx_aligned16(v_cache)) {
         const int per_kv = (int)(heads / kv_heads), nh = per_kv >= 4 ? 4 : (per_kv >= 2 ? 2 : 1);
         const dim3 tgrid((unsigned)(kv_heads * ((per_kv + nh - 1) / nh)), (unsigned)n_tok, (unsigned)n_split);
-        const size_t tlds = (size_t)(4 * nh * dim + 8 * nh) * sizeof(float);
-#define NVX_TIED_ROWS_L(NH, LPR)                                                                                                                \
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((tied_rows_attn_kernel<A_, NH, sizeof(A_) == 2 ? 8 : 4, LPR>), tgrid, dim3(256), tlds, (hipStream_t)stream, \
-                                         (const A_*)q, (const A_*)k_cache, k_rn, kv_indices, kv_start, kv_len, qo_indptr, tok_seq, scale, (A_*)out,  \
-                                         (int)heads, (int)kv_heads, (int)dim, n_split, part, (int)window, (int)chunk, slopes))
-#define NVX_TIED_ROWS(NH)                            \
-    do {                                             \
-        if (dim <= 64) NVX_TIED_ROWS_L(NH, 8);       \
-        else if (dim <= 128) NVX_TIED_ROWS_L(NH, 16); \
-        else if (dim <= 256) NVX_TIED_ROWS_L(NH, 32); \
-        else NVX_TIED_ROWS_L(NH, 64);                \
+        const size_t tlds = (size_t)(4 * nh * vdim + 8 * nh) * sizeof(float);
+        const int64_t longest = dim > vdim ? dim : vdim;
+#define NVX_ROWS_ATTN_T(NH, LPR, U, TIED)                                                                                                       \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((rows_attn_kernel<A_, NH, sizeof(A_) == 2 ? U : 4, LPR, TIED>), tgrid, dim3(256), tlds, (hipStream_t)stream, \
+                                         (const A_*)q, (const A_*)k_cache, (const A_*)v_cache, k_rn, kv_indices, kv_start, kv_len, qo_indptr, tok_seq, scale, \
+                                         (A_*)out, (int)heads, (int)kv_heads, (int)dim, (int)vdim, n_split, part, (int)window, (int)chunk, slopes, sink, \
+                                         sink_score, sinks, (int)keep_first, out_mul, out_stride))
+#define NVX_ROWS_ATTN_L(NH, LPR) do { if (tied) NVX_ROWS_ATTN_T(NH, LPR, 8, true); else NVX_ROWS_ATTN_T(NH, LPR, 4, false); } while (0)
+#define NVX_ROWS_ATTN(NH)                                 \
+    do {                                                  \
+        if (longest <= 64) NVX_ROWS_ATTN_L(NH, 8);        \
+        else if (longest <= 128) NVX_ROWS_ATTN_L(NH, 16); \
+        else if (longest <= 256) NVX_ROWS_ATTN_L(NH, 32); \
+        else NVX_ROWS_ATTN_L(NH, 64);                     \
     } while (0)
-        if (nh == 4) NVX_TIED_ROWS(4);
-        else if (nh == 2) NVX_TIED_ROWS(2);
-        else NVX_TIED_ROWS(1);
-#undef NVX_TIED_ROWS_L
-#undef NVX_TIED_ROWS
+        if (nh == 4) NVX_ROWS_ATTN(4);
+        else if (nh == 2) NVX_ROWS_ATTN(2);
+        else NVX_ROWS_ATTN(1);
+#undef NVX_ROWS_ATTN_L
+#undef NVX_ROWS_ATTN_T
+#undef NVX_ROWS_ATTN
         if (n_split > 1)
             NVX_FMT_CALL(fmt, hipLaunchKernelGGL(softcap_merge_kernel<A_>, dim3((unsigned)(n_tok * heads)), dim3(64), 0, (hipStream_t)stream,
                                                  (const float*)part, n_split, (A_*)out, (int)vdim, (int)heads, vcs, v_interleaved, (const A_*)gate,

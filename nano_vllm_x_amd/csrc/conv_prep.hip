@@ -42,9 +42,8 @@ template <typename A> struct ConvPrep {
         return hd < heads + kv_heads ? hd * dim : (heads + kv_heads) * dim + (hd - heads - kv_heads) * vdim;
     }
     // where token t's part goes (null: nowhere, a padding row's keys and values)
-    __device__ __forceinline__ A* target(int64_t t, int hd) const {
+    __device__ __forceinline__ A* target(int64_t t, int64_t slot, int hd) const {
         if (hd < heads) return q_out + (t * heads + hd) * dim;
-        const int64_t slot = slots[t];
         if (slot < 0) return nullptr;
         if (hd < heads + kv_heads) return k_cache + (slot * kv_heads + (hd - heads)) * dim;
         return v_cache + (slot * kv_heads + (hd - heads - kv_heads)) * vdim;
@@ -82,7 +81,7 @@ __global__ __launch_bounds__(256) void conv_attn_prep_kernel(ConvPrep<A> p, int6
     }
     // a rotation keeps the length of every pair, so the root mean square is that of the row before it
     const float rn = turned && p.norm ? 1.0f / sqrtf(wave_sum(ss) / (float)n + p.eps) : 1.0f;
-    A* o = p.target(t, hd);
+    A* o = p.target(t, p.slots[t], hd);
     if (!o) return;
     __builtin_amdgcn_wave_barrier();
     __threadfence_block();
@@ -98,18 +97,26 @@ __global__ __launch_bounds__(256) void conv_attn_prep_kernel(ConvPrep<A> p, int6
 }
 
 // Sizes in multiples of eight, up to four taps: a part of a row per LPR neighbouring lanes of eight channels each.  A lane group walks
-// `run` consecutive tokens with the taps and the last inputs in registers, so weights and rows are read once; where another sequence
-// begins, the history comes from that sequence.  With `own_tail` (one token per sequence) the lane also writes the new history back: no
+// RUN consecutive tokens with the taps and the last inputs in registers, so weights are read once for them and rows little more than once;
+// everything of the walk is asked for before the first token is worked on.  Where another sequence begins, the history comes from
+// that sequence.  With `own_tail` (one token per sequence) the lane also writes the new history back: no
 // other lane touches its channels of that slot.
-template <typename A, int LPR, int TAPS>
-__global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, int run, int64_t n_groups, int own_tail) {
+typedef float f4_any __attribute__((ext_vector_type(4), aligned(4)));       // four floats in one access, on any border of four bytes
+__device__ __forceinline__ void load8(const float* __restrict__ src, float (&dst)[8]) {
+    const f4_any a = *reinterpret_cast<const f4_any*>(src), b = *reinterpret_cast<const f4_any*>(src + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) { dst[e] = a[e]; dst[4 + e] = b[e]; }
+}
+template <typename A, int LPR, int TAPS, int RUN>
+__global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, unsigned n_groups, int own_tail) {
     typedef A vec8 __attribute__((ext_vector_type(8)));
     constexpr int HN = TAPS - 1;
-    const int64_t item = ((int64_t)blockIdx.x * 256 + threadIdx.x) / LPR;
+    const unsigned item = blockIdx.x * (256 / LPR) + threadIdx.x / LPR;
     const int l = threadIdx.x % LPR;
     const bool item_on = item < n_groups;
-    const int64_t t0 = item_on ? item / p.per() * run : 0;
-    const int hd = item_on ? (int)(item % p.per()) : 0;
+    const unsigned run_no = item_on ? item / (unsigned)p.per() : 0u;
+    const int64_t t0 = (int64_t)run_no * RUN;
+    const int hd = item_on ? (int)(item - run_no * p.per()) : 0;
     const bool turned = hd < p.heads + p.kv_heads;
     const int n = turned ? p.dim : p.vdim, ch = p.channels(), c0 = p.first(hd) + l * 8;
     const bool on = item_on && l * 8 < n;
@@ -117,19 +124,28 @@ __global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, 
     const int partner = (threadIdx.x & 63) + (rot_here ? (low ? p.half / 8 : -(p.half / 8)) : 0), m0 = low ? l * 8 : l * 8 - p.half;
     float w[TAPS][8], hist[HN > 0 ? HN : 1][8];
 #pragma unroll
-    for (int i = 0; i < TAPS; ++i)
+    for (int i = 0; i < TAPS; ++i) load8(p.w + (int64_t)i * ch + (on ? c0 : 0), w[i]);      // (a lane without channels keeps channel 0's, unused)
+    vec8 rows[RUN];
+    int seqs[RUN];
+    int64_t slots[RUN];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) w[i][e] = on ? p.w[(int64_t)i * ch + c0 + e] : 0.f;
+    for (int k = 0; k < RUN; ++k) {
+        const int64_t t = t0 + k < p.n_tok ? t0 + k : p.n_tok - 1;
+        seqs[k] = p.tok_seq ? p.tok_seq[t] : (int)t;
+        slots[k] = p.slots[t];
+        rows[k] = *reinterpret_cast<const vec8*>(p.x + t * p.x_stride + (on ? c0 : 0));
+    }
     int last_b = -1;
     SeqSpan s{0, 0, 0, -1};
-    for (int k = 0; k < run; ++k) {
+#pragma unroll
+    for (int k = 0; k < RUN; ++k) {
         const int64_t t = t0 + k;
         const bool here = on && t < p.n_tok;
         float y[8], cur[8];
 #pragma unroll
         for (int e = 0; e < 8; ++e) { y[e] = 0.f; cur[e] = 0.f; }
         if (here) {
-            const int b = p.tok_seq ? p.tok_seq[t] : (int)t;
+            const int b = seqs[k];
             if (b != last_b) {               // the first token of this walk, or of another sequence: its history
                 last_b = b;
                 s = seq_span(b, p.qo_indptr, p.pos0, p.state_slot);
@@ -141,14 +157,15 @@ __global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, 
                         const vec8 v = *reinterpret_cast<const vec8*>(p.x + (s.q0 + src) * p.x_stride + c0);
 #pragma unroll
                         for (int e = 0; e < 8; ++e) hist[i][e] = (float)v[e];
+                    } else if (has_state) {
+                        load8(p.state + ((int64_t)s.slot * HN + HN + src) * ch + c0, hist[i]);
                     } else {
-                        const float* st = p.state + ((int64_t)(has_state ? s.slot : 0) * HN + (has_state ? HN + src : 0)) * ch + c0;
 #pragma unroll
-                        for (int e = 0; e < 8; ++e) hist[i][e] = has_state ? st[e] : 0.f;
+                        for (int e = 0; e < 8; ++e) hist[i][e] = 0.f;
                     }
                 }
             }
-            const vec8 v = *reinterpret_cast<const vec8*>(p.x + t * p.x_stride + c0);
+            const vec8 v = rows[k];
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
                 cur[e] = (float)v[e];
@@ -162,9 +179,11 @@ __global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, 
             }
             if (own_tail && HN > 0 && s.slot >= 0) {
 #pragma unroll
-                for (int i = 0; i < HN; ++i)
-#pragma unroll
-                    for (int e = 0; e < 8; ++e) p.state[((int64_t)s.slot * HN + i) * ch + c0 + e] = hist[i][e];
+                for (int i = 0; i < HN; ++i) {
+                    float* st = p.state + ((int64_t)s.slot * HN + i) * ch + c0;
+                    *reinterpret_cast<f4_any*>(st) = f4_any{hist[i][0], hist[i][1], hist[i][2], hist[i][3]};
+                    *reinterpret_cast<f4_any*>(st + 4) = f4_any{hist[i][4], hist[i][5], hist[i][6], hist[i][7]};
+                }
             }
         }
         float ss = 0.f;
@@ -180,13 +199,13 @@ __global__ __launch_bounds__(256) void conv_attn_prep_vec_kernel(ConvPrep<A> p, 
         if (!here) continue;
         if (p.half && rot_here) {
             const float* tr = p.turn.cos + t * p.turn.stride + m0;
+            float c[8], sn[8];
+            load8(tr, c);
+            load8(tr + p.turn.sin_off, sn);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) {
-                const float c = tr[e], sn = tr[p.turn.sin_off + e];
-                y[e] = low ? y[e] * c - z[e] * sn : y[e] * c + z[e] * sn;
-            }
+            for (int e = 0; e < 8; ++e) y[e] = low ? y[e] * c[e] - z[e] * sn[e] : y[e] * c[e] + z[e] * sn[e];
         }
-        A* o = p.target(t, hd);
+        A* o = p.target(t, slots[k], hd);
         if (!o) continue;
         vec8 r;
 #pragma unroll
@@ -204,11 +223,14 @@ template <typename A> static void launch_conv_prep(const ConvPrep<A>& p, bool ve
         return;
     }
     const int lpr = longest <= 64 ? 8 : (longest <= 128 ? 16 : (longest <= 256 ? 32 : 64));
-    int run = 8;                             // walks of eight tokens, shorter ones where that leaves too few workgroups
-    while (run > 1 && (!p.qo_indptr || (p.n_tok + run - 1) / run * per * lpr < 256 * 1024)) run >>= 1;
+    const int run = p.qo_indptr && p.n_tok * per * lpr >= 256 * 1024 ? 4 : 1;      // (walks of four tokens where they leave workgroups enough)
     const int64_t groups = (p.n_tok + run - 1) / run * per;
     const dim3 grid((unsigned)((groups * lpr + 255) / 256));
-#define NVX_CONV_T(LPR, T) hipLaunchKernelGGL((conv_attn_prep_vec_kernel<A, LPR, T>), grid, dim3(256), 0, st, p, run, groups, own_tail)
+#define NVX_CONV_T(LPR, T)                                                                                                                    \
+    do {                                                                                                                                      \
+        if (run == 4) hipLaunchKernelGGL((conv_attn_prep_vec_kernel<A, LPR, T, 4>), grid, dim3(256), 0, st, p, (unsigned)groups, own_tail);    \
+        else hipLaunchKernelGGL((conv_attn_prep_vec_kernel<A, LPR, T, 1>), grid, dim3(256), 0, st, p, (unsigned)groups, own_tail);             \
+    } while (0)
 #define NVX_CONV(LPR)                                 \
     do {                                              \
         if (p.taps_n == 1) NVX_CONV_T(LPR, 1);        \
@@ -246,7 +268,7 @@ extern "C" int nvx_conv_attn_prep(const void* x, int64_t x_stride, int fmt, cons
     NVX_REQUIRE(n_tok >= 0 && n_seq >= 0 && n_seq <= 65535 && heads > 0 && kv_heads > 0 && dim > 0 && dim <= 4096 && vdim > 0 && vdim <= 4096 &&
                     taps_n >= 1 && taps_n <= 64 && n_slots >= 0, NVX_EINVAL, "nvx_conv_attn_prep: bad sizes (heads of at most 4096, 1 to 64 taps)");
     const int64_t channels = heads * dim + kv_heads * (dim + vdim), per = heads + 2 * kv_heads;
-    NVX_REQUIRE(channels < (1 << 30) && x_stride >= channels && n_tok * per < (1ll << 32), NVX_EINVAL, "nvx_conv_attn_prep: row stride, or too many rows");
+    NVX_REQUIRE(channels < (1 << 30) && x_stride >= channels && n_tok * per < (1ll << 31), NVX_EINVAL, "nvx_conv_attn_prep: row stride, or too many rows");
     NVX_REQUIRE(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || (turn && turn_stride >= turn_sin_off + rot_dims / 2)), NVX_EINVAL,
                 "nvx_conv_attn_prep: the rotated part must be even and within a head, and needs its table");
     if (n_tok == 0 || n_seq == 0) return NVX_OK;

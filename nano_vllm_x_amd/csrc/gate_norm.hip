@@ -266,7 +266,7 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const float* x_in, c
 //   predecessor is the step's own or, for the first token of a portion, the id that the sequence's state slot keeps (its bits in a
 //   float32 word).  The workgroup of a portion's first token reads that word before it replaces it by the portion's last id, and no
 //   other workgroup touches it.
-template <typename A>
+template <typename A, int V>
 __global__ __launch_bounds__(256) void embed_sum_kernel(const int64_t* __restrict__ ids, const A* __restrict__ table, int64_t vocab,
                                                        const A* __restrict__ pair, int64_t buckets, int64_t mul_prev, int64_t mul_cur,
                                                        float* prev_id, const A* __restrict__ pos_table, int64_t n_pos,
@@ -305,14 +305,18 @@ __global__ __launch_bounds__(256) void embed_sum_kernel(const int64_t* __restric
     const A* er = table + id * width;
     const A* pr = pair ? pair + pair_row * width : nullptr;
     const A* lr = pos_table ? pos_table + p * width : nullptr;
+    typedef A veca __attribute__((ext_vector_type(V)));
+    typedef float vecf __attribute__((ext_vector_type(V)));
     float ss = 0.f;
-    for (int c = threadIdx.x; c < width; c += 256) {
-        float v = ld_f(er, c);
-        if (pr) v += ld_f(pr, c);
-        if (lr) v += ld_f(lr, c);
-        x[t * (int64_t)width + c] = v;
-        su[c] = v;
-        ss += v * v;
+    for (int c = threadIdx.x * V; c < width; c += 256 * V) {
+        const veca a = *reinterpret_cast<const veca*>(er + c);
+        vecf v;
+        for (int i = 0; i < V; ++i) v[i] = (float)a[i];
+        if (pr) { const veca u = *reinterpret_cast<const veca*>(pr + c); for (int i = 0; i < V; ++i) v[i] += (float)u[i]; }
+        if (lr) { const veca u = *reinterpret_cast<const veca*>(lr + c); for (int i = 0; i < V; ++i) v[i] += (float)u[i]; }
+        *reinterpret_cast<vecf*>(x + t * (int64_t)width + c) = v;
+        *reinterpret_cast<vecf*>(su + c) = v;
+        for (int i = 0; i < V; ++i) ss += v[i] * v[i];
     }
     __syncthreads();
     row_end<A>(su, ss, red, w, b, eps, split, h, t, width);
@@ -631,9 +635,13 @@ extern "C" int nvx_embed_sum(const int64_t* ids, const void* table, int fmt, int
     NVX_REQUIRE(!pos_table || (positions && n_pos > 0), NVX_EINVAL, "nvx_embed_sum: the position table needs positions");
     NVX_REQUIRE(!h || width % 4 != 0 || (nvx_aligned16(w) && nvx_aligned16(w_bias)), NVX_EINVAL,
                 "nvx_embed_sum: the norm's weight and bias must start on a 16-byte border");
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL(embed_sum_kernel<A_>, dim3((unsigned)n_tok), dim3(256), (size_t)width * sizeof(float), (hipStream_t)stream, ids,
-                                         (const A_*)table, vocab, (const A_*)pair, buckets, mul_prev, mul_cur, prev_id, (const A_*)pos_table, n_pos,
-                                         positions, tok_seq, qo_indptr, pos0, state_slot, x, w, w_bias, eps, split, (A_*)h, (int)width));
+#define NVX_EMBED_SUM(V)                                                                                                                       \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((embed_sum_kernel<A_, V>), dim3((unsigned)n_tok), dim3(256), (size_t)width * sizeof(float), (hipStream_t)stream, ids, \
+                                         (const A_*)table, vocab, (const A_*)pair, buckets, mul_prev, mul_cur, prev_id, (const A_*)pos_table, n_pos,   \
+                                         positions, tok_seq, qo_indptr, pos0, state_slot, x, w, w_bias, eps, split, (A_*)h, (int)width))
+    if (width % 4 == 0 && nvx_aligned16(table) && nvx_aligned16(pair) && nvx_aligned16(pos_table) && nvx_aligned16(x)) NVX_EMBED_SUM(4);
+    else NVX_EMBED_SUM(1);
+#undef NVX_EMBED_SUM
     return nvx_check_launch("nvx_embed_sum");
 }
 

@@ -153,7 +153,7 @@ __device__ __forceinline__ float glu_act(float g, float u, float limit, float al
     return g * sigmoid_f(alpha * g) * (u + shift);
 }
 
-// A token's experts row by row.  w_gu: (experts, 2 * ff, width) rows [gate | up]; w_d: (experts, width, ff).  Two launches, both
+// A token's experts row by row (float32, and sizes that fit no 16-byte loads).  w_gu: (experts, 2 * ff, width) rows [gate | up]; w_d: (experts, width, ff).  Two launches, both
 // with a workgroup per 32 weight rows so that a step of a few tokens still fills the chip: the hidden activations of every
 // (token, choice) pair into a float32 workspace, then the output rows summed over a token's choices.  A wave takes 8 rows; its
 // lanes walk a row 8 elements at a time (16-byte loads) where the format is 16-bit and the rows are 16-byte aligned.
@@ -281,6 +281,140 @@ __global__ __launch_bounds__(256) void moe_rows_down_kernel(const float* __restr
         const int c = blockIdx.x * MOE_ROWS + wave * (MOE_ROWS / 4) + i;
         if (c < width && lane == 0) st_f(out, t * (int64_t)width + c, o[i]);
     }
+}
+
+// ---- a step of few tokens on the matrix cores (16-bit formats) -------------------------------------------------------------------
+// The experts' weights are the bytes that count, and tokens share experts: a workgroup takes 16 weight rows of ONE expert and all (token,
+// choice) pairs that chose it, 16 at a time, so a weight is read once for them.  Its four waves share the depth in blocks of 128 (every
+// fourth block each): per 32 of them one v_mfma_f32_16x16x32 takes 16 rows (operand A: lane (row, quarter) loads 16 bytes of its row) against
+// 16 pairs (operand B: the same of the pair's input), the loads of a block in flight together; the waves' sums meet in LDS in one
+// order, so a pair's result does not depend on the batch.  Three launches: hidden activations per pair, output rows per pair, and the sum
+// over a token's choices.
+typedef __attribute__((ext_vector_type(8))) __bf16 moe_bf16x8;
+typedef __attribute__((ext_vector_type(8))) _Float16 moe_f16x8;
+template <typename A> __device__ __forceinline__ nvx_f32x4 moe_mfma32(nvx_u32x4 a, nvx_u32x4 b, nvx_f32x4 c) {
+    if constexpr (__is_same(A, __bf16))
+        return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(moe_bf16x8, a), __builtin_bit_cast(moe_bf16x8, b), c, 0, 0, 0);
+    else
+        return __builtin_amdgcn_mfma_f32_16x16x32_f16(__builtin_bit_cast(moe_f16x8, a), __builtin_bit_cast(moe_f16x8, b), c, 0, 0, 0);
+}
+constexpr int MT_PAD = 17;       // floats per row of a 16 x 16 tile of partial sums in LDS
+
+// the pairs of expert e in their order -> list; returns how many (the same in every thread)
+__device__ __forceinline__ int pairs_of_expert(const int32_t* __restrict__ idx, int n_pairs, int e, int* list) {
+    __shared__ int wave_n[4];
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    int base = 0;
+    for (int r0 = 0; r0 < n_pairs; r0 += 256) {
+        const int r = r0 + threadIdx.x;
+        const bool mine = r < n_pairs && idx[r] == e;
+        const unsigned long long mask = __ballot(mine);
+        if (lane == 0) wave_n[wave] = __popcll(mask);
+        __syncthreads();
+        int at = base;
+        for (int w = 0; w < wave; ++w) at += wave_n[w];
+        if (mine) list[at + __popcll(mask & ((1ull << lane) - 1ull))] = r;
+        base += wave_n[0] + wave_n[1] + wave_n[2] + wave_n[3];
+        __syncthreads();
+    }
+    return base;
+}
+
+// sums of NM row tiles (rows of `a[m]` at the lane's row) against one tile of inputs at `b`, this wave's blocks of the depth `n`
+template <typename A, int NM>
+__device__ __forceinline__ void moe_tile_sums(const A* const (&a)[NM], const A* __restrict__ b, float b_mul, bool scaled, int n, int wave, int g, nvx_f32x4 (&acc)[NM]) {
+    const nvx_u32x4 none = {0u, 0u, 0u, 0u};
+    for (int k0 = wave * 128; k0 < n; k0 += 512) {
+        nvx_u32x4 av[NM][4], bv[4];
+#pragma unroll
+        for (int s = 0; s < 4; ++s) {
+            const int k = k0 + 32 * s + 8 * g;
+            const bool in = k < n;                     // (n is a multiple of eight)
+#pragma unroll
+            for (int m = 0; m < NM; ++m) av[m][s] = in ? *reinterpret_cast<const nvx_u32x4*>(a[m] + k) : none;
+            bv[s] = in ? *reinterpret_cast<const nvx_u32x4*>(b + k) : none;
+        }
+        if (scaled) {
+            typedef A vec8 __attribute__((ext_vector_type(8)));
+#pragma unroll
+            for (int s = 0; s < 4; ++s) {
+                vec8 v = __builtin_bit_cast(vec8, bv[s]);
+#pragma unroll
+                for (int i = 0; i < 8; ++i) v[i] = (A)(b_mul * (float)v[i]);
+                bv[s] = __builtin_bit_cast(nvx_u32x4, v);
+            }
+        }
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+#pragma unroll
+            for (int m = 0; m < NM; ++m) acc[m] = moe_mfma32<A>(av[m][s], bv[s], acc[m]);
+    }
+}
+
+template <typename A>
+__global__ __launch_bounds__(256) void moe_tile_up_kernel(const A* __restrict__ h, int64_t h_stride, const int32_t* __restrict__ idx,
+                                                         const float* __restrict__ wts, int top, int n_pairs, const A* __restrict__ w_gu, float limit,
+                                                         float alpha, float shift, int weight_out, A* __restrict__ y, int width, int ff) {
+    extern __shared__ int list[];                      // n_pairs
+    __shared__ float part[4][2][16 * MT_PAD];
+    const int e = blockIdx.y, j0 = blockIdx.x * 16;
+    const int count = pairs_of_expert(idx, n_pairs, e, list);
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+    const int row = j0 + c < ff ? j0 + c : ff - 1;
+    const A* const rows[2] = {w_gu + ((int64_t)e * 2 * ff + row) * width, w_gu + ((int64_t)e * 2 * ff + ff + row) * width};
+    for (int m0 = 0; m0 < count; m0 += 16) {
+        const int pair = list[m0 + c < count ? m0 + c : count - 1];
+        nvx_f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+        moe_tile_sums<A, 2>(rows, h + (int64_t)(pair / top) * h_stride, weight_out ? 1.0f : wts[pair], !weight_out, width, wave, g, acc);
+#pragma unroll
+        for (int m = 0; m < 2; ++m)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) part[wave][m][(4 * g + r) * MT_PAD + c] = acc[m][r];      // (row 4 g + r, pair c)
+        __syncthreads();
+        const int rr = threadIdx.x & 15, cc = threadIdx.x >> 4, at = rr * MT_PAD + cc;
+        if (m0 + cc < count && j0 + rr < ff) {
+            const float gs = part[0][0][at] + part[1][0][at] + part[2][0][at] + part[3][0][at];
+            const float us = part[0][1][at] + part[1][1][at] + part[2][1][at] + part[3][1][at];
+            y[(int64_t)list[m0 + cc] * ff + j0 + rr] = (A)glu_act((float)(A)gs, (float)(A)us, limit, alpha, shift);
+        }
+        __syncthreads();
+    }
+}
+
+template <typename A>
+__global__ __launch_bounds__(256) void moe_tile_down_kernel(const A* __restrict__ y, const int32_t* __restrict__ idx, int n_pairs,
+                                                           const A* __restrict__ w_d, float* __restrict__ o, int width, int ff) {
+    extern __shared__ int list[];                      // n_pairs
+    __shared__ float part[4][16 * MT_PAD];
+    const int e = blockIdx.y, j0 = blockIdx.x * 16;
+    const int count = pairs_of_expert(idx, n_pairs, e, list);
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, c = lane & 15, g = lane >> 4;
+    const int row = j0 + c < width ? j0 + c : width - 1;
+    const A* const rows[1] = {w_d + ((int64_t)e * width + row) * ff};
+    for (int m0 = 0; m0 < count; m0 += 16) {
+        const int pair = list[m0 + c < count ? m0 + c : count - 1];
+        nvx_f32x4 acc[1] = {{0.f, 0.f, 0.f, 0.f}};
+        moe_tile_sums<A, 1>(rows, y + (int64_t)pair * ff, 1.0f, false, ff, wave, g, acc);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) part[wave][(4 * g + r) * MT_PAD + c] = acc[0][r];
+        __syncthreads();
+        const int rr = threadIdx.x & 15, cc = threadIdx.x >> 4, at = rr * MT_PAD + cc;
+        if (m0 + cc < count && j0 + rr < width)
+            o[(int64_t)list[m0 + cc] * width + j0 + rr] = (float)(A)(part[0][at] + part[1][at] + part[2][at] + part[3][at]);
+        __syncthreads();
+    }
+}
+
+// out[t] = sum over a token's choices of (weight_out ? wts : 1) * o[pair]
+template <typename A>
+__global__ __launch_bounds__(256) void moe_pair_sum_kernel(const float* __restrict__ o, const float* __restrict__ wts, int top, int weight_out,
+                                                          A* __restrict__ out, int width) {
+    const int64_t t = blockIdx.y;
+    const int c = blockIdx.x * 256 + threadIdx.x;
+    if (c >= width) return;
+    float v = 0.f;
+    for (int k = 0; k < top; ++k) v += (weight_out ? wts[t * top + k] : 1.0f) * o[(t * top + k) * width + c];
+    st_f(out, t * (int64_t)width + c, v);
 }
 
 // xs[dst[r]] = wts[r] * h[r / top]  for every (token, choice) pair r: the experts' inputs in expert order
@@ -440,9 +574,24 @@ extern "C" int64_t nvx_moe_expert_rows_max_width(int64_t ff) {
 
 template <typename A>
 static void launch_moe_rows(const void* h, int64_t h_stride, const int32_t* idx, const float* wts, int top, const void* w_gu, const void* w_d,
-                            float limit, float alpha, float shift, int weight_out, float* ws, void* out, int64_t n_tok, int width, int ff,
+                            int n_exp, float limit, float alpha, float shift, int weight_out, float* ws, void* out, int64_t n_tok, int width, int ff,
                             hipStream_t s) {
     const bool vec = sizeof(A) == 2 && width % 8 == 0 && ff % 8 == 0 && nvx_aligned16(w_gu) && nvx_aligned16(w_d);
+    if constexpr (sizeof(A) == 2) {
+        const int64_t pairs = n_tok * top;
+        if (vec && h_stride % 8 == 0 && nvx_aligned16(h) && nvx_aligned16(ws) && pairs <= 8192 && n_exp <= 65535) {
+            A* y = reinterpret_cast<A*>(ws);
+            float* o = ws + pairs * ff;
+            const size_t lds = (size_t)pairs * sizeof(int);
+            hipLaunchKernelGGL(moe_tile_up_kernel<A>, dim3((unsigned)((ff + 15) / 16), (unsigned)n_exp), dim3(256), lds, s, (const A*)h, h_stride, idx, wts, top,
+                               (int)pairs, (const A*)w_gu, limit, alpha, shift, weight_out, y, width, ff);
+            hipLaunchKernelGGL(moe_tile_down_kernel<A>, dim3((unsigned)((width + 15) / 16), (unsigned)n_exp), dim3(256), lds, s, (const A*)y, idx, (int)pairs,
+                               (const A*)w_d, o, width, ff);
+            hipLaunchKernelGGL(moe_pair_sum_kernel<A>, dim3((unsigned)((width + 255) / 256), (unsigned)n_tok), dim3(256), 0, s, (const float*)o, wts, top, weight_out,
+                               (A*)out, width);
+            return;
+        }
+    }
     const dim3 up((unsigned)((ff + MOE_ROWS - 1) / MOE_ROWS), (unsigned)top, (unsigned)n_tok);
     const dim3 down((unsigned)((width + MOE_ROWS - 1) / MOE_ROWS), (unsigned)n_tok);
     if (vec) {
@@ -462,12 +611,12 @@ extern "C" int nvx_moe_expert_rows(const void* h, int64_t h_stride, int fmt, con
                                    const void* w_gu, const void* w_d, int64_t n_exp, float limit, float alpha, float shift, int weight_out,
                                    float* ws, void* out, int64_t n_tok, int64_t width, int64_t ff, nvx_stream_t stream) {
     NVX_REQUIRE(fmt >= 0 && fmt <= 2, NVX_EINVAL, "nvx_moe_expert_rows: fmt must be 0, 1 or 2");
-    NVX_REQUIRE(n_tok >= 0 && n_tok <= 65535 && top > 0 && top <= 65535 && n_exp > 0 && width > 0 && ff > 0 && h_stride >= width, NVX_EINVAL,
+    NVX_REQUIRE(n_tok >= 0 && n_tok <= 65535 && top > 0 && top <= 65535 && n_exp > 0 && n_exp < (1 << 20) && width > 0 && ff > 0 && h_stride >= width, NVX_EINVAL,
                 "nvx_moe_expert_rows: bad sizes (at most 65535 tokens a step)");
     NVX_REQUIRE(width <= nvx_moe_expert_rows_max_width(ff), NVX_EUNSUPPORTED, "nvx_moe_expert_rows: a row or the hidden size does not fit LDS");
     if (n_tok == 0) return NVX_OK;
     NVX_REQUIRE(h && idx && wts && w_gu && w_d && ws && out, NVX_EINVAL, "nvx_moe_expert_rows: null pointer");
-    NVX_FMT_CALL(fmt, launch_moe_rows<A_>(h, h_stride, idx, wts, (int)top, w_gu, w_d, limit, alpha, shift, weight_out, ws, out, n_tok, (int)width, (int)ff,
+    NVX_FMT_CALL(fmt, launch_moe_rows<A_>(h, h_stride, idx, wts, (int)top, w_gu, w_d, (int)n_exp, limit, alpha, shift, weight_out, ws, out, n_tok, (int)width, (int)ff,
                                           (hipStream_t)stream));
     return nvx_check_launch("nvx_moe_expert_rows");
 }

@@ -50,7 +50,7 @@ class ExpertBank(nn.Module):
     write them anew (the buffers end in ROW_STEP spare rows), so every row ends as its own expert's.  The library then sees a
     handful of row counts instead of a new one per expert, layer and step, which halves what a product's launch costs the host."""
 
-    ROWS_PATH_TOKENS = 32
+    ROWS_PATH_TOKENS = 32           # ... 64 in 16-bit formats, where an expert's rows serve up to 16 pairs at a time
     ROW_STEP = 64
 
     def __init__(self, width: int, experts: int, top: int, ff: int, limit: float, alpha: float, shift: float):
@@ -68,7 +68,7 @@ class ExpertBank(nn.Module):
             self._order_fit = ops.moe_order_fits(self.experts)      # more experts than the ordering kernel holds: pair by pair
             if not (self._rows_fit or self._order_fit):
                 raise NotImplementedError(f"{self.experts} experts of {self.ff} x {self.width}: neither expert path is built for these sizes")
-        return self._rows_fit and (decode_step or t <= self.ROWS_PATH_TOKENS or not self._order_fit)
+        return self._rows_fit and (decode_step or t <= (1 if self.w_gu.dtype == torch.float32 else 2) * self.ROWS_PATH_TOKENS or not self._order_fit)
 
     def run(self, h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, decode_step: bool, weight_out: bool, order=None) -> torch.Tensor:
         """`order` = (dst, counts as a list): the expert order of idx where the caller has it already (ops.moe_order)."""

@@ -1404,14 +1404,15 @@ def _moe_weights(w_gu, w_d, what: str):
 def moe_expert_rows(h, idx, wts, w_gu, w_d, limit: float, alpha: float, shift: float = 1.0, weight_out: bool = False):
     """out[t] = sum over token t's chosen experts of expert(score * h[t]) (or of score * expert(h[t]) if `weight_out`); w_gu
     (experts, 2 * ff, width) = gate | up rows, w_d (experts, width, ff); activation min(g, limit) sigmoid(alpha min(g, limit))
-    (clamp(u, +-limit) + shift).  The chosen experts' rows are streamed per (token, choice) pair: the form for steps of few tokens."""
+    (clamp(u, +-limit) + shift).  The form for steps of few tokens, without a host read: in 16-bit formats an expert's rows are read once for up to
+    16 of its (token, choice) pairs, else per pair."""
     _dev(h, idx, wts, w_gu, w_d)
     n_exp, ff, width = _moe_weights(w_gu, w_d, "moe_expert_rows")
     t, top = idx.shape
     _need(h.shape == (t, width) and h.stride(1) == 1 and h.dtype == w_gu.dtype, "moe_expert_rows: h shape / format")
     _need(idx.dtype == torch.int32 and idx.is_contiguous() and wts.dtype == F32 and wts.is_contiguous() and wts.shape == idx.shape, "moe_expert_rows: choices")
     out = torch.empty((t, width), dtype=h.dtype, device=h.device)
-    ws = torch.empty((t, top, ff), dtype=F32, device=h.device)      # the hidden activations between the two launches
+    ws = torch.empty((t * top * (ff + width),), dtype=F32, device=h.device)      # hidden activations and output rows between the launches
     lib = _lib.load()
     _lib.check(lib.nvx_moe_expert_rows(_ptr(h), h.stride(0), _fmt(h), _ptr(idx), _ptr(wts), top, _ptr(w_gu), _ptr(w_d), n_exp, float(limit),
                                        float(alpha), float(shift), int(bool(weight_out)), _ptr(ws), _ptr(out), t, width, ff, _stream()),

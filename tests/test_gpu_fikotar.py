@@ -195,7 +195,7 @@ def test_queries_keys_and_values_through_convolution_rotation_and_norm(fmt, head
 
 
 def test_long_walks_of_the_convolution_cross_sequences():
-    """A step of thousands of tokens, where a lane group walks eight tokens at a time over the borders of many short sequences."""
+    """A step of thousands of tokens, where a lane group walks several tokens at a time over the borders of many short sequences."""
     from nano_vllm_x_amd import ops
     g = torch.Generator().manual_seed(1)
     heads, kvh, dim, vdim, taps = 8, 4, 64, 64, 4
@@ -437,6 +437,35 @@ def test_shared_expert_hidden_rows_behind_their_gate(fmt, ff, t):
     want = torch.sigmoid(z[:, 4:].double()) * fo.silu(x[:, 8:8 + ff].double()) * x[:, 8 + ff:].double()
     near(wide[:, 8:8 + ff].float().cpu(), want, 1e-4 if fmt == torch.float32 else 1e-2)
     assert (wide[:, :8] == 3.0).all() and (wide[:, 8 + ff:] == 3.0).all()
+
+
+@pytest.mark.parametrize("fmt", [torch.bfloat16, torch.float32])
+@pytest.mark.parametrize("width,ff,n_exp,top,t", [(64, 48, 4, 2, 1), (72, 40, 3, 3, 37), (128, 16, 20, 2, 9), (520, 264, 2, 1, 50), (40, 8, 1, 1, 33), (36, 20, 5, 2, 6)])
+@pytest.mark.parametrize("weight_out", [True, False])
+def test_experts_of_a_step_of_few_tokens(fmt, width, ff, n_exp, top, t, weight_out):
+    """An expert that every token chooses (more pairs than a tile of 16 holds), experts nobody chooses, depths that end inside a block of 128
+    and inside 32, sizes without 16-byte rows; against the restatement on the same values, weights on the outputs and on the inputs;
+    a token's result is the same bits alone and beside others."""
+    from nano_vllm_x_amd import ops
+    g = torch.Generator().manual_seed(width + t)
+    h = torch.randn(t, width, generator=g).to(fmt)
+    w_gu, w_d = (torch.randn(n_exp, 2 * ff, width, generator=g) * width ** -0.5).to(fmt), (torch.randn(n_exp, width, ff, generator=g) * ff ** -0.5).to(fmt)
+    idx = torch.stack([torch.cat([torch.zeros(1, dtype=torch.long), 1 + torch.randperm(n_exp - 1, generator=g)[:top - 1] // 1]) if n_exp > 1 else torch.zeros(1, dtype=torch.long)
+                       for _ in range(t)])
+    wts = torch.rand(t, top, generator=g) + 0.1
+    rounded = lambda z: z.to(fmt).double()            # what a product hands on in the activations' format
+    want = torch.zeros(t, width, dtype=torch.float64)
+    for r in range(t):
+        for e, s in zip(idx[r].tolist(), wts[r]):
+            x = h[r].double() if weight_out else rounded(s * h[r].float())
+            hidden = rounded(fo.silu(rounded(w_gu[e, :ff].double() @ x)) * rounded(w_gu[e, ff:].double() @ x))
+            want[r] += (s.double() if weight_out else 1.0) * rounded(w_d[e].double() @ hidden)
+    args = [x.cuda() for x in (h, idx.to(torch.int32), wts, w_gu, w_d)]
+    got = ops.moe_expert_rows(*args, float("inf"), 1.0, 0.0, weight_out)
+    near(got.float().cpu(), want, 1e-3 if fmt == torch.float32 else 3e-2, "experts")
+    alone = torch.cat([ops.moe_expert_rows(args[0][r:r + 1], args[1][r:r + 1].contiguous(), args[2][r:r + 1].contiguous(), *args[3:], float("inf"), 1.0, 0.0, weight_out)
+                       for r in range(min(t, 5))])
+    assert torch.equal(alone, got[:len(alone)])
 
 
 # ---- one mechanism at a time ---------------------------------------------------------------------------------------------
