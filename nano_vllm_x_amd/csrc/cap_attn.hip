@@ -446,9 +446,10 @@ __global__ __launch_bounds__(256) void rows_attn_kernel(const A* __restrict__ q,
         slope[n] = slopes ? slopes[h] : 0.f;
         m[n] = -INFINITY;
         sum[n] = 0.f;
+        const vec8 qr = *reinterpret_cast<const vec8*>(q + (t * heads + h) * (int64_t)dim + (on ? l * 8 : 0));
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
-            qv[n][i] = on ? ld_f(q, (t * heads + h) * (int64_t)dim + l * 8 + i) * scale : 0.f;
+            qv[n][i] = on ? (float)qr[i] * scale : 0.f;
             acc[n][i] = 0.f;
         }
     }
@@ -1011,7 +1012,8 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
     NVX_REQUIRE(n_split >= 1 && n_split <= 64 && (n_split == 1 || part), NVX_EINVAL, "nvx_softcap_attn: a key split needs its workspace");
     // without what the kernel does not do: a row is read once for up to four heads
     const bool tied = k_rn && k_cache == v_cache && dim == vdim;
-    if ((tied || !k_rn) && dim % 8 == 0 && vdim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && nvx_aligned16(k_cache) && nvx_aligned16(v_cache)) {
+    if ((tied || !k_rn) && dim % 8 == 0 && vdim % 8 == 0 && dim <= 512 && cap <= 0.f && !r1 && !vcs && !gate && nvx_aligned16(q) && nvx_aligned16(k_cache) &&
+        nvx_aligned16(v_cache)) {
         const int per_kv = (int)(heads / kv_heads), nh = per_kv >= 4 ? 4 : (per_kv >= 2 ? 2 : 1);
         const dim3 tgrid((unsigned)(kv_heads * ((per_kv + nh - 1) / nh)), (unsigned)n_tok, (unsigned)n_split);
         const size_t tlds = (size_t)(4 * nh * vdim + 8 * nh) * sizeof(float);
@@ -1021,7 +1023,7 @@ extern "C" int nvx_softcap_attn(const void* q, const void* k_cache, const void* 
                                          (const A_*)q, (const A_*)k_cache, (const A_*)v_cache, k_rn, kv_indices, kv_start, kv_len, qo_indptr, tok_seq, scale, \
                                          (A_*)out, (int)heads, (int)kv_heads, (int)dim, (int)vdim, n_split, part, (int)window, (int)chunk, slopes, sink, \
                                          sink_score, sinks, (int)keep_first, out_mul, out_stride))
-#define NVX_ROWS_ATTN_L(NH, LPR) do { if (tied) NVX_ROWS_ATTN_T(NH, LPR, 8, true); else NVX_ROWS_ATTN_T(NH, LPR, 4, false); } while (0)
+#define NVX_ROWS_ATTN_L(NH, LPR) do { if (tied) NVX_ROWS_ATTN_T(NH, LPR, 8, true); else NVX_ROWS_ATTN_T(NH, LPR, (NH == 4 ? 4 : 8), false); } while (0)
 #define NVX_ROWS_ATTN(NH)                                 \
     do {                                                  \
         if (longest <= 64) NVX_ROWS_ATTN_L(NH, 8);        \

@@ -94,6 +94,47 @@ __device__ __forceinline__ void wave_best(float& v, int& i) {       // the large
         if (oi >= 0 && (i < 0 || ov > v || (ov == v && oi < i))) { v = ov; i = oi; }
     }
 }
+// The softmax router without groups, a wave per token (n_exp <= 1024): logits and choices stay in registers and lane exchanges.
+__global__ __launch_bounds__(256) void moe_route_softmax_wave_kernel(const float* __restrict__ logits, int64_t logits_stride, int n_exp, int top,
+                                                                    float norm_eps, int32_t* __restrict__ idx, float* __restrict__ wts, int64_t n_tok) {
+    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t >= n_tok) return;                                // (waves share nothing)
+    const int lane = threadIdx.x & 63;
+    float z[16];
+    float zmax = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+        z[i] = i * 64 + lane < n_exp ? logits[t * logits_stride + i * 64 + lane] : -INFINITY;
+        zmax = fmaxf(zmax, z[i]);
+    }
+    zmax = wave_max(zmax);
+    float denom = 0.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+        if (i * 64 < n_exp) denom += expf(z[i] - zmax);    // (past the last expert: exp(-inf) = 0)
+    denom = wave_sum(denom);
+    unsigned taken = 0;                                    // of this lane's experts
+    float sum = 0.f, mine = 0.f;
+    int mine_e = 0;
+    for (int k = 0; k < top; ++k) {
+        float v = -INFINITY;
+        int e = -1;
+#pragma unroll
+        for (int i = 0; i < 16; ++i)
+            if (i * 64 + lane < n_exp && !((taken >> i) & 1u) && (e < 0 || z[i] > v)) { v = z[i]; e = i * 64 + lane; }
+        wave_best(v, e);
+        if (e < 0) e = 0;
+        if (lane == (e & 63)) taken |= 1u << (e >> 6);
+        const float sc = expf(v - zmax) / denom;
+        sum += sc;
+        if (lane == (k & 63)) { mine = sc; mine_e = e; }   // (top <= 64: choice k is lane k's to write)
+    }
+    if (lane < top) {
+        idx[t * top + lane] = mine_e;
+        wts[t * top + lane] = mine / (sum + norm_eps);
+    }
+}
+
 __global__ __launch_bounds__(256) void moe_route_sigmoid_kernel(const float* __restrict__ logits, const float* __restrict__ correction, int n_exp,
                                                                int top, int n_groups, int keep_groups, float w_scale, int32_t* __restrict__ idx,
                                                                float* __restrict__ wts, int64_t n_tok) {
@@ -549,6 +590,11 @@ extern "C" int nvx_moe_route_softmax(const float* logits, int64_t logits_stride,
                 NVX_EINVAL, "nvx_moe_route_softmax: groups must divide the experts (at most 256 groups) and the kept groups must hold `top` experts");
     if (n_tok == 0) return NVX_OK;
     NVX_REQUIRE(logits && idx && wts && logits_stride >= n_exp, NVX_EINVAL, "nvx_moe_route_softmax: null pointer or row stride");
+    if ((n_groups <= 1 || keep_groups == n_groups) && n_exp <= 1024 && top <= 64) {
+        hipLaunchKernelGGL(moe_route_softmax_wave_kernel, dim3((unsigned)((n_tok + 3) / 4)), dim3(256), 0, (hipStream_t)stream, logits, logits_stride, (int)n_exp,
+                           (int)top, norm_eps, idx, wts, n_tok);
+        return nvx_check_launch("nvx_moe_route_softmax");
+    }
     hipLaunchKernelGGL(moe_route_softmax_kernel, dim3((unsigned)((n_tok + 255) / 256)), dim3(256), 0, (hipStream_t)stream, logits, logits_stride, (int)n_exp,
                        (int)top, (int)n_groups, (int)keep_groups, norm_eps, idx, wts, n_tok);
     return nvx_check_launch("nvx_moe_route_softmax");

@@ -500,11 +500,12 @@ __global__ __launch_bounds__(256) void rwkv_scan_kernel(const A* __restrict__ rx
 // the state at every chunk's start (and writes the sequence's final state), phase 3 walks every chunk from there with the read-out.
 // Because the decay is a constant, the carry over a chunk of n tokens is decay^n S + (the chunk's own contribution).  phase 0: one
 // workgroup walks the whole portion (single tokens, short portions).
+// A thread keeps NC value columns: the rows it reads from LDS then serve NC of them.
 // With `half` > 0 the pairs (m, m + half) of every staged query and key are rotated by the token's angles (turn), in float32, and keys are
 // multiplied by k_mul.
 // `tb` tokens are staged at a time: 32 where the key size leaves LDS for them (more than the other recurrences take: an activation
 // is applied as they are staged, and fewer, longer stages hide more of the loads), fewer for wide keys.
-template <typename A, int PHASE>
+template <typename A, int PHASE, int NC>
 __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x, int64_t x_stride, int q_off, int k_off, int v_off, int act,
                                                         const float* __restrict__ decay, float* __restrict__ S,
                                                         const int32_t* __restrict__ qo_indptr, const int64_t* __restrict__ pos0,
@@ -528,14 +529,16 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
         sp.n = sp.n - first < chunk ? sp.n - first : chunk;
     }
     const ScanThread th = scan_thread(p_lanes, vdim);
+    const int e0 = blockIdx.x * cb * NC + th.col;              // this thread's value columns: e0, e0 + cb, ...
     // where the state comes from and goes to: the pool (phase 0), nothing and ws (1), ws and nothing (3)
     float* Sp = phase ? ws + ((int64_t)blockIdx.z * heads + hd) * dim * vdim : S + ((int64_t)sp.slot * heads + hd) * dim * vdim;
-    float s[KR];
+    float s[NC][KR];
     const bool cont = phase == 3 || (phase == 0 && sp.pos0 > 0);
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
-        s[r] = (cont && row < dim && th.active) ? Sp[(int64_t)row * vdim + th.e] : 0.f;
+#pragma unroll
+        for (int n = 0; n < NC; ++n) s[n][r] = (cont && row < dim && e0 + n * cb < vdim) ? Sp[(int64_t)row * vdim + e0 + n * cb] : 0.f;
     }
     zero_rows(sq, 2 * tb * rs);
     const float g = decay[hd];
@@ -545,7 +548,7 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
         const A* xr = x + (sp.q0 + t0) * x_stride;
         if (phase != 1) stage_key_rows(sq, rs, xr + q_off + hd * dim, x_stride, nt, dim, vec, act);      // (phase 1 wants the state only)
         stage_key_rows(sk, rs, xr + k_off + hd * dim, x_stride, nt, dim, vec, act, k_mul);
-        stage_value_cols(sv, cb, xr + v_off + hd * vdim + blockIdx.x * cb, x_stride, nt, vdim - (int)blockIdx.x * cb, vec, act);
+        stage_value_cols(sv, cb * NC, xr + v_off + hd * vdim + blockIdx.x * cb * NC, x_stride, nt, vdim - (int)blockIdx.x * cb * NC, vec, act);
         __syncthreads();
         if (half) {
             for (int i = threadIdx.x; i < nt * half; i += blockDim.x) {
@@ -566,29 +569,39 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(const A* __restrict__ x
             __syncthreads();
         }
         for (int tt = 0; tt < nt; ++tt) {
-            const float v = sv[tt * cb + th.col];
+            float v[NC], o[NC];
+#pragma unroll
+            for (int n = 0; n < NC; ++n) { v[n] = sv[(tt * NC + n) * cb + th.col]; o[n] = 0.f; }
             const float* kk = sk + tt * rs + th.p * KS;
             const float* qq = sq + tt * rs + th.p * KS;
             if (phase == 1) {
 #pragma unroll
-                for (int r = 0; r < KR; ++r) s[r] = g * s[r] + kk[r] * v;
+                for (int r = 0; r < KR; ++r)
+#pragma unroll
+                    for (int n = 0; n < NC; ++n) s[n][r] = g * s[n][r] + kk[r] * v[n];
                 continue;
             }
-            float o = 0.f;
 #pragma unroll
-            for (int r = 0; r < KR; ++r) {
-                s[r] = g * s[r] + kk[r] * v;
-                o += s[r] * qq[r];
+            for (int r = 0; r < KR; ++r)
+#pragma unroll
+                for (int n = 0; n < NC; ++n) {
+                    s[n][r] = g * s[n][r] + kk[r] * v[n];
+                    o[n] += s[n][r] * qq[r];
+                }
+#pragma unroll
+            for (int n = 0; n < NC; ++n) {
+                const float sum = lanes_sum(o[n], p_lanes);
+                if (th.p == 0 && e0 + n * cb < vdim) out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + e0 + n * cb] = sum;
             }
-            o = lanes_sum(o, p_lanes);
-            if (th.p == 0 && th.active) out[(sp.q0 + t0 + tt) * (int64_t)heads * vdim + (int64_t)hd * vdim + th.e] = o;
         }
     }
     if (phase == 3) return;
 #pragma unroll
     for (int r = 0; r < KR; ++r) {
         const int row = th.r0 + r;
-        if (row < dim && th.active) Sp[(int64_t)row * vdim + th.e] = s[r];
+#pragma unroll
+        for (int n = 0; n < NC; ++n)
+            if (row < dim && e0 + n * cb < vdim) Sp[(int64_t)row * vdim + e0 + n * cb] = s[n][r];
     }
 }
 
@@ -702,14 +715,24 @@ __global__ __launch_bounds__(256) void decay_chunk_carry_kernel(const float* __r
     const float g = decay[i / ((int64_t)dim * vdim)];
     float* Sp = S + (int64_t)sp.slot * per + i;
     float run = sp.pos0 > 0 ? *Sp : 0.f;
-    for (int ck = 0; (int64_t)ck * chunk < sp.n; ++ck) {
-        const int64_t n = sp.n - (int64_t)ck * chunk < chunk ? sp.n - (int64_t)ck * chunk : chunk;
-        float* w = ws + ((int64_t)blockIdx.y * n_chunk_max + ck) * per + i;
-        const float own = *w;
-        *w = run;
-        float gn = 1.f;
-        for (int64_t k = 0; k < n; ++k) gn *= g;     // the same products, in the same order, as n steps of the recurrence
-        run = gn * run + own;
+    float* w = ws + (int64_t)blockIdx.y * n_chunk_max * per + i;
+    const int n_chunks = (int)((sp.n + chunk - 1) / chunk), last = (int)(sp.n - (int64_t)(n_chunks - 1) * chunk);
+    float g_chunk = 1.f, g_last = 1.f;               // decay over a chunk: the same products, in the same order, as that many steps of the recurrence
+    for (int k = 0; k < chunk; ++k) {
+        g_chunk *= g;
+        if (k + 1 == last) g_last = g_chunk;
+    }
+    constexpr int U = 8;                             // chunks whose contributions are asked for together
+    for (int c0 = 0; c0 < n_chunks; c0 += U) {
+        float own[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) own[u] = c0 + u < n_chunks ? w[(c0 + u) * per] : 0.f;
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            if (c0 + u >= n_chunks) continue;
+            w[(c0 + u) * per] = run;
+            run = (c0 + u + 1 == n_chunks ? g_last : g_chunk) * run + own[u];
+        }
     }
     *Sp = run;
 }
@@ -988,24 +1011,28 @@ extern "C" int nvx_decay_scan(const void* x, int64_t x_stride, int fmt, int64_t 
     NVX_REQUIRE(x && decay && S && out, NVX_EINVAL, "nvx_decay_scan: null pointer");
     NVX_REQUIRE(q_off >= 0 && k_off >= 0 && v_off >= 0 && x_stride >= q_off + heads * dim && x_stride >= k_off + heads * dim &&
                     x_stride >= v_off + heads * vdim, NVX_EINVAL, "nvx_decay_scan: q, k or v lies outside a row");
+    const int nc = chunk && vdim > 1 ? 2 : 1;      // value columns per thread: a staged row then serves two of them
+    NVX_REQUIRE(scan_launch(dim, (vdim + nc - 1) / nc, &g), NVX_EUNSUPPORTED, "nvx_decay_scan: key size above 512");
     const int tb = g.p_lanes <= 4 ? 32 : (g.p_lanes == 8 ? 16 : TB);
-    const size_t lds = (size_t)(2 * tb * g.p_lanes * KS + tb * g.cb) * sizeof(float);
+    const size_t lds = (size_t)(2 * tb * g.p_lanes * KS + tb * g.cb * nc) * sizeof(float);
     NVX_REQUIRE(chunk == 0 || (chunk > 0 && chunk < (1 << 30) && n_chunk_max > 0 && n_seq * n_chunk_max <= 65535 && ws && qo_indptr), NVX_EINVAL,
                 "nvx_decay_scan: chunks need a ragged step, their workspace, and at most 65535 of them");
-    const dim3 grid((unsigned)((vdim + g.cb - 1) / g.cb), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
-#define NVX_DECAY_SCAN(PHASE)                                                                                                                      \
-    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((decay_scan_kernel<A_, PHASE>), grid, dim3(g.threads), lds, (hipStream_t)stream, (const A_*)x, x_stride,   \
+    const dim3 grid((unsigned)((vdim + g.cb * nc - 1) / (g.cb * nc)), (unsigned)heads, (unsigned)(chunk ? n_seq * n_chunk_max : n_seq));
+#define NVX_DECAY_SCAN(PHASE, NC)                                                                                                                   \
+    NVX_FMT_CALL(fmt, hipLaunchKernelGGL((decay_scan_kernel<A_, PHASE, NC>), grid, dim3(g.threads), lds, (hipStream_t)stream, (const A_*)x, x_stride,   \
                                          (int)q_off, (int)k_off, (int)v_off, act, decay, S, qo_indptr, pos0, state_slot, out, (int)heads, (int)dim,  \
-                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb), (int)chunk, (int)n_chunk_max, ws, tr, \
+                                         (int)vdim, g.p_lanes, tb, (int)stage_vec_ok<A_>(x, x_stride, q_off, k_off, v_off, dim, vdim, g.cb * nc), (int)chunk, (int)n_chunk_max, ws, tr, \
                                          rot_dims / 2, k_mul))
     if (!chunk) {
-        NVX_DECAY_SCAN(0);
+        NVX_DECAY_SCAN(0, 1);
     } else {
-        NVX_DECAY_SCAN(1);
+        if (nc == 2) NVX_DECAY_SCAN(1, 2);
+        else NVX_DECAY_SCAN(1, 1);
         hipLaunchKernelGGL(decay_chunk_carry_kernel, dim3((unsigned)((heads * dim * vdim + 255) / 256), (unsigned)n_seq), dim3(256), 0,
                            (hipStream_t)stream, decay, S, ws, qo_indptr, pos0, state_slot, (int)heads, (int)dim, (int)vdim, (int)chunk,
                            (int)n_chunk_max);
-        NVX_DECAY_SCAN(3);
+        if (nc == 2) NVX_DECAY_SCAN(3, 2);
+        else NVX_DECAY_SCAN(3, 1);
     }
 #undef NVX_DECAY_SCAN
     return nvx_check_launch("nvx_decay_scan");

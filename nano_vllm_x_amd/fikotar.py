@@ -136,17 +136,18 @@ class FikotarLayer(nn.Module):
 
     def forward(self, h: torch.Tensor, turns: TurnTables, table, md, decode_step: bool):
         """(mixers and shared expert, experts or None): what the stream takes up behind this layer."""
+        z = plan = None
+        if self.moe is not None:      # first of all: the experts' counts reach the host while the mixers run
+            z = ops.skinny_proj(h, self.moe.router)
+            plan = self.moe.plan(z[:, :self.moe.experts], decode_step)
         x, at, to = self.in_proj(h), self.in_at, self.out_at
         o = torch.empty((h.shape[0], to[-1]), dtype=h.dtype, device=h.device)
         self.left.attend(x, at[0], turns.at(table, self.left.rot_key), md, o[:, to[0]:to[1]])
         self.right.mix(x, at[1], turns.at(table, self.right.rot_key), md, o[:, to[1]:to[2]])
-        y2 = None
-        if self.moe is not None:
-            z = ops.skinny_proj(h, self.moe.router)
-            if self.shared is not None:
-                self.shared.hidden(x, at[2], z[:, self.moe.experts], o[:, to[2]:to[3]])
-            y2 = self.moe(h, decode_step, logits=z[:, :self.moe.experts])
-        return self.out_proj(o), y2
+        if self.shared is not None:
+            self.shared.hidden(x, at[2], z[:, self.moe.experts], o[:, to[2]:to[3]])
+        y = self.out_proj(o)
+        return y, self.moe(h, decode_step, plan=plan) if self.moe is not None else None
 
 
 class FikotarForCausalLM(nn.Module):

@@ -60,6 +60,25 @@ class ExpertBank(nn.Module):
         self.w_gu = nn.Parameter(torch.empty(experts, 2 * ff, width))      # rows of an expert: gate | up
         self.w_d = nn.Parameter(torch.empty(experts, width, ff))
         self._rows_fit = None
+        self._counts_host = self._counts_ready = None
+
+    def order_ahead(self, idx: torch.Tensor, decode_step: bool):
+        """The expert order of a step's choices, asked for ahead of other work: (dst, function that gives the counts), or None for a step that
+        needs none.  The counts travel to the host behind the order kernel; what the caller queues between this call and `run` keeps
+        the device busy, so that reading them there waits for the order alone and not for an idle device."""
+        if self.by_rows(idx.shape[0], decode_step):
+            return None
+        if self._counts_host is None:
+            self._counts_host = torch.empty(self.experts, dtype=torch.int32, pin_memory=True)
+            self._counts_ready = torch.cuda.Event()
+        dst, counts = ops.moe_order(idx, self.experts)
+        self._counts_host.copy_(counts, non_blocking=True)
+        self._counts_ready.record()
+
+        def read():
+            self._counts_ready.synchronize()
+            return self._counts_host.tolist()
+        return dst, read
 
     def by_rows(self, t: int, decode_step: bool) -> bool:
         """Whether a step of t tokens streams the chosen experts' rows (else: per-expert products over the expert order)."""
@@ -71,7 +90,8 @@ class ExpertBank(nn.Module):
         return self._rows_fit and (decode_step or t <= (1 if self.w_gu.dtype == torch.float32 else 2) * self.ROWS_PATH_TOKENS or not self._order_fit)
 
     def run(self, h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, decode_step: bool, weight_out: bool, order=None) -> torch.Tensor:
-        """`order` = (dst, counts as a list): the expert order of idx where the caller has it already (ops.moe_order)."""
+        """`order` = (dst, counts as a list, or a function that gives them): the expert order of idx where the caller has it already
+        (ops.moe_order, order_ahead)."""
         t = h.shape[0]
         if self.by_rows(t, decode_step):
             return ops.moe_expert_rows(h, idx, wts, self.w_gu, self.w_d, self.limit, self.alpha, self.shift, weight_out)
@@ -80,6 +100,8 @@ class ExpertBank(nn.Module):
             counts = counts.tolist()
         else:
             dst, counts = order
+            if callable(counts):
+                counts = counts()
         step = self.ROW_STEP
         xs = ops.moe_scatter_rows(h, None if weight_out else wts, dst, spare_rows=step)
         spans, a = [], 0
@@ -173,10 +195,16 @@ class GroupedSoftmaxMoE(ExpertBank):
         self.norm_eps = float(norm_eps)
         self.router = nn.Parameter(torch.zeros(experts, width, dtype=torch.float32))
 
-    def forward(self, h: torch.Tensor, decode_step: bool = False, logits=None) -> torch.Tensor:
-        """`logits` (T, experts): the router's, where the caller has made them beside other numbers per token."""
-        idx, wts = ops.moe_route_softmax(ops.skinny_proj(h, self.router) if logits is None else logits, self.top, self.groups, self.keep, self.norm_eps)
-        return self.run(h, idx, wts, decode_step, weight_out=True)
+    def plan(self, logits: torch.Tensor, decode_step: bool) -> dict:
+        """A step's choices and their expert order from the router's logits (T, experts), ahead of `forward`."""
+        idx, wts = ops.moe_route_softmax(logits, self.top, self.groups, self.keep, self.norm_eps)
+        return {"idx": idx, "wts": wts, "order": self.order_ahead(idx, decode_step)}
+
+    def forward(self, h: torch.Tensor, decode_step: bool = False, plan=None) -> torch.Tensor:
+        if plan is None:
+            idx, wts = ops.moe_route_softmax(ops.skinny_proj(h, self.router), self.top, self.groups, self.keep, self.norm_eps)
+            return self.run(h, idx, wts, decode_step, weight_out=True)
+        return self.run(h, plan["idx"], plan["wts"], decode_step, weight_out=True, order=plan["order"])
 
 
 class GatedSharedExpert(nn.Module):

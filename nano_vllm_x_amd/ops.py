@@ -979,9 +979,9 @@ def token_shift_mix(h, mu, state, layout: StepLayout):
 
 
 SCAN_CHUNK_FROM = 256       # portions from this length on are cut into chunks that run side by side
-SCAN_CHUNKS = ((65536, 32), (131072, 64), (None, 128))      # (tokens x heads of a step up to ..., tokens of a chunk): short chunks while
-# the step is too small to fill the chip with long ones, long chunks (fewer carried states) from there on (4 x 1 024 tokens, 8
-# heads: 895 us in one walk, 301 in chunks of 128, 150 in chunks of 32; 16 x 1 024 tokens: 446 us at 128 and 64, 474 at 32)
+SCAN_CHUNKS = ((49152, 32), (98304, 64), (None, 128))      # (tokens x heads of a step up to ..., tokens of a chunk): short chunks while
+# the step is too small to fill the chip with long ones, long chunks (fewer carried states) from there on (4 x 1 024 tokens: 8 heads 97 us
+# at 32, 151 at 64, 267 at 128; 16 heads 238, 164, 287; 32 heads 400, 418, 302)
 GLA_SCAN_CHUNKS = ((32768, 32), (None, 64))       # (4 x 1 024 tokens: 8 heads 116 us at 32, 164 at 64; 16 heads 222 and 178)
 MLSTM_SCAN_CHUNKS = ((None, 64),)                 # (the same: 191 and 167; 312 and 291; one walk per portion: 1 420)
 SCAN_WS_BYTES = 1 << 30     # the chunks' states may take this much; longer chunks otherwise
